@@ -1,8 +1,9 @@
 // Attention of single tokens over the paged cache in bfloat16, split over the keys.
 // Compiled for one head size: -DNHV_HEAD_DIM=<multiple of 16>.
 //
-// One wave works on (token, key/value head, split of the keys). The G query heads
-// that share the key/value head (G <= 16) are the 16 columns of the MFMA tiles:
+// One wave works on (token, key/value head, up to 16 of the query heads that share it, split of
+// the keys). The query heads are the 16 columns of the MFMA tiles (more than 16 heads on one
+// key/value head, as over a cached latent, are several waves that read the same keys):
 //   S^T[key, head]  = K[key, :] . Q[head, :]        K rows straight from the cache (v_mfma_f32_16x16x32_bf16)
 //   running maximum per head in float (two shuffles), sums kept per lane
 //   O^T[d, head]   += V^T[d, key] . P^T[key, head]   V^T from the wave's own LDS tile, P in registers
@@ -17,9 +18,11 @@
 // float; a second kernel merges the splits in rising order. Keys that are not visible
 // are loaded as zeros (the cache's unused slots may hold anything).
 // What a layer may ask for besides (the entry point ..._more): a cap on the scores (s <- cap tanh(s / cap), after the
-// scale; taken on the float scores where they leave the first product), one more term exp(sink) in the softmax's
-// denominator (it joins in the merge, as a split without values would) and a gate per (token, head) whose sigmoid
-// multiplies the head's result (in the merge, with the division by the sum).
+// scale; taken on the float scores where they leave the first product), a bias that grows with the distance (BIASED:
+// slopes[head] * (query position - key position) is taken off the float score after scale and cap), one more term
+// exp(sink) in the softmax's denominator (one score for the layer or one per head; it joins in the merge, as a split
+// without values would) and a gate per (token, head) whose sigmoid multiplies the head's result (in the merge, with the
+// division by the sum).
 #include "nhv_common.h"
 #include "nhv_no_alloc.h"
 #include <math.h>
@@ -63,12 +66,13 @@ __device__ __forceinline__ int slot_of(const int* bt, int key, int page_size, in
 
 // CAPPED: the scores pass cap tanh(s scale / cap). cap_l2 = cap log2(e); tanh_k = 2 log2(e) scale / cap, so that
 // tanh(x) = 1 - 2 / (1 + exp(2 x)) costs one exp2 and one reciprocal (an overflowing exp2 gives the limit 1).
-template <bool CAPPED>
+template <bool CAPPED, bool BIASED>
 __global__ __launch_bounds__(64) void decode_attention_kernel(
     const bf16_t* __restrict__ q, const bf16_t* __restrict__ k_cache, const bf16_t* __restrict__ v_cache,
     float* __restrict__ part_o, float* __restrict__ part_ml, const int* __restrict__ token_req,
     const int* __restrict__ positions, const int* __restrict__ block_tables, int max_blocks, int Hq, int Hkv,
-    int page_size, int page_shift, float scale_log2e, int window, int split_len, int n_splits, float cap_l2, float tanh_k) {
+    int page_size, int page_shift, float scale_log2e, int window, int split_len, int n_splits, float cap_l2, float tanh_k,
+    const float* __restrict__ slopes) {
   __shared__ __attribute__((aligned(16))) bf16_t vt_s[D * VPITCH];
   const int lane = threadIdx.x;
   // blocks go to the eight XCDs in turn by their linear index: with the split as the slowest index every XCD
@@ -78,8 +82,11 @@ __global__ __launch_bounds__(64) void decode_attention_kernel(
   // 2 D Hkv bytes of a page, and an XCD that read one and the same head for every token took 4 to 5 % longer at
   // 32 and 64 requests (116 against 111 us at 64) than one whose blocks go over all heads
   const int t = blockIdx.y, split = blockIdx.z;
-  const int kvh = (int)((blockIdx.x + blockIdx.y + blockIdx.z) % gridDim.x);
-  const int G = Hq / Hkv;
+  const int group = (int)((blockIdx.x + blockIdx.y + blockIdx.z) % gridDim.x);
+  const int per_kv = (int)gridDim.x / Hkv;         // groups of up to 16 query heads on one key/value head
+  const int kvh = group / per_kv;
+  const int head0 = kvh * (Hq / Hkv) + (group % per_kv) * 16;                  // this wave's query heads: head0 + (0 .. G - 1)
+  const int G = min(16, Hq / Hkv - (group % per_kv) * 16);
   const int pos = positions[t];
   const int lo = nhv_first_key(pos, window);
   const int first = max(lo, split * split_len);
@@ -93,9 +100,10 @@ __global__ __launch_bounds__(64) void decode_attention_kernel(
 #pragma unroll
   for (int s = 0; s < DSTEPS; ++s) {
     const int d = s * 32 + grp * 8;
-    qb[s] = (col < G && d < D) ? load8(q + ((size_t)t * Hq + kvh * G + col) * D + d) : zero8();
+    qb[s] = (col < G && d < D) ? load8(q + ((size_t)t * Hq + head0 + col) * D + d) : zero8();
   }
 
+  const float slope_l2 = BIASED && col < G ? slopes[head0 + col] * 1.4426950408889634f : 0.f;
   float m_run = -INFINITY, l_part = 0.f;     // of head `col` (base 2); l_part is this lane's share of the sum
   floatx4 o[DTILES];                          // o[dt][j]: entry dt * 16 + 4 grp + j of head `col`
 #pragma unroll
@@ -171,6 +179,7 @@ __global__ __launch_bounds__(64) void decode_attention_kernel(
         float scaled = s4[kt][j] * scale_log2e;
         if (CAPPED)
           scaled = __builtin_fmaf(-2.0f * cap_l2, __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(s4[kt][j] * tanh_k)), cap_l2);
+        if (BIASED) scaled = __builtin_fmaf(slope_l2, (float)(key - pos), scaled);
         const float v = (key >= first && key <= last) ? scaled : -INFINITY;
         s4[kt][j] = v;
         m_tile = fmaxf(m_tile, v);
@@ -229,7 +238,7 @@ __global__ __launch_bounds__(64) void decode_attention_kernel(
   l_part += __shfl_xor(l_part, 16, 64);
   l_part += __shfl_xor(l_part, 32, 64);
   if (col < G) {
-    const size_t item = ((size_t)t * Hq + kvh * G + col) * n_splits + split;
+    const size_t item = ((size_t)t * Hq + head0 + col) * n_splits + split;
     if (grp == 0) {
       part_ml[item * 2] = m_run;
       part_ml[item * 2 + 1] = l_part;
@@ -254,7 +263,7 @@ template <int W>
 __global__ __launch_bounds__(64 * W) void merge_splits_kernel(const float* __restrict__ part_o, const float* __restrict__ part_ml,
                                                               bf16_t* __restrict__ out, const int* __restrict__ positions,
                                                               int window, int split_len, int n_splits, int Hq, float sink_l2,
-                                                              const bf16_t* __restrict__ gate, long long gate_ld) {
+                                                              const float* __restrict__ sinks, const bf16_t* __restrict__ gate, long long gate_ld) {
   __shared__ float4 sum_s[W > 1 ? W - 1 : 1][MPIECES][64];
   const int item = blockIdx.x;               // t * Hq + h
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
@@ -270,6 +279,7 @@ __global__ __launch_bounds__(64 * W) void merge_splits_kernel(const float* __res
   m = wave_max(m);
   float l = 0.f;
   for (int s = s0 + lane; s <= s1; s += 64) l += ml[s * 2 + 1] * exp2f(ml[s * 2] - m);
+  if (sinks) sink_l2 = sinks[item % Hq] * 1.4426950408889634f;
   l = wave_sum(l) + exp2f(sink_l2 - m);       // (no sink: sink_l2 is -inf and the term 0)
   float inv = 1.0f / l;
   if (gate) inv /= 1.0f + expf(-(float)gate[(size_t)t * gate_ld + item % Hq]);
@@ -336,7 +346,7 @@ __global__ __launch_bounds__(64 * W) void merge_splits_at_once_kernel(const floa
                                                                       const float* __restrict__ part_ml,
                                                                       bf16_t* __restrict__ out, const int* __restrict__ positions,
                                                                       int window, int split_len, int n_splits, int Hq, float sink_l2,
-                                                                      const bf16_t* __restrict__ gate, long long gate_ld) {
+                                                                      const float* __restrict__ sinks, const bf16_t* __restrict__ gate, long long gate_ld) {
   __shared__ float4 sum_s[W > 1 ? W - 1 : 1][MPIECES][64];
   __shared__ float ml_s[W > 1 ? W - 1 : 1][2];
   const int item = blockIdx.x;               // t * Hq + h
@@ -423,6 +433,7 @@ __global__ __launch_bounds__(64 * W) void merge_splits_at_once_kernel(const floa
     }
   }
   if (sub == 0) {
+    if (sinks) sink_l2 = sinks[item % Hq] * 1.4426950408889634f;
     l += exp2f(sink_l2 - m_final);                         // (no sink: sink_l2 is -inf and the term 0)
     float inv = 1.0f / l;
     if (gate) inv /= 1.0f + expf(-(float)gate[(size_t)(item / Hq) * gate_ld + item % Hq]);
@@ -445,25 +456,29 @@ static int launch_decode_attention(const void* q, const void* k_cache, const voi
                                    float* part_ml, const void* token_req, const void* positions,
                                    const void* block_tables, int max_blocks, int T, int Hq, int Hkv, int page_size,
                                    float scale, int window, int split_len, int n_splits, hipStream_t s, float cap = 0.f,
-                                   int has_sink = 0, float sink = 0.f, const void* gate = nullptr, long long gate_ld = 0) {
+                                   int has_sink = 0, float sink = 0.f, const void* sinks = nullptr, const void* slopes = nullptr,
+                                   const void* gate = nullptr, long long gate_ld = 0) {
   int page_shift = -1;
   for (int b = 0; b < 31; ++b)
     if (page_size == (1 << b)) page_shift = b;
-  dim3 grid(Hkv, T, n_splits);
+  dim3 grid(Hkv * ((Hq / Hkv + 15) / 16), T, n_splits);
   const float log2e = 1.4426950408889634f;
-#define NHV_DECODE_LAUNCH(CAPPED_)                                                                                    \
-  hipLaunchKernelGGL(decode_attention_kernel<CAPPED_>, grid, dim3(64), 0, s, (const bf16_t*)q, (const bf16_t*)k_cache, \
+#define NHV_DECODE_LAUNCH(CAPPED_, BIASED_)                                                                           \
+  hipLaunchKernelGGL((decode_attention_kernel<CAPPED_, BIASED_>), grid, dim3(64), 0, s, (const bf16_t*)q, (const bf16_t*)k_cache, \
                      (const bf16_t*)v_cache, part_o, part_ml, (const int*)token_req,                                  \
                      (const int*)positions, (const int*)block_tables, max_blocks, Hq, Hkv, page_size, page_shift,     \
-                     scale * log2e, window, split_len, n_splits, cap * log2e, cap > 0.f ? 2.0f * log2e * scale / cap : 0.f)
-  if (cap > 0.f) NHV_DECODE_LAUNCH(true);
-  else NHV_DECODE_LAUNCH(false);
+                     scale * log2e, window, split_len, n_splits, cap * log2e, cap > 0.f ? 2.0f * log2e * scale / cap : 0.f, \
+                     (const float*)slopes)
+  if (cap > 0.f && slopes) NHV_DECODE_LAUNCH(true, true);
+  else if (cap > 0.f) NHV_DECODE_LAUNCH(true, false);
+  else if (slopes) NHV_DECODE_LAUNCH(false, true);
+  else NHV_DECODE_LAUNCH(false, false);
 #undef NHV_DECODE_LAUNCH
   NHV_LAUNCH_CHECK("decode_attention");
   const unsigned items = (unsigned)((size_t)T * Hq);
   const float sink_l2 = has_sink ? sink * log2e : -INFINITY;
 #define NHV_MERGE_ARGS (const float*)part_o, (const float*)part_ml, (bf16_t*)out, (const int*)positions, window, split_len, n_splits, Hq, \
-                       sink_l2, (const bf16_t*)gate, gate_ld
+                       sink_l2, (const float*)sinks, (const bf16_t*)gate, gate_ld
 #define NHV_MERGE_AT_ONCE(W_, NL_) \
   hipLaunchKernelGGL((merge_splits_at_once_kernel<W_, NL_>), dim3(items), dim3(64 * W_), 0, s, NHV_MERGE_ARGS)
   // few splits: everything asked for at once, by four waves from the point where one wave's lanes would take more
@@ -489,10 +504,8 @@ static int check_decode_attention(int max_blocks, int T, int Hq, int Hkv, int pa
                                   int n_splits) {
   NHV_REQUIRE(T > 0 && Hq > 0 && Hkv > 0 && page_size > 0 && max_blocks > 0, "decode attention: bad sizes");
   NHV_REQUIRE(Hq % Hkv == 0, "decode attention: %d query heads are not a multiple of %d key heads", Hq, Hkv);
-  const int G = Hq / Hkv;
-  NHV_REQUIRE(G <= 16, "decode attention: %d query heads per key head are beyond this kernel's limit of 16", G);
   NHV_REQUIRE(split_len > 0 && split_len % RK == 0, "decode attention: split length %d must be a multiple of %d", split_len, RK);
-  NHV_REQUIRE(n_splits > 0 && n_splits <= 65535 && Hkv <= 65535 && T <= 65535, "decode attention: grid too large");
+  NHV_REQUIRE(n_splits > 0 && n_splits <= 65535 && Hq <= 65535 && T <= 65535, "decode attention: grid too large");
   return 0;
 }
 
@@ -508,18 +521,20 @@ extern "C" int nhv_decode_attention_bf16(const void* q, const void* k_cache, con
                                  (hipStream_t)stream);
 }
 
-// The same with a cap on the scores (0: none), one more term exp(sink) in the denominator (has_sink) and a gate per
+// The same with a cap on the scores (0: none), one more term exp(sink) in the denominator (has_sink: sink; sinks: one
+// float per head in its place; null: none), a bias by distance (slopes: one float per head; null: none) and a gate per
 // (token, head): gate[t * gate_ld + h] in bfloat16, whose sigmoid multiplies the head's result (null: none).
 extern "C" int nhv_decode_attention_bf16_more(const void* q, const void* k_cache, const void* v_cache, void* out, void* part_o,
                                               void* part_ml, const void* token_req, const void* positions,
                                               const void* block_tables, int max_blocks, int T, int Hq, int Hkv, int page_size,
                                               float scale, int window, int split_len, int n_splits, float cap, int has_sink,
-                                              float sink, const void* gate, long long gate_ld, void* stream) {
+                                              float sink, const void* sinks, const void* slopes, const void* gate, long long gate_ld,
+                                              void* stream) {
   if (check_decode_attention(max_blocks, T, Hq, Hkv, page_size, window, split_len, n_splits)) return 1;
   NHV_REQUIRE(cap >= 0.f && (!gate || gate_ld >= Hq), "decode attention: cap %g, gate rows %lld apart for %d heads", (double)cap, gate_ld, Hq);
   return launch_decode_attention(q, k_cache, v_cache, out, (float*)part_o, (float*)part_ml, token_req, positions,
                                  block_tables, max_blocks, T, Hq, Hkv, page_size, scale, window, split_len, n_splits,
-                                 (hipStream_t)stream, cap, has_sink, sink, gate, gate_ld);
+                                 (hipStream_t)stream, cap, has_sink, sink, sinks, slopes, gate, gate_ld);
 }
 
 // ---- the entry point that allocates nothing (nhv_no_alloc.h) ----

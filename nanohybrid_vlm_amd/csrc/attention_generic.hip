@@ -7,9 +7,11 @@
 // start of the request), else 0. Value heads may have another size (E) than key heads (D).
 // Keys are taken in blocks of 64 aligned to absolute positions, always in rising
 // order, so the result for a position does not depend on the batch or the portion.
-// Options that a layer may name: a cap on the scores (s <- cap tanh(s / cap), after the scale), one more term in the
-// softmax's denominator (a sink: a key of a given score that has no value), and a gate per (token, head) whose
-// sigmoid multiplies the head's result (read from rows ``gate_ld`` entries apart).
+// Options that a layer may name: a cap on the scores (s <- cap tanh(s / cap), after the scale), a bias that grows with
+// the distance (slopes[h] * (p - key position) is taken off the score after scale and cap), one more term in the
+// softmax's denominator (a sink: a key of a given score that has no value; one score for the layer, or one per head in
+// ``sinks``), and a gate per (token, head) whose sigmoid multiplies the head's result (read from rows ``gate_ld``
+// entries apart).
 // This is the attention of the 32-bit path and the fallback of the bfloat16 path.
 #include "nhv_common.h"
 #include <math.h>
@@ -21,7 +23,8 @@ __global__ __launch_bounds__(256) void paged_attention_generic_kernel(
     const T* __restrict__ q, const T* __restrict__ k_cache, const T* __restrict__ v_cache, T* __restrict__ out,
     const int* __restrict__ token_req, const int* __restrict__ positions, const int* __restrict__ block_tables,
     int max_blocks, int n_items, int Hq, int Hkv, int D, int E, int page_size, float scale, int window, int chunk,
-    float cap, int has_sink, float sink, const T* __restrict__ gate, long long gate_ld) {
+    float cap, int has_sink, float sink, const float* __restrict__ sinks, const float* __restrict__ slopes,
+    const T* __restrict__ gate, long long gate_ld) {
   extern __shared__ float q_s[];            // 4 waves x D floats
   const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
   const int item = blockIdx.x * 4 + wave;
@@ -58,6 +61,7 @@ __global__ __launch_bounds__(256) void paged_attention_generic_kernel(
       for (int d = 0; d < D; ++d) dot = fmaf(qs[d], to_f32(kr[d]), dot);
       s = dot * scale;
       if (cap > 0.f) s = cap * tanhf(s / cap);
+      if (slopes) s = fmaf(-slopes[h], (float)(pos - kp), s);
     }
     const float m_new = fmaxf(m, wave_max(s));     // finite: every block holds at least one visible key
     const float alpha = expf(m - m_new);           // 0 on the first block
@@ -79,7 +83,8 @@ __global__ __launch_bounds__(256) void paged_attention_generic_kernel(
       }
     }
   }
-  if (has_sink) {                                  // the sink joins the denominator as one more key would, without a value
+  if (sinks) sink = sinks[h];
+  if (has_sink || sinks) {                         // the sink joins the denominator as one more key would, without a value
     const float m_new = fmaxf(m, sink);
     const float alpha = expf(m - m_new);
     l = l * alpha + expf(sink - m_new);
@@ -100,7 +105,8 @@ extern "C" int nhv_paged_attention_generic(const void* q, const void* k_cache, c
                                            const void* token_req, const void* positions, const void* block_tables,
                                            int max_blocks, int T, int Hq, int Hkv, int D, int E, int page_size,
                                            float scale, int window, int chunk, float cap, int has_sink, float sink,
-                                           const void* gate, long long gate_ld, int dtype, void* stream) {
+                                           const void* sinks, const void* slopes, const void* gate, long long gate_ld,
+                                           int dtype, void* stream) {
   NHV_REQUIRE(cap >= 0.f && (!gate || gate_ld >= Hq), "attention: cap %g, gate rows %lld apart for %d heads", (double)cap, gate_ld, Hq);
   NHV_REQUIRE(T > 0 && Hq > 0 && Hkv > 0 && D > 0 && page_size > 0 && max_blocks > 0,
               "attention: bad sizes T=%d Hq=%d Hkv=%d D=%d page=%d blocks=%d", T, Hq, Hkv, D, page_size, max_blocks);
@@ -117,12 +123,12 @@ extern "C" int nhv_paged_attention_generic(const void* q, const void* k_cache, c
     hipLaunchKernelGGL(paged_attention_generic_kernel<float>, dim3(blocks), dim3(256), lds, s, (const float*)q,
                        (const float*)k_cache, (const float*)v_cache, (float*)out, (const int*)token_req,
                        (const int*)positions, (const int*)block_tables, max_blocks, (int)n_items, Hq, Hkv, D, E, page_size,
-                       scale, window, chunk, cap, has_sink, sink, (const float*)gate, gate_ld);
+                       scale, window, chunk, cap, has_sink, sink, (const float*)sinks, (const float*)slopes, (const float*)gate, gate_ld);
   else if (dtype == NHV_BF16)
     hipLaunchKernelGGL(paged_attention_generic_kernel<bf16_t>, dim3(blocks), dim3(256), lds, s, (const bf16_t*)q,
                        (const bf16_t*)k_cache, (const bf16_t*)v_cache, (bf16_t*)out, (const int*)token_req,
                        (const int*)positions, (const int*)block_tables, max_blocks, (int)n_items, Hq, Hkv, D, E, page_size,
-                       scale, window, chunk, cap, has_sink, sink, (const bf16_t*)gate, gate_ld);
+                       scale, window, chunk, cap, has_sink, sink, (const float*)sinks, (const float*)slopes, (const bf16_t*)gate, gate_ld);
   else
     return nhv_fail("attention: unknown dtype %d", dtype);
   NHV_LAUNCH_CHECK("paged_attention_generic");

@@ -35,9 +35,11 @@
 // nearest key inside it (their P is 0): unused cache slots may hold anything, and 0 * NaN
 // would poison the sums.
 // What a layer may ask for besides (MORE; the entry point ..._more): a cap on the scores (s <- cap tanh(s / cap), after
-// the scale; taken on the float scores where they leave the first product), one more term exp(sink) in the softmax's
-// denominator (it joins the row's sum at the end, against the row's reference point) and a gate per (token, head) whose
-// sigmoid multiplies the head's result (with the division by the sum).
+// the scale; taken on the float scores where they leave the first product), a bias that grows with the distance (BIASED:
+// slopes[head] * (query position - key position) is taken off the float score after scale and cap), one more term
+// exp(sink) in the softmax's denominator (one score for the layer or one per head; it is the row's first reference point,
+// and joins the row's sum at the end) and a gate per (token, head) whose sigmoid multiplies the head's result (with the
+// division by the sum).
 #include "nhv_common.h"
 #include <math.h>
 #include <type_traits>
@@ -92,14 +94,18 @@ __device__ __forceinline__ int slot_of(P bt, int key, int page_size, int page_sh
 // look-up that every load of a key depends on costs an LDS read instead of a trip to memory.
 // MORE: cap_ratio = cap / scale (0: no cap) and tanh_k = 2 log2(e) scale / cap, so that the capped score, still to be
 // multiplied by the scale as every score is, costs one exp2 and one reciprocal: tanh(x) = 1 - 2 / (1 + exp(2 x)), and an
-// exp2 that overflows gives the limit 1; sink_l2 = sink log2(e), or -inf for none; gate (may be null).
-template <bool BT_IN_LDS, int RT, bool MORE>
+// exp2 that overflows gives the limit 1; sink_l2 = sink log2(e), or -inf for none (sinks, may be null: one per head in
+// its place); gate (may be null). BIASED: slopes per head; the scores are then brought to base-2 exponents, scale and
+// bias in, before the exponentials (a bias that depends on the key cannot be left to the row's reference point).
+template <bool BT_IN_LDS, int RT, bool MORE, bool BIASED>
 __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(2))) void prefill_attention_kernel(
     const bf16_t* __restrict__ q, const bf16_t* __restrict__ k_cache, const bf16_t* __restrict__ v_cache,
     bf16_t* __restrict__ out, const int* __restrict__ cu_seqlens_q, const int* __restrict__ context_lens,
     const int* __restrict__ block_tables, int max_blocks, int Hq, int Hkv, int page_size, int page_shift,
-    float scale_log2e, int window, float cap_ratio, float tanh_k, float sink_l2, const bf16_t* __restrict__ gate,
-    long long gate_ld) {
+    float scale_log2e, int window, float cap_ratio, float tanh_k, float sink_l2, const float* __restrict__ sinks,
+    const float* __restrict__ slopes, const bf16_t* __restrict__ gate, long long gate_ld) {
+  static_assert(MORE || !BIASED, "the bias is one of the further options");
+  constexpr float LOG2E = 1.4426950408889634f;
   constexpr int DL = SUPPORTED ? D : 16;                   // keeps the unsupported sizes compilable; they are never launched
   constexpr int TILE = SUPPORTED ? BN * DL : 16;           // elements of a tile
   __shared__ __attribute__((aligned(16))) bf16_t k_s0[TILE], k_s1[TILE], v_s0[TILE], v_s1[TILE];
@@ -175,11 +181,19 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(2))) void p
                      : zero8();
     }
   }
+  // what turns a score into the exponent of its term: the bias needs it before that, then nothing is left to do
+  const float to_exponent = BIASED ? 1.0f : scale_log2e;
+  float slope_l2[RT], row_sink[RT];
+#pragma unroll
+  for (int r = 0; r < RT; ++r) {
+    slope_l2[r] = BIASED ? slopes[head[r]] * LOG2E : 0.f;
+    row_sink[r] = MORE ? (sinks ? sinks[head[r]] * LOG2E : sink_l2) : -INFINITY;
+  }
   float m_run[RT], l_part[RT];                             // of row `col` (base 2); l_part is this lane's share of the row's sum
   floatx4 o[RT][DTILES];                                   // o[r][dt][j]: entry dt * 16 + 4 grp + j of row `col`
 #pragma unroll
   for (int r = 0; r < RT; ++r) {
-    m_run[r] = -INFINITY;
+    m_run[r] = row_sink[r];                                // (no sink: -inf, the first tile gives the reference)
     l_part[r] = 0.f;
 #pragma unroll
     for (int dt = 0; dt < DTILES; ++dt) o[r][dt] = floatx4{0.f, 0.f, 0.f, 0.f};
@@ -268,6 +282,17 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(2))) void p
             s4[r][kt][j] = __builtin_fmaf(-2.0f * cap_ratio,
                                           __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(s4[r][kt][j] * tanh_k)), cap_ratio);
     }
+    if (BIASED) {
+#pragma unroll
+      for (int r = 0; r < RT; ++r) {
+        const float nearest = slope_l2[r] * (float)(kb + grp * 4 - row_pos[r]);      // of this lane's first key; the others follow by steps
+#pragma unroll
+        for (int kt = 0; kt < KT; ++kt)
+#pragma unroll
+          for (int j = 0; j < 4; ++j)
+            s4[r][kt][j] = __builtin_fmaf(s4[r][kt][j], scale_log2e, __builtin_fmaf(slope_l2[r], (float)(kt * 16 + j), nearest));
+      }
+    }
     bf16x8 pa[RT][KT / 2];                                 // P of keys (32 a + 4 grp + j) and (32 a + 16 + 4 grp + j)
     float alpha[RT];
     bool grow[RT];
@@ -290,7 +315,7 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(2))) void p
       for (int kt = 0; kt < KT; ++kt)
 #pragma unroll
         for (int j = 0; j < 4; ++j) {
-          const float p = __builtin_amdgcn_exp2f(__builtin_fmaf(s4[r][kt][j], scale_log2e, -m_run[r]));
+          const float p = __builtin_amdgcn_exp2f(__builtin_fmaf(s4[r][kt][j], to_exponent, -m_run[r]));
           psum += p;
           pa[r][kt / 2][(kt % 2) * 4 + j] = (__bf16)p;
         }
@@ -303,7 +328,7 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(2))) void p
         for (int kt = 0; kt < KT; ++kt)
 #pragma unroll
           for (int j = 0; j < 4; ++j) m_tile = fmaxf(m_tile, s4[r][kt][j]);
-        m_tile *= scale_log2e;
+        m_tile *= to_exponent;
         m_tile = fmaxf(m_tile, __shfl_xor(m_tile, 16, 64));
         m_tile = fmaxf(m_tile, __shfl_xor(m_tile, 32, 64));
         const float m_new = fmaxf(m_run[r], m_tile);
@@ -314,7 +339,7 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(2))) void p
         for (int kt = 0; kt < KT; ++kt)
 #pragma unroll
           for (int j = 0; j < 4; ++j) {
-            const float p = __builtin_amdgcn_exp2f(__builtin_fmaf(s4[r][kt][j], scale_log2e, -m_safe));
+            const float p = __builtin_amdgcn_exp2f(__builtin_fmaf(s4[r][kt][j], to_exponent, -m_safe));
             psum += p;
             pa[r][kt / 2][(kt % 2) * 4 + j] = (__bf16)p;
           }
@@ -385,7 +410,7 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(2))) void p
     l += __shfl_xor(l, 16, 64);
     l += __shfl_xor(l, 32, 64);
     if (row_ok[r]) {
-      if (MORE) l += __builtin_amdgcn_exp2f(sink_l2 - m_run[r]);      // (a row that is stored has seen its own key: m_run is a number)
+      if (MORE) l += __builtin_amdgcn_exp2f(row_sink[r] - m_run[r]);      // (a row that is stored has seen its own key: m_run is a number)
       float inv = 1.0f / l;
       if (MORE && gate) inv /= 1.0f + expf(-(float)gate[(size_t)(q_begin + row_tok[r]) * gate_ld + head[r]]);
       bf16_t* dst = out + ((size_t)(q_begin + row_tok[r]) * Hq + head[r]) * D;
@@ -405,8 +430,8 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(2))) void p
 static int launch_prefill_attention(const void* q, const void* k_cache, const void* v_cache, void* out,
                                     const void* cu_seqlens_q, const void* context_lens, const void* block_tables,
                                     int max_blocks, int B, int max_q_len, int Hq, int Hkv, int page_size, float scale,
-                                    int window, void* stream, bool more, float cap, int has_sink, float sink, const void* gate,
-                                    long long gate_ld) {
+                                    int window, void* stream, bool more, float cap, int has_sink, float sink,
+                                    const void* sinks, const void* slopes, const void* gate, long long gate_ld) {
   NHV_REQUIRE(B > 0 && max_q_len > 0 && Hq > 0 && Hkv > 0 && page_size > 0 && max_blocks > 0, "prefill attention: bad sizes");
   NHV_REQUIRE(Hq % Hkv == 0, "prefill attention: %d query heads are not a multiple of %d key heads", Hq, Hkv);
   NHV_REQUIRE(prefill::SUPPORTED, "prefill attention: head size %d is beyond this kernel's limit of 256", prefill::D);
@@ -423,17 +448,18 @@ static int launch_prefill_attention(const void* q, const void* k_cache, const vo
   NHV_REQUIRE(gx <= 0x7fffffff && Hkv <= 65535 && B <= 65535, "prefill attention: grid too large");
   const float log2e = 1.4426950408889634f;
   const bool capped = more && cap > 0.f;
-#define NHV_PREFILL_LAUNCH_AS(BT, RT_, MORE_)                                                                          \
-  hipLaunchKernelGGL((prefill::prefill_attention_kernel<BT, RT_, MORE_>), dim3((unsigned)gx, Hkv, B), dim3(256), 0,  \
+#define NHV_PREFILL_LAUNCH_AS(BT, RT_, MORE_, BIASED_)                                                                 \
+  hipLaunchKernelGGL((prefill::prefill_attention_kernel<BT, RT_, MORE_, BIASED_>), dim3((unsigned)gx, Hkv, B), dim3(256), 0, \
                      (hipStream_t)stream, (const bf16_t*)q, (const bf16_t*)k_cache, (const bf16_t*)v_cache, (bf16_t*)out, \
                      (const int*)cu_seqlens_q, (const int*)context_lens, (const int*)block_tables, max_blocks, Hq, Hkv, \
                      page_size, page_shift, scale * log2e, window, capped ? cap / scale : 0.f,                         \
                      capped ? 2.0f * log2e * scale / cap : 0.f, more && has_sink ? sink * log2e : -INFINITY,           \
-                     (const bf16_t*)gate, gate_ld)
-#define NHV_PREFILL_LAUNCH(BT, RT_)            \
-  do {                                         \
-    if (more) NHV_PREFILL_LAUNCH_AS(BT, RT_, true); \
-    else NHV_PREFILL_LAUNCH_AS(BT, RT_, false);     \
+                     (const float*)sinks, (const float*)slopes, (const bf16_t*)gate, gate_ld)
+#define NHV_PREFILL_LAUNCH(BT, RT_)                               \
+  do {                                                            \
+    if (slopes) NHV_PREFILL_LAUNCH_AS(BT, RT_, true, true);       \
+    else if (more) NHV_PREFILL_LAUNCH_AS(BT, RT_, true, false);   \
+    else NHV_PREFILL_LAUNCH_AS(BT, RT_, false, false);            \
   } while (0)
   const bool bt_in_lds = max_blocks <= prefill::BT_LDS;
   if (two) {
@@ -454,18 +480,20 @@ extern "C" int nhv_prefill_attention_bf16(const void* q, const void* k_cache, co
                                           int max_blocks, int B, int max_q_len, int Hq, int Hkv, int page_size, float scale,
                                           int window, void* stream) {
   return launch_prefill_attention(q, k_cache, v_cache, out, cu_seqlens_q, context_lens, block_tables, max_blocks, B, max_q_len,
-                                  Hq, Hkv, page_size, scale, window, stream, false, 0.f, 0, 0.f, nullptr, 0);
+                                  Hq, Hkv, page_size, scale, window, stream, false, 0.f, 0, 0.f, nullptr, nullptr, nullptr, 0);
 }
 
 // The same with a cap on the scores (0: none; a positive scale is then needed), one more term exp(sink) in the
-// denominator (has_sink) and a gate per (token, head): gate[t * gate_ld + h] in bfloat16 (null: none).
+// denominator (has_sink: sink; sinks: one float per head in its place; null: none), a bias by distance (slopes: one float
+// per head; null: none) and a gate per (token, head): gate[t * gate_ld + h] in bfloat16 (null: none).
 extern "C" int nhv_prefill_attention_bf16_more(const void* q, const void* k_cache, const void* v_cache, void* out,
                                                const void* cu_seqlens_q, const void* context_lens, const void* block_tables,
                                                int max_blocks, int B, int max_q_len, int Hq, int Hkv, int page_size,
-                                               float scale, int window, float cap, int has_sink, float sink, const void* gate,
-                                               long long gate_ld, void* stream) {
+                                               float scale, int window, float cap, int has_sink, float sink,
+                                               const void* sinks, const void* slopes, const void* gate, long long gate_ld,
+                                               void* stream) {
   NHV_REQUIRE(cap >= 0.f && (cap == 0.f || scale > 0.f) && (!gate || gate_ld >= Hq),
               "prefill attention: cap %g with scale %g, gate rows %lld apart for %d heads", (double)cap, (double)scale, gate_ld, Hq);
   return launch_prefill_attention(q, k_cache, v_cache, out, cu_seqlens_q, context_lens, block_tables, max_blocks, B, max_q_len,
-                                  Hq, Hkv, page_size, scale, window, stream, true, cap, has_sink, sink, gate, gate_ld);
+                                  Hq, Hkv, page_size, scale, window, stream, true, cap, has_sink, sink, sinks, slopes, gate, gate_ld);
 }

@@ -2,6 +2,7 @@
 // the fused q/k-norm + rotation + cache-write kernel. All in two element types
 // (float, bfloat16); statistics, angles and sums are float.
 #include "nhv_common.h"
+#include "nhv_gates.h"
 
 // ---------------------------------------------------------------- embedding
 // scale: the row is multiplied by it in float and rounded once (1: the row is copied as it is)
@@ -39,11 +40,11 @@ extern "C" int nhv_embed(const void* ids, const void* table, void* out, int T, i
 // residual_mode 0: no residual. 1: s = x + residual, and s replaces the residual.
 // 2: s = x starts a residual (the first norm of a model). The residual may be kept
 // in float while the rows are bfloat16: the sum is then carried unrounded from
-// layer to layer. The weight is multiplied after rounding to the element type, as
-// a separate rounded product.
+// layer to layer. ``rounds_between``: the weight is multiplied after rounding to the
+// element type, as a separate rounded product; else the norm is rounded once, at its end.
 template <typename T, typename W, typename R>
 __global__ void rmsnorm_kernel(const T* __restrict__ x, R* __restrict__ residual, int residual_mode,
-                               const W* __restrict__ w, T* __restrict__ y, int H, float eps) {
+                               const W* __restrict__ w, T* __restrict__ y, int H, float eps, int rounds_between) {
   extern __shared__ float row[];          // H floats + 16
   float* scratch = row + H;
   const size_t base = (size_t)blockIdx.x * H;
@@ -58,8 +59,8 @@ __global__ void rmsnorm_kernel(const T* __restrict__ x, R* __restrict__ residual
   const float total = block_sum(ss, scratch);
   const float r = 1.0f / sqrtf(total / (float)H + eps);
   for (int i = threadIdx.x; i < H; i += blockDim.x) {
-    const T n = from_f32<T>(row[i] * r);
-    y[base + i] = from_f32<T>(to_f32(n) * to_f32(w[i]));
+    const float n = row[i] * r;
+    y[base + i] = from_f32<T>((rounds_between ? to_f32(from_f32<T>(n)) : n) * to_f32(w[i]));
   }
 }
 
@@ -103,7 +104,7 @@ __device__ __forceinline__ void store8f<float>(float* p, const float* in) {
 
 template <typename T, typename W, typename R, int MAXC>
 __global__ __launch_bounds__(1024) void rmsnorm_vec_kernel(const T* __restrict__ x, R* __restrict__ residual, int residual_mode,
-                                                           const W* __restrict__ w, T* __restrict__ y, int H, float eps) {
+                                                           const W* __restrict__ w, T* __restrict__ y, int H, float eps, int rounds_between) {
   __shared__ float scratch[16];
   const size_t base = (size_t)blockIdx.x * H;
   const int nch = H / 8;
@@ -141,14 +142,14 @@ __global__ __launch_bounds__(1024) void rmsnorm_vec_kernel(const T* __restrict__
     if (ch < nch) {
       float o[8];
 #pragma unroll
-      for (int e = 0; e < 8; ++e) o[e] = to_f32(from_f32<T>(v[c][e] * r)) * wv[c][e];
+      for (int e = 0; e < 8; ++e) o[e] = (rounds_between ? to_f32(from_f32<T>(v[c][e] * r)) : v[c][e] * r) * wv[c][e];
       store8f<T>(y + base + ch * 8, o);
     }
   }
 }
 
 extern "C" int nhv_rmsnorm(const void* x, void* residual, int residual_mode, int residual_dtype, const void* w, void* y,
-                           int T, int H, float eps, int dtype, int w_dtype, void* stream) {
+                           int T, int H, float eps, int rounds_between, int dtype, int w_dtype, void* stream) {
   NHV_REQUIRE(T > 0 && H > 0, "rmsnorm: bad sizes T=%d H=%d", T, H);
   NHV_REQUIRE(residual_mode >= 0 && residual_mode <= 2, "rmsnorm: bad residual mode %d", residual_mode);
   NHV_REQUIRE((residual_mode == 0) == (residual == nullptr), "rmsnorm: residual and its mode do not agree");
@@ -167,13 +168,13 @@ extern "C" int nhv_rmsnorm(const void* x, void* residual, int residual_mode, int
   do {                                                                                                                  \
     if (vec && maxc == 1)                                                                                               \
       hipLaunchKernelGGL((rmsnorm_vec_kernel<TT, WW, RR, 1>), dim3(T), dim3(vthreads), 0, s, (const TT*)x, (RR*)residual, \
-                         residual_mode, (const WW*)w, (TT*)y, H, eps);                                                  \
+                         residual_mode, (const WW*)w, (TT*)y, H, eps, rounds_between);                                  \
     else if (vec && maxc == 2)                                                                                          \
       hipLaunchKernelGGL((rmsnorm_vec_kernel<TT, WW, RR, 2>), dim3(T), dim3(vthreads), 0, s, (const TT*)x, (RR*)residual, \
-                         residual_mode, (const WW*)w, (TT*)y, H, eps);                                                  \
+                         residual_mode, (const WW*)w, (TT*)y, H, eps, rounds_between);                                  \
     else                                                                                                                \
       hipLaunchKernelGGL((rmsnorm_kernel<TT, WW, RR>), dim3(T), dim3(threads), lds, s, (const TT*)x, (RR*)residual,     \
-                         residual_mode, (const WW*)w, (TT*)y, H, eps);                                                  \
+                         residual_mode, (const WW*)w, (TT*)y, H, eps, rounds_between);                                  \
   } while (0)
   if (dtype == NHV_F32 && w_dtype == NHV_F32 && residual_dtype == NHV_F32) LAUNCH(float, float, float);
   else if (dtype == NHV_BF16 && w_dtype == NHV_BF16 && residual_dtype == NHV_F32) LAUNCH(bf16_t, bf16_t, float);
@@ -187,93 +188,80 @@ extern "C" int nhv_rmsnorm(const void* x, void* residual, int residual_mode, int
 }
 
 // ---------------------------------------------------------------- act(gate) * up
-// gu: [T, 2I], gate = first I columns, up = last I. Float inside, rounded once.
-// act 0: SiLU, z sigmoid(z). act 1: GELU in its tanh form, 0.5 z (1 + tanh(sqrt(2 / pi) (z + 0.044715 z^3))).
-template <int ACT>
-__device__ __forceinline__ float gate_act(float z) {
-  if (ACT == 1) return 0.5f * z * (1.0f + tanhf(0.7978845608028654f * (z + 0.044715f * z * z * z)));
-  return z / (1.0f + expf(-z));
-}
-
-template <typename T, int ACT = 0>
-__global__ void silu_mul_kernel(const T* __restrict__ gu, T* __restrict__ out, int I, size_t total) {
+// gu: [T, 2I], gate = first I columns, up = last I; bias (may be null): [2I], joins both in float first. Float inside,
+// rounded once. The gates are those of nhv_gates.h.
+template <typename T, int ACT>
+__global__ void gate_mul_kernel(const T* __restrict__ gu, const T* __restrict__ bias, T* __restrict__ out, int I, size_t total,
+                                const NhvGate gate) {
   for (size_t idx = (size_t)blockIdx.x * blockDim.x + threadIdx.x; idx < total; idx += (size_t)gridDim.x * blockDim.x) {
     const size_t t = idx / I, i = idx % I;
-    const float g = to_f32(gu[t * 2 * I + i]);
-    const float u = to_f32(gu[t * 2 * I + I + i]);
-    out[idx] = from_f32<T>(gate_act<ACT>(g) * u);
+    float g = to_f32(gu[t * 2 * I + i]), u = to_f32(gu[t * 2 * I + I + i]);
+    if (bias) {
+      g += to_f32(bias[i]);
+      u += to_f32(bias[I + i]);
+    }
+    out[idx] = from_f32<T>(nhv_gated<ACT>(g, u, gate));
   }
 }
 
 // the same, eight entries a thread (widths that are a multiple of 8)
-template <typename T, int ACT = 0>
-__global__ void silu_mul_vec_kernel(const T* __restrict__ gu, T* __restrict__ out, int I, size_t total8) {
+template <typename T, int ACT>
+__global__ void gate_mul_vec_kernel(const T* __restrict__ gu, const T* __restrict__ bias, T* __restrict__ out, int I,
+                                    size_t total8, const NhvGate gate) {
   const int per_row = I / 8;
   for (size_t idx = (size_t)blockIdx.x * blockDim.x + threadIdx.x; idx < total8; idx += (size_t)gridDim.x * blockDim.x) {
     const size_t t = idx / per_row, c = idx % per_row;
     float g[8], u[8], o[8];
     load8f<T>(gu + t * 2 * I + c * 8, g);
     load8f<T>(gu + t * 2 * I + I + c * 8, u);
+    if (bias) {
+      float bg[8], bu[8];
+      load8f<T>(bias + c * 8, bg);
+      load8f<T>(bias + I + c * 8, bu);
 #pragma unroll
-    for (int e = 0; e < 8; ++e) o[e] = gate_act<ACT>(g[e]) * u[e];
+      for (int e = 0; e < 8; ++e) {
+        g[e] += bg[e];
+        u[e] += bu[e];
+      }
+    }
+#pragma unroll
+    for (int e = 0; e < 8; ++e) o[e] = nhv_gated<ACT>(g[e], u[e], gate);
     store8f<T>(out + t * I + c * 8, o);
   }
 }
 
-extern "C" int nhv_silu_mul(const void* gu, void* out, int T, int I, int dtype, void* stream) {
-  NHV_REQUIRE(T > 0 && I > 0, "silu_mul: bad sizes T=%d I=%d", T, I);
-  if (I % 8 == 0 && (uintptr_t)gu % 16 == 0 && (uintptr_t)out % 16 == 0) {
-    const size_t total8 = (size_t)T * (I / 8);
-    const int vblocks = (int)((total8 + 255) / 256 > 65535 * 16 ? 65535 * 16 : (total8 + 255) / 256);
-    hipStream_t vs = (hipStream_t)stream;
-    if (dtype == NHV_F32)
-      hipLaunchKernelGGL(silu_mul_vec_kernel<float>, dim3(vblocks), dim3(256), 0, vs, (const float*)gu, (float*)out, I, total8);
-    else if (dtype == NHV_BF16)
-      hipLaunchKernelGGL(silu_mul_vec_kernel<bf16_t>, dim3(vblocks), dim3(256), 0, vs, (const bf16_t*)gu, (bf16_t*)out, I, total8);
-    else
-      return nhv_fail("silu_mul: unknown dtype %d", dtype);
-    NHV_LAUNCH_CHECK("silu_mul");
-    return 0;
+template <typename T, int ACT>
+static void launch_gate_mul(const void* gu, const void* bias, void* out, int rows, int I, const NhvGate& gate, hipStream_t s) {
+  if (I % 8 == 0 && (uintptr_t)gu % 16 == 0 && (uintptr_t)out % 16 == 0 && (uintptr_t)bias % 16 == 0) {
+    const size_t total8 = (size_t)rows * (I / 8);
+    const int blocks = (int)((total8 + 255) / 256 > 65535 * 16 ? 65535 * 16 : (total8 + 255) / 256);
+    hipLaunchKernelGGL((gate_mul_vec_kernel<T, ACT>), dim3(blocks), dim3(256), 0, s, (const T*)gu, (const T*)bias, (T*)out, I,
+                       total8, gate);
+    return;
   }
-  const size_t total = (size_t)T * I;
+  const size_t total = (size_t)rows * I;
   const int blocks = (int)((total + 255) / 256 > 65535 * 4 ? 65535 * 4 : (total + 255) / 256);
-  hipStream_t s = (hipStream_t)stream;
-  if (dtype == NHV_F32)
-    hipLaunchKernelGGL(silu_mul_kernel<float>, dim3(blocks), dim3(256), 0, s, (const float*)gu, (float*)out, I, total);
-  else if (dtype == NHV_BF16)
-    hipLaunchKernelGGL(silu_mul_kernel<bf16_t>, dim3(blocks), dim3(256), 0, s, (const bf16_t*)gu, (bf16_t*)out, I, total);
-  else
-    return nhv_fail("silu_mul: unknown dtype %d", dtype);
-  NHV_LAUNCH_CHECK("silu_mul");
-  return 0;
+  hipLaunchKernelGGL((gate_mul_kernel<T, ACT>), dim3(blocks), dim3(256), 0, s, (const T*)gu, (const T*)bias, (T*)out, I, total,
+                     gate);
 }
 
-// the same with the tanh form of GELU on the gate
-extern "C" int nhv_gelu_tanh_mul(const void* gu, void* out, int T, int I, int dtype, void* stream) {
-  NHV_REQUIRE(T > 0 && I > 0, "gelu_tanh_mul: bad sizes T=%d I=%d", T, I);
-  if (I % 8 == 0 && (uintptr_t)gu % 16 == 0 && (uintptr_t)out % 16 == 0) {
-    const size_t total8 = (size_t)T * (I / 8);
-    const int vblocks = (int)((total8 + 255) / 256 > 65535 * 16 ? 65535 * 16 : (total8 + 255) / 256);
-    hipStream_t vs = (hipStream_t)stream;
-    if (dtype == NHV_F32)
-      hipLaunchKernelGGL((silu_mul_vec_kernel<float, 1>), dim3(vblocks), dim3(256), 0, vs, (const float*)gu, (float*)out, I, total8);
-    else if (dtype == NHV_BF16)
-      hipLaunchKernelGGL((silu_mul_vec_kernel<bf16_t, 1>), dim3(vblocks), dim3(256), 0, vs, (const bf16_t*)gu, (bf16_t*)out, I, total8);
-    else
-      return nhv_fail("gelu_tanh_mul: unknown dtype %d", dtype);
-    NHV_LAUNCH_CHECK("gelu_tanh_mul");
-    return 0;
-  }
-  const size_t total = (size_t)T * I;
-  const int blocks = (int)((total + 255) / 256 > 65535 * 4 ? 65535 * 4 : (total + 255) / 256);
+extern "C" int nhv_gate_mul(const void* gu, const void* bias, void* out, int T, int I, int act, float limit, float alpha,
+                            float offset, int dtype, void* stream) {
+  NHV_REQUIRE(T > 0 && I > 0, "gate_mul: bad sizes T=%d I=%d", T, I);
+  NHV_REQUIRE(act >= 0 && act <= 2, "gate_mul: unknown gate %d", act);
+  NHV_REQUIRE(dtype == NHV_F32 || dtype == NHV_BF16, "gate_mul: unknown dtype %d", dtype);
+  const NhvGate gate = {act, limit, alpha, offset};
   hipStream_t s = (hipStream_t)stream;
-  if (dtype == NHV_F32)
-    hipLaunchKernelGGL((silu_mul_kernel<float, 1>), dim3(blocks), dim3(256), 0, s, (const float*)gu, (float*)out, I, total);
-  else if (dtype == NHV_BF16)
-    hipLaunchKernelGGL((silu_mul_kernel<bf16_t, 1>), dim3(blocks), dim3(256), 0, s, (const bf16_t*)gu, (bf16_t*)out, I, total);
-  else
-    return nhv_fail("gelu_tanh_mul: unknown dtype %d", dtype);
-  NHV_LAUNCH_CHECK("gelu_tanh_mul");
+#define LAUNCH(ACT)                                                                     \
+  do {                                                                                  \
+    if (dtype == NHV_F32) launch_gate_mul<float, ACT>(gu, bias, out, T, I, gate, s);    \
+    else launch_gate_mul<bf16_t, ACT>(gu, bias, out, T, I, gate, s);                    \
+  } while (0)
+  if (act == 2) LAUNCH(2);
+  else if (act == 1) LAUNCH(1);
+  else LAUNCH(0);
+#undef LAUNCH
+  NHV_LAUNCH_CHECK("gate_mul");
   return 0;
 }
 

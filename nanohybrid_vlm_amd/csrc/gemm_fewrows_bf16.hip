@@ -1,4 +1,4 @@
-// y[M, N] = x[M, K] . w[N, K]^T (+ bias), or silu(x . wg^T) * (x . wu^T), in bfloat16 for up to 16
+// y[M, N] = x[M, K] . w[N, K]^T (+ bias), or a gate of x . wg^T and x . wu^T (nhv_gates.h), in bfloat16 for up to 16
 // rows of x: the matrix products of a decoding step, whose time is the time to stream w from memory once.
 //
 // A block owns NT tiles of 16 rows of w (with GLU also their partners in the second matrix) and all
@@ -76,6 +76,12 @@ __device__ __forceinline__ void set_row_scales(const Fusion& f, const float (&sh
     sum = wave_sum(sum);
     if (m < M && lane == 0) r_s[m] = 1.0f / sqrtf(sum / (float)K + f.eps);
   }
+}
+
+// A gated product's two finished sums (the first with its bias in): the second one's bias lies N further.
+__device__ __forceinline__ float finish_gated(float g, float u, const bf16_t* bias, int n, int N, const NhvGate& gate) {
+  if (bias && n < N) u += (float)bias[N + n];
+  return nhv_gated(g, u, gate);
 }
 
 // What the wave that writes a tile adds to and multiplies with, asked for before the tile's weights: the residual's
@@ -218,7 +224,7 @@ __global__ __launch_bounds__(64 * WAVES) void gemm_fewrows_kernel(const bf16_t* 
     const int n = n0 + nt * 16 + grp * 4 + j;           // the tile's row 4 grp + j is output n, its column is row col of x
     float r = v[0][j] * rs;
     if (bias && n < N) r += (float)bias[n];
-    if (GLU) r = nhv_glu_gate(r, f.glu_act) * (v[NA - 1][j] * rs);
+    if (GLU) r = finish_gated(r, v[NA - 1][j] * rs, bias, n, N, f.gate);
     else if (f.plain_act) r = nhv_plain_act(r, f.plain_act);
     out[j] = r;
   }
@@ -345,7 +351,7 @@ __global__ __launch_bounds__(64 * WAVES) void gemm_fewrows_resident_kernel(const
       const int n = n0 + grp * 4 + j;
       float r = v[0][j] * rs;
       if (bias && n < N) r += (float)bias[n];
-      if (GLU) r = nhv_glu_gate(r, f.glu_act) * (v[NA - 1][j] * rs);
+      if (GLU) r = finish_gated(r, v[NA - 1][j] * rs, bias, n, N, f.gate);
       else if (f.plain_act) r = nhv_plain_act(r, f.plain_act);
       out[j] = r;
     }
@@ -450,7 +456,7 @@ __global__ __launch_bounds__(64 * WAVES) void gemm_fewrows_pieces_kernel(const b
       const int n = n0 + grp * 4 + j;
       float r = v[0][j] * rs;
       if (bias && n < N) r += (float)bias[n];
-      if (GLU) r = nhv_glu_gate(r, f.glu_act) * (v[NA - 1][j] * rs);
+      if (GLU) r = finish_gated(r, v[NA - 1][j] * rs, bias, n, N, f.gate);
       else if (f.plain_act) r = nhv_plain_act(r, f.plain_act);
       out[j] = r;
     }
@@ -563,7 +569,7 @@ __global__ __launch_bounds__(64 * WAVES) void gemm_fewrows_passes_kernel(const b
         const int n = n0 + grp * 4 + j;
         float r = v[0][j] * rs;
         if (bias && n < N) r += (float)bias[n];
-        if (GLU) r = nhv_glu_gate(r, f.glu_act) * (v[NA - 1][j] * rs);
+        if (GLU) r = finish_gated(r, v[NA - 1][j] * rs, bias, n, N, f.gate);
         else if (f.plain_act) r = nhv_plain_act(r, f.plain_act);
         out[j] = r;
       }

@@ -180,15 +180,16 @@ extern "C" int nhv_gemm_skinny_glu_bf16(const void* x, const void* w, void* y, i
   return 0;
 }
 
-// The same for up to 16 rows with the gate's activation named: 0 SiLU, 1 the tanh form of GELU.
-extern "C" int nhv_gemm_fewrows_glu_act_bf16(const void* x, const void* w, void* y, int M, int N, int K, int out_dtype, int act,
-                                             void* stream) {
+// The same for up to 16 rows with the gate named (nhv_gates.h) and an optional bias [2N] (of the gate's, then of the up
+// sums).
+extern "C" int nhv_gemm_fewrows_gated_bf16(const void* x, const void* w, const void* bias, void* y, int M, int N, int K,
+                                           int out_dtype, int act, float limit, float alpha, float offset, void* stream) {
   if (sk_check("few-rows gated gemm", x, w, M, N, K, out_dtype)) return 1;
-  NHV_REQUIRE(M <= 16 && (act == 0 || act == 1), "few-rows gated gemm: %d rows (up to 16), activation %d", M, act);
+  NHV_REQUIRE(M <= 16 && act >= 0 && act <= 2, "few-rows gated gemm: %d rows (up to 16), gate %d", M, act);
   NhvGemmFusion f = {};
-  f.glu_act = act;
-  if (nhv_gemm_fewrows_launch(true, x, w, nullptr, y, M, N, K, out_dtype, (hipStream_t)stream, f)) return 1;
-  NHV_LAUNCH_CHECK("gemm_fewrows_glu_act_bf16");
+  f.gate = {act, limit, alpha, offset};
+  if (nhv_gemm_fewrows_launch(true, x, w, bias, y, M, N, K, out_dtype, (hipStream_t)stream, f)) return 1;
+  NHV_LAUNCH_CHECK("gemm_fewrows_gated_bf16");
   return 0;
 }
 
@@ -206,8 +207,8 @@ extern "C" int nhv_gemm_fewrows_act_bf16(const void* x, const void* w, void* y, 
 }
 
 // ---- products of up to 16 rows that take over the kernels around them (nhv_gemm_fusion.h) ----
-// y = r . (x . w^T) (+ bias), or with glu silu(r . (x . w[0:N]^T)) * (r . (x . w[N:2N]^T)), for 1 <= M <= 16 rows in
-// bfloat16. With ss_in: x is a sum (times its norm's weight) whose rows still lack their scales: r per row from ss_in
+// y = r . (x . w^T) (+ bias), or with glu a gate (nhv_gates.h) of r . (x . w[0:N]^T) and r . (x . w[N:2N]^T) (bias: [2N]),
+// for 1 <= M <= 16 rows in bfloat16. With ss_in: x is a sum (times its norm's weight) whose rows still lack their scales: r per row from ss_in
 // [M, tiles_in] (the tiles' shares of the row's sum of squares over its K entries) and eps; without: r = 1.
 // With residual: the product is not stored; it is added to residual [M, N] (float or bfloat16, rewritten), the sum
 // times next_w [N] (if given), rounded, goes to sum_out [M, N] (bfloat16) and the tiles' shares of its rows' sums of
@@ -215,10 +216,13 @@ extern "C" int nhv_gemm_fewrows_act_bf16(const void* x, const void* w, void* y, 
 extern "C" int nhv_gemm_fewrows_fused_bf16(const void* x, const void* ss_in, int tiles_in, float eps, const void* w,
                                            const void* bias, void* y, int M, int N, int K, int out_dtype, int glu,
                                            void* residual, int residual_dtype, void* sum_out, void* ss_out,
-                                           const void* next_w, int next_w_dtype, void* stream) {
+                                           const void* next_w, int next_w_dtype, int act, float limit, float alpha,
+                                           float offset, void* stream) {
   if (sk_check("fused few-rows gemm", x, w, M, N, K, out_dtype)) return 1;
   NHV_REQUIRE(M <= 16, "fused few-rows gemm: %d rows are beyond this kernel's limit of 16", M);
   NhvGemmFusion f = {};
+  NHV_REQUIRE(act >= 0 && act <= 2, "fused few-rows gemm: unknown gate %d", act);
+  f.gate = {act, limit, alpha, offset};
   if (ss_in) {
     NHV_REQUIRE(tiles_in > 0 && eps > 0.f, "fused few-rows gemm: the rows' scales need the tiles' count and eps");
     f.ss_in = (const float*)ss_in;
@@ -239,7 +243,7 @@ extern "C" int nhv_gemm_fewrows_fused_bf16(const void* x, const void* ss_in, int
   } else {
     NHV_REQUIRE(y != nullptr, "fused few-rows gemm: no place for the result");
   }
-  if (nhv_gemm_fewrows_launch(glu != 0, x, w, glu ? nullptr : bias, y, M, N, K, out_dtype, (hipStream_t)stream, f)) return 1;
+  if (nhv_gemm_fewrows_launch(glu != 0, x, w, bias, y, M, N, K, out_dtype, (hipStream_t)stream, f)) return 1;
   NHV_LAUNCH_CHECK("gemm_fewrows_fused_bf16");
   return 0;
 }

@@ -1,12 +1,14 @@
 // Kernels of attention over a cached latent: every token stores one row [c | r], c the normed low-rank latent that
 // keys and values of all heads are made of, r a rotated key part shared by all heads (it may be absent).
-//   nhv_latent_prepare      the packed down projections of a step's rows -> the normed query latent, and the row
-//                           [RMS-normed c | rotated r] stored at the step's slots
+//   nhv_latent_prepare      the packed down projections of a step's rows -> the normed query latent (if there is one), and
+//                           the row [RMS-normed c | rotated r] stored at the step's slots
 //   nhv_head_gemm           y[t, h, :] = M_h x[t, h, :] for a matrix per head (strides say which way M_h lies), with an
-//                           optional sigmoid gate per (token, head) on the result
+//                           optional sigmoid gate on the result, one per (token, head) or one per entry
 //   nhv_head_gemm_fewrows   the same for up to 16 rows, with the turning of the queries' rotated part in the same launch
-//   nhv_rotate_interleaved  the rotated part of every query head, turned by position and copied beside the rest
-// Pairs (2i, 2i + 1) turn by angle = position * freqs[i]; cosine and sine are multiplied by ``gain``. The frequencies
+//   nhv_head_gemm_bf16      the same on the matrix cores for any number of rows, turning included
+//   nhv_rotate_heads        the rotated part of every query head, turned by position and copied beside the rest
+// Pairs (2i, 2i + 1), or (i, i + r / 2) of the r rotated entries where ``halves`` is set, turn by angle = position *
+// freqs[i]; cosine and sine are multiplied by ``gain``. The frequencies
 // come as doubles and the product with the position is taken and brought into [-pi, pi] in double (a float product
 // of a position in the thousands is off by 1e-4 of a turn), then sine and cosine in float. Norm statistics and sums
 // are float; rows are float or bfloat16.
@@ -21,69 +23,97 @@ __device__ __forceinline__ void nhv_turn_angle(int pos, double f, float gain, fl
   *cs *= gain;
 }
 
-// a: [T, A] float. Query latent: columns q_off .. q_off + q_rank, normed with wq into cq [T, q_rank]. Latent:
-// columns c_off .. c_off + kv_rank normed with wc, then ``rot`` columns turned; both stored at slot_mapping[t] in
-// ``cache`` (rows of ``row`` entries; entries beyond kv_rank + rot are left alone). kv_rank 0: nothing is stored.
+// entries of the rotated part that pair p is made of
+__device__ __forceinline__ int nhv_pair_first(int p, int rot, int halves) { return halves ? p : 2 * p; }
+__device__ __forceinline__ int nhv_pair_second(int p, int rot, int halves) { return halves ? p + rot / 2 : 2 * p + 1; }
+
+// The gate on entry n of head h's result at row m: none (null), mode 1: one float per (row, head), gate[m gs_t + h];
+// mode 2: one per entry, of the rows' type, gate[m gs_t + h N + n].
 template <typename T>
-__global__ void latent_prepare_kernel(const float* __restrict__ a, int A, int q_off, int q_rank, int c_off, int kv_rank,
+__device__ __forceinline__ float nhv_head_gate_of(const void* gate, int mode, long long gs_t, int m, int h, int N, int n) {
+  const float z = mode == 2 ? to_f32(reinterpret_cast<const T*>(gate)[(size_t)m * gs_t + (size_t)h * N + n])
+                            : reinterpret_cast<const float*>(gate)[(size_t)m * gs_t + h];
+  return 1.0f / (1.0f + expf(-z));
+}
+
+// Pair p of head h at row t, turned from x (entry x_rot_off on) into y (entry y_rot_off on).
+template <typename T>
+__device__ __forceinline__ void nhv_turn_pair(const T* s, T* d, int p, int rot, int halves, int pos, const double* freqs, float gain) {
+  float sn, cs;
+  nhv_turn_angle(pos, freqs[p], gain, &sn, &cs);
+  const int a = nhv_pair_first(p, rot, halves), b = nhv_pair_second(p, rot, halves);
+  const float u = to_f32(s[a]), v = to_f32(s[b]);
+  d[a] = from_f32<T>(u * cs - v * sn);
+  d[b] = from_f32<T>(v * cs + u * sn);
+}
+
+// a: [T, A] rows of type TA. Query latent (q_rank > 0): columns q_off .. q_off + q_rank, normed with wq into cq [T, q_rank]. Latent:
+// columns c_off .. c_off + kv_rank normed with wc, then ``rot`` columns turned; both stored at slot_mapping[t] in
+// ``cache`` (rows of ``row`` entries; entries beyond kv_rank + rot become zeros). kv_rank 0: nothing is stored.
+template <typename T, typename TA>
+__global__ void latent_prepare_kernel(const TA* __restrict__ a, int A, int q_off, int q_rank, int c_off, int kv_rank,
                                       int rot, const float* __restrict__ wq, const float* __restrict__ wc, float eps,
                                       const double* __restrict__ freqs, float gain, const int* __restrict__ positions,
                                       const int* __restrict__ slot_mapping, T* __restrict__ cache, int row,
-                                      T* __restrict__ cq) {
+                                      T* __restrict__ cq, int halves) {
   __shared__ float scratch[16];
   const int t = blockIdx.x;
-  const float* src = a + (size_t)t * A;
+  const TA* src = a + (size_t)t * A;
   float ss = 0.f;
-  for (int i = threadIdx.x; i < q_rank; i += blockDim.x) {
-    const float v = src[q_off + i];
-    ss += v * v;
+  if (q_rank > 0) {                          // the same for the whole grid
+    for (int i = threadIdx.x; i < q_rank; i += blockDim.x) {
+      const float v = to_f32(src[q_off + i]);
+      ss += v * v;
+    }
+    const float rq = 1.0f / sqrtf(block_sum(ss, scratch) / (float)q_rank + eps);
+    for (int i = threadIdx.x; i < q_rank; i += blockDim.x)
+      cq[(size_t)t * q_rank + i] = from_f32<T>(to_f32(src[q_off + i]) * rq * wq[i]);
   }
-  const float rq = 1.0f / sqrtf(block_sum(ss, scratch) / (float)q_rank + eps);
-  for (int i = threadIdx.x; i < q_rank; i += blockDim.x)
-    cq[(size_t)t * q_rank + i] = from_f32<T>(src[q_off + i] * rq * wq[i]);
   if (kv_rank == 0 || slot_mapping == nullptr) return;
   const int slot = slot_mapping[t];          // the same for the whole block
   if (slot < 0) return;
   ss = 0.f;
   for (int i = threadIdx.x; i < kv_rank; i += blockDim.x) {
-    const float v = src[c_off + i];
+    const float v = to_f32(src[c_off + i]);
     ss += v * v;
   }
   const float rc = 1.0f / sqrtf(block_sum(ss, scratch) / (float)kv_rank + eps);
   T* dst = cache + (size_t)slot * row;
-  for (int i = threadIdx.x; i < kv_rank; i += blockDim.x) dst[i] = from_f32<T>(src[c_off + i] * rc * wc[i]);
+  for (int i = threadIdx.x; i < kv_rank; i += blockDim.x) dst[i] = from_f32<T>(to_f32(src[c_off + i]) * rc * wc[i]);
   const int pos = positions[t];
   for (int i = threadIdx.x; i < rot / 2; i += blockDim.x) {
     float sn, cs;
     nhv_turn_angle(pos, freqs[i], gain, &sn, &cs);
-    const float u = src[c_off + kv_rank + 2 * i], v = src[c_off + kv_rank + 2 * i + 1];
-    dst[kv_rank + 2 * i] = from_f32<T>(u * cs - v * sn);
-    dst[kv_rank + 2 * i + 1] = from_f32<T>(v * cs + u * sn);
+    const int first = nhv_pair_first(i, rot, halves), second = nhv_pair_second(i, rot, halves);
+    const float u = to_f32(src[c_off + kv_rank + first]), v = to_f32(src[c_off + kv_rank + second]);
+    dst[kv_rank + first] = from_f32<T>(u * cs - v * sn);
+    dst[kv_rank + second] = from_f32<T>(v * cs + u * sn);
   }
+  // (entries of the row beyond the rotated part: zeros, which meet zeros in the queries)
+  for (int i = kv_rank + rot + threadIdx.x; i < row; i += blockDim.x) dst[i] = from_f32<T>(0.f);
 }
 
-extern "C" int nhv_latent_prepare(const void* a, int A, int q_off, int q_rank, int c_off, int kv_rank, int rot,
+extern "C" int nhv_latent_prepare(const void* a, int a_dtype, int A, int q_off, int q_rank, int c_off, int kv_rank, int rot,
                                   const void* wq, const void* wc, float eps, const void* freqs, float gain,
-                                  const void* positions, const void* slot_mapping, void* cache, int row, void* cq, int T,
-                                  int dtype, void* stream) {
-  NHV_REQUIRE(T > 0 && A > 0 && q_rank > 0 && kv_rank >= 0 && rot >= 0 && rot % 2 == 0,
+                                  const void* positions, const void* slot_mapping, void* cache, int row, void* cq, int halves,
+                                  int T, int dtype, void* stream) {
+  NHV_REQUIRE(T > 0 && A > 0 && q_rank >= 0 && kv_rank >= 0 && q_rank + kv_rank > 0 && rot >= 0 && rot % 2 == 0,
               "latent_prepare: bad sizes T=%d A=%d q_rank=%d kv_rank=%d rot=%d", T, A, q_rank, kv_rank, rot);
-  NHV_REQUIRE(q_off >= 0 && q_off + q_rank <= A && (kv_rank == 0 || (c_off >= 0 && c_off + kv_rank + rot <= A)),
+  NHV_REQUIRE((q_rank == 0 || (q_off >= 0 && q_off + q_rank <= A)) && (kv_rank == 0 || (c_off >= 0 && c_off + kv_rank + rot <= A)),
               "latent_prepare: columns %d+%d and %d+%d+%d of %d", q_off, q_rank, c_off, kv_rank, rot, A);
   NHV_REQUIRE(kv_rank == 0 || slot_mapping == nullptr || (cache != nullptr && row >= kv_rank + rot),
               "latent_prepare: cache rows of %d entries for %d + %d", row, kv_rank, rot);
   NHV_REQUIRE(rot == 0 || kv_rank == 0 || freqs != nullptr, "latent_prepare: a rotated part without frequencies");
   hipStream_t s = (hipStream_t)stream;
-  if (dtype == NHV_F32)
-    hipLaunchKernelGGL(latent_prepare_kernel<float>, dim3(T), dim3(256), 0, s, (const float*)a, A, q_off, q_rank, c_off,
-                       kv_rank, rot, (const float*)wq, (const float*)wc, eps, (const double*)freqs, gain,
-                       (const int*)positions, (const int*)slot_mapping, (float*)cache, row, (float*)cq);
-  else if (dtype == NHV_BF16)
-    hipLaunchKernelGGL(latent_prepare_kernel<bf16_t>, dim3(T), dim3(256), 0, s, (const float*)a, A, q_off, q_rank, c_off,
-                       kv_rank, rot, (const float*)wq, (const float*)wc, eps, (const double*)freqs, gain,
-                       (const int*)positions, (const int*)slot_mapping, (bf16_t*)cache, row, (bf16_t*)cq);
-  else
-    return nhv_fail("latent_prepare: unknown dtype %d", dtype);
+#define LAUNCH(TT, TA)                                                                                                     \
+  hipLaunchKernelGGL((latent_prepare_kernel<TT, TA>), dim3(T), dim3(256), 0, s, (const TA*)a, A, q_off, q_rank, c_off,      \
+                     kv_rank, rot, (const float*)wq, (const float*)wc, eps, (const double*)freqs, gain,                    \
+                     (const int*)positions, (const int*)slot_mapping, (TT*)cache, row, (TT*)cq, halves)
+  if (dtype == NHV_F32 && a_dtype == NHV_F32) LAUNCH(float, float);
+  else if (dtype == NHV_BF16 && a_dtype == NHV_F32) LAUNCH(bf16_t, float);
+  else if (dtype == NHV_BF16 && a_dtype == NHV_BF16) LAUNCH(bf16_t, bf16_t);
+  else return nhv_fail("latent_prepare: unknown dtypes %d, %d", a_dtype, dtype);
+#undef LAUNCH
   NHV_LAUNCH_CHECK("latent_prepare");
   return 0;
 }
@@ -91,7 +121,7 @@ extern "C" int nhv_latent_prepare(const void* a, int A, int q_off, int q_rank, i
 // ---------------------------------------------------------------- a matrix per head
 // y[t * ys_t + h * ys_h + n] = sum over k of x[t * xs_t + h * xs_h + k] * w[h * ws_h + n * ws_n + k * ws_k], k rising,
 // one thread per output, so a row's result does not depend on its batch. A block owns 32 rows x 64 outputs of one head
-// and walks over k in pieces of 16 through LDS. gate: y *= sigmoid(gate[t * gs_t + h]).
+// and walks over k in pieces of 16 through LDS. gate: y *= the sigmoid of a gate (nhv_head_gate_of).
 #define HG_TM 32
 #define HG_TN 64
 #define HG_TK 16
@@ -99,8 +129,8 @@ template <typename T>
 __global__ __launch_bounds__(256) void head_gemm_kernel(const T* __restrict__ x, long long xs_t, long long xs_h,
                                                         const T* __restrict__ w, long long ws_h, long long ws_n,
                                                         long long ws_k, T* __restrict__ y, long long ys_t, long long ys_h,
-                                                        const float* __restrict__ gate, long long gs_t, int rows, int N,
-                                                        int K) {
+                                                        const void* __restrict__ gate, int gate_mode, long long gs_t,
+                                                        int rows, int N, int K) {
   __shared__ float xs[HG_TM][HG_TK];
   __shared__ float wt[HG_TN][HG_TK + 1];
   const int h = blockIdx.z;
@@ -138,24 +168,24 @@ __global__ __launch_bounds__(256) void head_gemm_kernel(const T* __restrict__ x,
     const int m = m0 + ty * (HG_TM / 4) + i;
     if (m >= rows) continue;
     float v = acc[i];
-    if (gate != nullptr) v *= 1.0f / (1.0f + expf(-gate[(size_t)m * gs_t + h]));
+    if (gate != nullptr) v *= nhv_head_gate_of<T>(gate, gate_mode, gs_t, m, h, N, n);
     y[(size_t)m * ys_t + (size_t)h * ys_h + n] = from_f32<T>(v);
   }
 }
 
 extern "C" int nhv_head_gemm(const void* x, long long xs_t, long long xs_h, const void* w, long long ws_h, long long ws_n,
-                             long long ws_k, void* y, long long ys_t, long long ys_h, const void* gate, long long gs_t,
-                             int rows, int H, int N, int K, int dtype, void* stream) {
+                             long long ws_k, void* y, long long ys_t, long long ys_h, const void* gate, int gate_mode,
+                             long long gs_t, int rows, int H, int N, int K, int dtype, void* stream) {
   NHV_REQUIRE(rows > 0 && H > 0 && N > 0 && K > 0 && H <= 65535, "head_gemm: bad sizes rows=%d H=%d N=%d K=%d", rows, H, N, K);
   const dim3 grid((rows + HG_TM - 1) / HG_TM, (N + HG_TN - 1) / HG_TN, H);
   NHV_REQUIRE(grid.y <= 65535, "head_gemm: %d outputs a head are too many", N);
   hipStream_t s = (hipStream_t)stream;
   if (dtype == NHV_F32)
     hipLaunchKernelGGL(head_gemm_kernel<float>, grid, dim3(256), 0, s, (const float*)x, xs_t, xs_h, (const float*)w, ws_h,
-                       ws_n, ws_k, (float*)y, ys_t, ys_h, (const float*)gate, gs_t, rows, N, K);
+                       ws_n, ws_k, (float*)y, ys_t, ys_h, gate, gate_mode, gs_t, rows, N, K);
   else if (dtype == NHV_BF16)
     hipLaunchKernelGGL(head_gemm_kernel<bf16_t>, grid, dim3(256), 0, s, (const bf16_t*)x, xs_t, xs_h, (const bf16_t*)w,
-                       ws_h, ws_n, ws_k, (bf16_t*)y, ys_t, ys_h, (const float*)gate, gs_t, rows, N, K);
+                       ws_h, ws_n, ws_k, (bf16_t*)y, ys_t, ys_h, gate, gate_mode, gs_t, rows, N, K);
   else
     return nhv_fail("head_gemm: unknown dtype %d", dtype);
   NHV_LAUNCH_CHECK("head_gemm");
@@ -167,7 +197,7 @@ extern "C" int nhv_head_gemm(const void* x, long long xs_t, long long xs_h, cons
 // thread that walked over k with loads from memory waited for memory at every step); then lane = output, wave = four
 // of the rows, k rising as above, so the sums are the same bits. One more block a head may turn the rotated part of x
 // and copy it beside the outputs (``rot`` entries from x_rot_off to y_rot_off), which saves the launch of
-// nhv_rotate_interleaved.
+// nhv_rotate_heads.
 template <typename V>
 __device__ __forceinline__ void hg_load8f(const V* p, float* out);
 template <>
@@ -189,22 +219,18 @@ template <typename T, bool VEC>
 __global__ __launch_bounds__(256) void head_gemm_fewrows_kernel(const T* __restrict__ x, long long xs_t, long long xs_h,
                                                                 const T* __restrict__ w, long long ws_h, long long ws_n,
                                                                 long long ws_k, T* __restrict__ y, long long ys_t,
-                                                                long long ys_h, const float* __restrict__ gate,
+                                                                long long ys_h, const void* __restrict__ gate, int gate_mode,
                                                                 long long gs_t, int rows, int N, int K, int n_chunks, int rot,
-                                                                int x_rot_off, int y_rot_off, const double* __restrict__ freqs,
+                                                                int x_rot_off, int y_rot_off, int halves,
+                                                                const double* __restrict__ freqs,
                                                                 float gain, const int* __restrict__ positions) {
   extern __shared__ float xs[];              // 16 x K floats, then the block's piece of the matrix
   const int h = blockIdx.y;
   if ((int)blockIdx.x == n_chunks) {         // the rotated part
     for (int i = threadIdx.x; i < rows * (rot / 2); i += blockDim.x) {
       const int t = i / (rot / 2), p = i % (rot / 2);
-      float sn, cs;
-      nhv_turn_angle(positions[t], freqs[p], gain, &sn, &cs);
-      const T* s = x + (size_t)t * xs_t + (size_t)h * xs_h + x_rot_off + 2 * p;
-      T* d = y + (size_t)t * ys_t + (size_t)h * ys_h + y_rot_off + 2 * p;
-      const float u = to_f32(s[0]), v = to_f32(s[1]);
-      d[0] = from_f32<T>(u * cs - v * sn);
-      d[1] = from_f32<T>(v * cs + u * sn);
+      nhv_turn_pair(x + (size_t)t * xs_t + (size_t)h * xs_h + x_rot_off, y + (size_t)t * ys_t + (size_t)h * ys_h + y_rot_off, p,
+                    rot, halves, positions[t], freqs, gain);
     }
     return;
   }
@@ -290,15 +316,15 @@ __global__ __launch_bounds__(256) void head_gemm_fewrows_kernel(const T* __restr
   for (int t = 0; t < 4; ++t) {
     if (t0 + t >= rows) break;
     float v = acc[t];
-    if (gate != nullptr) v *= 1.0f / (1.0f + expf(-gate[(size_t)(t0 + t) * gs_t + h]));
+    if (gate != nullptr) v *= nhv_head_gate_of<T>(gate, gate_mode, gs_t, t0 + t, h, N, n);
     y[(size_t)(t0 + t) * ys_t + (size_t)h * ys_h + n] = from_f32<T>(v);
   }
 }
 
 extern "C" int nhv_head_gemm_fewrows(const void* x, long long xs_t, long long xs_h, const void* w, long long ws_h,
                                      long long ws_n, long long ws_k, void* y, long long ys_t, long long ys_h, const void* gate,
-                                     long long gs_t, int rows, int H, int N, int K, int rot, int x_rot_off, int y_rot_off,
-                                     const void* freqs, float gain, const void* positions, int dtype, void* stream) {
+                                     int gate_mode, long long gs_t, int rows, int H, int N, int K, int rot, int x_rot_off,
+                                     int y_rot_off, int halves, const void* freqs, float gain, const void* positions, int dtype, void* stream) {
   const size_t item = dtype == NHV_F32 ? 4 : 2;
   const size_t lds = 16 * (size_t)K * sizeof(float) + (64 + 16 / item) * (size_t)K * item;
   NHV_REQUIRE(rows > 0 && rows <= 16 && H > 0 && H <= 65535 && N > 0 && K > 0 && lds <= 96 * 1024,
@@ -316,8 +342,8 @@ extern "C" int nhv_head_gemm_fewrows(const void* x, long long xs_t, long long xs
     if (lds > 64 * 1024)                                                                                                  \
       (void)hipFuncSetAttribute((const void*)head_gemm_fewrows_kernel<TYPE, VEC>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds); \
     hipLaunchKernelGGL((head_gemm_fewrows_kernel<TYPE, VEC>), grid, dim3(256), lds, s, (const TYPE*)x, xs_t, xs_h,          \
-                       (const TYPE*)w, ws_h, ws_n, ws_k, (TYPE*)y, ys_t, ys_h, (const float*)gate, gs_t, rows, N, K, n_chunks, \
-                       rot, x_rot_off, y_rot_off, (const double*)freqs, gain, (const int*)positions);                      \
+                       (const TYPE*)w, ws_h, ws_n, ws_k, (TYPE*)y, ys_t, ys_h, gate, gate_mode, gs_t, rows, N, K, n_chunks,   \
+                       rot, x_rot_off, y_rot_off, halves, (const double*)freqs, gain, (const int*)positions);                      \
   } while (0)
   if (dtype == NHV_F32) {
     if (vec) NHV_HG_LAUNCH(float, true); else NHV_HG_LAUNCH(float, false);
@@ -331,70 +357,171 @@ extern "C" int nhv_head_gemm_fewrows(const void* x, long long xs_t, long long xs
   return 0;
 }
 
-// ---------------------------------------------------------------- the gate alone
-// y[t, h, :] *= sigmoid(gate[t * gs_t + h]) for rows that a library product has made
-template <typename T>
-__global__ void head_gate_kernel(T* __restrict__ y, const float* __restrict__ gate, long long gs_t, int H, int N, size_t total) {
-  for (size_t i = (size_t)blockIdx.x * blockDim.x + threadIdx.x; i < total; i += (size_t)gridDim.x * blockDim.x) {
-    const size_t th = i / N;
-    const float g = gate[(th / H) * gs_t + th % H];
-    y[i] = from_f32<T>(to_f32(y[i]) * (1.0f / (1.0f + expf(-g))));
+// ---------------------------------------------------------------- a matrix per head on the matrix cores
+// The same in bfloat16 for matrices that are contiguous in k (M_h[n, k] = w[h N K + n K + k]), any number of rows, K and
+// every stride a multiple of 8 and every start 16 bytes aligned (the host checks). A wave owns MT x 16 rows and NT x 16
+// outputs of one head; the matrix rows are the 16 x 32 operand and the rows of x the 32 x 16 one, both asked for from
+// memory in the operands' own layout, 16 bytes a lane (a head's matrix is small and is found in L2 by all but the first
+// rows' blocks). A lane then holds four consecutive outputs of one row. Sums run over k in rising order whatever MT and
+// NT are, so a row's result does not depend on how many rows there are. One more block of outputs turns the rotated part.
+typedef __attribute__((__vector_size__(8 * sizeof(__bf16)))) __bf16 hg_bf16x8;
+typedef __attribute__((__vector_size__(4 * sizeof(__bf16)))) __bf16 hg_bf16x4;
+typedef __attribute__((__vector_size__(4 * sizeof(float)))) float hg_floatx4;
+
+// U: steps of 32 columns whose loads are all under way before the first product.
+template <int MT, int NT, int WAVES, int U>
+__global__ __launch_bounds__(64 * WAVES) void head_gemm_mfma_kernel(const bf16_t* __restrict__ x, long long xs_t, long long xs_h,
+                                                                    const bf16_t* __restrict__ w, bf16_t* __restrict__ y,
+                                                                    long long ys_t, long long ys_h,
+                                                                    const void* __restrict__ gate, int gate_mode,
+                                                                    long long gs_t, int rows, int N, int K, int n_chunks, int rot,
+                                                                    int x_rot_off, int y_rot_off, int halves,
+                                                                    const double* __restrict__ freqs, float gain,
+                                                                    const int* __restrict__ positions) {
+  const int h = blockIdx.z;
+  const int m0 = blockIdx.y * 16 * MT;
+  if ((int)blockIdx.x == n_chunks) {         // the rotated part of these rows
+    const int here = min(16 * MT, rows - m0), half = rot / 2;
+    for (int i = threadIdx.x; i < here * half; i += 64 * WAVES) {
+      const int t = m0 + i / half;
+      nhv_turn_pair(x + (size_t)t * xs_t + (size_t)h * xs_h + x_rot_off, y + (size_t)t * ys_t + (size_t)h * ys_h + y_rot_off,
+                    i % half, rot, halves, positions[t], freqs, gain);
+    }
+    return;
+  }
+  const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
+  const int col = lane & 15, grp = lane >> 4;
+  const int n0 = (blockIdx.x * WAVES + wave) * 16 * NT;
+  if (n0 >= N) return;
+  const bf16_t* wrow[NT];
+  bool n_ok[NT];
+#pragma unroll
+  for (int nt = 0; nt < NT; ++nt) {
+    const int n = n0 + nt * 16 + col;
+    n_ok[nt] = n < N;
+    wrow[nt] = w + ((size_t)h * N + (n_ok[nt] ? n : 0)) * K;
+  }
+  const bf16_t* xrow[MT];
+  bool m_ok[MT];
+#pragma unroll
+  for (int mt = 0; mt < MT; ++mt) {
+    const int m = m0 + mt * 16 + col;
+    m_ok[mt] = m < rows;
+    xrow[mt] = x + (size_t)(m_ok[mt] ? m : 0) * xs_t + (size_t)h * xs_h;
+  }
+  hg_floatx4 acc[MT][NT];
+#pragma unroll
+  for (int mt = 0; mt < MT; ++mt)
+#pragma unroll
+    for (int nt = 0; nt < NT; ++nt) acc[mt][nt] = hg_floatx4{0.f, 0.f, 0.f, 0.f};
+  hg_bf16x8 zero;
+#pragma unroll
+  for (int i = 0; i < 8; ++i) zero[i] = (__bf16)0.f;
+  for (int k0 = 0; k0 < K; k0 += 32 * U) {
+    hg_bf16x8 a[U][NT], b[U][MT];
+#pragma unroll
+    for (int u = 0; u < U; ++u) {
+      const int k = k0 + u * 32 + grp * 8;
+      const bool k_ok = k < K;               // K is a multiple of 8: a piece is inside or outside as a whole
+#pragma unroll
+      for (int nt = 0; nt < NT; ++nt) a[u][nt] = (n_ok[nt] && k_ok) ? *reinterpret_cast<const hg_bf16x8*>(wrow[nt] + k) : zero;
+#pragma unroll
+      for (int mt = 0; mt < MT; ++mt) b[u][mt] = (m_ok[mt] && k_ok) ? *reinterpret_cast<const hg_bf16x8*>(xrow[mt] + k) : zero;
+    }
+#pragma unroll
+    for (int u = 0; u < U; ++u)
+#pragma unroll
+      for (int mt = 0; mt < MT; ++mt)
+#pragma unroll
+        for (int nt = 0; nt < NT; ++nt)
+          acc[mt][nt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a[u][nt], b[u][mt], acc[mt][nt], 0, 0, 0);
+  }
+#pragma unroll
+  for (int mt = 0; mt < MT; ++mt) {
+    const int m = m0 + mt * 16 + col;
+    if (!m_ok[mt]) continue;
+#pragma unroll
+    for (int nt = 0; nt < NT; ++nt) {
+      const int n = n0 + nt * 16 + grp * 4;
+      float v[4];
+#pragma unroll
+      for (int j = 0; j < 4; ++j) {
+        v[j] = acc[mt][nt][j];
+        if (gate != nullptr && n + j < N) v[j] *= nhv_head_gate_of<bf16_t>(gate, gate_mode, gs_t, m, h, N, n + j);
+      }
+      bf16_t* dst = y + (size_t)m * ys_t + (size_t)h * ys_h + n;
+      if (n + 3 < N && ((uintptr_t)dst & 7) == 0) {
+        hg_bf16x4 four;
+#pragma unroll
+        for (int j = 0; j < 4; ++j) four[j] = (__bf16)v[j];
+        *reinterpret_cast<hg_bf16x4*>(dst) = four;
+      } else {
+#pragma unroll
+        for (int j = 0; j < 4; ++j)
+          if (n + j < N) dst[j] = (bf16_t)v[j];
+      }
+    }
   }
 }
 
-extern "C" int nhv_head_gate(void* y, const void* gate, long long gs_t, int rows, int H, int N, int dtype, void* stream) {
-  NHV_REQUIRE(rows > 0 && H > 0 && N > 0 && gate != nullptr, "head_gate: bad sizes rows=%d H=%d N=%d", rows, H, N);
-  const size_t total = (size_t)rows * H * N;
-  const int blocks = (int)((total + 255) / 256 > 65535 * 4 ? 65535 * 4 : (total + 255) / 256);
+extern "C" int nhv_head_gemm_bf16(const void* x, long long xs_t, long long xs_h, const void* w, void* y, long long ys_t,
+                                  long long ys_h, const void* gate, int gate_mode, long long gs_t, int rows, int H, int N, int K,
+                                  int rot, int x_rot_off, int y_rot_off, int halves, const void* freqs, float gain,
+                                  const void* positions, void* stream) {
+  NHV_REQUIRE(rows > 0 && H > 0 && H <= 65535 && N > 0 && K > 0, "head_gemm_bf16: bad sizes rows=%d H=%d N=%d K=%d", rows, H, N, K);
+  NHV_REQUIRE(K % 8 == 0 && xs_t % 8 == 0 && xs_h % 8 == 0 && (uintptr_t)x % 16 == 0 && (uintptr_t)w % 16 == 0,
+              "head_gemm_bf16: K=%d and the strides %lld, %lld must be multiples of 8, the operands 16 bytes aligned", K, xs_t, xs_h);
+  NHV_REQUIRE(rot >= 0 && rot % 2 == 0 && (rot == 0 || (freqs != nullptr && positions != nullptr)),
+              "head_gemm_bf16: a rotated part of %d entries needs frequencies and positions", rot);
   hipStream_t s = (hipStream_t)stream;
-  if (dtype == NHV_F32)
-    hipLaunchKernelGGL(head_gate_kernel<float>, dim3(blocks), dim3(256), 0, s, (float*)y, (const float*)gate, gs_t, H, N, total);
-  else if (dtype == NHV_BF16)
-    hipLaunchKernelGGL(head_gate_kernel<bf16_t>, dim3(blocks), dim3(256), 0, s, (bf16_t*)y, (const float*)gate, gs_t, H, N, total);
-  else
-    return nhv_fail("head_gate: unknown dtype %d", dtype);
-  NHV_LAUNCH_CHECK("head_gate");
+#define LAUNCH(MT, NT, WAVES, U)                                                                                          \
+  do {                                                                                                                    \
+    const int n_chunks = (N + 16 * NT * WAVES - 1) / (16 * NT * WAVES);                                                   \
+    const dim3 grid(n_chunks + (rot > 0 ? 1 : 0), (rows + 16 * MT - 1) / (16 * MT), H);                                   \
+    NHV_REQUIRE(grid.y <= 65535, "head_gemm_bf16: %d rows are too many", rows);                                           \
+    hipLaunchKernelGGL((head_gemm_mfma_kernel<MT, NT, WAVES, U>), grid, dim3(64 * WAVES), 0, s, (const bf16_t*)x, xs_t, xs_h, \
+                       (const bf16_t*)w, (bf16_t*)y, ys_t, ys_h, gate, gate_mode, gs_t, rows, N, K, n_chunks, rot,        \
+                       x_rot_off, y_rot_off, halves, (const double*)freqs, gain, (const int*)positions);                  \
+  } while (0)
+  if (rows <= 16) LAUNCH(1, 1, 1, 4);
+  else if (rows <= 64) LAUNCH(2, 1, 4, 4);
+  else LAUNCH(4, 2, 4, 2);
+#undef LAUNCH
+  NHV_LAUNCH_CHECK("head_gemm_bf16");
   return 0;
 }
 
 // ---------------------------------------------------------------- the rotated part of the queries
-// dst[t, h, d_off + j] = turned src[t, h, s_off + j], j < rot; src rows of ``s_row`` entries a head, dst of ``d_row``.
+// d[t, h, j] = turned s[t, h, j], j < rot; the rows of a (token, head) are s_t, s_h and d_t, d_h entries apart.
 template <typename T>
-__global__ void rotate_interleaved_kernel(const T* __restrict__ src, int s_row, int s_off, T* __restrict__ dst, int d_row,
-                                          int d_off, int rot, const double* __restrict__ freqs, float gain,
-                                          const int* __restrict__ positions, int H, size_t total) {
+__global__ void rotate_heads_kernel(const T* __restrict__ src, long long s_t, long long s_h, T* __restrict__ dst, long long d_t,
+                                    long long d_h, int rot, int halves, const double* __restrict__ freqs, float gain,
+                                    const int* __restrict__ positions, int H, size_t total) {
   const int half = rot / 2;
   for (size_t i = (size_t)blockIdx.x * blockDim.x + threadIdx.x; i < total; i += (size_t)gridDim.x * blockDim.x) {
     const int p = (int)(i % half);
-    const size_t th = i / half;
-    const int t = (int)(th / H);
-    float sn, cs;
-    nhv_turn_angle(positions[t], freqs[p], gain, &sn, &cs);
-    const T* s = src + th * s_row + s_off + 2 * p;
-    T* d = dst + th * d_row + d_off + 2 * p;
-    const float u = to_f32(s[0]), v = to_f32(s[1]);
-    d[0] = from_f32<T>(u * cs - v * sn);
-    d[1] = from_f32<T>(v * cs + u * sn);
+    const size_t t = i / half / H, h = i / half % H;
+    nhv_turn_pair(src + t * s_t + h * s_h, dst + t * d_t + h * d_h, p, rot, halves, positions[t], freqs, gain);
   }
 }
 
-extern "C" int nhv_rotate_interleaved(const void* src, int s_row, int s_off, void* dst, int d_row, int d_off, int rot,
-                                      const void* freqs, float gain, const void* positions, int T, int H, int dtype,
-                                      void* stream) {
-  NHV_REQUIRE(T > 0 && H > 0 && rot > 0 && rot % 2 == 0, "rotate_interleaved: bad sizes T=%d H=%d rot=%d", T, H, rot);
-  NHV_REQUIRE(s_off >= 0 && s_off + rot <= s_row && d_off >= 0 && d_off + rot <= d_row,
-              "rotate_interleaved: %d entries at %d of %d into %d of %d", rot, s_off, s_row, d_off, d_row);
+extern "C" int nhv_rotate_heads(const void* src, long long s_t, long long s_h, void* dst, long long d_t, long long d_h, int rot,
+                                int halves, const void* freqs, float gain, const void* positions, int T, int H, int dtype,
+                                void* stream) {
+  NHV_REQUIRE(T > 0 && H > 0 && rot > 0 && rot % 2 == 0, "rotate_heads: bad sizes T=%d H=%d rot=%d", T, H, rot);
+  NHV_REQUIRE(s_h >= rot && d_h >= rot && s_t >= s_h && d_t >= d_h, "rotate_heads: %d entries of rows %lld, %lld into %lld, %lld",
+              rot, s_t, s_h, d_t, d_h);
   const size_t total = (size_t)T * H * (rot / 2);
   const int blocks = (int)((total + 255) / 256 > 65535 * 4 ? 65535 * 4 : (total + 255) / 256);
   hipStream_t s = (hipStream_t)stream;
   if (dtype == NHV_F32)
-    hipLaunchKernelGGL(rotate_interleaved_kernel<float>, dim3(blocks), dim3(256), 0, s, (const float*)src, s_row, s_off,
-                       (float*)dst, d_row, d_off, rot, (const double*)freqs, gain, (const int*)positions, H, total);
+    hipLaunchKernelGGL(rotate_heads_kernel<float>, dim3(blocks), dim3(256), 0, s, (const float*)src, s_t, s_h, (float*)dst, d_t,
+                       d_h, rot, halves, (const double*)freqs, gain, (const int*)positions, H, total);
   else if (dtype == NHV_BF16)
-    hipLaunchKernelGGL(rotate_interleaved_kernel<bf16_t>, dim3(blocks), dim3(256), 0, s, (const bf16_t*)src, s_row, s_off,
-                       (bf16_t*)dst, d_row, d_off, rot, (const double*)freqs, gain, (const int*)positions, H, total);
+    hipLaunchKernelGGL(rotate_heads_kernel<bf16_t>, dim3(blocks), dim3(256), 0, s, (const bf16_t*)src, s_t, s_h, (bf16_t*)dst, d_t,
+                       d_h, rot, halves, (const double*)freqs, gain, (const int*)positions, H, total);
   else
-    return nhv_fail("rotate_interleaved: unknown dtype %d", dtype);
-  NHV_LAUNCH_CHECK("rotate_interleaved");
+    return nhv_fail("rotate_heads: unknown dtype %d", dtype);
+  NHV_LAUNCH_CHECK("rotate_heads");
   return 0;
 }

@@ -5,8 +5,8 @@
 //    weighted sum over that list;
 //  - nhv_rotary_split_write: splits a packed q | k | v projection whose value heads may have another size than
 //    the key heads, adds biases, turns queries and keys (angles from the position and a list of frequencies,
-//    taken in float here: no table, so no bound on positions) and optionally the values, and stores keys and
-//    values at the step's slots.
+//    taken in float here: no table, so no bound on positions) and optionally the values, scales queries by their
+//    position, mixes values with another layer's, and stores keys and values at the step's slots.
 // Statistics, angles and sums are float; rows are float or bfloat16.
 #include "nhv_common.h"
 #include <math.h>
@@ -155,13 +155,29 @@ extern "C" int nhv_depth_mix(const void* x, const void* a, const void* b, void* 
 // normed) on its own; Hq and Hkv count maps. The n maps of a key head are stored side by side as one key of n D entries
 // (there are Hkv / n key heads, and as many value heads); a query map goes out as a head of n D entries of its own
 // with zeros in the other maps' places, so that its product with the stored key is its product with its own map.
+// ``q_every`` > 0: queries at position p are multiplied by 1 + q_coef ln(floor((p + 1) / q_every) + 1). ``v_first``: value
+// head g becomes (1 - lam) v + lam v1, v1 the entries of value head g at v_first[t * v_first_ld + g E ...] (rows of
+// another layer's projection, of the same token), lam the number at v_lam; all in float, rounded once.
+struct SplitMore {
+  float q_coef;
+  double q_every;
+  const void* v_first;
+  long long v_first_ld;
+  const float* v_lam;
+};
+
+__device__ __forceinline__ float query_temperature(int pos, const SplitMore& more) {
+  if (!(more.q_every > 0.0)) return 1.0f;
+  return 1.0f + more.q_coef * logf((float)floor(((double)pos + 1.0) / more.q_every) + 1.0f);
+}
+
 template <typename T>
 __global__ void rotary_split_write_kernel(const T* __restrict__ qkv, const T* __restrict__ bias,
                                           const float* __restrict__ qk_freqs, int rot, const float* __restrict__ v_freqs,
                                           const int* __restrict__ positions, const int* __restrict__ slot_mapping,
                                           T* __restrict__ q_out, T* __restrict__ k_cache, T* __restrict__ v_cache, int Hq,
                                           int Hkv, int Hv, int D, int E, int heads, int ld, int interleaved, int unit,
-                                          float unit_eps, int v_from_k, int maps) {
+                                          float unit_eps, int v_from_k, int maps, const SplitMore more) {
   extern __shared__ float staged[];            // D floats where heads are normed: the head after bias and rotation
   const int t = blockIdx.x / heads, head = blockIdx.x % heads;
   const float p = (float)positions[t];
@@ -169,7 +185,10 @@ __global__ void rotary_split_write_kernel(const T* __restrict__ qkv, const T* __
   bool normed = false, pairs_adjacent = false;
   const float* freqs;
   T* dst;
+  const T* first = nullptr;                    // what a value head is mixed with, by lam
+  float factor = 1.0f, lam = 0.0f;
   if (head < Hq) {
+    factor = query_temperature(positions[t], more);
     col = head * D; size = D; half = rot / 2; freqs = qk_freqs; normed = unit; pairs_adjacent = interleaved;
     T* whole = q_out + ((size_t)t * Hq + head) * maps * D;
     dst = whole + (head % maps) * D;
@@ -188,12 +207,20 @@ __global__ void rotary_split_write_kernel(const T* __restrict__ qkv, const T* __
       col = v_from_k ? Hq * D + g * D : (Hq + Hkv) * D + g * E;
       size = E; half = v_freqs ? E / 2 : 0; freqs = v_freqs;
       dst = v_cache + ((size_t)slot * Hv + g) * E;
+      if (more.v_first) {
+        first = reinterpret_cast<const T*>(more.v_first) + (size_t)t * more.v_first_ld + g * E;
+        lam = *more.v_lam;
+      }
     }
   }
   const T* src = qkv + (size_t)t * ld + col;
   const T* bs = bias ? bias + col : nullptr;
   // the bias joins a projection that was rounded to the rows' type, and the sum is rounded again (the product's own result)
-  auto value = [&](int i) { return bs ? to_f32(from_f32<T>(to_f32(src[i]) + to_f32(bs[i]))) : to_f32(src[i]); };
+  auto value = [&](int i) {
+    float v = bs ? to_f32(from_f32<T>(to_f32(src[i]) + to_f32(bs[i]))) : to_f32(src[i]);
+    if (first) v = (1.0f - lam) * v + lam * to_f32(first[i]);
+    return v;
+  };
   if (!normed) {                               // nothing of the head depends on all of it: every entry goes out at once
     for (int i = threadIdx.x; i < size - half; i += blockDim.x) {
       if (i < half) {
@@ -201,10 +228,10 @@ __global__ void rotary_split_write_kernel(const T* __restrict__ qkv, const T* __
         const float u = value(a), v = value(b);
         float sn, cs;
         sincosf(p * freqs[i], &sn, &cs);
-        dst[a] = from_f32<T>(u * cs - v * sn);
-        dst[b] = from_f32<T>(v * cs + u * sn);
+        dst[a] = from_f32<T>((u * cs - v * sn) * factor);
+        dst[b] = from_f32<T>((v * cs + u * sn) * factor);
       } else {
-        dst[i + half] = from_f32<T>(value(i + half));
+        dst[i + half] = from_f32<T>(value(i + half) * factor);
       }
     }
     return;
@@ -227,7 +254,7 @@ __global__ void rotary_split_write_kernel(const T* __restrict__ qkv, const T* __
       ss = fmaf(x, x, ss);
     }
   }
-  const float r = 1.0f / sqrtf(wave_sum(ss) / (float)size + unit_eps);
+  const float r = factor / sqrtf(wave_sum(ss) / (float)size + unit_eps);
   __syncthreads();
   for (int i = threadIdx.x; i < size; i += blockDim.x) dst[i] = from_f32<T>(staged[i] * r);
 }
@@ -235,7 +262,8 @@ __global__ void rotary_split_write_kernel(const T* __restrict__ qkv, const T* __
 extern "C" int nhv_rotary_split_write(const void* qkv, const void* bias, const void* qk_freqs, int rot, const void* v_freqs,
                                       const void* positions, const void* slot_mapping, void* q_out, void* k_cache,
                                       void* v_cache, int T, int Hq, int Hkv, int D, int E, int with_kv, int more_columns,
-                                      int interleaved, int unit, float unit_eps, int v_from_k, int maps, int dtype,
+                                      int interleaved, int unit, float unit_eps, int v_from_k, int maps, float q_coef,
+                                      double q_every, const void* v_first, long long v_first_ld, const void* v_lam, int dtype,
                                       void* stream) {
   NHV_REQUIRE(more_columns >= 0, "rotary_split_write: %d columns after the projection", more_columns);
   NHV_REQUIRE(T > 0 && Hq > 0 && Hkv > 0 && D > 0 && E > 0, "rotary_split_write: bad sizes T=%d Hq=%d Hkv=%d D=%d E=%d", T, Hq, Hkv, D, E);
@@ -247,6 +275,10 @@ extern "C" int nhv_rotary_split_write(const void* qkv, const void* bias, const v
   NHV_REQUIRE(!v_from_k || (E == D && maps == 1), "rotary_split_write: values that are the keys as projected have the keys' size and one map");
   NHV_REQUIRE(!unit || unit_eps >= 0.f, "rotary_split_write: eps %g", (double)unit_eps);
   const int Hv = Hkv / maps;
+  NHV_REQUIRE(!v_first || (with_kv && v_lam && !v_freqs && v_first_ld >= (long long)Hv * E),
+              "rotary_split_write: values mixed with others need both, unturned, and rows of at least %d entries (%lld)", Hv * E, v_first_ld);
+  NHV_REQUIRE(q_every >= 0.0, "rotary_split_write: queries scaled in steps of %g positions", q_every);
+  const SplitMore more = {q_coef, q_every, v_first, v_first_ld, (const float*)v_lam};
   const int heads = with_kv ? Hq + Hkv + Hv : Hq;
   const int ld = (with_kv ? Hq * D + Hkv * D + (v_from_k ? 0 : Hv * E) : Hq * D) + more_columns;   // (columns that belong to another reader)
   NHV_REQUIRE((long long)T * heads < (1ll << 31), "rotary_split_write: too many tokens");
@@ -257,7 +289,7 @@ extern "C" int nhv_rotary_split_write(const void* qkv, const void* bias, const v
   hipLaunchKernelGGL(rotary_split_write_kernel<TT>, dim3((unsigned)((size_t)T * heads)), dim3(NHV_WAVE), lds, s,     \
                      (const TT*)qkv, (const TT*)bias, (const float*)qk_freqs, rot, (const float*)v_freqs,            \
                      (const int*)positions, (const int*)slot_mapping, (TT*)q_out, (TT*)k_cache, (TT*)v_cache, Hq, Hkv, Hv, \
-                     D, E, heads, ld, interleaved, unit, unit_eps, v_from_k, maps)
+                     D, E, heads, ld, interleaved, unit, unit_eps, v_from_k, maps, more)
   if (dtype == NHV_F32) LAUNCH(float);
   else if (dtype == NHV_BF16) LAUNCH(bf16_t);
   else return nhv_fail("rotary_split_write: unknown dtype %d", dtype);

@@ -161,15 +161,18 @@ class NativeBackend:
     def soft_cap(self, x, cap):
         self._call("nhv_soft_cap", _ptr(x), ctypes.c_size_t(x.numel()), ctypes.c_float(cap), _stream())
 
-    def rmsnorm(self, x, residual, residual_mode, w, y, eps):
+    def rmsnorm(self, x, residual, residual_mode, w, y, eps, rounds_between=True):
         T, H = x.shape
         self._call("nhv_rmsnorm", _ptr(x), _ptr(residual), residual_mode,
                    F32 if residual is None else dtype_code(residual), _ptr(w), _ptr(y), T, H, ctypes.c_float(eps),
-                   dtype_code(x), dtype_code(w), _stream())
+                   int(rounds_between), dtype_code(x), dtype_code(w), _stream())
 
     def silu_mul(self, gu, out):
+        self.gate_mul(gu, None, out, Gate())
+
+    def gate_mul(self, gu, bias, out, gate):
         T, I = out.shape
-        self._call("nhv_silu_mul", _ptr(gu), _ptr(out), T, I, dtype_code(gu), _stream())
+        self._call("nhv_gate_mul", _ptr(gu), _ptr(bias), _ptr(out), T, I, *gate.args(), dtype_code(gu), _stream())
 
     def gather_rows(self, x, rows, out):
         self._call("nhv_gather_rows", _ptr(x), _ptr(rows), _ptr(out), out.shape[0], x.shape[1], x.shape[0],
@@ -185,28 +188,25 @@ class NativeBackend:
                    dtype_code(qkv), wd, _stream())
 
     def paged_attention(self, q, k_cache, v_cache, out, batch: AttentionBatch, block_tables, scale, window, chunk=0,
-                        cap=0.0, sink=None, gate=None):
-        """``cap``: scores become cap tanh(score / cap); ``sink``: the score of one more term in the denominator;
+                        cap=0.0, sink=None, slopes=None, gate=None):
+        """``cap``: scores become cap tanh(score / cap); ``slopes`` [heads] float32: slope times the distance is taken off
+        the score; ``sink``: the score of one more term in the denominator (a number, or a tensor [heads] float32);
         ``gate`` = (tensor [tokens, columns] of q's element type, first column): the sigmoid of column + head
         multiplies the head's result."""
         T, Hq, D = q.shape
         _, page_size, Hkv, _ = k_cache.shape
         E = v_cache.shape[3]
-        plain = not cap and sink is None and gate is None
-        more = () if plain else (ctypes.c_float(cap or 0.0), int(sink is not None), ctypes.c_float(sink or 0.0), *_gate_args(gate))
+        sinks, sink = (sink, None) if isinstance(sink, torch.Tensor) else (None, sink)
+        options = (ctypes.c_float(cap or 0.0), int(sink is not None), ctypes.c_float(sink or 0.0), _ptr(sinks), _ptr(slopes),
+                   *_gate_args(gate))
+        plain = not cap and sink is None and sinks is None and slopes is None and gate is None
+        more = () if plain else options
         # the kernels on the matrix cores take value heads of the key heads' size; a chunk goes to them as a negative window
         fast = q.dtype == torch.bfloat16 and E == D and D % 16 == 0 and D <= 256
         if chunk:
             window = -chunk
-        if fast and batch.max_q_len == 1 and Hq // Hkv <= 16 and T <= 65535:
+        if fast and batch.max_q_len == 1 and T <= 65535:
             return self._decode_attention(q, k_cache, v_cache, out, batch, block_tables, scale, window, more)
-        if fast and plain and batch.max_q_len == 1 and Hkv == 1 and T <= 65535:
-            # more than 16 query heads on one key/value head (a cached latent): sixteen heads at a time
-            for h0 in range(0, Hq, 16):
-                part = torch.empty((T, min(16, Hq - h0), E), dtype=out.dtype, device=out.device)
-                self._decode_attention(q[:, h0:h0 + 16].contiguous(), k_cache, v_cache, part, batch, block_tables, scale, window)
-                out[:, h0:h0 + 16] = part
-            return None
         if fast and batch.num_requests <= 65535 and Hkv <= 65535:
             # prompt portions (and whatever single tokens share their batch) on the matrix cores
             return self._call("nhv_prefill_attention_bf16" + ("_more" if more else ""), _ptr(q), _ptr(k_cache), _ptr(v_cache),
@@ -215,8 +215,7 @@ class NativeBackend:
                               ctypes.c_float(scale), window, *more, _stream(), lib=self.attention_lib(D))
         self._call("nhv_paged_attention_generic", _ptr(q), _ptr(k_cache), _ptr(v_cache), _ptr(out),
                    _ptr(batch.token_req), _ptr(batch.positions), _ptr(block_tables), block_tables.shape[1], T, Hq, Hkv,
-                   D, E, page_size, ctypes.c_float(scale), 0 if chunk else window, chunk, ctypes.c_float(cap or 0.0),
-                   int(sink is not None), ctypes.c_float(sink or 0.0), *_gate_args(gate), dtype_code(q), _stream())
+                   D, E, page_size, ctypes.c_float(scale), 0 if chunk else window, chunk, *options, dtype_code(q), _stream())
 
     # -- layers that are not the pre-norm kind: norms with one number, sums over depth, rotation without a table --
     def scalar_rmsnorm(self, x, gain, y, eps):
@@ -238,11 +237,15 @@ class NativeBackend:
 
     def rotary_split_write(self, qkv, bias, qk_freqs, rot, v_freqs, positions, slot_mapping, q_out, k_cache, v_cache,
                            Hq, Hkv, D, E, with_kv, more_columns=0, interleaved=False, unit_eps=None, values_from_keys=False,
-                           maps=1):
+                           maps=1, temperature=None, mix=None):
+        coef, every = temperature if temperature is not None else (0.0, 0.0)
+        (first, column), lam = mix if mix is not None else ((None, 0), None)
+        first_p = None if first is None else ctypes.c_void_p(first.data_ptr() + column * first.element_size())
         self._call("nhv_rotary_split_write", _ptr(qkv), _ptr(bias), _ptr(qk_freqs), rot, _ptr(v_freqs), _ptr(positions),
                    _ptr(slot_mapping), _ptr(q_out), _ptr(k_cache), _ptr(v_cache), qkv.shape[0], Hq, Hkv, D, E,
                    int(with_kv), more_columns, int(interleaved), int(unit_eps is not None), ctypes.c_float(unit_eps or 0.0),
-                   int(values_from_keys), maps, dtype_code(qkv), _stream())
+                   int(values_from_keys), maps, ctypes.c_float(coef), ctypes.c_double(every), first_p,
+                   ctypes.c_longlong(0 if first is None else first.shape[1]), _ptr(lam), dtype_code(qkv), _stream())
 
     # -- what heads' results pass before the output projection; a layer normed on both sides of its sublayers --
     def differential_combine(self, a, lam, out, eps, post, gate=None):
@@ -332,50 +335,51 @@ class NativeBackend:
     def add_streams(self, x, a, b):
         self._call("nhv_add_streams", _ptr(x), _ptr(a), _ptr(b), ctypes.c_size_t(x.numel()), dtype_code(a), _stream())
 
-    def act_mul(self, gu, out, act):
-        T, I = out.shape
-        self._call("nhv_gelu_tanh_mul" if act == 1 else "nhv_silu_mul", _ptr(gu), _ptr(out), T, I, dtype_code(gu), _stream())
-
     # -- attention over a cached latent --
     def latent_prepare(self, a, q_off, q_rank, c_off, kv_rank, rot, wq, wc, eps, freqs, gain, positions, slot_mapping,
-                       cache, cq):
-        self._call("nhv_latent_prepare", _ptr(a), a.shape[1], q_off, q_rank, c_off, kv_rank, rot, _ptr(wq), _ptr(wc),
-                   ctypes.c_float(eps), _ptr(freqs), ctypes.c_float(gain), _ptr(positions), _ptr(slot_mapping), _ptr(cache),
-                   0 if cache is None else cache.shape[-1], _ptr(cq), a.shape[0], dtype_code(cq), _stream())
+                       cache, cq, row_dtype, halves=False):
+        self._call("nhv_latent_prepare", _ptr(a), dtype_code(a), a.shape[1], q_off, q_rank, c_off, kv_rank, rot, _ptr(wq),
+                   _ptr(wc), ctypes.c_float(eps), _ptr(freqs), ctypes.c_float(gain), _ptr(positions), _ptr(slot_mapping),
+                   _ptr(cache), 0 if cache is None else cache.shape[-1], _ptr(cq), int(halves), a.shape[0],
+                   _DTYPE_CODE[row_dtype], _stream())
 
-    def head_gemm(self, x, x_off, x_row, w, w_head, w_n, w_k, y, y_off, y_row, gate, gate_off, N, K, turn=None):
-        """y[t, h, y_off : y_off + N] = M_h x[t, h, x_off : x_off + K]; x and y are [rows, heads, x_row / y_row].
-        ``turn`` = (rot, x_rot_off, y_rot_off, freqs, gain, positions): also y[t, h, y_rot_off ...] = the ``rot`` entries
-        of x from x_rot_off on, turned. Returns whether the turning was done (up to 16 rows: in the same launch)."""
+    def head_gemm(self, x, x_off, w, w_head, w_n, w_k, y, y_off, gate, N, K, turn=None):
+        """y[t, h, y_off : y_off + N] = M_h x[t, h, x_off : x_off + K]; x and y are [rows, heads, row] with rows of
+        contiguous entries. ``gate`` = (tensor [rows, columns], first column, mode): mode 1, a float per head; mode 2, an
+        entry of x's type per result. ``turn`` = (rot, x_rot_off, y_rot_off, freqs, gain, positions, halves): also
+        y[t, h, y_rot_off ...] = the ``rot`` entries of x from x_rot_off on, turned. Returns whether the turning was done
+        (in the same launch)."""
         T, H = x.shape[0], x.shape[1]
         item = x.element_size()
         LL = ctypes.c_longlong
-        gate_p = None if gate is None else ctypes.c_void_p(gate.data_ptr() + 4 * gate_off)
         x_p, y_p = ctypes.c_void_p(x.data_ptr() + item * x_off), ctypes.c_void_p(y.data_ptr() + item * y_off)
-        gs_t = LL(0 if gate is None else gate.shape[1])
-        if T <= 16 and 16 * K * 4 + (64 * item + 16) * K <= 96 * 1024:      # (the kernel keeps the rows and a piece of the matrix in LDS)
-            rot, xr, yr, freqs, gain, positions = turn if turn is not None else (0, 0, 0, None, 1.0, None)
-            self._call("nhv_head_gemm_fewrows", x_p, LL(H * x_row), LL(x_row), _ptr(w), LL(w_head), LL(w_n), LL(w_k), y_p,
-                       LL(H * y_row), LL(y_row), gate_p, gs_t, T, H, N, K, rot, xr - x_off, yr - y_off, _ptr(freqs),
-                       ctypes.c_float(gain), _ptr(positions), dtype_code(x), _stream())
+        xs, ys = (LL(x.stride(0)), LL(x.stride(1))), (LL(y.stride(0)), LL(y.stride(1)))
+        gate_args = (None, 0, LL(0))
+        if gate is not None:
+            rows, col, mode = gate
+            gate_args = (ctypes.c_void_p(rows.data_ptr() + col * rows.element_size()), mode, LL(rows.shape[1]))
+        rot, xr, yr, freqs, gain, positions, halves = turn if turn is not None else (0, x_off, y_off, None, 1.0, None, False)
+        turn_args = (rot, xr - x_off, yr - y_off, int(halves), _ptr(freqs), ctypes.c_float(gain), _ptr(positions))
+        if (x.dtype == torch.bfloat16 and w_k == 1 and w_n == K and w_head == N * K and K % 8 == 0 and x.stride(0) % 8 == 0
+                and x.stride(1) % 8 == 0 and (x.data_ptr() + item * x_off) % 16 == 0 and w.data_ptr() % 16 == 0):
+            # matrices contiguous in k: the matrix cores, whatever the number of rows
+            self._call("nhv_head_gemm_bf16", x_p, *xs, _ptr(w), y_p, *ys, *gate_args, T, H, N, K, *turn_args, _stream())
             return True
-        if x.dtype == torch.bfloat16 and not self.own_kernels_only and (gate is None or (y_off == 0 and y_row == N)):
-            # many rows: the library's batched product, one matrix per head, on strided views
-            xv = x[:, :, x_off:x_off + K].transpose(0, 1)                         # [H, T, K]
-            wv = torch.as_strided(w, (H, K, N), (w_head, w_k, w_n))
-            yv = y[:, :, y_off:y_off + N].transpose(0, 1)
-            yv.copy_(torch.bmm(xv, wv))
-            if gate is not None:
-                self._call("nhv_head_gate", _ptr(y), gate_p, gs_t, T, H, N, dtype_code(y), _stream())
-            return False
-        self._call("nhv_head_gemm", x_p, LL(H * x_row), LL(x_row), _ptr(w), LL(w_head), LL(w_n), LL(w_k), y_p, LL(H * y_row),
-                   LL(y_row), gate_p, gs_t, T, H, N, K, dtype_code(x), _stream())
+        ws = (LL(w_head), LL(w_n), LL(w_k))
+        if T <= 16 and 16 * K * 4 + (64 * item + 16) * K <= 96 * 1024:      # (the kernel keeps the rows and a piece of the matrix in LDS)
+            self._call("nhv_head_gemm_fewrows", x_p, *xs, _ptr(w), *ws, y_p, *ys, *gate_args, T, H, N, K, *turn_args,
+                       dtype_code(x), _stream())
+            return True
+        self._call("nhv_head_gemm", x_p, *xs, _ptr(w), *ws, y_p, *ys, *gate_args, T, H, N, K, dtype_code(x), _stream())
         return False
 
-    def rotate_interleaved(self, src, s_off, dst, d_off, rot, freqs, gain, positions):
-        T, H, s_row = src.shape
-        self._call("nhv_rotate_interleaved", _ptr(src), s_row, s_off, _ptr(dst), dst.shape[2], d_off, rot, _ptr(freqs),
-                   ctypes.c_float(gain), _ptr(positions), T, H, dtype_code(src), _stream())
+    def rotate_heads(self, src, s_off, dst, d_off, rot, freqs, gain, positions, halves=False):
+        T, H = src.shape[0], src.shape[1]
+        LL = ctypes.c_longlong
+        self._call("nhv_rotate_heads", ctypes.c_void_p(src.data_ptr() + s_off * src.element_size()), LL(src.stride(0)),
+                   LL(src.stride(1)), ctypes.c_void_p(dst.data_ptr() + d_off * dst.element_size()), LL(dst.stride(0)),
+                   LL(dst.stride(1)), rot, int(halves), _ptr(freqs), ctypes.c_float(gain), _ptr(positions), T, H,
+                   dtype_code(src), _stream())
 
     # -- a feed-forward of many small experts --
     def route_topk(self, logits, ids, scores, bias=None, mode=0):
@@ -432,7 +436,7 @@ class NativeBackend:
         # split is longer than 1,024 keys. Measured at 2,176 and 8,192 keys, 1 to 64 requests, 8 key/value heads: the
         # best split length is 64 to 128 keys for 8 x 2,176 keys in all, 256 for 32 x 2,176 (62 against 64 us with
         # 512), 512 for 48 and 64 x 2,176 (110 against 118 us with 1,024) and for 16 x 8,192, 1,024 for 32 x 8,192.
-        want = max(1, T * Hkv * span // 1024)
+        want = max(1, T * Hkv * -(-(Hq // Hkv) // 16) * span // 1024)      # (a wave takes up to 16 heads of a key/value head)
         want = min(want, max(256, want * 2 // 3))
         # (splits of one round of 32 keys for one request of 2,100 keys, 525 waves: 3.64 against 3.66 ms a step; for two
         # requests 3.77 against 3.75: not taken)
@@ -730,31 +734,33 @@ class NativeBackend:
         reader_own, reader_library = reader_times
         return own + reader_own <= min(own, library) + self.norm_kernel_ms + min(reader_own, reader_library)
 
-    def fused_linear(self, x, w, bias, out, gated=False, row_scales=None, residual=None, sum_out=None, ss_out=None, next_w=None):
+    def fused_linear(self, x, w, bias, out, gated=False, row_scales=None, residual=None, sum_out=None, ss_out=None, next_w=None,
+                     gate=None):
         """The own few-rows product with what it may take over. ``row_scales`` = (squares [M, tiles], eps): x is a
         sum whose rows still lack their norm's scales, which are applied to the finished sums. ``residual``: the
         result is added to it (in place); ``sum_out`` gets the sum times ``next_w`` (the next norm's weight), rounded,
-        and ``ss_out`` the tiles' shares of the rows' sums of squares (``out`` is then not written)."""
+        and ``ss_out`` the tiles' shares of the rows' sums of squares (``out`` is then not written). ``gated``: w holds
+        two matrices (and ``bias`` their two biases), ``gate`` (a ``Gate``; None: SiLU) says what is made of their sums."""
         M, K = x.shape
         N = w.shape[0] // 2 if gated else w.shape[0]
         ss, eps = row_scales if row_scales is not None else (None, 0.0)
         self._call("nhv_gemm_fewrows_fused_bf16", _ptr(x), _ptr(ss), 0 if ss is None else ss.shape[1], ctypes.c_float(eps),
                    _ptr(w), _ptr(bias), _ptr(out), M, N, K, BF16 if out is None else dtype_code(out), int(gated),
                    _ptr(residual), F32 if residual is None else dtype_code(residual), _ptr(sum_out), _ptr(ss_out),
-                   _ptr(next_w), F32 if next_w is None else dtype_code(next_w), _stream())
+                   _ptr(next_w), F32 if next_w is None else dtype_code(next_w), *(gate or Gate()).args(), _stream())
 
     def scale_rows(self, x, squares, eps, out):
         self._call("nhv_scale_rows", _ptr(x), _ptr(squares), squares.shape[1], ctypes.c_float(eps), _ptr(out), x.shape[0],
                    x.shape[1], _stream())
 
-    def gated_linear(self, x, w, out, act: int = 0) -> bool:
-        """act(x Wg^T) * (x Wu^T) in one kernel, if this batch is one for the few-rows kernel; else False.
-        ``act``: 0 SiLU, 1 the tanh form of GELU (up to 16 rows)."""
+    def gated_linear(self, x, w, out, gate=None, bias=None) -> bool:
+        """A gate (a ``Gate``; None: SiLU) of x Wg^T and x Wu^T (+ bias) in one kernel, if this batch is one for the
+        few-rows kernel; else False. (SiLU without bias may also be one for the kernel of up to 64 rows.)"""
         M, K = x.shape
-        if act != 0:
+        if bias is not None or (gate is not None and gate.act != 0):
             if x.dtype == torch.bfloat16 and K % 8 == 0 and x.data_ptr() % 16 == 0 and w.data_ptr() % 16 == 0 and M <= self.few_rows:
-                self._call("nhv_gemm_fewrows_glu_act_bf16", _ptr(x), _ptr(w), _ptr(out), M, out.shape[1], K, dtype_code(out),
-                           act, _stream())
+                self._call("nhv_gemm_fewrows_gated_bf16", _ptr(x), _ptr(w), _ptr(bias), _ptr(out), M, out.shape[1], K,
+                           dtype_code(out), *(gate or Gate()).args(), _stream())
                 return True
             return False
         if (x.dtype == torch.bfloat16 and K % 8 == 0 and x.data_ptr() % 16 == 0 and w.data_ptr() % 16 == 0
@@ -988,12 +994,14 @@ def soft_cap_(logits: torch.Tensor, cap: float) -> torch.Tensor:
 
 
 def rmsnorm(x: torch.Tensor, w: torch.Tensor, eps: float, residual: torch.Tensor | None = None,
-            start_residual: bool = False, residual_float32: bool = True):
+            start_residual: bool = False, residual_float32: bool = True, rounds_between: bool = True):
     """``rmsnorm(x, w, eps)``: the norm of x.
     ``residual=r``: r += x in place (the sum is taken in float and normed unrounded; r keeps it in its own element
     type) and the norm of the sum is returned.
     ``start_residual=True``: returns (norm of x, the residual that later norms add to): a new float32 tensor holding
-    x, or, with ``residual_float32=False``, x itself (which later calls then add to in place)."""
+    x, or, with ``residual_float32=False``, x itself (which later calls then add to in place).
+    ``rounds_between``: the normed row is rounded to x's element type, then multiplied with the weight and rounded
+    again; False: it is rounded once, at the end."""
     _need(x.dim() == 2, "rmsnorm: x must be [tokens, width]")
     _dense(x, "rmsnorm: x")
     _dense(w, "rmsnorm: weight", (x.shape[1],))
@@ -1001,21 +1009,22 @@ def rmsnorm(x: torch.Tensor, w: torch.Tensor, eps: float, residual: torch.Tensor
           lambda: f"rmsnorm: weight of {w.dtype} with activations of {x.dtype}")
     dtype_code(x)
     y = torch.empty_like(x)
+    more = {} if rounds_between else {"rounds_between": False}
     if start_residual:
         _need(residual is None, "rmsnorm: a residual is either started or added to")
         if not residual_float32 and x.dtype != torch.float32:
-            backend().rmsnorm(x, None, 0, w, y, float(eps))
+            backend().rmsnorm(x, None, 0, w, y, float(eps), **more)
             return y, x
         residual = torch.empty(x.shape, dtype=torch.float32, device=x.device)
-        backend().rmsnorm(x, residual, 2, w, y, float(eps))
+        backend().rmsnorm(x, residual, 2, w, y, float(eps), **more)
         return y, residual
     if residual is not None:
         _dense(residual, "rmsnorm: residual", tuple(x.shape))
         _need(residual.dtype == x.dtype or residual.dtype == torch.float32,
               lambda: f"rmsnorm: residual of {residual.dtype} with rows of {x.dtype}")
-        backend().rmsnorm(x, residual, 1, w, y, float(eps))
+        backend().rmsnorm(x, residual, 1, w, y, float(eps), **more)
         return y
-    backend().rmsnorm(x, None, 0, w, y, float(eps))
+    backend().rmsnorm(x, None, 0, w, y, float(eps), **more)
     return y
 
 
@@ -1090,12 +1099,13 @@ def qk_rope_write(qkv, bias, q_norm_w, k_norm_w, eps, cos_sin, positions, slot_m
 
 def paged_attention(q, k_cache, v_cache, batch: AttentionBatch, block_tables, scale: float,
                     window: int | None = None, chunk: int | None = None, softcap: float | None = None,
-                    sink: float | None = None, gate: tuple | None = None) -> torch.Tensor:
+                    sink=None, slopes: torch.Tensor | None = None, gate: tuple | None = None) -> torch.Tensor:
     """Every query reads its request's keys up to its own position: all of them, the last ``window``, or (``chunk``)
     those of its own block of ``chunk`` positions counted from the request's start. The value heads may have another
     size than the key heads: the result is [tokens, heads, value size].
-    ``softcap``: a score s (after the scale) becomes softcap tanh(s / softcap). ``sink``: the softmax's denominator
-    holds one more term exp(sink), a key of that score without a value. ``gate`` = (rows [tokens, columns] of q's
+    ``softcap``: a score s (after the scale) becomes softcap tanh(s / softcap). ``slopes`` [heads] float32: slopes[h]
+    times the distance to the key is then taken off the score. ``sink``: the softmax's denominator holds one more term
+    exp(sink), a key of that score (one number, or a float32 tensor [heads]) without a value and without bias. ``gate`` = (rows [tokens, columns] of q's
     element type, first column): head h's result at token t is multiplied by sigmoid(rows[t, first column + h])."""
     _need(q.dim() == 3, "attention: q must be [tokens, heads, head_dim]")
     T, Hq, D = q.shape
@@ -1125,8 +1135,14 @@ def paged_attention(q, k_cache, v_cache, batch: AttentionBatch, block_tables, sc
     if softcap is not None:
         _need(softcap > 0, lambda: f"attention: the cap on scores must be positive, got {softcap}")
         more["cap"] = float(softcap)
-    if sink is not None:
+    if isinstance(sink, torch.Tensor):
+        _float32(sink, "attention: sinks", (Hq,))
+        more["sink"] = sink
+    elif sink is not None:
         more["sink"] = float(sink)
+    if slopes is not None:
+        _float32(slopes, "attention: slopes", (Hq,))
+        more["slopes"] = slopes
     if gate is not None:
         rows, col = gate
         _need(rows.dim() == 2 and rows.shape[0] == T and 0 <= col and col + Hq <= rows.shape[1],
@@ -1183,44 +1199,57 @@ def linear(x, w: torch.Tensor, bias: torch.Tensor | None = None, out_dtype=None,
     return out
 
 
-def gated_linear(x, w: torch.Tensor, activation: str = "silu") -> torch.Tensor:
-    """act(x . w[:I]^T) * (x . w[I:]^T) for a packed gate | up matrix w[2 I, K]: fused into one kernel for
-    few rows, else the matrix product followed by ``act_mul``. ``x`` may be a ``Normed`` (see ``linear``; with SiLU)."""
-    _need(activation in ACTIVATIONS, lambda: f"gated_linear: activation {activation!r} is not known ({sorted(ACTIVATIONS)} are)")
-    if activation != "silu":
-        x = dense(x)
-        _need(x.dim() == 2 and w.dim() == 2 and w.shape[0] % 2 == 0, "gated_linear: x must be [rows, in] and w [2 * out, in]")
-        _need(x.shape[1] == w.shape[1], lambda: f"gated_linear: x has {x.shape[1]} columns but w has {w.shape[1]}")
-        _dense(x, "gated_linear: x")
-        _dense(w, "gated_linear: w", dtype=x.dtype)
-        dtype_code(x)
-        fused = getattr(backend(), "gated_linear", None)
-        if fused is not None:
-            out = torch.empty((x.shape[0], w.shape[0] // 2), dtype=x.dtype, device=x.device)
-            if fused(x, w, out, ACTIVATIONS[activation]):
-                return out
-        return act_mul(linear(x, w), activation)
-    if isinstance(x, Normed):
-        normed, x = x, x.summed.weighted
-        _need(w.dim() == 2 and w.shape[0] % 2 == 0 and x.shape[1] == w.shape[1], "gated_linear: w must be [2 * out, in]")
-        _dense(w, "gated_linear: w", dtype=x.dtype)
-        if _may_fuse(x, w) and _fusion_pays(x, w, True):
-            out = torch.empty((x.shape[0], w.shape[0] // 2), dtype=x.dtype, device=x.device)
-            backend().fused_linear(x, w, None, out, gated=True, row_scales=(normed.summed.squares, float(normed.summed.eps)))
-            return out
-        x = normed.tensor()
+@dataclass(frozen=True)
+class Gate:
+    """What a gated feed-forward makes of a gate g and an up value u, in float: act 0, silu(g) u; act 1, the tanh form of
+    GELU of g, times u; act 2, with g' = min(g, limit) and u' = clamp(u, -limit, limit): g' sigmoid(alpha g') (u' + offset)."""
+
+    act: int = 0
+    limit: float = 0.0
+    alpha: float = 0.0
+    offset: float = 0.0
+
+    def args(self):
+        return self.act, ctypes.c_float(self.limit), ctypes.c_float(self.alpha), ctypes.c_float(self.offset)
+
+
+def gate_of(activation) -> Gate:
+    """``activation``: a ``Gate``, or the name of one without constants ("silu", "gelu_tanh")."""
+    if isinstance(activation, Gate):
+        return activation
+    _need(activation in ACTIVATIONS, lambda: f"gated product: activation {activation!r} is not known ({sorted(ACTIVATIONS)} are)")
+    return Gate(ACTIVATIONS[activation])
+
+
+def gated_linear(x, w: torch.Tensor, activation="silu", bias: torch.Tensor | None = None) -> torch.Tensor:
+    """A gate (``gate_of(activation)``) of x . w[:I]^T + bias[:I] and x . w[I:]^T + bias[I:] for a packed gate | up matrix
+    w[2 I, K]: fused into one kernel for few rows, else the matrix product followed by ``act_mul``. ``x`` may be a
+    ``Normed`` (see ``linear``)."""
+    gate = gate_of(activation)
+    plain = gate.act == 0 and bias is None
+    normed = x if isinstance(x, Normed) else None
+    if normed is not None:
+        x = normed.summed.weighted
     _need(x.dim() == 2 and w.dim() == 2 and w.shape[0] % 2 == 0, "gated_linear: x must be [rows, in] and w [2 * out, in]")
     _need(x.shape[1] == w.shape[1], lambda: f"gated_linear: x has {x.shape[1]} columns but w has {w.shape[1]}")
     _dense(x, "gated_linear: x")
     _dense(w, "gated_linear: w", dtype=x.dtype)
     dtype_code(x)
+    if bias is not None:
+        _dense(bias, "gated_linear: bias", (w.shape[0],), x.dtype)
+    if normed is not None:
+        if _may_fuse(x, w) and _fusion_pays(x, w, True):
+            out = torch.empty((x.shape[0], w.shape[0] // 2), dtype=x.dtype, device=x.device)
+            backend().fused_linear(x, w, bias, out, gated=True, row_scales=(normed.summed.squares, float(normed.summed.eps)),
+                                   **({} if plain else {"gate": gate}))
+            return out
+        x = normed.tensor()
     fused = getattr(backend(), "gated_linear", None)
     if fused is not None:
         out = torch.empty((x.shape[0], w.shape[0] // 2), dtype=x.dtype, device=x.device)
-        if fused(x, w, out):
+        if fused(x, w, out) if plain else fused(x, w, out, gate, bias):
             return out
-    return silu_mul(linear(x, w))
-
+    return act_mul(linear(x, w), gate, bias)
 
 
 # ------------------------------------------------------------------ two norms side by side, a hashed pair embedding
@@ -1296,31 +1325,36 @@ def add_streams_(x: torch.Tensor, a: torch.Tensor, b: torch.Tensor | None = None
     return x
 
 
-def act_mul(gate_up: torch.Tensor, activation: str) -> torch.Tensor:
-    """act(gate) * up for rows [gate | up]; ``activation``: "silu" or "gelu_tanh"."""
-    _need(activation in ACTIVATIONS, lambda: f"act_mul: activation {activation!r} is not known ({sorted(ACTIVATIONS)} are)")
-    if activation == "silu":
+def act_mul(gate_up: torch.Tensor, activation, bias: torch.Tensor | None = None) -> torch.Tensor:
+    """The gate (``gate_of(activation)``) of rows [gate | up], to which ``bias`` [2 width] is added first, in float."""
+    gate = gate_of(activation)
+    if gate.act == 0 and bias is None:
         return silu_mul(gate_up)
     _need(gate_up.dim() == 2 and gate_up.shape[1] % 2 == 0, "act_mul: input must be [tokens, 2 * width]")
     _dense(gate_up, "act_mul: input")
     dtype_code(gate_up)
+    if bias is not None:
+        _dense(bias, "act_mul: bias", (gate_up.shape[1],), gate_up.dtype)
     out = torch.empty((gate_up.shape[0], gate_up.shape[1] // 2), dtype=gate_up.dtype, device=gate_up.device)
-    backend().act_mul(gate_up, out, ACTIVATIONS[activation])
+    backend().gate_mul(gate_up, bias, out, gate)
     return out
 
 
 # ------------------------------------------------------------------ attention over a cached latent
-def latent_prepare(a: torch.Tensor, q_off: int, q_rank: int, c_off: int, kv_rank: int, rot: int, wq: torch.Tensor,
+def latent_prepare(a: torch.Tensor, q_off: int, q_rank: int, c_off: int, kv_rank: int, rot: int, wq: torch.Tensor | None,
                    wc: torch.Tensor | None, eps: float, freqs: torch.Tensor | None, gain: float, positions: torch.Tensor,
-                   slot_mapping: torch.Tensor | None, cache: torch.Tensor | None, out_dtype) -> torch.Tensor:
-    """``a`` [tokens, columns] float32 holds the packed down projections of the step's rows. Returns the query latent
-    (columns q_off ..., RMS-normed with ``wq``) as [tokens, q_rank] in ``out_dtype``; where ``kv_rank`` > 0 and a
-    ``slot_mapping`` is given, stores [RMS-normed columns c_off ... | the ``rot`` columns after them, turned pairwise
-    (2i, 2i + 1) by position * freqs[i], cosine and sine times ``gain``] at the tokens' slots of ``cache``."""
+                   slot_mapping: torch.Tensor | None, cache: torch.Tensor | None, out_dtype, halves: bool = False):
+    """``a`` [tokens, columns] (float32 or ``out_dtype``) holds the packed down projections of the step's rows. Returns the
+    query latent (columns q_off ..., RMS-normed with ``wq``) as [tokens, q_rank] in ``out_dtype`` (``q_rank`` 0: there is
+    none, None is returned); where ``kv_rank`` > 0 and a ``slot_mapping`` is given, stores [RMS-normed columns c_off ... |
+    the ``rot`` columns after them, turned pairwise by position * freqs[i], cosine and sine times ``gain`` | zeros] at the
+    tokens' slots of ``cache``. Pairs are (2i, 2i + 1), or (i, i + rot / 2) with ``halves``."""
     T = a.shape[0]
     _need(a.dim() == 2, "latent_prepare: a must be [tokens, columns]")
-    _dense(a, "latent_prepare: a", dtype=torch.float32)
-    _float32(wq, "latent_prepare: query norm weight", (q_rank,))
+    _need(a.dtype in (torch.float32, out_dtype), lambda: f"latent_prepare: a of {a.dtype} for rows of {out_dtype}")
+    _dense(a, "latent_prepare: a")
+    if q_rank:
+        _float32(wq, "latent_prepare: query norm weight", (q_rank,))
     _dense(positions, "latent_prepare: positions", (T,), torch.int32)
     _need(out_dtype in _DTYPE_CODE, lambda: f"latent_prepare: rows of {out_dtype}")
     store = kv_rank > 0 and slot_mapping is not None
@@ -1332,25 +1366,38 @@ def latent_prepare(a: torch.Tensor, q_off: int, q_rank: int, c_off: int, kv_rank
         _dense(cache, "latent_prepare: cache", dtype=out_dtype)
         if rot:
             _dense(freqs, "latent_prepare: frequencies", (rot // 2,), torch.float64)
-    cq = torch.empty((T, q_rank), dtype=out_dtype, device=a.device)
-    backend().latent_prepare(a, q_off, q_rank, c_off, kv_rank if store else 0, rot if store else 0, wq, wc if store else None,
-                             float(eps), freqs if store and rot else None, float(gain), positions,
-                             slot_mapping if store else None, cache if store else None, cq)
+    _need(q_rank > 0 or store, "latent_prepare: nothing to do")
+    cq = torch.empty((T, q_rank), dtype=out_dtype, device=a.device) if q_rank else None
+    backend().latent_prepare(a, q_off, q_rank, c_off, kv_rank if store else 0, rot if store else 0, wq if q_rank else None,
+                             wc if store else None, float(eps), freqs if store and rot else None, float(gain), positions,
+                             slot_mapping if store else None, cache if store else None, cq, out_dtype,
+                             **({"halves": True} if halves else {}))
     return cq
 
 
-def head_gemm(x: torch.Tensor, w: torch.Tensor, transposed: bool, N: int, K: int, x_off: int = 0, out: torch.Tensor | None = None,
-              out_off: int = 0, gate: torch.Tensor | None = None, gate_off: int = 0, turn: tuple | None = None) -> torch.Tensor:
-    """One small matrix per head: out[t, h, out_off : out_off + N] = M_h x[t, h, x_off : x_off + K], sums in float.
-    ``w`` is [heads * K, N] with M_h = w[h K : (h + 1) K]^T (``transposed``: x is multiplied from the left by the
-    block's transpose) or [heads * N, K] with M_h = w[h N : (h + 1) N]. ``gate`` [tokens, columns] float32: the result
-    of (t, h) is multiplied by sigmoid(gate[t, gate_off + h]). ``out``: [tokens, heads, row] to write into.
-    ``turn`` = (rot, x_rot_off, out_rot_off, freqs, gain, positions): also out[t, h, out_rot_off + j] = x[t, h,
-    x_rot_off + j] turned, j < rot, as ``rotate_interleaved`` does (for few rows in the same launch)."""
-    _need(x.dim() == 3, "head_gemm: x must be [tokens, heads, row]")
-    T, H, x_row = x.shape
-    _dense(x, "head_gemm: x")
+def _head_rows(x: torch.Tensor, name: str) -> None:
+    """[tokens, heads, row] with contiguous rows; tokens and heads may lie any distance apart (a view of packed rows)."""
+    _need(x.dim() == 3, lambda: f"{name} must be [tokens, heads, row]")
+    want = backend().device_type
+    _need(x.device.type == want, lambda: f"{name}: must live on a '{want}' device, is on {x.device}")
+    _need(x.shape[2] == 1 or x.stride(2) == 1, lambda: f"{name}: the entries of a head must be contiguous")
+    _need(x.shape[1] == 1 or x.stride(1) >= x.shape[2], lambda: f"{name}: heads overlap")
     dtype_code(x)
+
+
+def head_gemm(x: torch.Tensor, w: torch.Tensor, transposed: bool, N: int, K: int, x_off: int = 0, out: torch.Tensor | None = None,
+              out_off: int = 0, gate: tuple | None = None, turn: tuple | None = None) -> torch.Tensor:
+    """One small matrix per head: out[t, h, out_off : out_off + N] = M_h x[t, h, x_off : x_off + K], sums in float. ``x``
+    [tokens, heads, row] may be a view of packed rows.
+    ``w`` is [heads * K, N] with M_h = w[h K : (h + 1) K]^T (``transposed``: x is multiplied from the left by the
+    block's transpose) or [heads * N, K] with M_h = w[h N : (h + 1) N] (the form that the matrix cores take). ``gate`` =
+    (tensor [tokens, columns], first column): float32 with one column a head, the result of (t, h) is multiplied by
+    sigmoid(gate[t, column + h]); with ``per entry`` as a third element, of x's element type with N columns a head, entry n
+    by sigmoid(gate[t, column + h N + n]). ``out``: [tokens, heads, row] to write into.
+    ``turn`` = (rot, x_rot_off, out_rot_off, freqs, gain, positions, halves): also out[t, h, out_rot_off + j] = x[t, h,
+    x_rot_off + j] turned, j < rot, as ``rotate_heads`` does (where the kernel can, in the same launch)."""
+    _head_rows(x, "head_gemm: x")
+    T, H, x_row = x.shape
     _need(0 <= x_off and x_off + K <= x_row, lambda: f"head_gemm: columns {x_off}+{K} of {x_row}")
     _dense(w, "head_gemm: w", (H * K, N) if transposed else (H * N, K), x.dtype)
     if out is None:
@@ -1359,41 +1406,44 @@ def head_gemm(x: torch.Tensor, w: torch.Tensor, transposed: bool, N: int, K: int
           lambda: f"head_gemm: out {tuple(out.shape)} for {N} columns at {out_off}")
     _dense(out, "head_gemm: out", dtype=x.dtype)
     if gate is not None:
-        _need(gate.dim() == 2 and gate.shape[0] == T and 0 <= gate_off and gate_off + H <= gate.shape[1],
-              lambda: f"head_gemm: gate {tuple(gate.shape)} for {H} heads at {gate_off}")
-        _dense(gate, "head_gemm: gate", dtype=torch.float32)
+        rows, col, per_entry = (*gate, "per head")[:3]
+        _need(per_entry in ("per head", "per entry"), lambda: f"head_gemm: a gate {per_entry!r}")
+        n = H * N if per_entry == "per entry" else H
+        _need(rows.dim() == 2 and rows.shape[0] == T and 0 <= col and col + n <= rows.shape[1],
+              lambda: f"head_gemm: gate {tuple(rows.shape)}, {n} columns at {col}")
+        _dense(rows, "head_gemm: gate", dtype=x.dtype if per_entry == "per entry" else torch.float32)
+        gate = (rows, int(col), 2 if per_entry == "per entry" else 1)
     if transposed:
         w_head, w_n, w_k = K * N, 1, N
     else:
         w_head, w_n, w_k = N * K, K, 1
     if turn is None:
-        backend().head_gemm(x, x_off, x_row, w, w_head, w_n, w_k, out, out_off, out.shape[2], gate, gate_off, N, K)
+        backend().head_gemm(x, x_off, w, w_head, w_n, w_k, out, out_off, gate, N, K)
         return out
-    rot, x_rot, out_rot, freqs, gain, positions = turn
+    rot, x_rot, out_rot, freqs, gain, positions, halves = turn
     _need(rot > 0 and rot % 2 == 0 and 0 <= x_rot and x_rot + rot <= x_row and 0 <= out_rot and out_rot + rot <= out.shape[2],
           lambda: f"head_gemm: {rot} turned entries at {x_rot} of {x_row} into {out_rot} of {out.shape[2]}")
     _dense(freqs, "head_gemm: frequencies", (rot // 2,), torch.float64)
     _dense(positions, "head_gemm: positions", (T,), torch.int32)
-    done = backend().head_gemm(x, x_off, x_row, w, w_head, w_n, w_k, out, out_off, out.shape[2], gate, gate_off, N, K,
-                               turn=(rot, x_rot, out_rot, freqs, float(gain), positions))
+    done = backend().head_gemm(x, x_off, w, w_head, w_n, w_k, out, out_off, gate, N, K,
+                               turn=(rot, x_rot, out_rot, freqs, float(gain), positions, bool(halves)))
     if not done:
-        backend().rotate_interleaved(x, x_rot, out, out_rot, rot, freqs, float(gain), positions)
+        backend().rotate_heads(x, x_rot, out, out_rot, rot, freqs, float(gain), positions, **({"halves": True} if halves else {}))
     return out
 
 
-def rotate_interleaved(src: torch.Tensor, s_off: int, dst: torch.Tensor, d_off: int, rot: int, freqs: torch.Tensor,
-                       gain: float, positions: torch.Tensor) -> torch.Tensor:
-    """dst[t, h, d_off + j] = src[t, h, s_off + j] turned, j < rot: pairs (2i, 2i + 1) by position * freqs[i]."""
-    _need(src.dim() == 3 and dst.dim() == 3 and tuple(src.shape[:2]) == tuple(dst.shape[:2]),
-          "rotate_interleaved: src and dst must be [tokens, heads, row]")
-    _dense(src, "rotate_interleaved: src")
-    _dense(dst, "rotate_interleaved: dst", dtype=src.dtype)
-    dtype_code(src)
+def rotate_heads(src: torch.Tensor, s_off: int, dst: torch.Tensor, d_off: int, rot: int, freqs: torch.Tensor,
+                 gain: float, positions: torch.Tensor, halves: bool = False) -> torch.Tensor:
+    """dst[t, h, d_off + j] = src[t, h, s_off + j] turned, j < rot: pairs (2i, 2i + 1), or (i, i + rot / 2) with ``halves``,
+    by position * freqs[i]."""
+    _head_rows(src, "rotate_heads: src")
+    _need(dst.dim() == 3 and tuple(src.shape[:2]) == tuple(dst.shape[:2]), "rotate_heads: src and dst must be [tokens, heads, row]")
+    _dense(dst, "rotate_heads: dst", dtype=src.dtype)
     _need(rot > 0 and rot % 2 == 0 and 0 <= s_off and s_off + rot <= src.shape[2] and 0 <= d_off and d_off + rot <= dst.shape[2],
-          lambda: f"rotate_interleaved: {rot} entries at {s_off} of {src.shape[2]} into {d_off} of {dst.shape[2]}")
-    _dense(freqs, "rotate_interleaved: frequencies", (rot // 2,), torch.float64)
-    _dense(positions, "rotate_interleaved: positions", (src.shape[0],), torch.int32)
-    backend().rotate_interleaved(src, s_off, dst, d_off, rot, freqs, float(gain), positions)
+          lambda: f"rotate_heads: {rot} entries at {s_off} of {src.shape[2]} into {d_off} of {dst.shape[2]}")
+    _dense(freqs, "rotate_heads: frequencies", (rot // 2,), torch.float64)
+    _dense(positions, "rotate_heads: positions", (src.shape[0],), torch.int32)
+    backend().rotate_heads(src, s_off, dst, d_off, rot, freqs, float(gain), positions, **({"halves": True} if halves else {}))
     return dst
 
 
@@ -1548,7 +1598,8 @@ def rotary_split_write(qkv: torch.Tensor, bias: torch.Tensor | None, qk_freqs: t
                        v_freqs: torch.Tensor | None, positions: torch.Tensor, slot_mapping, k_cache, v_cache,
                        num_heads: int, num_kv_heads: int, head_dim: int, value_dim: int, with_kv: bool = True,
                        more_columns: int = 0, interleaved: bool = False, unit_eps: float | None = None,
-                       values_from_keys: bool = False, maps: int = 1) -> torch.Tensor:
+                       values_from_keys: bool = False, maps: int = 1, temperature: tuple | None = None,
+                       mix: tuple | None = None) -> torch.Tensor:
     """Splits the packed projection q | k | v (``with_kv``) or q alone (followed by ``more_columns`` columns that
     another reader takes), adds the bias, turns pair (i, i + r) of every
     query and key head by position * qk_freqs[i] (r = len(qk_freqs); the coordinates from 2 r on pass), turns the
@@ -1561,7 +1612,10 @@ def rotary_split_write(qkv: torch.Tensor, bias: torch.Tensor | None, qk_freqs: t
     maps. A key head's n maps are stored side by side as one key of n ``head_dim`` entries (the caches have
     num_kv_heads / n heads, and the projection as many value heads); every query map is returned as a head of its own,
     [tokens, num_heads, n head_dim], with zeros in the other maps' places, so that its product with a stored key is the
-    product with its own map."""
+    product with its own map. ``temperature`` = (coef, every): queries at position p are multiplied by
+    1 + coef ln(floor((p + 1) / every) + 1). ``mix`` = ((rows [tokens, columns], first column), lam): the value stored is
+    (1 - lam) v + lam v1, v1 the same entries of ``rows`` (another layer's packed projection of the same tokens), lam one
+    float32 number on the device."""
     T = qkv.shape[0]
     _need(maps >= 1 and num_heads % maps == 0 and num_kv_heads % maps == 0,
           lambda: f"rotary_split_write: {maps} maps with {num_heads} and {num_kv_heads} heads")
@@ -1578,6 +1632,19 @@ def rotary_split_write(qkv: torch.Tensor, bias: torch.Tensor | None, qk_freqs: t
         more["values_from_keys"] = True
     if maps != 1:
         more["maps"] = int(maps)
+    if temperature is not None:
+        _need(temperature[1] > 0, lambda: f"rotary_split_write: queries scaled in steps of {temperature[1]} positions")
+        more["temperature"] = (float(temperature[0]), float(temperature[1]))
+    if mix is not None:
+        (rows, col), lam = mix
+        _need(with_kv and v_freqs is None, "rotary_split_write: values that are mixed are the layer's own and are not turned")
+        n = (num_kv_heads // maps) * value_dim
+        _need(rows.dim() == 2 and rows.shape[0] == T and 0 <= col and col + n <= rows.shape[1],
+              lambda: f"rotary_split_write: values {tuple(rows.shape)} to mix with, {n} columns from {col}")
+        _dense(rows, "rotary_split_write: values to mix with", dtype=qkv.dtype)
+        _need(lam.numel() == 1, "rotary_split_write: values are mixed by one number")
+        _dense(lam, "rotary_split_write: lambda", dtype=torch.float32)
+        more["mix"] = ((rows, int(col)), lam)
     _need(more_columns >= 0, "rotary_split_write: a negative number of further columns")
     _dense(qkv, "rotary_split_write: qkv", (T, width + more_columns))
     dtype_code(qkv)

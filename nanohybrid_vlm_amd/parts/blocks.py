@@ -11,21 +11,29 @@ from .base import BLOCKS, ParamSpec, Part
 class PreNormBlock(Part):
     """r += mixer(norm(r)); r += feed_forward(norm(r)), with each addition folded into
     the next norm (nanovllm/models/qwen3.py:152-159): the block takes and returns
-    (hidden, residual), and ``residual`` is None before the first block."""
+    (hidden, residual), and ``residual`` is None before the first block. The feed-forward
+    may be absent."""
 
     # the norms this arrangement takes, by the names of its constructor's arguments: the model builds one per slot
     # from the layer's description (``LayerSpec.norms[slot]``, else ``LayerSpec.norm``)
     norm_slots = ("mixer_norm", "feed_forward_norm")
 
-    def __init__(self, mixer, feed_forward, mixer_norm, feed_forward_norm):
+    def __init__(self, mixer, feed_forward, mixer_norm, feed_forward_norm, keeps_unused_norm: bool = False):
+        """``keeps_unused_norm``: a block without feed-forward holds its second norm's tensors all the same (a
+        checkpoint that stores them), unused."""
         self.mixer = mixer
         self.feed_forward = feed_forward
         self.mixer_norm = mixer_norm
         self.feed_forward_norm = feed_forward_norm
+        self.keeps_unused_norm = bool(keeps_unused_norm)
 
     def children(self):
-        return {"mixer_norm": self.mixer_norm, "mixer": self.mixer,
-                "feed_forward_norm": self.feed_forward_norm, "feed_forward": self.feed_forward}
+        out = {"mixer_norm": self.mixer_norm, "mixer": self.mixer}
+        if self.feed_forward is not None or self.keeps_unused_norm:
+            out["feed_forward_norm"] = self.feed_forward_norm
+        if self.feed_forward is not None:
+            out["feed_forward"] = self.feed_forward
+        return out
 
     @property
     def takes_summed(self) -> bool:
@@ -45,6 +53,8 @@ class PreNormBlock(Part):
             x, residual = self.mixer_norm.forward_start(hidden)
         else:
             x, residual = self.mixer_norm.forward_add(hidden, residual, **_deferred(self.mixer_norm, mixer))
+        if ff is None:
+            return mixer.forward(x, step, cache, **_add_to(mixer, next_norm, residual, next_reader)), residual
         x = mixer.forward(x, step, cache, **_add_to(mixer, self.feed_forward_norm, residual, ff))
         x, residual = self.feed_forward_norm.forward_add(x, residual, **_deferred(self.feed_forward_norm, ff))
         x = ff.forward(x, step, **_add_to(ff, next_norm, residual, next_reader))

@@ -13,21 +13,34 @@ class SwiGLU(Part):
     ``intermediate_size`` rows are the gate (nanovllm/layers/linear.py:102-108,
     nanovllm/layers/activation.py:10-11)."""
 
-    def __init__(self, hidden_size: int, intermediate_size: int, activation: str = "silu"):
-        """``activation``: what the gate passes, "silu" (the reference's) or "gelu_tanh"."""
-        if activation not in ops.ACTIVATIONS:
-            raise ValueError(f"activation {activation!r} is not known ({sorted(ops.ACTIVATIONS)} are)")
+    def __init__(self, hidden_size: int, intermediate_size: int, activation: str = "silu", bias: bool = False,
+                 limit: float | None = None, alpha: float = 1.0, offset: float = 0.0):
+        """``activation``: what the gate passes, "silu" (the reference's), "gelu_tanh", or "clamped_swish": with
+        g' = min(g, ``limit``) and u' = clamp(u, -limit, limit), the result is g' sigmoid(``alpha`` g') (u' + ``offset``).
+        ``bias``: all three projections have biases."""
+        if activation == "clamped_swish":
+            if limit is None or not limit > 0:
+                raise ValueError(f"a clamped gate needs a positive limit, got {limit}")
+            self.gate = ops.Gate(2, float(limit), float(alpha), float(offset))
+        elif activation in ops.ACTIVATIONS:
+            self.gate = ops.gate_of(activation)
+        else:
+            raise ValueError(f"activation {activation!r} is not known ({sorted(ops.ACTIVATIONS)} and 'clamped_swish' are)")
         self.hidden_size = hidden_size
         self.intermediate_size = intermediate_size
-        self.activation = activation
-        self.gate_up_weight = None
-        self.down_weight = None
+        self.activation, self.bias = activation, bool(bias)
+        self.gate_up_weight = self.gate_up_bias = None
+        self.down_weight = self.down_bias = None
 
     def param_specs(self):
-        return {
+        specs = {
             "gate_up.weight": ParamSpec((2 * self.intermediate_size, self.hidden_size)),
             "down.weight": ParamSpec((self.hidden_size, self.intermediate_size)),
         }
+        if self.bias:
+            specs["gate_up.bias"] = ParamSpec((2 * self.intermediate_size,), init="zeros")
+            specs["down.bias"] = ParamSpec((self.hidden_size,), init="zeros")
+        return specs
 
     takes_deferred_norm = True    # x goes straight into a product, which can norm it
     adds_to_residual = True       # the down projection can make the addition to the residual stream
@@ -37,9 +50,8 @@ class SwiGLU(Part):
         return self.gate_up_weight, True
 
     def forward(self, x, step, add_to=None):
-        if self.activation != "silu":
-            return ops.linear(ops.gated_linear(x, self.gate_up_weight, self.activation), self.down_weight, add_to=add_to)
-        return ops.linear(ops.gated_linear(x, self.gate_up_weight), self.down_weight, add_to=add_to)
+        y = ops.gated_linear(x, self.gate_up_weight, self.gate, self.gate_up_bias)
+        return ops.linear(y, self.down_weight, self.down_bias, add_to=add_to)
 
 
 @FEED_FORWARDS.register("plain_mlp")

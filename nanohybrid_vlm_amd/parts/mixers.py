@@ -1,6 +1,7 @@
 """Token mixers. ``GQAAttention`` follows nanovllm/models/qwen3.py:14-88 and
 nanovllm/layers/attention.py:43-75. ``RotaryAttention`` is softmax attention in a more general make (value heads of
-their own size, biases, a chunk mask, turned values, keys and values lent by another layer), ``GatedDeltaRule`` a
+their own size, biases, a window or a chunk, sinks, a bias by distance, turned or mixed values, keys and values lent by
+another layer), ``GatedDeltaRule`` a
 recurrent mixer with a matrix of state per head, ``NormedPair`` two mixers side by side, ``DifferentialAttention`` the
 difference of two softmax maps per head over the same values."""
 from __future__ import annotations
@@ -101,13 +102,20 @@ class RotaryAttention(Part):
     last ``num_heads * value_dim`` rows of the packed projection. ``rotation``: which coordinates make a pair,
     "halves" (i, i + r / 2) or "interleaved" (2i, 2i + 1). ``unit_norm_eps``: after the rotation every query and key head
     is divided by its root mean square (this eps under the root). ``values_are_keys``: there is no value projection; a
-    token's values are its keys as projected, before rotation and norm (``value_dim`` equals ``head_dim``)."""
+    token's values are its keys as projected, before rotation and norm (``value_dim`` equals ``head_dim``).
+    ``learned_sink``: the sink's score is a parameter, one number per head. ``distance_bias``: slope_h times the distance
+    to the key is taken off head h's scores (after scale and cap), slope_h = 2^(-8 (h + 1) / num_heads), h from 0.
+    ``temperature`` (coef, every): queries at position p are multiplied by 1 + coef ln(floor((p + 1) / every) + 1).
+    ``mix_values``: "first": the layer's values are kept for later layers of the same step; "later": what is stored (and
+    read) is (1 - lam) v + lam v1, v1 the same token's values of the layer that said "first", lam a parameter (the "first"
+    layer holds one as well, unused)."""
 
     def __init__(self, hidden_size: int, num_heads: int, num_kv_heads: int, head_dim: int, value_dim: int, scale: float,
                  bias: bool, position, chunk: int | None = None, window: int | None = None, rotate_values: bool = False,
                  own_kv: bool = True, softcap: float | None = None, sink: float | None = None, head_gate: bool = False,
                  element_gate: bool = False, rotation: str = "halves", unit_norm_eps: float | None = None,
-                 values_are_keys: bool = False):
+                 values_are_keys: bool = False, learned_sink: bool = False, distance_bias: bool = False,
+                 temperature: tuple | None = None, mix_values: str | None = None):
         if num_heads % num_kv_heads:
             raise ValueError(f"{num_heads} heads are not a multiple of {num_kv_heads} key/value heads")
         if window and chunk:
@@ -133,7 +141,18 @@ class RotaryAttention(Part):
         self.softcap, self.sink, self.head_gate = softcap, sink, bool(head_gate)
         self.element_gate, self.rotation, self.unit_norm_eps = bool(element_gate), rotation, unit_norm_eps
         self.values_are_keys = bool(values_are_keys)
+        if learned_sink and sink is not None:
+            raise ValueError("a sink is one number for the layer or a parameter per head, not both")
+        if temperature is not None and not temperature[1] > 0:
+            raise ValueError(f"queries are scaled in steps of a positive number of positions, got {temperature[1]}")
+        if mix_values not in (None, "first", "later"):
+            raise ValueError(f"mix_values {mix_values!r} is not known ('first' and 'later' are)")
+        if mix_values and (values_are_keys or rotate_values or bias or not own_kv):
+            raise ValueError("values that are mixed with another layer's are projections of their own, without bias, and not turned")
+        self.learned_sink, self.distance_bias, self.mix_values = bool(learned_sink), bool(distance_bias), mix_values
+        self.temperature = None if temperature is None else (float(temperature[0]), float(temperature[1]))
         self.qkv_weight = self.qkv_bias = self.o_weight = None
+        self.sinks = self.slopes = self.vmix = None
 
     def _packed_width(self) -> int:
         width = self.num_heads * self.head_dim
@@ -150,17 +169,41 @@ class RotaryAttention(Part):
                  "o.weight": ParamSpec((self.hidden_size, self.num_heads * self.value_dim))}
         if self.bias:
             specs["qkv.bias"] = ParamSpec((self._packed_width(),), init="zeros")
+        if self.learned_sink:
+            specs["sink"] = ParamSpec((self.num_heads,), always_float32=True, init_mean=0.0, init_std=1.0)
+        if self.mix_values:
+            specs["vmix"] = ParamSpec((), always_float32=True, init_mean=0.4, init_std=0.1)
         return specs
 
     def bind(self, params):
         self.qkv_weight, self.o_weight = params["qkv.weight"], params["o.weight"]
         self.qkv_bias = params.get("qkv.bias")
+        self.sinks, self.vmix = params.get("sink"), params.get("vmix")
+        if self.distance_bias:
+            self.slopes = distance_slopes(self.num_heads).to(self.qkv_weight.device)
 
     def cache_need(self):
         return PagedKVNeed(self.num_kv_heads, self.head_dim, self.window,
                            None if self.value_dim == self.head_dim else self.value_dim, self.chunk)
 
-    def forward(self, x, step, cache: CacheView):
+    takes_deferred_norm = True    # x goes straight into a product, which can norm it
+    adds_to_residual = True       # the output projection can make the addition to the residual stream
+
+    def first_product(self):
+        """(weight, gated) of the product that x goes into."""
+        return self.qkv_weight, False
+
+    def _values_to_mix(self, qkv, step) -> dict:
+        """Where this layer's values start among its packed columns is where the later layers' argument points to."""
+        if self.mix_values == "first":
+            step.scratch["first_values"] = (qkv, (self.num_heads + self.num_kv_heads) * self.head_dim)
+        if self.mix_values != "later":
+            return {}
+        if "first_values" not in step.scratch:
+            raise ValueError("a layer that mixes values runs before the layer whose values it mixes in")
+        return {"mix": (step.scratch["first_values"], self.vmix)}
+
+    def forward(self, x, step, cache: CacheView, add_to=None):
         tables = step.groups[cache.group]
         writes = self.own_kv and cache.writes
         if not self.own_kv and cache.writes:
@@ -178,17 +221,23 @@ class RotaryAttention(Part):
         q = ops.rotary_split_write(qkv, bias, freqs, v_freqs, step.token_positions, tables.slot_mapping, cache.k, cache.v,
                                    self.num_heads, self.num_kv_heads, self.head_dim, self.value_dim, with_kv=writes,
                                    more_columns=gates, interleaved=self.rotation == "interleaved",
-                                   unit_eps=self.unit_norm_eps, values_from_keys=self.values_are_keys)
+                                   unit_eps=self.unit_norm_eps, values_from_keys=self.values_are_keys,
+                                   temperature=self.temperature, **self._values_to_mix(qkv, step))
         # (the gates stay where the projection left them: the attention kernels read them from the packed rows)
         o = ops.paged_attention(q, cache.k, cache.v, step.attention, tables.block_tables, self.scale, self.window, self.chunk,
-                                softcap=self.softcap, sink=self.sink,
-                                gate=(qkv, qkv.shape[1] - gates) if self.head_gate else None)
+                                softcap=self.softcap, sink=self.sinks if self.learned_sink else self.sink,
+                                slopes=self.slopes, gate=(qkv, qkv.shape[1] - gates) if self.head_gate else None)
         if self.rotate_values:
             ops.turn_back_(o, v_freqs, step.token_positions)
         o = o.view(o.shape[0], self.num_heads * self.value_dim)
         if self.element_gate:
             ops.gate_rows_(o, (qkv, qkv.shape[1] - gates))
-        return ops.linear(o, self.o_weight)
+        return ops.linear(o, self.o_weight, add_to=add_to)
+
+
+def distance_slopes(heads: int) -> torch.Tensor:
+    """[heads] float32: 2^(-8 (h + 1) / heads), h from 0."""
+    return (2.0 ** (-8.0 * torch.arange(1, heads + 1, dtype=torch.float64) / heads)).to(torch.float32)
 
 
 @MIXERS.register("differential_attention")

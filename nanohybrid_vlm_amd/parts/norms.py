@@ -15,14 +15,17 @@ class RMSNorm(Part):
     takes_summed = True           # ``forward_add`` takes an ``ops.Summed`` (a sum that a product has made already)
     defers_to_products = True     # ``forward_add(..., deferred=True)`` may return an ``ops.Normed``
 
-    def __init__(self, size: int, eps: float, residual_float32: bool = True):
+    def __init__(self, size: int, eps: float, residual_float32: bool = True, rounds_between: bool = True):
         """``residual_float32`` (an engine option, offered to every part when a model is built): True: the residual
         stream is carried in float32 whatever the rows' element type, so the sum goes from layer to layer
         unrounded. False: it is carried in the rows' element type, rounded after every addition, as the
-        reference carries it (layernorm.py:34-40; the norm itself still takes the unrounded float sum)."""
+        reference carries it (layernorm.py:34-40; the norm itself still takes the unrounded float sum).
+        ``rounds_between``: the normed row is rounded before it meets the weight and once more after it, as the
+        reference does (layernorm.py:22-25); False: the weight joins in float and the row is rounded once."""
         self.size = size
         self.eps = eps
         self.residual_float32 = bool(residual_float32)
+        self.rounds_between = bool(rounds_between)
         self.weight = None
 
     def param_specs(self):
@@ -30,10 +33,11 @@ class RMSNorm(Part):
 
     def forward_start(self, x: torch.Tensor):
         """The first norm of a model: returns (norm(x), x as the residual that later norms add to)."""
-        return ops.rmsnorm(x, self.weight, self.eps, start_residual=True, residual_float32=self.residual_float32)
+        return ops.rmsnorm(x, self.weight, self.eps, start_residual=True, residual_float32=self.residual_float32,
+                           rounds_between=self.rounds_between)
 
     def forward(self, x) -> torch.Tensor:
-        return ops.rmsnorm(ops.dense(x), self.weight, self.eps)
+        return ops.rmsnorm(ops.dense(x), self.weight, self.eps, rounds_between=self.rounds_between)
 
     def add_to(self, residual: torch.Tensor, reader=None) -> ops.AddTo:
         """What the part before this norm is handed so that its last product can make the addition to ``residual``
@@ -52,7 +56,7 @@ class RMSNorm(Part):
                 raise ValueError("a sum that a product made for another norm, or into another residual stream")
             normed = ops.Normed(x)
             return (normed if deferred else normed.tensor()), residual
-        y = ops.rmsnorm(x, self.weight, self.eps, residual=residual)
+        y = ops.rmsnorm(x, self.weight, self.eps, residual=residual, rounds_between=self.rounds_between)
         return y, residual
 
 

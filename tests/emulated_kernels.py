@@ -23,14 +23,15 @@ class EmulatedBackend:
     def soft_cap(self, x, cap):
         x.copy_(cap * torch.tanh(x / cap))
 
-    def rmsnorm(self, x, residual, residual_mode, w, y, eps):
+    def rmsnorm(self, x, residual, residual_mode, w, y, eps, rounds_between=True):
         s = x.float()
         if residual_mode == 1:
             s = s + residual.float()
         if residual_mode != 0:
             residual.copy_(s.to(residual.dtype))
         r = torch.rsqrt(s.pow(2).mean(-1, keepdim=True) + eps)
-        y.copy_(((s * r).to(x.dtype).float() * w.float()).to(x.dtype))
+        n = (s * r).to(x.dtype).float() if rounds_between else s * r
+        y.copy_((n * w.float()).to(x.dtype))
 
     def silu_mul(self, gu, out):
         I = out.shape[1]
@@ -81,7 +82,7 @@ class EmulatedBackend:
             v_cache.view(-1, Hkv, D)[slots] = v[ok].to(dt)
 
     def paged_attention(self, q, k_cache, v_cache, out, batch, block_tables, scale, window, chunk=0, cap=0.0, sink=None,
-                        gate=None):
+                        slopes=None, gate=None):
         T, Hq, D = q.shape
         page_size, Hkv = k_cache.shape[1], k_cache.shape[2]
         group = Hq // Hkv
@@ -101,12 +102,15 @@ class EmulatedBackend:
                 s = (kh @ q[t, h].float()) * scale
                 if cap:
                     s = cap * torch.tanh(s / cap)
+                if slopes is not None:
+                    s = s - slopes[h] * (p - kp).float()
                 if sink is None:
                     o = torch.softmax(s, dim=0) @ vh
                 else:
-                    m = max(float(s.max()), sink)
+                    z = float(sink[h]) if isinstance(sink, torch.Tensor) else sink
+                    m = max(float(s.max()), z)
                     e = torch.exp(s - m)
-                    o = (e @ vh) / (e.sum() + math.exp(sink - m))
+                    o = (e @ vh) / (e.sum() + math.exp(z - m))
                 if gate is not None:
                     o = o * torch.sigmoid(gate[0][t, gate[1] + h].float())
                 out[t, h] = o.to(out.dtype)
@@ -180,48 +184,63 @@ class EmulatedBackend:
             return 0.5 * z * (1.0 + torch.tanh(0.7978845608028654 * (z + 0.044715 * z ** 3)))
         return z * torch.sigmoid(z)
 
-    def act_mul(self, gu, out, act):
+    @classmethod
+    def _gated(cls, g, u, gate):
+        if gate is not None and gate.act == 2:
+            g, u = torch.clamp(g, max=gate.limit), torch.clamp(u, -gate.limit, gate.limit)
+            return g * torch.sigmoid(gate.alpha * g) * (u + gate.offset)
+        return cls._act(g, 0 if gate is None else gate.act) * u
+
+    def gate_mul(self, gu, bias, out, gate):
         I = out.shape[1]
-        out.copy_((self._act(gu[:, :I].float(), act) * gu[:, I:].float()).to(out.dtype))
+        x = gu.float() if bias is None else gu.float() + bias.float()
+        out.copy_(self._gated(x[:, :I], x[:, I:], gate).to(out.dtype))
 
     # -- attention over a cached latent
     @staticmethod
-    def _turn_pairs(t, positions, freqs, gain):
+    def _turn_pairs(t, positions, freqs, gain, halves=False):
         ang = positions.double()[:, None] * freqs[None, :]
         cos, sin = (ang.cos() * gain).float(), (ang.sin() * gain).float()
         while cos.dim() < t.dim():
             cos, sin = cos.unsqueeze(1), sin.unsqueeze(1)
-        u, v = t[..., 0::2], t[..., 1::2]
+        n = freqs.shape[0]
+        first, second = (slice(0, n), slice(n, 2 * n)) if halves else (slice(0, 2 * n, 2), slice(1, 2 * n, 2))
+        u, v = t[..., first], t[..., second]
         out = torch.empty_like(t)
-        out[..., 0::2] = u * cos - v * sin
-        out[..., 1::2] = v * cos + u * sin
+        out[..., first] = u * cos - v * sin
+        out[..., second] = v * cos + u * sin
         return out
 
     def latent_prepare(self, a, q_off, q_rank, c_off, kv_rank, rot, wq, wc, eps, freqs, gain, positions, slot_mapping,
-                       cache, cq):
-        q = a[:, q_off:q_off + q_rank]
-        cq.copy_((q / torch.sqrt(q.pow(2).mean(-1, keepdim=True) + eps) * wq).to(cq.dtype))
+                       cache, cq, row_dtype, halves=False):
+        a = a.float()
+        if q_rank:
+            q = a[:, q_off:q_off + q_rank]
+            cq.copy_((q / torch.sqrt(q.pow(2).mean(-1, keepdim=True) + eps) * wq).to(cq.dtype))
         if kv_rank == 0 or slot_mapping is None:
             return
         c = a[:, c_off:c_off + kv_rank]
         rows = [c / torch.sqrt(c.pow(2).mean(-1, keepdim=True) + eps) * wc]
         if rot:
-            rows.append(self._turn_pairs(a[:, c_off + kv_rank:c_off + kv_rank + rot], positions, freqs, gain))
+            rows.append(self._turn_pairs(a[:, c_off + kv_rank:c_off + kv_rank + rot], positions, freqs, gain, halves))
+        rows.append(torch.zeros(a.shape[0], cache.shape[-1] - kv_rank - rot))
         rows = torch.cat(rows, dim=-1).to(cache.dtype)
         ok = slot_mapping >= 0
-        cache.view(-1, cache.shape[-1])[slot_mapping[ok].long(), :kv_rank + rot] = rows[ok]
+        cache.view(-1, cache.shape[-1])[slot_mapping[ok].long()] = rows[ok]
 
-    def head_gemm(self, x, x_off, x_row, w, w_head, w_n, w_k, y, y_off, y_row, gate, gate_off, N, K, turn=None):
+    def head_gemm(self, x, x_off, w, w_head, w_n, w_k, y, y_off, gate, N, K, turn=None):
         T, H = x.shape[0], x.shape[1]
         m = torch.as_strided(w, (H, N, K), (w_head, w_n, w_k)).float()
         r = torch.einsum("thk,hnk->thn", x[:, :, x_off:x_off + K].float(), m)
         if gate is not None:
-            r = r * torch.sigmoid(gate[:, gate_off:gate_off + H])[:, :, None]
+            rows, col, mode = gate
+            z = rows[:, col:col + (H * N if mode == 2 else H)].float()
+            r = r * torch.sigmoid(z.reshape(T, H, -1))
         y[:, :, y_off:y_off + N] = r.to(y.dtype)
-        return False                               # (the turning is left to rotate_interleaved)
+        return False                               # (the turning is left to rotate_heads)
 
-    def rotate_interleaved(self, src, s_off, dst, d_off, rot, freqs, gain, positions):
-        dst[:, :, d_off:d_off + rot] = self._turn_pairs(src[:, :, s_off:s_off + rot].float(), positions, freqs, gain).to(dst.dtype)
+    def rotate_heads(self, src, s_off, dst, d_off, rot, freqs, gain, positions, halves=False):
+        dst[:, :, d_off:d_off + rot] = self._turn_pairs(src[:, :, s_off:s_off + rot].float(), positions, freqs, gain, halves).to(dst.dtype)
 
     # -- a feed-forward of many small experts
     def route_topk(self, logits, ids, scores, bias=None, mode=0):
@@ -262,7 +281,7 @@ class EmulatedBackend:
 
     def rotary_split_write(self, qkv, bias, qk_freqs, rot, v_freqs, positions, slot_mapping, q_out, k_cache, v_cache,
                            Hq, Hkv, D, E, with_kv, more_columns=0, interleaved=False, unit_eps=None, values_from_keys=False,
-                           maps=1):
+                           maps=1, temperature=None, mix=None):
         T, dt = qkv.shape[0], qkv.dtype
         x = qkv.float()
         if more_columns:
@@ -285,6 +304,9 @@ class EmulatedBackend:
             return t
 
         q = prepared(x[:, :Hq * D].reshape(T, Hq, D))
+        if temperature is not None:
+            coef, every = temperature
+            q = q * (1.0 + coef * torch.log(torch.floor((positions.double() + 1) / every) + 1).float())[:, None, None]
         if maps > 1:                 # every map a head of its own, with zeros in the other maps' places
             wide = torch.zeros(T, Hq, maps, D)
             for s in range(Hq):
@@ -300,6 +322,9 @@ class EmulatedBackend:
                 v = x[:, (Hq + Hkv) * D:].reshape(T, Hkv // maps, E)
             if v_freqs is not None:
                 v = self._turned(v, positions, v_freqs)
+            if mix is not None:
+                (rows, col), lam = mix
+                v = (1.0 - lam) * v + lam * rows[:, col:col + v.shape[1] * E].float().reshape(v.shape)
             ok = slot_mapping >= 0
             slots = slot_mapping[ok].long()
             k_cache.view(-1, Hkv // maps, maps * D)[slots] = k[ok].to(dt)
@@ -443,18 +468,18 @@ class EmulatedBackend:
     few_rows = 16
     fuse_norms = True
 
-    def fused_linear(self, x, w, bias, out, gated=False, row_scales=None, residual=None, sum_out=None, ss_out=None, next_w=None):
+    def fused_linear(self, x, w, bias, out, gated=False, row_scales=None, residual=None, sum_out=None, ss_out=None, next_w=None,
+                     gate=None):
         dt = x.dtype
         y = x.float() @ w.float().T
         if row_scales is not None:
             ss, eps = row_scales
             y = y * torch.rsqrt(ss.sum(-1, keepdim=True) / x.shape[1] + eps)
+        if bias is not None:
+            y = y + bias.float()
         if gated:
             half = w.shape[0] // 2
-            g, u = y[:, :half], y[:, half:]
-            y = g * torch.sigmoid(g) * u
-        elif bias is not None:
-            y = y + bias.float()
+            y = self._gated(y[:, :half], y[:, half:], gate)
         if residual is None:
             out.copy_(y.to(out.dtype))
             return
