@@ -413,7 +413,7 @@ def bench_projections(args):
 
 
 def bench_design(args):
-    """A Pevazen model beside a Qwen3 model of equal sizes: prefill of one prompt, decoding at a fixed batch, and the
+    """A model of one of the designs beside its closest model(s) of equal sizes: prefill of one prompt, decoding at a fixed batch, and the
     device time of every own kernel in one eager step of each kind (library products are what is left of the step)."""
     import types
     import torch
@@ -423,13 +423,25 @@ def bench_design(args):
     from nanohybrid_vlm_amd.engine.runner import StepEntry
     from nanohybrid_vlm_amd.native import ops
 
-    name = args.shape if args.shape.startswith(("pevazen", "fazovik", "vugelix", "pukarax")) else "pevazen-1b"
+    name = args.shape if args.shape.startswith(("pevazen", "fazovik", "vugelix", "pukarax", "gabelorn")) else "pevazen-1b"
     design = name.split("-")[0]
     new = json.loads(json.dumps(named_shapes()[name]))
     layers = args.layers or min(8, len(new["layers"]))
     new["layers"] = new["layers"][:layers]
     beside = "qwen3"
-    if design == "vugelix":
+    further = []                                       # a second model beside it
+    if design == "gabelorn":
+        # the two kinds of layer have a like each: Fazovik's latent attention (with as many heads of the same sizes, on as
+        # long a row) and Qwen3's grouped heads; both twins have dense feed-forwards of the same inner size in every layer
+        beside = "fazovik"
+        a, b = new["layers"][0]["mixer"], new["layers"][1]["mixer"]
+        ff = new["layers"][0]["mlp"]["ff"]
+        mixer = {"dim": a["dim"], "heads": a["heads"], "kv_rank": a["kv_rank"], "q_rank": new["width"] * 3 // 8,
+                 "rot": a["rot"], "rot_dim": a["rot_dim"], "scale": a["scale"], "vdim": a["vdim"]}
+        twin = {"architecture": "Fazovik", "layers": [{"type": "latent_attention", "mixer": mixer, "mlp": {"kind": "dense", "ff": ff}}] * layers,
+                "norm": {"eps": 1e-6}, "vocab": new["vocab"], "width": new["width"]}
+        further = [("qwen3", qwen3_shape(layers, new["width"], b["heads"], b["kv_heads"], b["dim"], ff, vocab=new["vocab"]))]
+    elif design == "vugelix":
         # the closest model the engine has is Pevazen's pair of mixers (attention beside a gated delta rule): the twin is
         # made of such layers alone, with this design's heads and head sizes on both sides, a chunk as long as the
         # window, and a (gated) feed-forward of the same inner size
@@ -462,7 +474,7 @@ def bench_design(args):
     context = args.context or (T + 512)
     pages = (batch + 1) * -(-context // args.block_size) + 1
     out = {}
-    for label, raw in ((design, new), (beside, twin)):
+    for label, raw in [(design, new), (beside, twin)] + further:
         llm = LLM(raw, random_weights=0, dtype=args.dtype, kvcache_block_size=args.block_size, max_num_seqs=max(batch, 1),
                   enforce_eager=args.eager, num_kvcache_blocks=pages, max_num_batched_tokens=max(args.token_budget, T, batch),
                   max_model_len=context, scheduler_policy="prefill_first")
@@ -509,13 +521,14 @@ def bench_design(args):
         llm.exit()
         del llm, runner
         torch.cuda.empty_cache()
-    line = {"metric": f"{design.capitalize()} ({name}, {layers} layers) beside {beside.capitalize()} of equal sizes: prefill of {T} tokens and decode at batch {batch}",
+    names = " and ".join(n.capitalize() for n in [beside] + [n for n, _ in further])
+    line = {"metric": f"{design.capitalize()} ({name}, {layers} layers) beside {names} of equal sizes: prefill of {T} tokens and decode at batch {batch}",
             "value": out[design]["decode_tok_s"], "unit": "tok/s", "n_gpus": 1, "steps": args.steps, "warmup": args.warmup,
             "ms_per_step": out[design]["decode_ms_per_step"], "higher_is_better": True, "scaling": "weak", "vs_baseline": None,
             "dtype": "bf16" if args.dtype == "bfloat16" else "fp32", "data": "synthetic: random token ids, random weights",
             "config": {"model": name, "layers": layers, "width": new["width"], "global_batch": batch, "prompt_len": T,
                        "seq_len": context, "parallelism": "single GPU", "graphs": not args.eager},
-            design: out[design], beside: out[beside]}
+            **out}
     print(json.dumps(line), flush=True)
     return 0
 

@@ -96,24 +96,24 @@ class EmulatedBackend:
                 lo = p - p % chunk
             kp = torch.arange(lo, p + 1)
             slots = block_tables[r, kp // page_size].long() * page_size + kp % page_size
-            for h in range(Hq):
-                kh = kf[slots, h // group].float()
-                vh = vf[slots, h // group].float()
-                s = (kh @ q[t, h].float()) * scale
-                if cap:
-                    s = cap * torch.tanh(s / cap)
-                if slopes is not None:
-                    s = s - slopes[h] * (p - kp).float()
-                if sink is None:
-                    o = torch.softmax(s, dim=0) @ vh
-                else:
-                    z = float(sink[h]) if isinstance(sink, torch.Tensor) else sink
-                    m = max(float(s.max()), z)
-                    e = torch.exp(s - m)
-                    o = (e @ vh) / (e.sum() + math.exp(z - m))
-                if gate is not None:
-                    o = o * torch.sigmoid(gate[0][t, gate[1] + h].float())
-                out[t, h] = o.to(out.dtype)
+            kt = kf[slots].float().repeat_interleave(group, dim=1)          # [keys, heads, D]
+            vt = vf[slots].float().repeat_interleave(group, dim=1)
+            s = torch.einsum("khd,hd->hk", kt, q[t].float()) * scale
+            if cap:
+                s = cap * torch.tanh(s / cap)
+            if slopes is not None:
+                s = s - slopes[:, None] * (p - kp).float()[None]
+            if sink is None:
+                weights = torch.softmax(s, dim=-1)
+            else:
+                z = sink[:, None] if isinstance(sink, torch.Tensor) else torch.full((Hq, 1), float(sink))
+                m = torch.maximum(s.max(dim=-1, keepdim=True).values, z)
+                e = torch.exp(s - m)
+                weights = e / (e.sum(-1, keepdim=True) + torch.exp(z - m))
+            o = torch.einsum("hk,khe->he", weights, vt)
+            if gate is not None:
+                o = o * torch.sigmoid(gate[0][t, gate[1]:gate[1] + Hq].float())[:, None]
+            out[t] = o.to(out.dtype)
 
     # -- layers that are not the pre-norm kind
     def scalar_rmsnorm(self, x, gain, y, eps):
