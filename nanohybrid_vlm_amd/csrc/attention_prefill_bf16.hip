@@ -34,9 +34,10 @@
 // comes as a negative window, else 0). Keys outside the block's range are replaced by the
 // nearest key inside it (their P is 0): unused cache slots may hold anything, and 0 * NaN
 // would poison the sums.
-// What a layer may ask for besides (MORE; the entry point ..._more): a cap on the scores (s <- cap tanh(s / cap), after
-// the scale; taken on the float scores where they leave the first product), a bias that grows with the distance (BIASED:
-// slopes[head] * (query position - key position) is taken off the float score after scale and cap), one more term
+// What a layer may ask for besides (MORE; the entry point ..._more): a cap on the scores (CAPPED: s <- cap tanh(s / cap), after
+// the scale; taken on the float scores where they leave the first product), a bias that grows with the distance (BIASED,
+// not together with a cap: slopes[head] * (query position - key position) is taken off the score; the first product's
+// float sums start from it, divided by the scale, so that it costs one operation a score), one more term
 // exp(sink) in the softmax's denominator (one score for the layer or one per head; it is the row's first reference point,
 // and joins the row's sum at the end) and a gate per (token, head) whose sigmoid multiplies the head's result (with the
 // division by the sum).
@@ -92,19 +93,18 @@ __device__ __forceinline__ int slot_of(P bt, int key, int page_size, int page_sh
 
 // BT_IN_LDS: the request's block table (up to the block's last key) is copied into LDS first, so that the
 // look-up that every load of a key depends on costs an LDS read instead of a trip to memory.
-// MORE: cap_ratio = cap / scale (0: no cap) and tanh_k = 2 log2(e) scale / cap, so that the capped score, still to be
+// CAPPED: cap_ratio = cap / scale and tanh_k = 2 log2(e) scale / cap, so that the capped score, still to be
 // multiplied by the scale as every score is, costs one exp2 and one reciprocal: tanh(x) = 1 - 2 / (1 + exp(2 x)), and an
 // exp2 that overflows gives the limit 1; sink_l2 = sink log2(e), or -inf for none (sinks, may be null: one per head in
-// its place); gate (may be null). BIASED: slopes per head; the scores are then brought to base-2 exponents, scale and
-// bias in, before the exponentials (a bias that depends on the key cannot be left to the row's reference point).
-template <bool BT_IN_LDS, int RT, bool MORE, bool BIASED>
+// its place); gate (may be null). BIASED: slopes per head, slope_ratio = 1 / scale.
+template <bool BT_IN_LDS, int RT, bool MORE, bool CAPPED, bool BIASED>
 __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(2))) void prefill_attention_kernel(
     const bf16_t* __restrict__ q, const bf16_t* __restrict__ k_cache, const bf16_t* __restrict__ v_cache,
     bf16_t* __restrict__ out, const int* __restrict__ cu_seqlens_q, const int* __restrict__ context_lens,
     const int* __restrict__ block_tables, int max_blocks, int Hq, int Hkv, int page_size, int page_shift,
     float scale_log2e, int window, float cap_ratio, float tanh_k, float sink_l2, const float* __restrict__ sinks,
-    const float* __restrict__ slopes, const bf16_t* __restrict__ gate, long long gate_ld) {
-  static_assert(MORE || !BIASED, "the bias is one of the further options");
+    const float* __restrict__ slopes, float slope_ratio, const bf16_t* __restrict__ gate, long long gate_ld) {
+  static_assert((MORE || !(BIASED || CAPPED)) && !(BIASED && CAPPED), "cap and bias are further options, one of them at most");
   constexpr float LOG2E = 1.4426950408889634f;
   constexpr int DL = SUPPORTED ? D : 16;                   // keeps the unsupported sizes compilable; they are never launched
   constexpr int TILE = SUPPORTED ? BN * DL : 16;           // elements of a tile
@@ -181,12 +181,10 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(2))) void p
                      : zero8();
     }
   }
-  // what turns a score into the exponent of its term: the bias needs it before that, then nothing is left to do
-  const float to_exponent = BIASED ? 1.0f : scale_log2e;
-  float slope_l2[RT], row_sink[RT];
+  float slope[RT], row_sink[RT];                           // (the slope as the unscaled scores see it)
 #pragma unroll
   for (int r = 0; r < RT; ++r) {
-    slope_l2[r] = BIASED ? slopes[head[r]] * LOG2E : 0.f;
+    slope[r] = BIASED ? slopes[head[r]] * slope_ratio : 0.f;
     row_sink[r] = MORE ? (sinks ? sinks[head[r]] * LOG2E : sink_l2) : -INFINITY;
   }
   float m_run[RT], l_part[RT];                             // of row `col` (base 2); l_part is this lane's share of the row's sum
@@ -259,10 +257,20 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(2))) void p
     constexpr bool MASKED = decltype(masked)::value;
     // ---- scores of the tile's keys for this wave's rows: every K operand serves all row tiles
     floatx4 s4[RT][KT];
+    float first_bias[RT];                                  // at this lane's first key of the tile; the others follow by steps
+#pragma unroll
+    for (int r = 0; r < RT; ++r) first_bias[r] = BIASED ? slope[r] * (float)(kb + grp * 4 - row_pos[r]) : 0.f;
 #pragma unroll
     for (int kt = 0; kt < KT; ++kt) {
 #pragma unroll
-      for (int r = 0; r < RT; ++r) s4[r][kt] = floatx4{0.f, 0.f, 0.f, 0.f};
+      for (int r = 0; r < RT; ++r) {
+        if (BIASED) {
+#pragma unroll
+          for (int j = 0; j < 4; ++j) s4[r][kt][j] = __builtin_fmaf(slope[r], (float)(kt * 16 + j), first_bias[r]);
+        } else {
+          s4[r][kt] = floatx4{0.f, 0.f, 0.f, 0.f};
+        }
+      }
 #pragma unroll
       for (int s = 0; s < DSTEPS; ++s) {
         const int piece = s * 4 + grp;
@@ -272,7 +280,7 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(2))) void p
         for (int r = 0; r < RT; ++r) s4[r][kt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(ka, qb[r][s], s4[r][kt], 0, 0, 0);
       }
     }
-    if (MORE && cap_ratio > 0.f) {
+    if (CAPPED) {
 #pragma unroll
       for (int r = 0; r < RT; ++r)
 #pragma unroll
@@ -281,17 +289,6 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(2))) void p
           for (int j = 0; j < 4; ++j)
             s4[r][kt][j] = __builtin_fmaf(-2.0f * cap_ratio,
                                           __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(s4[r][kt][j] * tanh_k)), cap_ratio);
-    }
-    if (BIASED) {
-#pragma unroll
-      for (int r = 0; r < RT; ++r) {
-        const float nearest = slope_l2[r] * (float)(kb + grp * 4 - row_pos[r]);      // of this lane's first key; the others follow by steps
-#pragma unroll
-        for (int kt = 0; kt < KT; ++kt)
-#pragma unroll
-          for (int j = 0; j < 4; ++j)
-            s4[r][kt][j] = __builtin_fmaf(s4[r][kt][j], scale_log2e, __builtin_fmaf(slope_l2[r], (float)(kt * 16 + j), nearest));
-      }
     }
     bf16x8 pa[RT][KT / 2];                                 // P of keys (32 a + 4 grp + j) and (32 a + 16 + 4 grp + j)
     float alpha[RT];
@@ -315,7 +312,7 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(2))) void p
       for (int kt = 0; kt < KT; ++kt)
 #pragma unroll
         for (int j = 0; j < 4; ++j) {
-          const float p = __builtin_amdgcn_exp2f(__builtin_fmaf(s4[r][kt][j], to_exponent, -m_run[r]));
+          const float p = __builtin_amdgcn_exp2f(__builtin_fmaf(s4[r][kt][j], scale_log2e, -m_run[r]));
           psum += p;
           pa[r][kt / 2][(kt % 2) * 4 + j] = (__bf16)p;
         }
@@ -328,7 +325,7 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(2))) void p
         for (int kt = 0; kt < KT; ++kt)
 #pragma unroll
           for (int j = 0; j < 4; ++j) m_tile = fmaxf(m_tile, s4[r][kt][j]);
-        m_tile *= to_exponent;
+        m_tile *= scale_log2e;
         m_tile = fmaxf(m_tile, __shfl_xor(m_tile, 16, 64));
         m_tile = fmaxf(m_tile, __shfl_xor(m_tile, 32, 64));
         const float m_new = fmaxf(m_run[r], m_tile);
@@ -339,7 +336,7 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(2))) void p
         for (int kt = 0; kt < KT; ++kt)
 #pragma unroll
           for (int j = 0; j < 4; ++j) {
-            const float p = __builtin_amdgcn_exp2f(__builtin_fmaf(s4[r][kt][j], to_exponent, -m_safe));
+            const float p = __builtin_amdgcn_exp2f(__builtin_fmaf(s4[r][kt][j], scale_log2e, -m_safe));
             psum += p;
             pa[r][kt / 2][(kt % 2) * 4 + j] = (__bf16)p;
           }
@@ -448,18 +445,19 @@ static int launch_prefill_attention(const void* q, const void* k_cache, const vo
   NHV_REQUIRE(gx <= 0x7fffffff && Hkv <= 65535 && B <= 65535, "prefill attention: grid too large");
   const float log2e = 1.4426950408889634f;
   const bool capped = more && cap > 0.f;
-#define NHV_PREFILL_LAUNCH_AS(BT, RT_, MORE_, BIASED_)                                                                 \
-  hipLaunchKernelGGL((prefill::prefill_attention_kernel<BT, RT_, MORE_, BIASED_>), dim3((unsigned)gx, Hkv, B), dim3(256), 0, \
+#define NHV_PREFILL_LAUNCH_AS(BT, RT_, MORE_, CAPPED_, BIASED_)                                                        \
+  hipLaunchKernelGGL((prefill::prefill_attention_kernel<BT, RT_, MORE_, CAPPED_, BIASED_>), dim3((unsigned)gx, Hkv, B), dim3(256), 0, \
                      (hipStream_t)stream, (const bf16_t*)q, (const bf16_t*)k_cache, (const bf16_t*)v_cache, (bf16_t*)out, \
                      (const int*)cu_seqlens_q, (const int*)context_lens, (const int*)block_tables, max_blocks, Hq, Hkv, \
                      page_size, page_shift, scale * log2e, window, capped ? cap / scale : 0.f,                         \
                      capped ? 2.0f * log2e * scale / cap : 0.f, more && has_sink ? sink * log2e : -INFINITY,           \
-                     (const float*)sinks, (const float*)slopes, (const bf16_t*)gate, gate_ld)
-#define NHV_PREFILL_LAUNCH(BT, RT_)                               \
-  do {                                                            \
-    if (slopes) NHV_PREFILL_LAUNCH_AS(BT, RT_, true, true);       \
-    else if (more) NHV_PREFILL_LAUNCH_AS(BT, RT_, true, false);   \
-    else NHV_PREFILL_LAUNCH_AS(BT, RT_, false, false);            \
+                     (const float*)sinks, (const float*)slopes, 1.0f / scale, (const bf16_t*)gate, gate_ld)
+#define NHV_PREFILL_LAUNCH(BT, RT_)                                      \
+  do {                                                                   \
+    if (slopes) NHV_PREFILL_LAUNCH_AS(BT, RT_, true, false, true);       \
+    else if (capped) NHV_PREFILL_LAUNCH_AS(BT, RT_, true, true, false);  \
+    else if (more) NHV_PREFILL_LAUNCH_AS(BT, RT_, true, false, false);   \
+    else NHV_PREFILL_LAUNCH_AS(BT, RT_, false, false, false);            \
   } while (0)
   const bool bt_in_lds = max_blocks <= prefill::BT_LDS;
   if (two) {
@@ -492,6 +490,8 @@ extern "C" int nhv_prefill_attention_bf16_more(const void* q, const void* k_cach
                                                float scale, int window, float cap, int has_sink, float sink,
                                                const void* sinks, const void* slopes, const void* gate, long long gate_ld,
                                                void* stream) {
+  NHV_REQUIRE(!slopes || (cap == 0.f && scale > 0.f), "prefill attention: a bias by distance needs a positive scale (%g) and no cap (%g)",
+              (double)scale, (double)cap);
   NHV_REQUIRE(cap >= 0.f && (cap == 0.f || scale > 0.f) && (!gate || gate_ld >= Hq),
               "prefill attention: cap %g with scale %g, gate rows %lld apart for %d heads", (double)cap, (double)scale, gate_ld, Hq);
   return launch_prefill_attention(q, k_cache, v_cache, out, cu_seqlens_q, context_lens, block_tables, max_blocks, B, max_q_len,

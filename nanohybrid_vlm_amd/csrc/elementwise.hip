@@ -204,39 +204,41 @@ __global__ void gate_mul_kernel(const T* __restrict__ gu, const T* __restrict__ 
   }
 }
 
-// the same, eight entries a thread (widths that are a multiple of 8)
+// the same, eight entries a thread (widths that are a multiple of 8): blockIdx.x walks along a row, and a block takes
+// rows blockIdx.y, + gridDim.y, ... (its piece of the biases is read once for all of them)
 template <typename T, int ACT>
-__global__ void gate_mul_vec_kernel(const T* __restrict__ gu, const T* __restrict__ bias, T* __restrict__ out, int I,
-                                    size_t total8, const NhvGate gate) {
-  const int per_row = I / 8;
-  for (size_t idx = (size_t)blockIdx.x * blockDim.x + threadIdx.x; idx < total8; idx += (size_t)gridDim.x * blockDim.x) {
-    const size_t t = idx / per_row, c = idx % per_row;
+__global__ __launch_bounds__(256) void gate_mul_vec_kernel(const T* __restrict__ gu, const T* __restrict__ bias, T* __restrict__ out,
+                                                           int I, int rows, const NhvGate gate) {
+  const int c = (blockIdx.x * 256 + threadIdx.x) * 8;
+  if (c >= I) return;
+  float bg[8], bu[8];
+#pragma unroll
+  for (int e = 0; e < 8; ++e) bg[e] = bu[e] = 0.f;
+  if (bias) {
+    load8f<T>(bias + c, bg);
+    load8f<T>(bias + I + c, bu);
+  }
+  for (int t = blockIdx.y; t < rows; t += gridDim.y) {
+    const T* row = gu + (size_t)t * 2 * I + c;
     float g[8], u[8], o[8];
-    load8f<T>(gu + t * 2 * I + c * 8, g);
-    load8f<T>(gu + t * 2 * I + I + c * 8, u);
-    if (bias) {
-      float bg[8], bu[8];
-      load8f<T>(bias + c * 8, bg);
-      load8f<T>(bias + I + c * 8, bu);
+    load8f<T>(row, g);
+    load8f<T>(row + I, u);
 #pragma unroll
-      for (int e = 0; e < 8; ++e) {
-        g[e] += bg[e];
-        u[e] += bu[e];
-      }
-    }
-#pragma unroll
-    for (int e = 0; e < 8; ++e) o[e] = nhv_gated<ACT>(g[e], u[e], gate);
-    store8f<T>(out + t * I + c * 8, o);
+    for (int e = 0; e < 8; ++e) o[e] = nhv_gated<ACT>(g[e] + bg[e], u[e] + bu[e], gate);
+    store8f<T>(out + (size_t)t * I + c, o);
   }
 }
 
 template <typename T, int ACT>
 static void launch_gate_mul(const void* gu, const void* bias, void* out, int rows, int I, const NhvGate& gate, hipStream_t s) {
   if (I % 8 == 0 && (uintptr_t)gu % 16 == 0 && (uintptr_t)out % 16 == 0 && (uintptr_t)bias % 16 == 0) {
-    const size_t total8 = (size_t)rows * (I / 8);
-    const int blocks = (int)((total8 + 255) / 256 > 65535 * 16 ? 65535 * 16 : (total8 + 255) / 256);
-    hipLaunchKernelGGL((gate_mul_vec_kernel<T, ACT>), dim3(blocks), dim3(256), 0, s, (const T*)gu, (const T*)bias, (T*)out, I,
-                       total8, gate);
+    // a block takes up to four rows where that leaves eight blocks for every compute unit
+    const int along = (I / 8 + 255) / 256;
+    int down = rows;
+    while (down > 1 && down * 4 > rows && (long long)along * ((down + 1) / 2) >= 2048) down = (down + 1) / 2;
+    if (down > 65535) down = 65535;
+    hipLaunchKernelGGL((gate_mul_vec_kernel<T, ACT>), dim3(along, down), dim3(256), 0, s, (const T*)gu, (const T*)bias, (T*)out, I,
+                       rows, gate);
     return;
   }
   const size_t total = (size_t)rows * I;

@@ -10,15 +10,24 @@
 // Pairs (2i, 2i + 1), or (i, i + r / 2) of the r rotated entries where ``halves`` is set, turn by angle = position *
 // freqs[i]; cosine and sine are multiplied by ``gain``. The frequencies
 // come as doubles and the product with the position is taken and brought into [-pi, pi] in double (a float product
-// of a position in the thousands is off by 1e-4 of a turn), then sine and cosine in float. Norm statistics and sums
+// of a position in the thousands is off by 1e-4 of a turn), then sine and cosine are taken. Norm statistics and sums
 // are float; rows are float or bfloat16.
 #include "nhv_common.h"
 #include <math.h>
 
+// The sine and cosine are float's own for float rows; for bfloat16 rows, whose rounding is a thousand times coarser, they
+// are the hardware's (which takes turns).
+template <typename T>
 __device__ __forceinline__ void nhv_turn_angle(int pos, double f, float gain, float* sn, float* cs) {
   const double a = (double)pos * f;
-  const double turns = rint(a * 0.15915494309189535);
-  sincosf((float)(a - turns * 6.283185307179586), sn, cs);
+  const double turns = a * 0.15915494309189535;
+  if (sizeof(T) == 2) {
+    const float part = (float)(turns - rint(turns));
+    *sn = __builtin_amdgcn_sinf(part) * gain;
+    *cs = __builtin_amdgcn_cosf(part) * gain;
+    return;
+  }
+  sincosf((float)(a - rint(turns) * 6.283185307179586), sn, cs);
   *sn *= gain;
   *cs *= gain;
 }
@@ -40,7 +49,7 @@ __device__ __forceinline__ float nhv_head_gate_of(const void* gate, int mode, lo
 template <typename T>
 __device__ __forceinline__ void nhv_turn_pair(const T* s, T* d, int p, int rot, int halves, int pos, const double* freqs, float gain) {
   float sn, cs;
-  nhv_turn_angle(pos, freqs[p], gain, &sn, &cs);
+  nhv_turn_angle<T>(pos, freqs[p], gain, &sn, &cs);
   const int a = nhv_pair_first(p, rot, halves), b = nhv_pair_second(p, rot, halves);
   const float u = to_f32(s[a]), v = to_f32(s[b]);
   d[a] = from_f32<T>(u * cs - v * sn);
@@ -83,7 +92,7 @@ __global__ void latent_prepare_kernel(const TA* __restrict__ a, int A, int q_off
   const int pos = positions[t];
   for (int i = threadIdx.x; i < rot / 2; i += blockDim.x) {
     float sn, cs;
-    nhv_turn_angle(pos, freqs[i], gain, &sn, &cs);
+    nhv_turn_angle<T>(pos, freqs[i], gain, &sn, &cs);
     const int first = nhv_pair_first(i, rot, halves), second = nhv_pair_second(i, rot, halves);
     const float u = to_f32(src[c_off + kv_rank + first]), v = to_f32(src[c_off + kv_rank + second]);
     dst[kv_rank + first] = from_f32<T>(u * cs - v * sn);
@@ -464,6 +473,138 @@ __global__ __launch_bounds__(64 * WAVES) void head_gemm_mfma_kernel(const bf16_t
   }
 }
 
+// The same for many rows (K <= HT_MAX_K): a block owns 64 rows of one head and walks over all of its outputs, 128 at a time.
+// The rows come into LDS once, whole rows of K entries; a wave takes 32 of the 128 outputs, with the matrix rows straight
+// from memory (L2), and the results go back through LDS so that rows are written in pieces of 16 bytes side by side.
+#define HT_ROWS 64
+#define HT_COLS 128
+#define HT_MAX_K 512
+template <int U>
+__global__ __launch_bounds__(256) void head_gemm_tile_kernel(const bf16_t* __restrict__ x, long long xs_t, long long xs_h,
+                                                             const bf16_t* __restrict__ w, bf16_t* __restrict__ y,
+                                                             long long ys_t, long long ys_h, const void* __restrict__ gate,
+                                                             int gate_mode, long long gs_t, int rows, int N, int K, int rot,
+                                                             int x_rot_off, int y_rot_off, int halves,
+                                                             const double* __restrict__ freqs, float gain,
+                                                             const int* __restrict__ positions, int vec_out, int vec_gate) {
+  extern __shared__ __attribute__((aligned(16))) unsigned char ht_lds[];
+  const int pitch = K + 8;                               // 16 bytes more than a row: the rows spread over the banks
+  bf16_t* xs = reinterpret_cast<bf16_t*>(ht_lds);        // [64][pitch]
+  constexpr int YP = HT_COLS + 8;
+  bf16_t* ys = xs + HT_ROWS * pitch;                     // [64][YP]
+  const int h = blockIdx.x, m0 = blockIdx.y * HT_ROWS;
+  const int here = min(HT_ROWS, rows - m0);
+  const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
+  const int col = lane & 15, grp = lane >> 4;
+  const int pieces = K / 8;
+  for (int i = threadIdx.x; i < HT_ROWS * pieces; i += 256) {
+    const int m = i / pieces, p = i % pieces;
+    hg_bf16x8 v;
+    if (m < here) v = *reinterpret_cast<const hg_bf16x8*>(x + (size_t)(m0 + m) * xs_t + (size_t)h * xs_h + p * 8);
+    else {
+#pragma unroll
+      for (int e = 0; e < 8; ++e) v[e] = (__bf16)0.f;
+    }
+    *reinterpret_cast<hg_bf16x8*>(xs + m * pitch + p * 8) = v;
+  }
+  // the rotated part of these rows, while the rows are on their way
+  for (int i = threadIdx.x; i < here * (rot / 2); i += 256) {
+    const int t = m0 + i / (rot / 2);
+    nhv_turn_pair(x + (size_t)t * xs_t + (size_t)h * xs_h + x_rot_off, y + (size_t)t * ys_t + (size_t)h * ys_h + y_rot_off,
+                  i % (rot / 2), rot, halves, positions[t], freqs, gain);
+  }
+  hg_bf16x8 zero;
+#pragma unroll
+  for (int i = 0; i < 8; ++i) zero[i] = (__bf16)0.f;
+  __syncthreads();
+  for (int c0 = 0; c0 < N; c0 += HT_COLS) {
+    const int n0 = c0 + wave * 32;
+    if (n0 < N) {                                        // the whole wave; every wave meets the barriers below
+      const bf16_t* wrow[2];
+      bool n_ok[2];
+#pragma unroll
+      for (int nt = 0; nt < 2; ++nt) {
+        const int n = n0 + nt * 16 + col;
+        n_ok[nt] = n < N;
+        wrow[nt] = w + ((size_t)h * N + (n_ok[nt] ? n : 0)) * K;
+      }
+      hg_floatx4 acc[4][2];
+#pragma unroll
+      for (int mt = 0; mt < 4; ++mt)
+#pragma unroll
+        for (int nt = 0; nt < 2; ++nt) acc[mt][nt] = hg_floatx4{0.f, 0.f, 0.f, 0.f};
+      // gates of four entries at once, asked for before the products
+      hg_bf16x4 g4[4][2];
+      if (vec_gate) {
+#pragma unroll
+        for (int mt = 0; mt < 4; ++mt)
+#pragma unroll
+          for (int nt = 0; nt < 2; ++nt) {
+            const int n = n0 + nt * 16 + grp * 4, m = m0 + min(mt * 16 + col, here - 1);
+            g4[mt][nt] = *reinterpret_cast<const hg_bf16x4*>(reinterpret_cast<const bf16_t*>(gate) + (size_t)m * gs_t + (size_t)h * N +
+                                                             (n < N ? n : 0));
+          }
+      }
+      for (int k0 = 0; k0 < K; k0 += 32 * U) {
+        hg_bf16x8 a[U][2];
+#pragma unroll
+        for (int u = 0; u < U; ++u) {
+          const int k = k0 + u * 32 + grp * 8;
+#pragma unroll
+          for (int nt = 0; nt < 2; ++nt) a[u][nt] = (n_ok[nt] && k < K) ? *reinterpret_cast<const hg_bf16x8*>(wrow[nt] + k) : zero;
+        }
+#pragma unroll
+        for (int u = 0; u < U; ++u) {
+          const int k = k0 + u * 32 + grp * 8;
+#pragma unroll
+          for (int mt = 0; mt < 4; ++mt) {
+            const hg_bf16x8 b = k < K ? *reinterpret_cast<const hg_bf16x8*>(xs + (mt * 16 + col) * pitch + k) : zero;
+#pragma unroll
+            for (int nt = 0; nt < 2; ++nt) acc[mt][nt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a[u][nt], b, acc[mt][nt], 0, 0, 0);
+          }
+        }
+      }
+#pragma unroll
+      for (int mt = 0; mt < 4; ++mt)
+#pragma unroll
+        for (int nt = 0; nt < 2; ++nt) {
+          hg_bf16x4 four;
+          float v[4];
+#pragma unroll
+          for (int j = 0; j < 4; ++j) v[j] = acc[mt][nt][j];
+          if (vec_gate) {
+#pragma unroll
+            for (int j = 0; j < 4; ++j)
+              v[j] *= __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(-1.4426950408889634f * (float)g4[mt][nt][j]));
+          } else if (gate != nullptr && mt * 16 + col < here) {
+            const int n = n0 + nt * 16 + grp * 4;
+#pragma unroll
+            for (int j = 0; j < 4; ++j)
+              if (n + j < N) v[j] *= nhv_head_gate_of<bf16_t>(gate, gate_mode, gs_t, m0 + mt * 16 + col, h, N, n + j);
+          }
+#pragma unroll
+          for (int j = 0; j < 4; ++j) four[j] = (__bf16)v[j];
+          *reinterpret_cast<hg_bf16x4*>(ys + (mt * 16 + col) * YP + wave * 32 + nt * 16 + grp * 4) = four;
+        }
+    }
+    __syncthreads();
+    const int width = min(HT_COLS, N - c0);
+    if (vec_out) {                                       // N and the rows of y are pieces of 16 bytes
+      for (int i = threadIdx.x; i < here * (width / 8); i += 256) {
+        const int m = i / (width / 8), p = i % (width / 8);
+        *reinterpret_cast<hg_bf16x8*>(y + (size_t)(m0 + m) * ys_t + (size_t)h * ys_h + c0 + p * 8) =
+            *reinterpret_cast<const hg_bf16x8*>(ys + m * YP + p * 8);
+      }
+    } else {
+      for (int i = threadIdx.x; i < here * width; i += 256) {
+        const int m = i / width, p = i % width;
+        y[(size_t)(m0 + m) * ys_t + (size_t)h * ys_h + c0 + p] = ys[m * YP + p];
+      }
+    }
+    __syncthreads();
+  }
+}
+
 extern "C" int nhv_head_gemm_bf16(const void* x, long long xs_t, long long xs_h, const void* w, void* y, long long ys_t,
                                   long long ys_h, const void* gate, int gate_mode, long long gs_t, int rows, int H, int N, int K,
                                   int rot, int x_rot_off, int y_rot_off, int halves, const void* freqs, float gain,
@@ -483,9 +624,27 @@ extern "C" int nhv_head_gemm_bf16(const void* x, long long xs_t, long long xs_h,
                        (const bf16_t*)w, (bf16_t*)y, ys_t, ys_h, gate, gate_mode, gs_t, rows, N, K, n_chunks, rot,        \
                        x_rot_off, y_rot_off, halves, (const double*)freqs, gain, (const int*)positions);                  \
   } while (0)
-  if (rows <= 16) LAUNCH(1, 1, 1, 4);
-  else if (rows <= 64) LAUNCH(2, 1, 4, 4);
-  else LAUNCH(4, 2, 4, 2);
+  if (rows > 64 && K <= HT_MAX_K) {
+    const size_t lds = (size_t)HT_ROWS * (K + 8 + HT_COLS + 8) * sizeof(bf16_t);
+    auto kernel = head_gemm_tile_kernel<4>;
+    // more than 64 KB of dynamic LDS has to be allowed once per kernel (and per process)
+    static const hipError_t allowed = hipFuncSetAttribute((const void*)kernel, hipFuncAttributeMaxDynamicSharedMemorySize,
+                                                          (int)(HT_ROWS * (HT_MAX_K + 8 + HT_COLS + 8) * sizeof(bf16_t)));
+    NHV_REQUIRE(allowed == hipSuccess, "head_gemm_bf16: %s", hipGetErrorString(allowed));
+    const dim3 grid(H, (rows + HT_ROWS - 1) / HT_ROWS);
+    NHV_REQUIRE(grid.y <= 65535, "head_gemm_bf16: %d rows are too many", rows);
+    const int vec_out = N % 8 == 0 && ys_t % 8 == 0 && ys_h % 8 == 0 && (uintptr_t)y % 16 == 0;
+    const int vec_gate = gate != nullptr && gate_mode == 2 && N % 4 == 0 && gs_t % 4 == 0 && (uintptr_t)gate % 8 == 0;
+    hipLaunchKernelGGL(kernel, grid, dim3(256), lds, s, (const bf16_t*)x, xs_t, xs_h, (const bf16_t*)w, (bf16_t*)y, ys_t, ys_h, gate,
+                       gate_mode, gs_t, rows, N, K, rot, x_rot_off, y_rot_off, halves, (const double*)freqs, gain,
+                       (const int*)positions, vec_out, vec_gate);
+  } else if (rows <= 16) {
+    LAUNCH(1, 1, 1, 4);
+  } else if (rows <= 64) {
+    LAUNCH(2, 1, 4, 4);
+  } else {
+    LAUNCH(4, 2, 4, 2);
+  }
 #undef LAUNCH
   NHV_LAUNCH_CHECK("head_gemm_bf16");
   return 0;

@@ -259,6 +259,52 @@ __global__ void rotary_split_write_kernel(const T* __restrict__ qkv, const T* __
   for (int i = threadIdx.x; i < size; i += blockDim.x) dst[i] = from_f32<T>(staged[i] * r);
 }
 
+// The same where nothing is turned or normed and heads are whole pieces of eight entries: a thread moves eight entries of
+// one row (16 bytes in bfloat16), whatever head they belong to. blockIdx.x walks along the row, blockIdx.y over tokens.
+template <typename T>
+__device__ __forceinline__ void split_load8(const T* p, float* v) {
+  struct alignas(sizeof(T) * 8) Pack { T e[8]; };
+  const Pack pack = *reinterpret_cast<const Pack*>(p);
+#pragma unroll
+  for (int i = 0; i < 8; ++i) v[i] = to_f32(pack.e[i]);
+}
+
+template <typename T>
+__global__ __launch_bounds__(256) void split_write_vec_kernel(const T* __restrict__ qkv, const int* __restrict__ positions,
+                                                              const int* __restrict__ slot_mapping, T* __restrict__ q_out,
+                                                              T* __restrict__ k_cache, T* __restrict__ v_cache, int nq, int nk,
+                                                              int nv, int ld, int T_rows, const SplitMore more) {
+  struct alignas(sizeof(T) * 8) Pack { T e[8]; };
+  const int c = (blockIdx.x * 256 + threadIdx.x) * 8;
+  if (c >= nq + nk + nv) return;
+  for (int t = blockIdx.y; t < T_rows; t += gridDim.y) {
+    Pack in = *reinterpret_cast<const Pack*>(qkv + (size_t)t * ld + c);
+    if (c < nq) {
+      const float factor = query_temperature(positions[t], more);
+      if (factor != 1.0f)
+#pragma unroll
+        for (int i = 0; i < 8; ++i) in.e[i] = from_f32<T>(to_f32(in.e[i]) * factor);
+      *reinterpret_cast<Pack*>(q_out + (size_t)t * nq + c) = in;
+      continue;
+    }
+    const int slot = slot_mapping[t];
+    if (slot < 0) continue;                    // a row that stores nothing (padding of a recorded step)
+    if (c < nq + nk) {
+      *reinterpret_cast<Pack*>(k_cache + (size_t)slot * nk + (c - nq)) = in;
+      continue;
+    }
+    const int at = c - nq - nk;
+    if (more.v_first) {
+      float first[8];
+      split_load8(reinterpret_cast<const T*>(more.v_first) + (size_t)t * more.v_first_ld + at, first);
+      const float lam = *more.v_lam;
+#pragma unroll
+      for (int i = 0; i < 8; ++i) in.e[i] = from_f32<T>((1.0f - lam) * to_f32(in.e[i]) + lam * first[i]);
+    }
+    *reinterpret_cast<Pack*>(v_cache + (size_t)slot * nv + at) = in;
+  }
+}
+
 extern "C" int nhv_rotary_split_write(const void* qkv, const void* bias, const void* qk_freqs, int rot, const void* v_freqs,
                                       const void* positions, const void* slot_mapping, void* q_out, void* k_cache,
                                       void* v_cache, int T, int Hq, int Hkv, int D, int E, int with_kv, int more_columns,
@@ -282,6 +328,22 @@ extern "C" int nhv_rotary_split_write(const void* qkv, const void* bias, const v
   const int heads = with_kv ? Hq + Hkv + Hv : Hq;
   const int ld = (with_kv ? Hq * D + Hkv * D + (v_from_k ? 0 : Hv * E) : Hq * D) + more_columns;   // (columns that belong to another reader)
   NHV_REQUIRE((long long)T * heads < (1ll << 31), "rotary_split_write: too many tokens");
+  const size_t item = dtype == NHV_F32 ? 4 : 2;
+  const uintptr_t starts = (uintptr_t)qkv | (uintptr_t)q_out | (uintptr_t)k_cache | (uintptr_t)v_cache | (uintptr_t)v_first;
+  if (with_kv && rot == 0 && !unit && !v_freqs && !bias && !v_from_k && maps == 1 && D % 8 == 0 && E % 8 == 0 && ld % 8 == 0 &&
+      v_first_ld % 8 == 0 && starts % (8 * item) == 0 && (dtype == NHV_F32 || dtype == NHV_BF16)) {
+    const int nq = Hq * D, nk = Hkv * D, nv = Hkv * E;
+    const dim3 grid(((nq + nk + nv) / 8 + 255) / 256, T < 65535 ? T : 65535);
+    hipStream_t s = (hipStream_t)stream;
+    if (dtype == NHV_F32)
+      hipLaunchKernelGGL(split_write_vec_kernel<float>, grid, dim3(256), 0, s, (const float*)qkv, (const int*)positions,
+                         (const int*)slot_mapping, (float*)q_out, (float*)k_cache, (float*)v_cache, nq, nk, nv, ld, T, more);
+    else
+      hipLaunchKernelGGL(split_write_vec_kernel<bf16_t>, grid, dim3(256), 0, s, (const bf16_t*)qkv, (const int*)positions,
+                         (const int*)slot_mapping, (bf16_t*)q_out, (bf16_t*)k_cache, (bf16_t*)v_cache, nq, nk, nv, ld, T, more);
+    NHV_LAUNCH_CHECK("split_write_vec");
+    return 0;
+  }
   const size_t lds = unit ? (size_t)D * sizeof(float) : 0;
   NHV_REQUIRE(lds <= 64 * 1024, "rotary_split_write: heads of %d entries are beyond this kernel's unit norm", D);
   hipStream_t s = (hipStream_t)stream;

@@ -203,6 +203,7 @@ class NativeBackend:
         more = () if plain else options
         # the kernels on the matrix cores take value heads of the key heads' size; a chunk goes to them as a negative window
         fast = q.dtype == torch.bfloat16 and E == D and D % 16 == 0 and D <= 256
+        fast = fast and (slopes is None or (not cap and scale > 0))
         if chunk:
             window = -chunk
         if fast and batch.max_q_len == 1 and T <= 65535:
@@ -653,10 +654,15 @@ class NativeBackend:
         M, K = x.shape
         N = w.shape[0]
         if x.dtype == torch.bfloat16 and K % 8 == 0 and x.data_ptr() % 16 == 0 and w.data_ptr() % 16 == 0:
-            if bias is None and not self.own_kernels_only and (M <= self.library_rows or out.dtype == torch.bfloat16):
+            # (a bias of few rows joins in the own kernel; of more rows in a kernel after whatever made the product)
+            if (not self.own_kernels_only and (M <= self.library_rows or out.dtype == torch.bfloat16)
+                    and (bias is None or (M > self.few_rows and out.dtype == torch.bfloat16))):
                 how = self._choose(x, w, out)
                 if how is not None and how >= 0:
-                    return self._library_product(x, w, out, how)
+                    self._library_product(x, w, out, how)
+                    if bias is not None:
+                        self._call("nhv_add_bias_rows", _ptr(out), _ptr(bias), M, N, dtype_code(out), _stream())
+                    return None
             if M <= self.few_rows or (M <= 64 and self.own_kernels_only):
                 return self._call("nhv_gemm_skinny_bf16", _ptr(x), _ptr(w), _ptr(bias), _ptr(out), M, N, K,
                                   dtype_code(out), _stream())
