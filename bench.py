@@ -19,10 +19,10 @@ For these two ``value`` is generated tokens a second over the whole run, prompts
 ``--workload projections`` is a diagnosis, not the benchmark: a layer's matrix products alone, cold, beside a kernel
 that only reads the same bytes (see ``bench_projections``).
 
-``--workload design --shape pevazen-1b|pevazen-8b|fazovik-1b|fazovik-8b|vugelix-1b|vugelix-8b|pukarax-1b|pukarax-8b [--layers L]``: a model of
-the Pevazen, the Fazovik, the Vugelix or the Pukarax design (see ``architectures/``) beside a Qwen3 model (for Vugelix:
+``--workload design --shape D-1b|D-8b [--layers L]``, D one of pevazen, fazovik, vugelix, pukarax and gabelorn: a model of
+that design (see ``architectures/``) beside a Qwen3 model (for Vugelix:
 a Pevazen model of pairs of mixers; for Pukarax: a Fazovik model, whose feed-forwards are dense and routed in turn as
-well) of the same width, heads, feed-forward size, experts, vocabulary and number of layers: one prompt of ``--prompt-tokens`` in one step, decoding at
+well; for Gabelorn: a Fazovik model with dense feed-forwards and a Qwen3 model) of the same width, heads, feed-forward size, experts, vocabulary and number of layers: one prompt of ``--prompt-tokens`` in one step, decoding at
 ``--batch`` requests, and the time of every own kernel in one eager step of each kind (see ``bench_design``).
 """
 import argparse

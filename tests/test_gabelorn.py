@@ -239,7 +239,7 @@ def _latent_plain(m, eps, rows, w):
 
 
 @pytest.mark.parametrize("where", WHERE)
-@pytest.mark.parametrize("sizes", [(3, 8, 4, 6, 10), (20, 16, 16, 16, 48), (1, 1, 2, 1, 1), (4, 32, 16, 24, 100), (2, 64, 32, 64, 160), (2, 5, 6, 7, 9)],
+@pytest.mark.parametrize("sizes", [(3, 8, 4, 6, 10), (20, 16, 16, 16, 48), (1, 1, 2, 1, 1), (4, 32, 16, 24, 100), (2, 64, 32, 64, 160), (2, 5, 6, 7, 9), (2, 8, 16, 8, 300)],
                          ids=lambda s: "H%d-D%d-R%d-E%d-C%d" % s)
 @pytest.mark.parametrize("window", [1, 7, 40, 1000])
 def test_latent_attention_alone(where, kernels, sizes, window):
