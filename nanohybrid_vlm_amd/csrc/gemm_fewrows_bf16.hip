@@ -170,6 +170,7 @@ __global__ __launch_bounds__(64 * WAVES) void gemm_fewrows_kernel(const bf16_t* 
     for (int na = 0; na < NA; ++na) wrow[na * NT + nt] = w + ((size_t)na * N + (n_ok[nt] ? n : 0)) * K;
   }
   const bool m_ok = col < M;
+  if (f.band_rows) x += (size_t)min(n0 / f.band_rows, f.bands - 1) * M * K;
   const bf16_t* xrow = x + (size_t)(m_ok ? col : 0) * K;
 
   floatx4 acc[TILES];
@@ -748,6 +749,13 @@ int nhv_gemm_fewrows_launch(bool glu, const void* x, const void* w, const void* 
   using namespace fewrows;
   // a product that takes over work of its neighbours is a kernel of its own kind (more registers): bfloat16 results only
   const bool fused = f.residual != nullptr || f.ss_in != nullptr;
+  if (f.band_rows) {
+    // (a block's tiles lie in one band)
+    if (glu || fused || f.band_rows % 16 != 0) return nhv_fail("few-rows gemm: bands of %d rows (multiples of 16, no gate, no fusion)", f.band_rows);
+    if (f.band_rows % 32 == 0 && (N + 15) / 16 > 512) launch<2, 8, 2, false>(s, x, w, bias, y, M, N, K, out_dtype, false, f);
+    else launch<1, 8, 8, false>(s, x, w, bias, y, M, N, K, out_dtype, false, f);
+    return 0;
+  }
   if (fused && out_dtype != NHV_BF16) return nhv_fail("few-rows gemm: a product that takes over its neighbours' work gives bfloat16");
   const ResidentPlan rp = resident_plan(glu, M, N, K);
 #define NHV_RESIDENT_CASE(WV_, UN_, GLU_, PIECES_)                                                                     \

@@ -206,6 +206,21 @@ extern "C" int nhv_gemm_fewrows_act_bf16(const void* x, const void* w, void* y, 
   return 0;
 }
 
+// y[M, N] for up to 16 rows of each of ``bands`` sets x [bands, M, K]: outputs band_rows s ... band_rows (s + 1) - 1 from set s,
+// the last set's outputs going on to N. band_rows: a multiple of 16.
+extern "C" int nhv_gemm_fewrows_banded_bf16(const void* x, const void* w, void* y, int M, int N, int K, int bands, int band_rows,
+                                            int out_dtype, void* stream) {
+  if (sk_check("few-rows gemm in bands", x, w, M, N, K, out_dtype)) return 1;
+  NHV_REQUIRE(M <= 16 && bands > 0 && band_rows > 0 && band_rows % 16 == 0 && (long long)band_rows * (bands - 1) < N,
+              "few-rows gemm in bands: %d rows (up to 16), %d bands of %d rows (a multiple of 16) of %d", M, bands, band_rows, N);
+  NhvGemmFusion f = {};
+  f.band_rows = band_rows;
+  f.bands = bands;
+  if (nhv_gemm_fewrows_launch(false, x, w, nullptr, y, M, N, K, out_dtype, (hipStream_t)stream, f)) return 1;
+  NHV_LAUNCH_CHECK("gemm_fewrows_banded_bf16");
+  return 0;
+}
+
 // ---- products of up to 16 rows that take over the kernels around them (nhv_gemm_fusion.h) ----
 // y = r . (x . w^T) (+ bias), or with glu a gate (nhv_gates.h) of r . (x . w[0:N]^T) and r . (x . w[N:2N]^T) (bias: [2N]),
 // for 1 <= M <= 16 rows in bfloat16. With ss_in: x is a sum (times its norm's weight) whose rows still lack their scales: r per row from ss_in

@@ -1,0 +1,651 @@
+// Linear recurrences: mixers whose state is one matrix S[D, E] per head and request that decays and takes one outer
+// product a token, without a softmax or a denominator. Two designs of them share the kernels (kind):
+//   kind 0, a fixed decay per head ("retention"):      S_t = g_h S_(t-1) + k_t v_t^T,           o_t = S_t^T q_t,
+//           q and k turned by position (pairs (i, i + rot / 2)), k multiplied by a constant;
+//   kind 1, a decay per key channel and token ("wkv"): o_t = (S_(t-1) + diag(u) k_t v_t^T)^T r_t, S_t = diag(w_t) S_(t-1) + k_t v_t^T,
+//           w = exp(-exp(W2 tanh(z) + w0)) with z the first product of a low-rank projection.
+// Kernels:
+//  - nhv_token_shift: rows mixed with the row before them, x + (x' - x) mu_i, for several mu at once; the row before a
+//    request's first row of the step is kept per request;
+//  - nhv_recurrence_prepare and nhv_recurrence_chunks: portions of prompts, 16 tokens at a time. The first works on all
+//    chunks at once: decays and their running products, the products of a chunk's tokens among themselves
+//    A[t, j] (j <= t), queries with the decay from the chunk's start R[t], keys with the decay to its end K[t], and
+//    the decay of the whole chunk. The second walks over a request's chunks in order: O = A V + R S, S = diag(decay) S + K^T V,
+//    as float matrix products (v_mfma_f32_16x16x4_f32);
+//  - nhv_recurrence_tokens: steps of one or a few tokens a request: everything from the projections to the normed and
+//    gated read-out in one launch, a block per (request, head);
+//  - nhv_readout_norm: o over its root mean square per head, times a weight per entry (optional), times g sigmoid(g).
+// Everything is float but the projections' rows. Decays are kept as base-2 logarithms and only differences that are
+// never positive are raised: a strong decay gives zeros, not overflows. The state is [slots, H, E, D], zero for a request whose
+// first token is at position 0. A request without tokens in the step is left alone. A token's sums within a step
+// depend on where the step's first token of its request lies, by rounding only.
+#include "nhv_common.h"
+#include "nhv_rotation.h"
+#include <math.h>
+
+typedef __attribute__((__vector_size__(4 * sizeof(float)))) float floatx4;
+
+#define NHV_LOG2E 1.4426950408889634f
+#define NHV_CHUNK 16
+#define NHV_RANK_PIECE 64
+
+__device__ __forceinline__ float exp2_of(float x) { return __builtin_amdgcn_exp2f(x); }   // (x <= 0; tiny results may become 0)
+__device__ __forceinline__ float silu_of(float z) { return z / (1.0f + expf(-z)); }
+
+// ---------------------------------------------------------------- rows mixed with the row before them
+// out[i, t, :] = h[t] + (h' - h[t]) mu[i], h' the request's row before t (of this step, or kept[slot]; zeros at position 0).
+// The thread that reads a kept row (the request's first row of the step) also writes what the next step needs: the
+// request's last row; no other thread touches the kept row.
+template <typename T, int V>
+__global__ __launch_bounds__(256) void token_shift_kernel(const T* __restrict__ h, const float* __restrict__ mu, float* kept,
+                                                          T* __restrict__ out, const int* __restrict__ token_req,
+                                                          const int* __restrict__ positions, const int* __restrict__ cu,
+                                                          const int* __restrict__ state_slots, int n_mu, int rows, int W) {
+  struct alignas(sizeof(T) * V) Pack { T e[V]; };
+  const int c = (blockIdx.x * 256 + threadIdx.x) * V;
+  if (c >= W) return;
+  for (int t = blockIdx.y; t < rows; t += gridDim.y) {
+    const int req = token_req[t], first = cu[req];
+    const Pack me = *reinterpret_cast<const Pack*>(h + (size_t)t * W + c);
+    float x[V], d[V];
+    if (t > first) {
+      const Pack before = *reinterpret_cast<const Pack*>(h + (size_t)(t - 1) * W + c);
+#pragma unroll
+      for (int i = 0; i < V; ++i) d[i] = to_f32(before.e[i]);
+    } else {
+      float* row = kept + (size_t)state_slots[req] * W + c;
+      const bool fresh = positions[t] == 0;
+#pragma unroll
+      for (int i = 0; i < V; ++i) d[i] = fresh ? 0.f : row[i];
+      const Pack last = *reinterpret_cast<const Pack*>(h + (size_t)(cu[req + 1] - 1) * W + c);
+#pragma unroll
+      for (int i = 0; i < V; ++i) row[i] = to_f32(last.e[i]);
+    }
+#pragma unroll
+    for (int i = 0; i < V; ++i) {
+      x[i] = to_f32(me.e[i]);
+      d[i] -= x[i];
+    }
+    for (int m = 0; m < n_mu; ++m) {
+      Pack y;
+#pragma unroll
+      for (int i = 0; i < V; ++i) y.e[i] = from_f32<T>(fmaf(d[i], mu[(size_t)m * W + c + i], x[i]));
+      *reinterpret_cast<Pack*>(out + ((size_t)m * rows + t) * W + c) = y;
+    }
+  }
+}
+
+extern "C" int nhv_token_shift(const void* h, const void* mu, void* kept, void* out, const void* token_req, const void* positions,
+                               const void* cu, const void* state_slots, int n_mu, int T, int W, int dtype, void* stream) {
+  NHV_REQUIRE(T > 0 && W > 0 && n_mu > 0, "token_shift: bad sizes T=%d W=%d mixes=%d", T, W, n_mu);
+  hipStream_t s = (hipStream_t)stream;
+  const bool wide = W % 8 == 0 && (((uintptr_t)h | (uintptr_t)out) & 31) == 0;
+#define LAUNCH(TT, VV)                                                                                                  \
+  hipLaunchKernelGGL((token_shift_kernel<TT, VV>), dim3((W / VV + 255) / 256, T < 65535 ? T : 65535), dim3(256), 0, s,   \
+                     (const TT*)h, (const float*)mu, (float*)kept, (TT*)out, (const int*)token_req, (const int*)positions, \
+                     (const int*)cu, (const int*)state_slots, n_mu, T, W)
+  if (dtype == NHV_F32) { if (wide) LAUNCH(float, 8); else LAUNCH(float, 1); }
+  else if (dtype == NHV_BF16) { if (wide) LAUNCH(bf16_t, 8); else LAUNCH(bf16_t, 1); }
+  else return nhv_fail("token_shift: unknown dtype %d", dtype);
+#undef LAUNCH
+  NHV_LAUNCH_CHECK("token_shift");
+  return 0;
+}
+
+// ---------------------------------------------------------------- what the recurrences read
+// Rows of q (or r), k, v and the gates' linear parts: entry (t, h, i) at ptr + t ld + h size + i, all of one type.
+struct RecurrenceIn {
+  const void* q;
+  const void* k;
+  const void* v;
+  const void* g;
+  long long ld;
+  // kind 0
+  const float* log2_decay;                   // [H]
+  const double* freqs;                       // [rot / 2]
+  const int* turn_positions;                 // [T]
+  int rot;
+  float k_scale;
+  // kind 1
+  const float* z;                            // [T, rank], rows z_ld apart: before the tanh
+  long long z_ld;
+  const void* w2;                            // [H D, rank] of the weights' type
+  int rank;
+  const float* w0;                           // [H D]
+  const float* u;                            // [H D]
+};
+
+
+// ---------------------------------------------------------------- portions of prompts: all chunks at once
+// One block of 256 threads per (chunk, head, request). A chunk's place in the outputs: cu[req] / 16 + req + its number in
+// the request (places never overlap: a request of n tokens has at most floor(n / 16) + 1 chunks).
+template <typename T, typename TW, int KIND>
+__global__ __launch_bounds__(256) void recurrence_prepare_kernel(const RecurrenceIn in, float* __restrict__ r_out,
+                                                                 float* __restrict__ k_out, float* __restrict__ a_out,
+                                                                 float* __restrict__ decay_out, const int* __restrict__ cu,
+                                                                 int H, int D, int Dp) {
+  extern __shared__ __attribute__((aligned(16))) float lds[];
+  const int req = blockIdx.z, h = blockIdx.y;
+  const int first = cu[req], t0 = first + blockIdx.x * NHV_CHUNK, end = cu[req + 1];
+  if (t0 >= end) return;                     // (the same for the whole block)
+  const int n = min(NHV_CHUNK, end - t0);
+  const size_t place = ((size_t)(first / NHV_CHUNK) + req + blockIdx.x) * H + h;
+  const int tid = threadIdx.x, LD = D | 1;   // (rows of an odd number of floats: sixteen rows lie in sixteen banks)
+  float* rs = lds;
+  float* ks = rs + NHV_CHUNK * LD;
+  float* ls = ks + NHV_CHUNK * LD;           // kind 1: running sums of the decays' logarithms, the token's own included
+  const T* q = (const T*)in.q + (size_t)h * D;
+  const T* k = (const T*)in.k + (size_t)h * D;
+  if (KIND == 0) {
+    const int half = in.rot / 2, per = D - half;
+    for (int x = tid; x < NHV_CHUNK * per; x += 256) {
+      const int t = x / per, i = x % per;
+      const size_t at = (size_t)(t0 + t) * in.ld;
+      if (i < half) {
+        float q1 = 0.f, q2 = 0.f, k1 = 0.f, k2 = 0.f, sn = 0.f, cs = 0.f;
+        if (t < n) {
+          nhv_turn_angle<float>(in.turn_positions[t0 + t], in.freqs[i], 1.0f, &sn, &cs);
+          q1 = to_f32(q[at + i]); q2 = to_f32(q[at + i + half]);
+          k1 = to_f32(k[at + i]); k2 = to_f32(k[at + i + half]);
+        }
+        rs[t * LD + i] = q1 * cs - q2 * sn;
+        rs[t * LD + i + half] = q2 * cs + q1 * sn;
+        ks[t * LD + i] = (k1 * cs - k2 * sn) * in.k_scale;
+        ks[t * LD + i + half] = (k2 * cs + k1 * sn) * in.k_scale;
+      } else {
+        rs[t * LD + i + half] = t < n ? to_f32(q[at + i + half]) : 0.f;
+        ks[t * LD + i + half] = t < n ? to_f32(k[at + i + half]) * in.k_scale : 0.f;
+      }
+    }
+  } else {
+    for (int x = tid; x < NHV_CHUNK * D; x += 256) {
+      const int t = x / D, d = x % D;
+      const size_t at = (size_t)(t0 + t) * in.ld + d;
+      rs[t * LD + d] = t < n ? to_f32(q[at]) : 0.f;
+      ks[t * LD + d] = t < n ? to_f32(k[at]) : 0.f;
+    }
+    // the decays' linear part: a thread takes channel d of some of the tokens
+    constexpr int TLD = NHV_RANK_PIECE + 4;
+    float* th = lds + ((3 * NHV_CHUNK * LD + 3) & ~3);
+    int groups = 256 / D;
+    if (groups < 1) groups = 1;
+    if (groups > NHV_CHUNK) groups = NHV_CHUNK;
+    const int per = (NHV_CHUNK + groups - 1) / groups;
+    const int d = tid % D, tok0 = (tid / D) * per;
+    const bool works = tid < D * groups && tok0 < NHV_CHUNK;
+    const TW* w2 = (const TW*)in.w2 + ((size_t)h * D + d) * in.rank;
+    float acc[NHV_CHUNK];
+#pragma unroll
+    for (int i = 0; i < NHV_CHUNK; ++i) acc[i] = 0.f;
+    for (int r0 = 0; r0 < in.rank; r0 += NHV_RANK_PIECE) {
+      const int piece = min(NHV_RANK_PIECE, in.rank - r0);
+      for (int x = tid; x < NHV_CHUNK * NHV_RANK_PIECE; x += 256) {
+        const int t = x / NHV_RANK_PIECE, r = x % NHV_RANK_PIECE;
+        th[t * TLD + r] = (t < n && r < piece) ? tanhf(in.z[(size_t)(t0 + t) * in.z_ld + r0 + r]) : 0.f;
+      }
+      __syncthreads();
+      if (works) {
+        for (int r = 0; r < piece; r += 4) {
+          float w[4];
+#pragma unroll
+          for (int i = 0; i < 4; ++i) w[i] = r + i < piece ? to_f32(w2[r0 + r + i]) : 0.f;
+#pragma unroll
+          for (int i = 0; i < NHV_CHUNK; ++i) {
+            if (i < per && tok0 + i < NHV_CHUNK) {
+              const float4 x = *reinterpret_cast<const float4*>(&th[(tok0 + i) * TLD + r]);
+              acc[i] = fmaf(w[0], x.x, fmaf(w[1], x.y, fmaf(w[2], x.z, fmaf(w[3], x.w, acc[i]))));
+            }
+          }
+        }
+      }
+      __syncthreads();
+    }
+    if (works) {
+      const float w0 = in.w0[h * D + d];
+#pragma unroll
+      for (int i = 0; i < NHV_CHUNK; ++i)
+        if (i < per && tok0 + i < NHV_CHUNK) ls[(tok0 + i) * LD + d] = tok0 + i < n ? -NHV_LOG2E * expf(acc[i] + w0) : 0.f;
+    }
+    __syncthreads();
+    if (tid < D) {
+      float sum = 0.f;
+#pragma unroll
+      for (int t = 0; t < NHV_CHUNK; ++t) {
+        sum += ls[t * LD + tid];
+        ls[t * LD + tid] = sum;
+      }
+    }
+  }
+  __syncthreads();
+  const float l2 = KIND == 0 ? in.log2_decay[h] : 0.f;
+  {                                          // A: a thread per (t, j)
+    const int t = tid >> 4, j = tid & 15;
+    float sum = 0.f;
+    if (t < n && j <= t) {
+      if (KIND == 0) {
+        for (int d = 0; d < D; ++d) sum = fmaf(rs[t * LD + d], ks[j * LD + d], sum);
+        sum *= exp2_of(l2 * (float)(t - j));
+      } else if (j == t) {
+        for (int d = 0; d < D; ++d) sum = fmaf(rs[t * LD + d] * in.u[h * D + d], ks[t * LD + d], sum);
+      } else {
+        for (int d = 0; d < D; ++d)
+          sum = fmaf(rs[t * LD + d] * exp2_of(ls[(t - 1) * LD + d] - ls[j * LD + d]), ks[j * LD + d], sum);
+      }
+    }
+    a_out[place * 256 + tid] = sum;
+  }
+  for (int x = tid; x < NHV_CHUNK * Dp; x += 256) {
+    const int t = x / Dp, d = x % Dp;
+    float r = 0.f, kk = 0.f;
+    if (t < n && d < D) {
+      const float from_start = KIND == 0 ? l2 * (float)(t + 1) : (t > 0 ? ls[(t - 1) * LD + d] : 0.f);
+      const float to_end = KIND == 0 ? l2 * (float)(n - 1 - t) : ls[(n - 1) * LD + d] - ls[t * LD + d];
+      r = rs[t * LD + d] * exp2_of(from_start);
+      kk = ks[t * LD + d] * exp2_of(to_end);
+    }
+    r_out[place * NHV_CHUNK * Dp + x] = r;
+    k_out[place * NHV_CHUNK * Dp + x] = kk;
+  }
+  for (int d = tid; d < Dp; d += 256)
+    decay_out[place * Dp + d] = d < D ? exp2_of(KIND == 0 ? l2 * (float)n : ls[(n - 1) * LD + d]) : 0.f;
+}
+
+// ---------------------------------------------------------------- portions of prompts: a request's chunks in order
+// A block owns 16 columns of S (value channels) of one head of one request; its four waves share D in tiles of 16 rows,
+// TPW tiles a wave, which stay in registers as the result of the matrix cores' products: lane l holds S[16 tile + 4 (l / 16) + i,
+// column l % 16]. With the rows of D taken in that same order the tile is also the right-hand operand of R S as it stands.
+// The waves' shares of O meet in LDS (two buffers, one barrier a chunk) and are added in the order of the waves.
+template <typename T, int TPW>
+__global__ __launch_bounds__(256) void recurrence_chunks_kernel(const float* __restrict__ r_in, const float* __restrict__ k_in,
+                                                                const float* __restrict__ a_in, const float* __restrict__ decay_in,
+                                                                const T* __restrict__ v, long long ld, float* __restrict__ state,
+                                                                float* __restrict__ out, const int* __restrict__ positions,
+                                                                const int* __restrict__ cu, const int* __restrict__ state_slots,
+                                                                int H, int D, int Dp, int E) {
+  __shared__ float red[2][4][NHV_CHUNK][17];
+  const int req = blockIdx.z, h = blockIdx.y, e0 = blockIdx.x * 16;
+  const int first = cu[req], end = cu[req + 1];
+  if (end <= first) return;                  // (the same for the whole block)
+  const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63, col = lane & 15, grp = lane >> 4;
+  const int tiles = Dp / 16, tile0 = wave * TPW;
+  const bool column = e0 + col < E;
+  float* mine = state + (((size_t)state_slots[req] * H + h) * E + (column ? e0 + col : 0)) * D;
+  const bool fresh = positions[first] == 0;
+  floatx4 S[TPW];
+#pragma unroll
+  for (int i = 0; i < TPW; ++i)
+#pragma unroll
+    for (int j = 0; j < 4; ++j) {
+      const int d = (tile0 + i) * 16 + grp * 4 + j;
+      S[i][j] = (!fresh && column && d < D) ? mine[d] : 0.f;
+    }
+  const int chunks = (end - first + NHV_CHUNK - 1) / NHV_CHUNK;
+  const size_t place0 = (size_t)(first / NHV_CHUNK) + req;
+  floatx4 r[TPW], g[TPW];
+  float kk[TPW][4], vv[4];
+  float a = 0.f;
+  const T* vcol = v + (size_t)h * E + e0 + (column ? col : 0);
+  auto ask = [&](int c) {
+    const size_t place = (place0 + c) * H + h;
+    const int t0 = first + c * NHV_CHUNK;
+#pragma unroll
+    for (int i = 0; i < TPW; ++i) {
+      if (tile0 + i < tiles) {
+        const int d = (tile0 + i) * 16;
+        r[i] = *reinterpret_cast<const floatx4*>(r_in + (place * NHV_CHUNK + col) * Dp + d + grp * 4);
+        g[i] = *reinterpret_cast<const floatx4*>(decay_in + place * Dp + d + grp * 4);
+#pragma unroll
+        for (int j = 0; j < 4; ++j) kk[i][j] = k_in[(place * NHV_CHUNK + grp * 4 + j) * Dp + d + col];
+      } else {
+        r[i] = g[i] = floatx4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+        for (int j = 0; j < 4; ++j) kk[i][j] = 0.f;
+      }
+    }
+#pragma unroll
+    for (int j = 0; j < 4; ++j) {
+      const int t = t0 + grp * 4 + j;
+      vv[j] = (column && t < end) ? to_f32(vcol[(size_t)t * ld]) : 0.f;
+    }
+    a = a_in[place * 256 + col * 16 + grp * 4 + wave];
+  };
+  ask(0);
+  for (int c = 0; c < chunks; ++c) {
+    floatx4 o = {0.f, 0.f, 0.f, 0.f}, o2 = {0.f, 0.f, 0.f, 0.f};
+    // this wave's share of A V: the tokens 4 grp + wave
+    o2 = __builtin_amdgcn_mfma_f32_16x16x4f32(a, wave == 0 ? vv[0] : wave == 1 ? vv[1] : wave == 2 ? vv[2] : vv[3], o2, 0, 0, 0);
+#pragma unroll
+    for (int i = 0; i < TPW; ++i) {
+      o = __builtin_amdgcn_mfma_f32_16x16x4f32(r[i][0], S[i][0], o, 0, 0, 0);
+      o2 = __builtin_amdgcn_mfma_f32_16x16x4f32(r[i][1], S[i][1], o2, 0, 0, 0);
+      o = __builtin_amdgcn_mfma_f32_16x16x4f32(r[i][2], S[i][2], o, 0, 0, 0);
+      o2 = __builtin_amdgcn_mfma_f32_16x16x4f32(r[i][3], S[i][3], o2, 0, 0, 0);
+    }
+#pragma unroll
+    for (int i = 0; i < TPW; ++i) {
+#pragma unroll
+      for (int j = 0; j < 4; ++j) S[i][j] *= g[i][j];
+    }
+#pragma unroll
+    for (int j = 0; j < 4; ++j)
+#pragma unroll
+      for (int i = 0; i < TPW; ++i) S[i] = __builtin_amdgcn_mfma_f32_16x16x4f32(kk[i][j], vv[j], S[i], 0, 0, 0);
+    if (c + 1 < chunks) ask(c + 1);
+#pragma unroll
+    for (int j = 0; j < 4; ++j) red[c & 1][wave][grp * 4 + j][col] = o[j] + o2[j];
+    __syncthreads();
+    const int t = first + c * NHV_CHUNK + (tid >> 4), e = e0 + (tid & 15);
+    if (t < end && e < E) {
+      float sum = 0.f;
+#pragma unroll
+      for (int w = 0; w < 4; ++w) sum += red[c & 1][w][tid >> 4][tid & 15];
+      out[((size_t)t * H + h) * E + e] = sum;
+    }
+  }
+#pragma unroll
+  for (int i = 0; i < TPW; ++i)
+#pragma unroll
+    for (int j = 0; j < 4; ++j) {
+      const int d = (tile0 + i) * 16 + grp * 4 + j;
+      if (column && d < D) mine[d] = S[i][j];
+    }
+}
+
+// ---------------------------------------------------------------- steps of a few tokens a request: one launch
+// A block per (head, request). Token by token: the token's vectors go to LDS (turned; decays worked out), then every column
+// of S meets them: a column belongs to R adjacent lanes of 16 entries each, columns beyond the block's lanes come in
+// further passes; then the read-outs' norm and gate.
+template <typename T, typename TW, typename TO, int KIND, int R>
+__global__ __launch_bounds__(1024) void recurrence_tokens_kernel(const RecurrenceIn in, float* __restrict__ state,
+                                                                 const float* __restrict__ norm_w, float eps, TO* __restrict__ y,
+                                                                 const int* __restrict__ positions, const int* __restrict__ cu,
+                                                                 const int* __restrict__ state_slots, int H, int D, int E) {
+  extern __shared__ __attribute__((aligned(16))) float lds[];
+  __shared__ float scratch[16];
+  const int req = blockIdx.y, h = blockIdx.x;
+  const int first = cu[req], end = cu[req + 1];
+  if (end <= first) return;                  // (the same for the whole block)
+  const int tid = threadIdx.x, threads = blockDim.x;
+  const int Dl = R * 16;
+  float* qs = lds;                           // what meets the state: r, or q times the decay
+  float* ks = qs + Dl;
+  float* gs = ks + Dl;                       // decays
+  float* os = gs + Dl;                       // read-outs, E floats
+  float* zs = os + E;                        // kind 1: tanh(z), rank floats
+  float* head = state + ((size_t)state_slots[req] * H + h) * E * D;
+  const bool whole4 = (D & 3) == 0;
+  const float decay = KIND == 0 ? exp2f(in.log2_decay[h]) : 0.f;
+  for (int t = first; t < end; ++t) {
+    const T* q = (const T*)in.q + (size_t)t * in.ld + (size_t)h * D;
+    const T* k = (const T*)in.k + (size_t)t * in.ld + (size_t)h * D;
+    float bonus = 0.f;                       // this thread's share of what the token's own k v^T counts for
+    if (KIND == 1) {
+      for (int r = tid; r < in.rank; r += threads) zs[r] = tanhf(in.z[(size_t)t * in.z_ld + r]);
+      __syncthreads();
+      // four lanes a channel
+      for (int x = tid; x < Dl * 4; x += threads) {
+        const int d = x >> 2;
+        float sum = 0.f;
+        if (d < D) {
+          const TW* w2 = (const TW*)in.w2 + ((size_t)h * D + d) * in.rank;
+#pragma unroll 4
+          for (int r = x & 3; r < in.rank; r += 4) sum = fmaf(to_f32(w2[r]), zs[r], sum);
+        }
+        sum += __shfl_xor(sum, 1, NHV_WAVE);
+        sum += __shfl_xor(sum, 2, NHV_WAVE);
+        if ((x & 3) == 0) {
+          float rr = 0.f, kk = 0.f;
+          if (d < D) {
+            rr = to_f32(q[d]);
+            kk = to_f32(k[d]);
+            bonus = fmaf(rr * in.u[h * D + d], kk, bonus);
+          }
+          qs[d] = rr;
+          ks[d] = kk;
+          gs[d] = d < D ? exp2_of(-NHV_LOG2E * expf(sum + in.w0[h * D + d])) : 0.f;
+        }
+      }
+    } else {
+      const int half = in.rot / 2;
+      for (int d = tid; d < Dl; d += threads) {
+        float a = 0.f, b = 0.f;
+        if (d < D) {
+          a = to_f32(q[d]);
+          b = to_f32(k[d]);
+          if (d < in.rot) {
+            const int i = d < half ? d : d - half;
+            float sn, cs;
+            nhv_turn_angle<float>(in.turn_positions[t], in.freqs[i], 1.0f, &sn, &cs);
+            const float a2 = to_f32(q[d < half ? d + half : i]), b2 = to_f32(k[d < half ? d + half : i]);
+            a = d < half ? a * cs - a2 * sn : a * cs + a2 * sn;
+            b = d < half ? b * cs - b2 * sn : b * cs + b2 * sn;
+          }
+          b *= in.k_scale;
+          bonus = fmaf(a, b, bonus);
+        }
+        qs[d] = a * decay;
+        ks[d] = b;
+        gs[d] = decay;
+      }
+    }
+    bonus = block_sum(bonus, scratch);       // (its barriers also make the vectors visible)
+    const bool fresh = t == first && positions[t] == 0;
+    const int cols = threads / R, part = tid % R;
+    float ss = 0.f;
+    for (int e0 = 0; e0 < E; e0 += cols) {
+      const int e = e0 + tid / R;
+      const bool column = e < E && tid / R < cols;
+      float* mine = head + (size_t)(column ? e : 0) * D + part * 16;
+      float S[16];
+#pragma unroll
+      for (int i = 0; i < 16; i += 4) {
+        const int d = part * 16 + i;
+        if (whole4) {
+          const float4 s4 = (!fresh && column && d < D) ? *reinterpret_cast<const float4*>(mine + i) : float4{0.f, 0.f, 0.f, 0.f};
+          S[i] = s4.x; S[i + 1] = s4.y; S[i + 2] = s4.z; S[i + 3] = s4.w;
+        } else {
+#pragma unroll
+          for (int j = 0; j < 4; ++j) S[i + j] = (!fresh && column && d + j < D) ? mine[i + j] : 0.f;
+        }
+      }
+      const float vv = column ? to_f32(((const T*)in.v)[(size_t)t * in.ld + (size_t)h * E + e]) : 0.f;
+      float sum = 0.f;
+#pragma unroll
+      for (int i = 0; i < 16; i += 4) {
+        const int d = part * 16 + i;
+        const float4 q4 = *reinterpret_cast<const float4*>(&qs[d]), k4 = *reinterpret_cast<const float4*>(&ks[d]),
+                     g4 = *reinterpret_cast<const float4*>(&gs[d]);
+        sum = fmaf(q4.x, S[i], fmaf(q4.y, S[i + 1], fmaf(q4.z, S[i + 2], fmaf(q4.w, S[i + 3], sum))));
+        S[i] = fmaf(g4.x, S[i], k4.x * vv);
+        S[i + 1] = fmaf(g4.y, S[i + 1], k4.y * vv);
+        S[i + 2] = fmaf(g4.z, S[i + 2], k4.z * vv);
+        S[i + 3] = fmaf(g4.w, S[i + 3], k4.w * vv);
+      }
+#pragma unroll
+      for (int o = 1; o < R; o <<= 1) sum += __shfl_xor(sum, o, NHV_WAVE);
+      sum = fmaf(bonus, vv, sum);
+      if (column) {
+#pragma unroll
+        for (int i = 0; i < 16; i += 4) {
+          const int d = part * 16 + i;
+          if (whole4) {
+            if (d < D) *reinterpret_cast<float4*>(mine + i) = float4{S[i], S[i + 1], S[i + 2], S[i + 3]};
+          } else {
+#pragma unroll
+            for (int j = 0; j < 4; ++j)
+              if (d + j < D) mine[i + j] = S[i + j];
+          }
+        }
+        if (part == 0) {
+          os[e] = sum;
+          ss = fmaf(sum, sum, ss);
+        }
+      }
+    }
+    const float inv = 1.0f / sqrtf(block_sum(ss, scratch) / (float)E + eps);
+    for (int e = tid; e < E; e += threads) {
+      const float gate = silu_of(to_f32(((const T*)in.g)[(size_t)t * in.ld + (size_t)h * E + e]));
+      y[((size_t)t * H + h) * E + e] = from_f32<TO>(os[e] * inv * (norm_w ? norm_w[(size_t)h * E + e] : 1.0f) * gate);
+    }
+    __syncthreads();                         // (the next token's vectors take this one's place)
+  }
+}
+
+// ---------------------------------------------------------------- the read-out's norm and gate, for many rows
+template <typename T, typename TO>
+__global__ __launch_bounds__(256) void readout_norm_kernel(const float* __restrict__ o, const T* __restrict__ gate, long long ld,
+                                                           const float* __restrict__ w, TO* __restrict__ y, int H, int E,
+                                                           float eps, int n_items) {
+  const int item = blockIdx.x * 4 + (threadIdx.x >> 6);
+  if (item >= n_items) return;
+  const int lane = threadIdx.x & 63, t = item / H, h = item % H;
+  const float* src = o + (size_t)item * E;
+  float ss = 0.f;
+  for (int e = lane; e < E; e += NHV_WAVE) ss = fmaf(src[e], src[e], ss);
+  const float r = 1.0f / sqrtf(wave_sum(ss) / (float)E + eps);
+  for (int e = lane; e < E; e += NHV_WAVE) {
+    const float z = to_f32(gate[(size_t)t * ld + (size_t)h * E + e]);
+    y[(size_t)item * E + e] = from_f32<TO>(src[e] * r * (w ? w[(size_t)h * E + e] : 1.0f) * silu_of(z));
+  }
+}
+
+static RecurrenceIn recurrence_in(const void* q, const void* k, const void* v, const void* g, long long ld, const void* log2_decay,
+                                  const void* freqs, const void* turn_positions, int rot, float k_scale, const void* z,
+                                  long long z_ld, const void* w2, int rank, const void* w0, const void* u) {
+  RecurrenceIn in;
+  in.q = q; in.k = k; in.v = v; in.g = g; in.ld = ld;
+  in.log2_decay = (const float*)log2_decay; in.freqs = (const double*)freqs; in.turn_positions = (const int*)turn_positions;
+  in.rot = rot; in.k_scale = k_scale;
+  in.z = (const float*)z; in.z_ld = z_ld; in.w2 = w2; in.rank = rank; in.w0 = (const float*)w0; in.u = (const float*)u;
+  return in;
+}
+
+#define NHV_RECURRENCE_CHECK(name)                                                                                          \
+  NHV_REQUIRE(B > 0 && H > 0 && D > 0 && E > 0 && B <= 65535 && H <= 65535, name ": bad sizes B=%d H=%d D=%d E=%d", B, H, D, E); \
+  NHV_REQUIRE(D <= 256, name ": key heads of %d entries (up to 256 are taken)", D);                                         \
+  NHV_REQUIRE(kind == 0 || kind == 1, name ": kind %d", kind);                                                              \
+  NHV_REQUIRE(dtype == NHV_F32 || dtype == NHV_BF16, name ": unknown dtype %d", dtype);                                     \
+  NHV_REQUIRE(kind == 1 || (log2_decay && rot >= 0 && rot % 2 == 0 && rot <= D && (rot == 0 || (freqs && turn_positions))),  \
+              name ": %d turned entries of %d", rot, D);                                                                    \
+  NHV_REQUIRE(kind == 0 || (z && w2 && w0 && u && rank > 0 && z_ld >= rank), name ": decays of rank %d", rank)
+
+// Chunks' places: T / 16 + B + 1. r_out, k_out [places, H, 16, Dp], a_out [places, H, 16, 16], decay_out [places, H, Dp], Dp the
+// head size rounded up to a multiple of 16.
+extern "C" int nhv_recurrence_prepare(int kind, const void* q, const void* k, long long ld, int dtype, const void* log2_decay,
+                                      const void* freqs, const void* turn_positions, int rot, float k_scale, const void* z,
+                                      long long z_ld, const void* w2, int w2_dtype, int rank, const void* w0, const void* u,
+                                      void* r_out, void* k_out, void* a_out, void* decay_out, const void* cu, int B, int H, int D,
+                                      int max_q_len, void* stream) {
+  const int E = 1;
+  NHV_RECURRENCE_CHECK("recurrence_prepare");
+  NHV_REQUIRE(max_q_len > 0 && ld >= (long long)H * D, "recurrence_prepare: rows of %lld entries for %d heads of %d", ld, H, D);
+  const RecurrenceIn in = recurrence_in(q, k, nullptr, nullptr, ld, log2_decay, freqs, turn_positions, rot, k_scale, z, z_ld, w2,
+                                        rank, w0, u);
+  const int Dp = (D + 15) / 16 * 16;
+  const size_t lds = ((((kind == 1 ? 3 : 2) * NHV_CHUNK * (size_t)(D | 1)) + 3) / 4 * 4 +
+                      (kind == 1 ? NHV_CHUNK * (NHV_RANK_PIECE + 4) : 0)) * sizeof(float);
+  const dim3 grid((max_q_len + NHV_CHUNK - 1) / NHV_CHUNK, H, B);
+  hipStream_t s = (hipStream_t)stream;
+#define LAUNCH(TT, TTW, KIND)                                                                                            \
+  hipLaunchKernelGGL((recurrence_prepare_kernel<TT, TTW, KIND>), grid, dim3(256), lds, s, in, (float*)r_out, (float*)k_out, \
+                     (float*)a_out, (float*)decay_out, (const int*)cu, H, D, Dp)
+  if (kind == 0) { if (dtype == NHV_F32) LAUNCH(float, float, 0); else LAUNCH(bf16_t, bf16_t, 0); }
+  else if (w2_dtype == NHV_F32) { if (dtype == NHV_F32) LAUNCH(float, float, 1); else LAUNCH(bf16_t, float, 1); }
+  else if (w2_dtype == NHV_BF16) { if (dtype == NHV_F32) LAUNCH(float, bf16_t, 1); else LAUNCH(bf16_t, bf16_t, 1); }
+  else return nhv_fail("recurrence_prepare: unknown dtype %d", w2_dtype);
+#undef LAUNCH
+  NHV_LAUNCH_CHECK("recurrence_prepare");
+  return 0;
+}
+
+extern "C" int nhv_recurrence_chunks(const void* r_in, const void* k_in, const void* a_in, const void* decay_in, const void* v,
+                                     long long ld, int dtype, void* state, void* out, const void* positions, const void* cu,
+                                     const void* state_slots, int B, int H, int D, int E, void* stream) {
+  NHV_REQUIRE(B > 0 && H > 0 && D > 0 && E > 0 && B <= 65535 && H <= 65535 && D <= 256 && ld >= (long long)H * E,
+              "recurrence_chunks: bad sizes B=%d H=%d D=%d (up to 256) E=%d, rows of %lld", B, H, D, E, ld);
+  const int Dp = (D + 15) / 16 * 16, tpw = (Dp / 16 + 3) / 4;
+  const dim3 grid((E + 15) / 16, H, B);
+  hipStream_t s = (hipStream_t)stream;
+#define LAUNCH(TT, N)                                                                                                     \
+  hipLaunchKernelGGL((recurrence_chunks_kernel<TT, N>), grid, dim3(256), 0, s, (const float*)r_in, (const float*)k_in,    \
+                     (const float*)a_in, (const float*)decay_in, (const TT*)v, ld, (float*)state, (float*)out,            \
+                     (const int*)positions, (const int*)cu, (const int*)state_slots, H, D, Dp, E)
+#define BY_TILES(TT)          \
+  if (tpw == 1) LAUNCH(TT, 1); \
+  else if (tpw == 2) LAUNCH(TT, 2); \
+  else if (tpw == 3) LAUNCH(TT, 3); \
+  else LAUNCH(TT, 4)
+  if (dtype == NHV_F32) { BY_TILES(float); }
+  else if (dtype == NHV_BF16) { BY_TILES(bf16_t); }
+  else return nhv_fail("recurrence_chunks: unknown dtype %d", dtype);
+#undef BY_TILES
+#undef LAUNCH
+  NHV_LAUNCH_CHECK("recurrence_chunks");
+  return 0;
+}
+
+extern "C" int nhv_recurrence_tokens(int kind, const void* q, const void* k, const void* v, const void* g, long long ld, int dtype,
+                                     const void* log2_decay, const void* freqs, const void* turn_positions, int rot, float k_scale,
+                                     const void* z, long long z_ld, const void* w2, int w2_dtype, int rank, const void* w0,
+                                     const void* u, void* state, const void* norm_w, float eps, void* y, int y_dtype,
+                                     const void* positions, const void* cu, const void* state_slots, int B, int H, int D, int E,
+                                     void* stream) {
+  NHV_RECURRENCE_CHECK("recurrence_tokens");
+  NHV_REQUIRE(y_dtype == NHV_F32 || y_dtype == NHV_BF16, "recurrence_tokens: unknown dtype %d", y_dtype);
+  const RecurrenceIn in = recurrence_in(q, k, v, g, ld, log2_decay, freqs, turn_positions, rot, k_scale, z, z_ld, w2, rank, w0, u);
+  int R = 1;
+  while (R * 16 < D) R <<= 1;
+  int threads = (E * R + 63) / 64 * 64;
+  if (threads > 1024) threads = 1024;
+  if (threads < 128) threads = 128;
+  const size_t lds = (3 * (size_t)R * 16 + E + (kind == 1 ? rank : 0)) * sizeof(float);
+  NHV_REQUIRE(lds <= 60 * 1024, "recurrence_tokens: value heads of %d and decays of rank %d are beyond this kernel", E, rank);
+  const dim3 grid(H, B);
+  hipStream_t s = (hipStream_t)stream;
+#define LAUNCH(TT, TTW, TTO, KIND, RR)                                                                                      \
+  hipLaunchKernelGGL((recurrence_tokens_kernel<TT, TTW, TTO, KIND, RR>), grid, dim3(threads), lds, s, in, (float*)state,    \
+                     (const float*)norm_w, eps, (TTO*)y, (const int*)positions, (const int*)cu, (const int*)state_slots, H, D, E)
+#define BY_R(TT, TTW, TTO, KIND)                       \
+  switch (R) {                                         \
+    case 1: LAUNCH(TT, TTW, TTO, KIND, 1); break;      \
+    case 2: LAUNCH(TT, TTW, TTO, KIND, 2); break;      \
+    case 4: LAUNCH(TT, TTW, TTO, KIND, 4); break;      \
+    case 8: LAUNCH(TT, TTW, TTO, KIND, 8); break;      \
+    default: LAUNCH(TT, TTW, TTO, KIND, 16); break;    \
+  }
+  const bool f = dtype == NHV_F32, fo = y_dtype == NHV_F32, fw = w2_dtype == NHV_F32;
+  if (kind == 0) {
+    if (f && fo) { BY_R(float, float, float, 0) }
+    else if (!f && !fo) { BY_R(bf16_t, bf16_t, bf16_t, 0) }
+    else if (f && !fo) { BY_R(float, bf16_t, bf16_t, 0) }
+    else return nhv_fail("recurrence_tokens: bfloat16 rows give bfloat16 rows");
+  } else {
+    if (f && fo && fw) { BY_R(float, float, float, 1) }
+    else if (f && !fo && !fw) { BY_R(float, bf16_t, bf16_t, 1) }
+    else if (!f && !fo && !fw) { BY_R(bf16_t, bf16_t, bf16_t, 1) }
+    else return nhv_fail("recurrence_tokens: rows, weights and results of types %d, %d, %d are not taken", dtype, w2_dtype, y_dtype);
+  }
+#undef BY_R
+#undef LAUNCH
+  NHV_LAUNCH_CHECK("recurrence_tokens");
+  return 0;
+}
+
+extern "C" int nhv_readout_norm(const void* o, const void* gate, long long ld, int gate_dtype, const void* w, void* y, int y_dtype,
+                                int T, int H, int E, float eps, void* stream) {
+  NHV_REQUIRE(T > 0 && H > 0 && E > 0 && (long long)T * H < (1ll << 31) && ld >= (long long)H * E,
+              "readout_norm: bad sizes T=%d H=%d E=%d, gate rows of %lld", T, H, E, ld);
+  const int n_items = T * H;
+  const dim3 grid((unsigned)((n_items + 3) / 4));
+  hipStream_t s = (hipStream_t)stream;
+#define LAUNCH(TT, TTO)                                                                                                    \
+  hipLaunchKernelGGL((readout_norm_kernel<TT, TTO>), grid, dim3(256), 0, s, (const float*)o, (const TT*)gate, ld,          \
+                     (const float*)w, (TTO*)y, H, E, eps, n_items)
+  if (gate_dtype == NHV_F32 && y_dtype == NHV_F32) LAUNCH(float, float);
+  else if (gate_dtype == NHV_F32 && y_dtype == NHV_BF16) LAUNCH(float, bf16_t);
+  else if (gate_dtype == NHV_BF16 && y_dtype == NHV_BF16) LAUNCH(bf16_t, bf16_t);
+  else return nhv_fail("readout_norm: gates of type %d and rows of type %d are not taken together", gate_dtype, y_dtype);
+#undef LAUNCH
+  NHV_LAUNCH_CHECK("readout_norm");
+  return 0;
+}

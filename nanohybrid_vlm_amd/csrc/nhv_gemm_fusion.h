@@ -25,6 +25,9 @@ struct NhvGemmFusion {
   NhvGate gate;          // what a gated product makes of its two sums (all zero: SiLU)
   int plain_act;         // what a product without a gate passes its result through (after the bias): 0 nothing, 1 SiLU,
                          // 2 the tanh form of GELU, 3 the square of max(z, 0)
+  // Bands: x holds several sets of M rows, [sets, M, K], and outputs band_rows s ... band_rows (s + 1) - 1 are made from
+  // set s (the last set has all outputs from there on). 0: one set. Only the kernel that takes x from memory knows bands.
+  int band_rows, bands;
 };
 
 __device__ __forceinline__ float nhv_plain_act(float z, int act) {

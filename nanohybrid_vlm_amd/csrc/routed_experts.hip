@@ -1,9 +1,11 @@
 // A feed-forward made of many small gated feed-forwards of which every token uses a few.
 //   nhv_route_topk        from a row's float router logits (plus an optional bias) the ``top`` largest: their numbers and
 //                         scores (the sigmoid of each, or the softmax over the chosen logits alone)
+//   nhv_route_groups      the same choice by softmax scores over all experts plus a correction, among the best groups of experts
 //   nhv_experts_gate_up   for every (token, chosen expert): act(s G_e h) * (s U_e h), s the score: the expert's input is
 //                         s h, and a product is linear in its rows, so the score multiplies the finished float sums
-//                         (no scores: s = 1, for a design whose scores weigh the experts' outputs)
+//                         (no scores: s = 1, for a design whose scores weigh the experts' outputs); or act(s U_e h), for
+//                         experts without a gate
 //   nhv_experts_down      out[t] = sum over the token's experts of [w[t, j]] D_e u[t, j] [+ one more row added to all]
 // One wave per output: a sum runs over its inner index in an order that depends on the sizes only, so a row's result
 // does not depend on its batch. Weights of all experts lie in one tensor, [experts, 2 ff, width] (gate rows, then up
@@ -66,7 +68,88 @@ extern "C" int nhv_route_topk(const void* logits, const void* bias, void* ids, v
   return 0;
 }
 
+// The choice by softmax scores over all experts: s = softmax(z), choice c = s + correction; experts form ``groups`` equal runs of
+// neighbours, a group counts by its largest c, only the ``keep`` best groups' experts can be chosen; scores are s, not renormalised.
+// One wave per token.
+__global__ void route_groups_kernel(const float* __restrict__ logits, const float* __restrict__ correction, int* __restrict__ ids,
+                                    float* __restrict__ scores, int T, int E, int top, int groups, int keep) {
+  extern __shared__ float route_lds[];        // waves x 2 E: c, then the groups' bests
+  const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
+  const int t = blockIdx.x * (blockDim.x >> 6) + wave;
+  if (t >= T) return;
+  float* c = route_lds + (size_t)wave * 2 * E;
+  float* best_of = c + E;
+  const float* z = logits + (size_t)t * E;
+  float m = -INFINITY;
+  for (int e = lane; e < E; e += NHV_WAVE) m = fmaxf(m, z[e]);
+  m = wave_max(m);
+  float sum = 0.f;
+  for (int e = lane; e < E; e += NHV_WAVE) sum += expf(z[e] - m);
+  sum = wave_sum(sum);
+  for (int e = lane; e < E; e += NHV_WAVE) c[e] = expf(z[e] - m) / sum + (correction ? correction[e] : 0.f);
+  __builtin_amdgcn_wave_barrier();
+  // the largest entry of ``list`` (the first among equals), in every lane
+  auto largest = [&](const float* list, int n) {
+    float best = -INFINITY;
+    int at = 0x7fffffff;
+    for (int e = lane; e < n; e += NHV_WAVE)
+      if (list[e] > best) { best = list[e]; at = e; }
+#pragma unroll
+    for (int o = 32; o > 0; o >>= 1) {
+      const float ov = __shfl_xor(best, o, NHV_WAVE);
+      const int oa = __shfl_xor(at, o, NHV_WAVE);
+      if (ov > best || (ov == best && oa < at)) { best = ov; at = oa; }
+    }
+    return at == 0x7fffffff ? 0 : at;        // (no number at all: the first)
+  };
+  if (keep < groups) {
+    const int size = E / groups;
+    for (int g = lane; g < groups; g += NHV_WAVE) {
+      float b = -INFINITY;
+      for (int i = 0; i < size; ++i) b = fmaxf(b, c[g * size + i]);
+      best_of[g] = b;
+    }
+    __builtin_amdgcn_wave_barrier();
+    // the kept groups are marked by NaN, which no comparison takes
+    for (int j = 0; j < keep; ++j) {
+      const int g = largest(best_of, groups);
+      if (lane == 0) best_of[g] = NAN;
+      __builtin_amdgcn_wave_barrier();
+    }
+    for (int e = lane; e < E; e += NHV_WAVE)
+      if (!isnan(best_of[e / size])) c[e] = -INFINITY;
+    __builtin_amdgcn_wave_barrier();
+  }
+  for (int j = 0; j < top; ++j) {
+    const int at = largest(c, E);
+    if (lane == 0) {
+      ids[(size_t)t * top + j] = at;
+      scores[(size_t)t * top + j] = expf(z[at] - m) / sum;
+      c[at] = -INFINITY;
+    }
+    __builtin_amdgcn_wave_barrier();
+  }
+}
+
+extern "C" int nhv_route_groups(const void* logits, const void* correction, void* ids, void* scores, int T, int E, int top, int groups,
+                                int keep, void* stream) {
+  NHV_REQUIRE(T > 0 && E > 0 && E <= 4096 && groups > 0 && E % groups == 0 && keep > 0 && keep <= groups && top > 0 &&
+                  top <= keep * (E / groups),
+              "route_groups: bad sizes T=%d E=%d (up to 4096) top=%d, %d of %d groups", T, E, top, keep, groups);
+  const int waves = E <= 1024 ? 4 : 1;
+  hipLaunchKernelGGL(route_groups_kernel, dim3((T + waves - 1) / waves), dim3(64 * waves), (size_t)waves * 2 * E * sizeof(float),
+                     (hipStream_t)stream, (const float*)logits, (const float*)correction, (int*)ids, (float*)scores, T, E, top,
+                     groups, keep);
+  NHV_LAUNCH_CHECK("route_groups");
+  return 0;
+}
+
+// act: 0 SiLU, 1 the tanh form of GELU, 2 the square of max(z, 0)
 __device__ __forceinline__ float nhv_expert_act(float z, int act) {
+  if (act == 2) {
+    const float r = fmaxf(z, 0.f);
+    return r * r;
+  }
   if (act == 1) return 0.5f * z * (1.0f + tanhf(0.7978845608028654f * (z + 0.044715f * z * z * z)));
   return z / (1.0f + expf(-z));
 }
@@ -91,7 +174,8 @@ __device__ __forceinline__ void ex_load8f<float>(const float* p, float* out) {
 }
 
 // u[t * top + j, f] for the pair (t, j): one wave per f.
-template <typename T>
+// GATED false: one matrix [F, W] an expert, u = act(s U_e h).
+template <typename T, bool GATED>
 __global__ __launch_bounds__(256) void experts_gate_up_kernel(const T* __restrict__ h, const int* __restrict__ ids,
                                                               const float* __restrict__ scores,
                                                               const T* __restrict__ gate_up, T* __restrict__ u, int W,
@@ -103,60 +187,61 @@ __global__ __launch_bounds__(256) void experts_gate_up_kernel(const T* __restric
   const int e = ids[pair];
   if (e < 0 || e >= E) return;
   const T* x = h + (size_t)(pair / top) * W;
-  const T* g = gate_up + ((size_t)e * 2 * F + f) * W;
-  const T* p = g + (size_t)F * W;
+  const T* g = gate_up + ((size_t)e * (GATED ? 2 : 1) * F + f) * W;
+  const T* p = GATED ? g + (size_t)F * W : g;
   float sg = 0.f, su = 0.f;
   if (W % 8 == 0) {                          // (rows then start at multiples of 16 or 32 bytes)
     for (int k = lane * 8; k < W; k += NHV_WAVE * 8) {
       float xv[8], gv[8], pv[8];
       ex_load8f(x + k, xv);
       ex_load8f(g + k, gv);
-      ex_load8f(p + k, pv);
+      if (GATED) ex_load8f(p + k, pv);
 #pragma unroll
       for (int i = 0; i < 8; ++i) {
         sg = fmaf(gv[i], xv[i], sg);
-        su = fmaf(pv[i], xv[i], su);
+        if (GATED) su = fmaf(pv[i], xv[i], su);
       }
     }
   } else {
     for (int k = lane; k < W; k += NHV_WAVE) {
       const float xv = to_f32(x[k]);
       sg = fmaf(to_f32(g[k]), xv, sg);
-      su = fmaf(to_f32(p[k]), xv, su);
+      if (GATED) su = fmaf(to_f32(p[k]), xv, su);
     }
   }
   sg = wave_sum(sg);
-  su = wave_sum(su);
+  if (GATED) su = wave_sum(su);
   if (lane == 0) {
     const float s = scores ? scores[pair] : 1.0f;
-    u[(size_t)pair * F + f] = from_f32<T>(nhv_expert_act(s * sg, act) * (s * su));
+    u[(size_t)pair * F + f] = from_f32<T>(GATED ? nhv_expert_act(s * sg, act) * (s * su) : nhv_expert_act(s * sg, act));
   }
 }
 
 extern "C" int nhv_experts_gate_up(const void* h, const void* ids, const void* scores, const void* gate_up, void* u,
-                                   int T, int W, int F, int top, int E, int act, int dtype, void* stream) {
+                                   int T, int W, int F, int top, int E, int act, int gated, int dtype, void* stream) {
   NHV_REQUIRE(T > 0 && W > 0 && F > 0 && top > 0 && E > 0, "experts_gate_up: bad sizes T=%d W=%d F=%d top=%d E=%d", T, W, F, top, E);
   NHV_REQUIRE((long long)T * top < (1ll << 31) && (F + 3) / 4 <= 65535, "experts_gate_up: T=%d top=%d F=%d are beyond this kernel's grid", T, top, F);
   const dim3 grid(T * top, (F + 3) / 4);
   hipStream_t s = (hipStream_t)stream;
-  if (dtype == NHV_F32)
-    hipLaunchKernelGGL(experts_gate_up_kernel<float>, grid, dim3(256), 0, s, (const float*)h, (const int*)ids,
-                       (const float*)scores, (const float*)gate_up, (float*)u, W, F, top, E, act);
-  else if (dtype == NHV_BF16)
-    hipLaunchKernelGGL(experts_gate_up_kernel<bf16_t>, grid, dim3(256), 0, s, (const bf16_t*)h, (const int*)ids,
-                       (const float*)scores, (const bf16_t*)gate_up, (bf16_t*)u, W, F, top, E, act);
+#define LAUNCH(TT, GATED)                                                                                             \
+  hipLaunchKernelGGL((experts_gate_up_kernel<TT, GATED>), grid, dim3(256), 0, s, (const TT*)h, (const int*)ids,       \
+                     (const float*)scores, (const TT*)gate_up, (TT*)u, W, F, top, E, act)
+  if (dtype == NHV_F32) { if (gated) LAUNCH(float, true); else LAUNCH(float, false); }
+  else if (dtype == NHV_BF16) { if (gated) LAUNCH(bf16_t, true); else LAUNCH(bf16_t, false); }
+#undef LAUNCH
   else
     return nhv_fail("experts_gate_up: unknown dtype %d", dtype);
   NHV_LAUNCH_CHECK("experts_gate_up");
   return 0;
 }
 
-// out[t, n] = sum over j < top (rising), each a sum over f [times weights[t, j]], [plus add[t, n]]: one wave per n.
+// out[t, n] = sum over j < top (rising), each a sum over f [times weights[t, j]], [plus add[t, n]]: one wave per n. With ``self``
+// a number e >= E stands for an expert without matrices whose output is self[t] (the token's input).
 template <typename T>
 __global__ __launch_bounds__(256) void experts_down_kernel(const T* __restrict__ u, const int* __restrict__ ids,
                                                            const T* __restrict__ down, T* __restrict__ out, int W, int F,
                                                            int top, int E, const float* __restrict__ weights,
-                                                           const T* __restrict__ add) {
+                                                           const T* __restrict__ add, const T* __restrict__ self) {
   const int t = blockIdx.x;
   const int n = blockIdx.y * 4 + (threadIdx.x >> 6);
   const int lane = threadIdx.x & 63;
@@ -164,6 +249,10 @@ __global__ __launch_bounds__(256) void experts_down_kernel(const T* __restrict__
   float total = 0.f;
   for (int j = 0; j < top; ++j) {
     const int e = ids[(size_t)t * top + j];
+    if (e >= E && self) {                    // an expert that hands its input on (the same value in every lane)
+      const float v = to_f32(self[(size_t)t * W + n]);
+      total += weights ? weights[(size_t)t * top + j] * v : v;
+    }
     if (e < 0 || e >= E) continue;
     const T* d = down + ((size_t)e * W + n) * F;
     const T* x = u + ((size_t)t * top + j) * F;
@@ -185,17 +274,18 @@ __global__ __launch_bounds__(256) void experts_down_kernel(const T* __restrict__
 }
 
 extern "C" int nhv_experts_down(const void* u, const void* ids, const void* down, void* out, int T, int W, int F, int top,
-                                int E, const void* weights, const void* add, int dtype, void* stream) {
+                                int E, const void* weights, const void* add, const void* self, int dtype, void* stream) {
   NHV_REQUIRE(T > 0 && W > 0 && F > 0 && top > 0 && E > 0, "experts_down: bad sizes T=%d W=%d F=%d top=%d E=%d", T, W, F, top, E);
   NHV_REQUIRE((W + 3) / 4 <= 65535, "experts_down: width %d is beyond this kernel's grid", W);
   const dim3 grid(T, (W + 3) / 4);
   hipStream_t s = (hipStream_t)stream;
   if (dtype == NHV_F32)
     hipLaunchKernelGGL(experts_down_kernel<float>, grid, dim3(256), 0, s, (const float*)u, (const int*)ids,
-                       (const float*)down, (float*)out, W, F, top, E, (const float*)weights, (const float*)add);
+                       (const float*)down, (float*)out, W, F, top, E, (const float*)weights, (const float*)add, (const float*)self);
   else if (dtype == NHV_BF16)
     hipLaunchKernelGGL(experts_down_kernel<bf16_t>, grid, dim3(256), 0, s, (const bf16_t*)u, (const int*)ids,
-                       (const bf16_t*)down, (bf16_t*)out, W, F, top, E, (const float*)weights, (const bf16_t*)add);
+                       (const bf16_t*)down, (bf16_t*)out, W, F, top, E, (const float*)weights, (const bf16_t*)add,
+                       (const bf16_t*)self);
   else
     return nhv_fail("experts_down: unknown dtype %d", dtype);
   NHV_LAUNCH_CHECK("experts_down");
@@ -267,14 +357,16 @@ extern "C" int nhv_experts_sort(const void* ids, int P, int E, int TM, void* sor
   return 0;
 }
 
-// x: GLU: the step's rows [tokens, K] (pair p reads row p / top); else one row per pair [pairs, K]. w: [experts, NA N, K].
-// y: one row per pair [pairs, N]. GLU: y = act(s g) * (s u) with the pair's score s.
-template <int MT, int NT, int WAVES, int UNROLL, bool GLU, typename TOut>
+// KIND 1 and 2 (an expert's first half, with and without a gate): x the step's rows [tokens, K] (pair p reads row p / top);
+// KIND 0 (its second half): one row per pair [pairs, K]. w: [experts, NA N, K], NA = 2 for KIND 1, else 1. y: one row per pair
+// [pairs, N]. KIND 1: y = act(s g) * (s u) with the pair's score s; KIND 2: y = act(s u).
+template <int MT, int NT, int WAVES, int UNROLL, int KIND, typename TOut>
 __global__ __launch_bounds__(64 * WAVES) void experts_grouped_kernel(const bf16_t* __restrict__ x, const bf16_t* __restrict__ w,
                                                                      TOut* __restrict__ y, const int* __restrict__ sorted,
                                                                      const int* __restrict__ tile_expert,
                                                                      const float* __restrict__ scores, int top, int N, int K,
                                                                      int act) {
+  constexpr bool GLU = KIND == 1, FIRST = KIND != 0;
   constexpr int NA = GLU ? 2 : 1;
   constexpr int TILES = NA * NT;
   static_assert(MT <= WAVES, "each of the first MT waves finishes one tile of rows");
@@ -301,7 +393,7 @@ __global__ __launch_bounds__(64 * WAVES) void experts_grouped_kernel(const bf16_
   for (int mt = 0; mt < MT; ++mt) {
     const int pair = places[mt * 16 + col];
     m_ok[mt] = pair >= 0;
-    xrow[mt] = x + (size_t)(m_ok[mt] ? (GLU ? pair / top : pair) : 0) * K;
+    xrow[mt] = x + (size_t)(m_ok[mt] ? (FIRST ? pair / top : pair) : 0) * K;
   }
   floatx4 acc[TILES][MT];
 #pragma unroll
@@ -331,7 +423,7 @@ __global__ __launch_bounds__(64 * WAVES) void experts_grouped_kernel(const bf16_
   }
   // wave ``mt`` adds the waves' partial sums of tile (nt, mt) in the order of the waves and writes that tile
   const int my_pair = wave < MT ? places[wave * 16 + col] : -1;
-  const float s = (GLU && scores && my_pair >= 0) ? scores[my_pair] : 1.0f;
+  const float s = (FIRST && scores && my_pair >= 0) ? scores[my_pair] : 1.0f;
 #pragma unroll
   for (int nt = 0; nt < NT; ++nt) {
     float v[NA][4];
@@ -360,6 +452,7 @@ __global__ __launch_bounds__(64 * WAVES) void experts_grouped_kernel(const bf16_
         if (n < N) {
           float r = v[0][j];
           if (GLU) r = nhv_expert_act(s * r, act) * (s * v[NA - 1][j]);
+          else if (FIRST) r = nhv_expert_act(s * r, act);
           y[(size_t)my_pair * N + n] = (TOut)r;
         }
       }
@@ -373,12 +466,13 @@ __global__ __launch_bounds__(64 * WAVES) void experts_grouped_kernel(const bf16_
 // tiles of pairs against BW / 16 / WN tiles of matrix rows (GLU: gate tiles and their up tiles). The larger the block's
 // tile, the fewer bytes cross from L2 for a product: 64 x 128 asks for 24 KB per 2^20 multiply-adds, 128 x 256 for 48 KB
 // per 2^22.
-template <bool GLU, typename TOut, int BM, int BW, int WM, int WN>
+template <int KIND, typename TOut, int BM, int BW, int WM, int WN>
 __global__ __launch_bounds__(64 * WM * WN) void experts_tiled_kernel(const bf16_t* __restrict__ x, const bf16_t* __restrict__ w,
                                                                      TOut* __restrict__ y, const int* __restrict__ sorted,
                                                                      const int* __restrict__ tile_expert,
                                                                      const float* __restrict__ scores, int top, int N, int K,
                                                                      int act) {
+  constexpr bool GLU = KIND == 1, FIRST = KIND != 0;
   constexpr int THREADS = 64 * WM * WN, BK = 64, LD = BK + 8;  // (rows of 144 bytes: 16-byte pieces stay aligned, banks shift)
   constexpr int RP = THREADS / 8;            // rows that the threads bring in one pass
   constexpr int XI = BM / RP, WI = BW / RP;
@@ -402,7 +496,7 @@ __global__ __launch_bounds__(64 * WM * WN) void experts_tiled_kernel(const bf16_
   for (int i = 0; i < XI; ++i) {
     const int pair = places[r0 + RP * i];
     xok[i] = pair >= 0;
-    xp[i] = x + (size_t)(xok[i] ? (GLU ? pair / top : pair) : 0) * K + kc;
+    xp[i] = x + (size_t)(xok[i] ? (FIRST ? pair / top : pair) : 0) * K + kc;
   }
   const bf16_t* wp[WI];
   bool wok[WI];
@@ -457,7 +551,7 @@ __global__ __launch_bounds__(64 * WM * WN) void experts_tiled_kernel(const bf16_
   for (int mt = 0; mt < MT; ++mt) {
     const int pair = places[(wm * MT + mt) * 16 + col];
     if (pair < 0) continue;
-    const float s = (GLU && scores) ? scores[pair] : 1.0f;
+    const float s = (FIRST && scores) ? scores[pair] : 1.0f;
 #pragma unroll
     for (int a = 0; a < NH; ++a)
 #pragma unroll
@@ -465,30 +559,31 @@ __global__ __launch_bounds__(64 * WM * WN) void experts_tiled_kernel(const bf16_
         const int n = n0 + (wn * NH + a) * 16 + grp * 4 + j;
         if (n >= N) continue;
         if (GLU) y[(size_t)pair * N + n] = (TOut)(nhv_expert_act(s * acc[a][mt][j], act) * (s * acc[NH + a][mt][j]));
+        else if (FIRST) y[(size_t)pair * N + n] = (TOut)nhv_expert_act(s * acc[a][mt][j], act);
         else y[(size_t)pair * N + n] = (TOut)acc[a][mt][j];
       }
   }
 }
 
-template <bool GLU, typename TOut>
+template <int KIND, typename TOut>
 static void tiled_launch(hipStream_t s, const void* x, const void* w, void* y, const void* sorted, const void* tile_expert,
                          const void* scores, int top, int N, int K, int act, int tiles_cap, int TM) {
-  const int out = GLU ? 64 : 128;
+  const int out = KIND == 1 ? 64 : 128;
   const dim3 grid(tiles_cap, (N + out - 1) / out);
   if (TM == 128)
-    hipLaunchKernelGGL((experts_tiled_kernel<GLU, TOut, 128, 128, 2, 4>), grid, dim3(512), 0, s, (const bf16_t*)x,
+    hipLaunchKernelGGL((experts_tiled_kernel<KIND, TOut, 128, 128, 2, 4>), grid, dim3(512), 0, s, (const bf16_t*)x,
                        (const bf16_t*)w, (TOut*)y, (const int*)sorted, (const int*)tile_expert, (const float*)scores, top, N, K, act);
   else
-    hipLaunchKernelGGL((experts_tiled_kernel<GLU, TOut, 64, 128, 1, 4>), grid, dim3(256), 0, s, (const bf16_t*)x,
+    hipLaunchKernelGGL((experts_tiled_kernel<KIND, TOut, 64, 128, 1, 4>), grid, dim3(256), 0, s, (const bf16_t*)x,
                        (const bf16_t*)w, (TOut*)y, (const int*)sorted, (const int*)tile_expert, (const float*)scores, top, N, K, act);
 }
 
-template <int MT, bool GLU, typename TOut>
+template <int MT, int KIND, typename TOut>
 static void grouped_launch(hipStream_t s, const void* x, const void* w, void* y, const void* sorted, const void* tile_expert,
                            const void* scores, int top, int N, int K, int act, int tiles_cap) {
-  constexpr int NT = GLU ? 2 : 4, WAVES = 8, UNROLL = 2;
+  constexpr int NT = KIND == 1 ? 2 : 4, WAVES = 8, UNROLL = 2;
   const dim3 grid(tiles_cap, (N + 16 * NT - 1) / (16 * NT));
-  hipLaunchKernelGGL((experts_grouped_kernel<MT, NT, WAVES, UNROLL, GLU, TOut>), grid, dim3(64 * WAVES), 0, s,
+  hipLaunchKernelGGL((experts_grouped_kernel<MT, NT, WAVES, UNROLL, KIND, TOut>), grid, dim3(64 * WAVES), 0, s,
                      (const bf16_t*)x, (const bf16_t*)w, (TOut*)y, (const int*)sorted, (const int*)tile_expert,
                      (const float*)scores, top, N, K, act);
 }
@@ -496,13 +591,15 @@ static void grouped_launch(hipStream_t s, const void* x, const void* w, void* y,
 // u [pairs, F] bfloat16 from the step's rows h [tokens, W]; TM: 16, 64 or 128 places a tile (as the sort was told).
 extern "C" int nhv_experts_grouped_gate_up(const void* h, const void* gate_up, void* u, const void* sorted,
                                            const void* tile_expert, const void* scores, int top, int W, int F, int act,
-                                           int TM, int tiles_cap, void* stream) {
+                                           int gated, int TM, int tiles_cap, void* stream) {
   NHV_REQUIRE(W > 0 && F > 0 && W % 8 == 0 && top > 0 && tiles_cap > 0 && (TM == 16 || TM == 64 || TM == 128),
               "experts_grouped_gate_up: bad sizes W=%d (a multiple of 8) F=%d top=%d TM=%d", W, F, top, TM);
   NHV_REQUIRE((F + 31) / 32 <= 65535, "experts_grouped_gate_up: F=%d is beyond this kernel's grid", F);
   hipStream_t s = (hipStream_t)stream;
-  if (TM >= 64) tiled_launch<true, bf16_t>(s, h, gate_up, u, sorted, tile_expert, scores, top, F, W, act, tiles_cap, TM);
-  else grouped_launch<1, true, bf16_t>(s, h, gate_up, u, sorted, tile_expert, scores, top, F, W, act, tiles_cap);
+  if (TM >= 64 && gated) tiled_launch<1, bf16_t>(s, h, gate_up, u, sorted, tile_expert, scores, top, F, W, act, tiles_cap, TM);
+  else if (TM >= 64) tiled_launch<2, bf16_t>(s, h, gate_up, u, sorted, tile_expert, scores, top, F, W, act, tiles_cap, TM);
+  else if (gated) grouped_launch<1, 1, bf16_t>(s, h, gate_up, u, sorted, tile_expert, scores, top, F, W, act, tiles_cap);
+  else grouped_launch<1, 2, bf16_t>(s, h, gate_up, u, sorted, tile_expert, scores, top, F, W, act, tiles_cap);
   NHV_LAUNCH_CHECK("experts_grouped_gate_up");
   return 0;
 }
@@ -514,30 +611,35 @@ extern "C" int nhv_experts_grouped_down(const void* u, const void* down, void* y
               "experts_grouped_down: bad sizes W=%d F=%d (a multiple of 8) TM=%d", W, F, TM);
   NHV_REQUIRE((W + 63) / 64 <= 65535, "experts_grouped_down: W=%d is beyond this kernel's grid", W);
   hipStream_t s = (hipStream_t)stream;
-  if (TM >= 64) tiled_launch<false, float>(s, u, down, y, sorted, tile_expert, nullptr, 1, W, F, 0, tiles_cap, TM);
-  else grouped_launch<1, false, float>(s, u, down, y, sorted, tile_expert, nullptr, 1, W, F, 0, tiles_cap);
+  if (TM >= 64) tiled_launch<0, float>(s, u, down, y, sorted, tile_expert, nullptr, 1, W, F, 0, tiles_cap, TM);
+  else grouped_launch<1, 0, float>(s, u, down, y, sorted, tile_expert, nullptr, 1, W, F, 0, tiles_cap);
   NHV_LAUNCH_CHECK("experts_grouped_down");
   return 0;
 }
 
-// out[t, n] = sum over j < top (rising) of [weights[t, j]] y[t * top + j, n], [plus add[t, n]]
+// out[t, n] = sum over j < top (rising) of [weights[t, j]] y[t * top + j, n], [plus add[t, n]]; with ``self`` the row of a pair whose
+// number (ids) is E or more is self[t]: such a pair has no row in y
 __global__ void experts_combine_kernel(const float* __restrict__ y, bf16_t* __restrict__ out, int W, int top, size_t total,
-                                       const float* __restrict__ weights, const bf16_t* __restrict__ add) {
+                                       const float* __restrict__ weights, const bf16_t* __restrict__ add,
+                                       const int* __restrict__ ids, int E, const bf16_t* __restrict__ self) {
   for (size_t i = (size_t)blockIdx.x * blockDim.x + threadIdx.x; i < total; i += (size_t)gridDim.x * blockDim.x) {
     const size_t t = i / W, n = i % W;
     float sum = 0.f;
-    for (int j = 0; j < top; ++j) sum += weights ? weights[t * top + j] * y[(t * top + j) * W + n] : y[(t * top + j) * W + n];
+    for (int j = 0; j < top; ++j) {
+      const float v = (self && ids[t * top + j] >= E) ? (float)self[i] : y[(t * top + j) * W + n];
+      sum += weights ? weights[t * top + j] * v : v;
+    }
     out[i] = (bf16_t)(add ? sum + (float)add[i] : sum);
   }
 }
 
 extern "C" int nhv_experts_combine(const void* y, void* out, int T, int W, int top, const void* weights, const void* add,
-                                   void* stream) {
+                                   const void* ids, int E, const void* self, void* stream) {
   NHV_REQUIRE(T > 0 && W > 0 && top > 0, "experts_combine: bad sizes T=%d W=%d top=%d", T, W, top);
   const size_t total = (size_t)T * W;
   const int blocks = (int)((total + 255) / 256 > 65535 * 4 ? 65535 * 4 : (total + 255) / 256);
   hipLaunchKernelGGL(experts_combine_kernel, dim3(blocks), dim3(256), 0, (hipStream_t)stream, (const float*)y, (bf16_t*)out,
-                     W, top, total, (const float*)weights, (const bf16_t*)add);
+                     W, top, total, (const float*)weights, (const bf16_t*)add, (const int*)ids, E, (const bf16_t*)self);
   NHV_LAUNCH_CHECK("experts_combine");
   return 0;
 }

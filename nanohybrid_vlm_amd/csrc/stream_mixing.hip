@@ -9,6 +9,7 @@
 //    position, mixes values with another layer's, and stores keys and values at the step's slots.
 // Statistics, angles and sums are float; rows are float or bfloat16.
 #include "nhv_common.h"
+#include "nhv_rotation.h"
 #include <math.h>
 
 // ---------------------------------------------------------------- norm with one number as its weight
@@ -357,6 +358,89 @@ extern "C" int nhv_rotary_split_write(const void* qkv, const void* bias, const v
   else return nhv_fail("rotary_split_write: unknown dtype %d", dtype);
 #undef LAUNCH
   NHV_LAUNCH_CHECK("rotary_split_write");
+  return 0;
+}
+
+// ---------------------------------------------------------------- queries and keys normed over their whole projection
+// Packed rows q (Hq D) | k (Hkv D) | v (Hkv E, absent where the values are the keys as projected), plus bias. All of q is
+// divided by its root mean square and multiplied by wq entry by entry, all of k likewise by wk; then pairs (i, i + rot / 2) of every head
+// turn by position * freqs[i] (doubles), cosine and sine times gain; q goes to q_out, keys and values to the step's slots. One
+// block a token: the sums of squares meet in LDS, and so do the token's sines and cosines, which all heads share.
+template <typename T>
+__global__ __launch_bounds__(256) void normed_split_write_kernel(const T* __restrict__ qkv, int ld, const T* __restrict__ bias,
+                                                                 const float* __restrict__ wq, const float* __restrict__ wk,
+                                                                 float eps, const double* __restrict__ freqs, int rot, float gain,
+                                                                 const int* __restrict__ positions,
+                                                                 const int* __restrict__ slot_mapping, T* __restrict__ q_out,
+                                                                 T* __restrict__ k_cache, T* __restrict__ v_cache, int Hq, int Hkv,
+                                                                 int D, int E, int v_from_k) {
+  extern __shared__ float turns[];             // rot / 2 sines, then as many cosines
+  __shared__ float scratch[16];
+  const int t = blockIdx.x, nq = Hq * D, nk = Hkv * D, half = rot / 2;
+  const T* row = qkv + (size_t)t * ld;
+  auto value = [&](int c) { return bias ? to_f32(row[c]) + to_f32(bias[c]) : to_f32(row[c]); };
+  for (int i = threadIdx.x; i < half; i += 256) nhv_turn_angle<float>(positions[t], freqs[i], gain, &turns[i], &turns[half + i]);
+  float sq = 0.f, sk = 0.f;
+  for (int c = threadIdx.x; c < nq; c += 256) {
+    const float v = value(c);
+    sq = fmaf(v, v, sq);
+  }
+  for (int c = nq + threadIdx.x; c < nq + nk; c += 256) {
+    const float v = value(c);
+    sk = fmaf(v, v, sk);
+  }
+  const float rq = 1.0f / sqrtf(block_sum(sq, scratch) / (float)nq + eps);
+  const float rk = 1.0f / sqrtf(block_sum(sk, scratch) / (float)nk + eps);    // (its barriers show the sines as well)
+  const int slot = slot_mapping[t];
+  const int per = D - half;                    // pairs, then what is not turned
+  const int heads = slot < 0 ? Hq : Hq + Hkv;  // (a row that stores nothing: padding of a recorded step)
+  for (int x = threadIdx.x; x < heads * per; x += 256) {
+    const int h = x / per, i = x % per;
+    const bool key = h >= Hq;
+    const float* w = key ? wk + (size_t)(h - Hq) * D : wq + (size_t)h * D;
+    const float r = key ? rk : rq;
+    T* dst = key ? k_cache + ((size_t)slot * Hkv + h - Hq) * D : q_out + ((size_t)t * Hq + h) * D;
+    const int c = h * D;
+    if (i < half) {
+      const float a = value(c + i), b = value(c + i + half);
+      const float u = a * r * w[i], v = b * r * w[i + half];
+      dst[i] = from_f32<T>(u * turns[half + i] - v * turns[i]);
+      dst[i + half] = from_f32<T>(v * turns[half + i] + u * turns[i]);
+      if (key && v_from_k) {
+        T* vd = v_cache + ((size_t)slot * Hkv + h - Hq) * E;
+        vd[i] = from_f32<T>(a);
+        vd[i + half] = from_f32<T>(b);
+      }
+    } else {
+      const float a = value(c + i + half);
+      dst[i + half] = from_f32<T>(a * r * w[i + half]);
+      if (key && v_from_k) v_cache[((size_t)slot * Hkv + h - Hq) * E + i + half] = from_f32<T>(a);
+    }
+  }
+  if (slot >= 0 && !v_from_k)
+    for (int c = threadIdx.x; c < Hkv * E; c += 256) v_cache[(size_t)slot * Hkv * E + c] = from_f32<T>(value(nq + nk + c));
+}
+
+extern "C" int nhv_normed_split_write(const void* qkv, long long ld, const void* bias, const void* wq, const void* wk, float eps,
+                                      const void* freqs, int rot, float gain, const void* positions, const void* slot_mapping,
+                                      void* q_out, void* k_cache, void* v_cache, int T, int Hq, int Hkv, int D, int E,
+                                      int v_from_k, int dtype, void* stream) {
+  NHV_REQUIRE(T > 0 && Hq > 0 && Hkv > 0 && D > 0 && E > 0, "normed_split_write: bad sizes T=%d Hq=%d Hkv=%d D=%d E=%d", T, Hq, Hkv, D, E);
+  NHV_REQUIRE(rot >= 0 && rot % 2 == 0 && rot <= D && (rot == 0 || freqs) && rot <= 8192, "normed_split_write: rotary size %d with head size %d", rot, D);
+  NHV_REQUIRE(!v_from_k || E == D, "normed_split_write: values that are the keys as projected have the keys' size");
+  NHV_REQUIRE(ld >= (long long)(Hq + Hkv) * D + (v_from_k ? 0 : Hkv * E) && ld < (1ll << 31), "normed_split_write: rows of %lld entries", ld);
+  NHV_REQUIRE(wq && wk && slot_mapping && k_cache && v_cache && eps >= 0.f, "normed_split_write: norm weights, slots and caches are needed");
+  hipStream_t s = (hipStream_t)stream;
+#define LAUNCH(TT)                                                                                                        \
+  hipLaunchKernelGGL(normed_split_write_kernel<TT>, dim3(T), dim3(256), (size_t)rot * sizeof(float), s, (const TT*)qkv, (int)ld, \
+                     (const TT*)bias, (const float*)wq, (const float*)wk, eps, (const double*)freqs, rot, gain,           \
+                     (const int*)positions, (const int*)slot_mapping, (TT*)q_out, (TT*)k_cache, (TT*)v_cache, Hq, Hkv, D, E, \
+                     v_from_k)
+  if (dtype == NHV_F32) LAUNCH(float);
+  else if (dtype == NHV_BF16) LAUNCH(bf16_t);
+  else return nhv_fail("normed_split_write: unknown dtype %d", dtype);
+#undef LAUNCH
+  NHV_LAUNCH_CHECK("normed_split_write");
   return 0;
 }
 

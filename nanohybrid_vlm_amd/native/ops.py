@@ -20,7 +20,7 @@ from . import library
 
 CORE_SOURCES = ["error.hip", "elementwise.hip", "gemm_generic.hip", "gemm_skinny_bf16.hip", "gemm_fewrows_bf16.hip", "attention_generic.hip",
                 "sampling.hip", "measure.hip", "stream_mixing.hip", "delta_rule.hip", "parallel_block.hip", "latent_attention.hip",
-                "routed_experts.hip", "hyper_streams.hip", "head_outputs.hip", "sandwich_norms.hip"]
+                "routed_experts.hip", "hyper_streams.hip", "head_outputs.hip", "sandwich_norms.hip", "linear_recurrence.hip"]
 BLAS_SOURCES = ["error.hip", "gemm_library.hip"]                                                   # the vendor's matrix library, algorithm by number
 BLAS_LINK = ["-lhipblaslt"]
 ATTENTION_SOURCES = ["error.hip", "attention_decode_bf16.hip", "attention_prefill_bf16.hip"]      # compiled once per head size
@@ -248,6 +248,13 @@ class NativeBackend:
                    int(values_from_keys), maps, ctypes.c_float(coef), ctypes.c_double(every), first_p,
                    ctypes.c_longlong(0 if first is None else first.shape[1]), _ptr(lam), dtype_code(qkv), _stream())
 
+    def normed_split_write(self, qkv, bias, wq, wk, eps, freqs, gain, positions, slot_mapping, q_out, k_cache, v_cache, Hq,
+                           Hkv, D, E, values_from_keys):
+        self._call("nhv_normed_split_write", _ptr(qkv), ctypes.c_longlong(qkv.shape[1]), _ptr(bias), _ptr(wq), _ptr(wk),
+                   ctypes.c_float(eps), _ptr(freqs), 0 if freqs is None else 2 * freqs.shape[0], ctypes.c_float(gain),
+                   _ptr(positions), _ptr(slot_mapping), _ptr(q_out), _ptr(k_cache), _ptr(v_cache), qkv.shape[0], Hq, Hkv, D, E,
+                   int(values_from_keys), dtype_code(qkv), _stream())
+
     # -- what heads' results pass before the output projection; a layer normed on both sides of its sublayers --
     def differential_combine(self, a, lam, out, eps, post, gate=None):
         T, H, E = out.shape
@@ -387,18 +394,22 @@ class NativeBackend:
         T, E = logits.shape
         self._call("nhv_route_topk", _ptr(logits), _ptr(bias), _ptr(ids), _ptr(scores), T, E, ids.shape[1], mode, _stream())
 
-    def experts_gate_up(self, h, ids, scores, gate_up, u, act):
-        T, W = h.shape
-        E, F2, _ = gate_up.shape
-        self._call("nhv_experts_gate_up", _ptr(h), _ptr(ids), _ptr(scores), _ptr(gate_up), _ptr(u), T, W, F2 // 2,
-                   ids.shape[1], E, act, dtype_code(h), _stream())
+    def route_groups(self, logits, correction, ids, scores, groups, keep):
+        T, E = logits.shape
+        self._call("nhv_route_groups", _ptr(logits), _ptr(correction), _ptr(ids), _ptr(scores), T, E, ids.shape[1], groups, keep,
+                   _stream())
 
-    def experts_grouped(self, h, ids, scores, gate_up, down, out, act, weights=None, add=None):
+    def experts_gate_up(self, h, ids, scores, gate_up, u, act, gated=True):
+        T, W = h.shape
+        self._call("nhv_experts_gate_up", _ptr(h), _ptr(ids), _ptr(scores), _ptr(gate_up), _ptr(u), T, W, u.shape[1],
+                   ids.shape[1], gate_up.shape[0], act, int(gated), dtype_code(h), _stream())
+
+    def experts_grouped(self, h, ids, scores, gate_up, down, out, act, weights=None, add=None, gated=True, self_rows=None):
         """Many rows in bfloat16: the pairs sorted by expert, then both products on the matrix cores, then the sum over
         a token's experts."""
         T, W = h.shape
-        E, F2, _ = gate_up.shape
-        F, top = F2 // 2, ids.shape[1]
+        E, F1, _ = gate_up.shape
+        F, top = (F1 // 2 if gated else F1), ids.shape[1]
         P = T * top
         # places a tile (runs of an expert's pairs are filled up to whole tiles): 128 or 64 where an expert has pairs
         # enough (block tiles of 128 x 128 and 64 x 128 matrix rows). Tiles of 128 pairs x 256 matrix rows, which the
@@ -411,17 +422,75 @@ class NativeBackend:
         self._call("nhv_experts_sort", _ptr(ids), P, E, TM, _ptr(sorted_pairs), tiles * TM, _ptr(tile_expert), tiles, _stream())
         u = torch.empty((P, F), dtype=h.dtype, device=h.device)
         self._call("nhv_experts_grouped_gate_up", _ptr(h), _ptr(gate_up), _ptr(u), _ptr(sorted_pairs), _ptr(tile_expert),
-                   _ptr(scores), top, W, F, act, TM, tiles, _stream())
+                   _ptr(scores), top, W, F, act, int(gated), TM, tiles, _stream())
         y = torch.empty((P, W), dtype=torch.float32, device=h.device)
         self._call("nhv_experts_grouped_down", _ptr(u), _ptr(down), _ptr(y), _ptr(sorted_pairs), _ptr(tile_expert), W, F, TM,
                    tiles, _stream())
-        self._call("nhv_experts_combine", _ptr(y), _ptr(out), T, W, top, _ptr(weights), _ptr(add), _stream())
+        self._call("nhv_experts_combine", _ptr(y), _ptr(out), T, W, top, _ptr(weights), _ptr(add), _ptr(ids), E,
+                   _ptr(self_rows), _stream())
 
-    def experts_down(self, u, ids, down, out, weights=None, add=None):
+    def experts_down(self, u, ids, down, out, weights=None, add=None, self_rows=None):
         T, W = out.shape
         E, _, F = down.shape
         self._call("nhv_experts_down", _ptr(u), _ptr(ids), _ptr(down), _ptr(out), T, W, F, ids.shape[1], E,
-                   _ptr(weights), _ptr(add), dtype_code(u), _stream())
+                   _ptr(weights), _ptr(add), _ptr(self_rows), dtype_code(u), _stream())
+
+    # -- linear recurrences --
+    def token_shift(self, h, mu, kept, out, batch, state_slots):
+        T, W = h.shape
+        self._call("nhv_token_shift", _ptr(h), _ptr(mu), _ptr(kept), _ptr(out), _ptr(batch.token_req), _ptr(batch.positions),
+                   _ptr(batch.cu_seqlens_q), _ptr(state_slots), mu.shape[0], T, W, dtype_code(h), _stream())
+
+    def banded_linear(self, x, w, out, band_rows) -> bool:
+        """One product whose outputs are made from several sets of rows (x [sets, rows, in]; ``band_rows`` outputs a set, the
+        last set has the rest), if this batch is one for the few-rows kernel; else False."""
+        sets, M, K = x.shape
+        if not (x.dtype == torch.bfloat16 and M <= self.few_rows and K % 8 == 0 and band_rows % 16 == 0
+                and x.data_ptr() % 16 == 0 and w.data_ptr() % 16 == 0):
+            return False
+        self._call("nhv_gemm_fewrows_banded_bf16", _ptr(x), _ptr(w), _ptr(out), M, w.shape[0], K, sets, band_rows,
+                   dtype_code(out), _stream())
+        return True
+
+    @staticmethod
+    def _recurrence_args(rule):
+        """The arguments of a ``Retention`` or ``WKV`` rule as the kernels take them (kind first)."""
+        LL = ctypes.c_longlong
+        if isinstance(rule, Retention):
+            return 0, (_ptr(rule.log2_decay), _ptr(rule.freqs), _ptr(rule.positions),
+                       0 if rule.freqs is None else 2 * rule.freqs.shape[0], ctypes.c_float(rule.k_scale), None, LL(0), None, 0,
+                       0, None, None)
+        return 1, (None, None, None, 0, ctypes.c_float(1.0), _ptr(rule.z), LL(rule.z.stride(0)), _ptr(rule.w2),
+                   dtype_code(rule.w2), rule.w2.shape[1], _ptr(rule.w0), _ptr(rule.u))
+
+    def recurrence_tokens(self, rule, q, k, v, gate, state, norm_w, eps, y, batch, state_slots):
+        _, H, E, D = state.shape
+        kind, args = self._recurrence_args(rule)
+        self._call("nhv_recurrence_tokens", kind, _ptr(q), _ptr(k), _ptr(v), _ptr(gate), ctypes.c_longlong(q.stride(0)),
+                   dtype_code(q), *args, _ptr(state), _ptr(norm_w), ctypes.c_float(eps), _ptr(y), dtype_code(y),
+                   _ptr(batch.positions), _ptr(batch.cu_seqlens_q), _ptr(state_slots), batch.num_requests, H, D, E, _stream())
+
+    def recurrence_chunks(self, rule, q, k, v, state, out, batch, state_slots):
+        _, H, E, D = state.shape
+        T, B, C = q.shape[0], batch.num_requests, 16
+        Dp = -(-D // 16) * 16
+        places = T // C + B + 1
+        kind, args = self._recurrence_args(rule)
+        r_s = torch.empty((places, H, C, Dp), dtype=torch.float32, device=q.device)
+        k_s = torch.empty_like(r_s)
+        a = torch.empty((places, H, C, C), dtype=torch.float32, device=q.device)
+        decay = torch.empty((places, H, Dp), dtype=torch.float32, device=q.device)
+        self._call("nhv_recurrence_prepare", kind, _ptr(q), _ptr(k), ctypes.c_longlong(q.stride(0)), dtype_code(q), *args,
+                   _ptr(r_s), _ptr(k_s), _ptr(a), _ptr(decay), _ptr(batch.cu_seqlens_q), B, H, D, max(1, batch.max_q_len),
+                   _stream())
+        self._call("nhv_recurrence_chunks", _ptr(r_s), _ptr(k_s), _ptr(a), _ptr(decay), _ptr(v), ctypes.c_longlong(v.stride(0)),
+                   dtype_code(v), _ptr(state), _ptr(out), _ptr(batch.positions), _ptr(batch.cu_seqlens_q), _ptr(state_slots), B,
+                   H, D, E, _stream())
+
+    def readout_norm(self, o, gate, w, y, eps):
+        T, H, E = o.shape
+        self._call("nhv_readout_norm", _ptr(o), _ptr(gate), ctypes.c_longlong(gate.stride(0)), dtype_code(gate), _ptr(w), _ptr(y),
+                   dtype_code(y), T, H, E, ctypes.c_float(eps), _stream())
 
     def _decode_attention(self, q, k_cache, v_cache, out, batch, block_tables, scale, window, more=()):
         """Single tokens in bfloat16: keys split over waves, then merged. ``more``: the arguments of a cap on the
@@ -1479,20 +1548,46 @@ def route_topk(logits: torch.Tensor, top: int, bias: torch.Tensor | None = None,
     return ids, scores
 
 
+def route_groups(logits: torch.Tensor, top: int, correction: torch.Tensor | None = None, groups: int = 1, keep: int = 1):
+    """(numbers [tokens, top] int32, scores [tokens, top] float32): scores s = softmax of all logits of a token; the ``top``
+    experts with the largest s + correction (``correction`` [experts] float32) are chosen, the largest first, the lower number
+    among equals, among the experts of the ``keep`` best of ``groups`` equal runs of neighbours (a group counts by the largest
+    s + correction in it). The scores returned are the chosen experts' s as they are."""
+    _need(logits.dim() == 2, "route_groups: logits must be [tokens, experts]")
+    _dense(logits, "route_groups: logits", dtype=torch.float32)
+    E = logits.shape[1]
+    _need(groups > 0 and E % groups == 0 and 0 < keep <= groups and 0 < top <= keep * (E // groups),
+          lambda: f"route_groups: {top} of {E} experts, {keep} of {groups} groups")
+    if correction is not None:
+        _float32(correction, "route_groups: correction", (E,))
+    ids = torch.empty((logits.shape[0], top), dtype=torch.int32, device=logits.device)
+    scores = torch.empty((logits.shape[0], top), dtype=torch.float32, device=logits.device)
+    if logits.shape[0]:
+        backend().route_groups(logits, correction, ids, scores, int(groups), int(keep))
+    return ids, scores
+
+
 def routed_experts(h: torch.Tensor, ids: torch.Tensor, scores: torch.Tensor, gate_up: torch.Tensor, down: torch.Tensor,
-                   activation: str = "silu", scores_on: str = "input", add: torch.Tensor | None = None) -> torch.Tensor:
+                   activation: str = "silu", scores_on: str = "input", add: torch.Tensor | None = None, gated: bool = True,
+                   identity: bool = False) -> torch.Tensor:
     """sum over a token's experts e (``ids``) of D_e (act(G_e x) * (U_e x)), x = score * h: the score multiplies the
     expert's input (``scores_on`` "input"); or of score * D_e (act(G_e h) * (U_e h)): the score weighs the expert's
     output ("output"). ``add`` [tokens, width]: one more row added to every token's sum before it is rounded (an expert
-    that all tokens use). ``gate_up`` [experts, 2 ff, width] (gate rows, then up rows), ``down`` [experts, width, ff]."""
+    that all tokens use). ``gate_up`` [experts, 2 ff, width] (gate rows, then up rows), ``down`` [experts, width, ff].
+    ``gated`` False: experts are D_e act(U_e x), and ``gate_up`` [experts, ff, width] holds the up matrices alone.
+    ``identity``: a number of at least ``experts`` stands for an expert without matrices whose output is h itself (scores
+    on the output)."""
     _need(scores_on in ("input", "output"), lambda: f"routed_experts: scores on {scores_on!r}")
+    _need(not identity or scores_on == "output", "routed_experts: an identity expert's score weighs its output")
     _need(h.dim() == 2, "routed_experts: h must be [tokens, width]")
     T, W = h.shape
     _dense(h, "routed_experts: h")
     dtype_code(h)
-    _need(activation in ACTIVATIONS, lambda: f"routed_experts: activation {activation!r}")
-    _need(gate_up.dim() == 3 and gate_up.shape[2] == W and gate_up.shape[1] % 2 == 0, "routed_experts: gate_up must be [experts, 2 ff, width]")
-    E, F = gate_up.shape[0], gate_up.shape[1] // 2
+    known = ACTIVATIONS if gated else PLAIN_ACTIVATIONS
+    _need(activation in known, lambda: f"routed_experts: activation {activation!r} ({sorted(known)} are known)")
+    per = 2 if gated else 1
+    _need(gate_up.dim() == 3 and gate_up.shape[2] == W and gate_up.shape[1] % per == 0, "routed_experts: gate_up must be [experts, 2 ff, width]")
+    E, F = gate_up.shape[0], gate_up.shape[1] // per
     _dense(gate_up, "routed_experts: gate_up", dtype=h.dtype)
     _dense(down, "routed_experts: down", (E, W, F), h.dtype)
     _need(ids.dim() == 2 and ids.shape[0] == T, "routed_experts: ids must be [tokens, top]")
@@ -1506,16 +1601,149 @@ def routed_experts(h: torch.Tensor, ids: torch.Tensor, scores: torch.Tensor, gat
     if add is not None:
         _dense(add, "routed_experts: add", (T, W), h.dtype)
         more["add"] = add
+    if identity:
+        more["self_rows"] = h
+    plain = {} if gated else {"gated": False}
     if not T:
         return out
+    act = known[activation]
     if (h.dtype == torch.bfloat16 and T > getattr(b, "few_rows", 0) and W % 8 == 0 and F % 8 == 0 and E <= 4096
             and hasattr(b, "experts_grouped")):
-        b.experts_grouped(h, ids, first, gate_up, down, out, ACTIVATIONS[activation], **more)
+        b.experts_grouped(h, ids, first, gate_up, down, out, act, **more, **plain)
         return out
     u = torch.empty((T * ids.shape[1], F), dtype=h.dtype, device=h.device)
-    b.experts_gate_up(h, ids, first, gate_up, u, ACTIVATIONS[activation])
+    b.experts_gate_up(h, ids, first, gate_up, u, act, **plain)
     b.experts_down(u, ids, down, out, **more)
     return out
+
+
+# ------------------------------------------------------------------ linear recurrences
+@dataclass
+class Retention:
+    """S_t = g_h S_(t-1) + k_t v_t^T, o_t = S_t^T q_t: ``log2_decay`` [heads] float32 holds log2 g_h; q and k are turned first
+    (pairs (i, i + r) by positions * freqs[i], float64, r of them; None: not at all) and k is multiplied by ``k_scale``."""
+
+    log2_decay: torch.Tensor
+    freqs: torch.Tensor | None
+    positions: torch.Tensor
+    k_scale: float = 1.0
+
+
+@dataclass
+class WKV:
+    """o_t = (S_(t-1) + diag(u) k_t v_t^T)^T r_t, S_t = diag(w_t) S_(t-1) + k_t v_t^T, w = exp(-exp(w2 tanh(z) + w0)): ``z``
+    [tokens, rank] float32 (rows may lie further apart), ``w2`` [heads * dim, rank], ``w0`` [heads * dim] and ``u``
+    [heads, dim] float32."""
+
+    z: torch.Tensor
+    w2: torch.Tensor
+    w0: torch.Tensor
+    u: torch.Tensor
+
+
+FEW_TOKENS = 4                # up to so many tokens a request, a recurrence is one kernel from projections to gated read-out
+RECURRENCE_KEY_DIM = 256      # the largest key head that the recurrences take
+
+
+def token_shift(h: torch.Tensor, mu: torch.Tensor, kept: torch.Tensor, batch: AttentionBatch, state_slots: torch.Tensor) -> torch.Tensor:
+    """[n, tokens, width]: h + (h' - h) mu_i for each row mu_i of ``mu`` [n, width] float32, h' the request's row before
+    (zeros at position 0). ``kept`` [slots, width] float32 holds every request's last row and is updated."""
+    _need(h.dim() == 2, "token_shift: h must be [tokens, width]")
+    T, W = h.shape
+    _dense(h, "token_shift: h")
+    dtype_code(h)
+    _need(mu.dim() == 2 and mu.shape[1] == W, lambda: f"token_shift: mu {tuple(mu.shape)} for rows of {W}")
+    _dense(mu, "token_shift: mu", dtype=torch.float32)
+    _need(kept.dim() == 2 and kept.shape[1] == W, lambda: f"token_shift: kept rows {tuple(kept.shape)}")
+    _dense(kept, "token_shift: kept rows", dtype=torch.float32)
+    _recurrence_batch("token_shift", T, batch, state_slots)
+    out = torch.empty((mu.shape[0], T, W), dtype=h.dtype, device=h.device)
+    if T:
+        backend().token_shift(h, mu, kept, out, batch, state_slots)
+    return out
+
+
+def _recurrence_batch(name: str, T: int, batch: AttentionBatch, state_slots: torch.Tensor) -> None:
+    _need(T == batch.num_tokens, lambda: f"{name}: {T} tokens but the batch has {batch.num_tokens}")
+    _dense(batch.token_req, f"{name}: token_req", (T,), torch.int32)
+    _dense(batch.positions, f"{name}: positions", (T,), torch.int32)
+    _dense(batch.cu_seqlens_q, f"{name}: cu_seqlens_q", (batch.num_requests + 1,), torch.int32)
+    _dense(state_slots, f"{name}: state_slots", (batch.num_requests,), torch.int32)
+
+
+def banded_linear(x: torch.Tensor, w: torch.Tensor, band_rows: int) -> list[torch.Tensor]:
+    """One product per set of rows: x [n, rows, in], w [out, in] whose outputs i * band_rows ... belong to set i and all outputs
+    from (n - 1) * band_rows on to the last set. Returns n tensors [rows, its outputs] (rows may lie further apart than
+    that; the first n - 1 are alike in type and spacing), the last one float32. Few rows in bfloat16: one kernel, and
+    all of them float32."""
+    _need(x.dim() == 3 and w.dim() == 2 and x.shape[2] == w.shape[1], lambda: f"banded_linear: x {tuple(x.shape)} and w {tuple(w.shape)}")
+    n, M, _ = x.shape
+    N, last = w.shape[0], (n - 1) * band_rows
+    _need(band_rows > 0 and last < N, lambda: f"banded_linear: {n} bands of {band_rows} of {N} outputs")
+    _dense(x, "banded_linear: x")
+    _dense(w, "banded_linear: w", dtype=x.dtype)
+    dtype_code(x)
+    starts = [i * band_rows for i in range(n)] + [N]
+    fused = getattr(backend(), "banded_linear", None)
+    if fused is not None and M:
+        out = torch.empty((M, N), dtype=torch.float32, device=x.device)
+        if fused(x, w, out, band_rows):
+            return [out[:, a:b] for a, b in zip(starts, starts[1:])]
+    return [linear(x[i], w[starts[i]:starts[i + 1]], out_dtype=torch.float32 if i == n - 1 else None) for i in range(n)]
+
+
+def _spaced_rows(t: torch.Tensor, name: str, shape: tuple, like: torch.Tensor) -> None:
+    want = backend().device_type
+    _need(t.device.type == want, lambda: f"{name}: must live on a '{want}' device, is on {t.device}")
+    _need(tuple(t.shape) == shape and (t.shape[1] == 1 or t.stride(1) == 1), lambda: f"{name}: {tuple(t.shape)}, {shape} is needed with dense rows")
+    _need(t.dtype == like.dtype and t.stride(0) == like.stride(0), lambda: f"{name}: rows of another type or spacing than the queries'")
+
+
+def linear_recurrence(rule, q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, gate: torch.Tensor, state: torch.Tensor, eps: float,
+                      batch: AttentionBatch, state_slots: torch.Tensor, out_dtype, norm_weight: torch.Tensor | None = None) -> torch.Tensor:
+    """A recurrent mixer between its projections, by ``rule`` (a ``Retention`` or a ``WKV``, whose q is r): the recurrence
+    over every request's tokens in order from and into ``state`` [slots, heads, value size, key size] float32 (zero for a
+    request whose first token is at position 0); every head's read-out over its root mean square (``eps``), times
+    ``norm_weight`` [heads * value size] float32 if given, times g sigmoid(g). q, k [tokens, heads * key size], v, gate
+    [tokens, heads * value size]: as projected, of one type and spacing. Returns [tokens, heads * value size]."""
+    _need(state.dim() == 4, "linear_recurrence: state must be [slots, heads, value size, key size]")
+    _dense(state, "linear_recurrence: state", dtype=torch.float32)
+    _, H, E, D = state.shape
+    T = q.shape[0]
+    dtype_code(q)
+    _need(D <= RECURRENCE_KEY_DIM, lambda: f"linear_recurrence: key heads of {D} entries (up to {RECURRENCE_KEY_DIM} are taken)")
+    for name, t, size in (("q", q, D), ("k", k, D), ("v", v, E), ("gate", gate, E)):
+        _spaced_rows(t, f"linear_recurrence: {name}", (T, H * size), q)
+    _recurrence_batch("linear_recurrence", T, batch, state_slots)
+    if isinstance(rule, Retention):
+        _float32(rule.log2_decay, "linear_recurrence: decays", (H,))
+        _dense(rule.positions, "linear_recurrence: positions", (T,), torch.int32)
+        if rule.freqs is not None:
+            _need(2 * rule.freqs.shape[0] <= D, lambda: f"linear_recurrence: {2 * rule.freqs.shape[0]} turned entries of {D}")
+            _dense(rule.freqs, "linear_recurrence: frequencies", dtype=torch.float64)
+    else:
+        rank = rule.w2.shape[1]
+        _dense(rule.w2, "linear_recurrence: w2", (H * D, rank))
+        dtype_code(rule.w2)
+        _need(rule.z.dtype == torch.float32 and tuple(rule.z.shape) == (T, rank) and (rank == 1 or rule.z.stride(1) == 1),
+              lambda: f"linear_recurrence: z {tuple(rule.z.shape)} of {rule.z.dtype} for rank {rank}")
+        _float32(rule.w0, "linear_recurrence: w0", (H * D,))
+        _float32(rule.u, "linear_recurrence: u", (H, D))
+    if norm_weight is not None:
+        _float32(norm_weight, "linear_recurrence: norm weight", (H * E,))
+    y = torch.empty((T, H * E), dtype=out_dtype, device=q.device)
+    dtype_code(y)
+    if T == 0:
+        return y
+    b = backend()
+    if batch.max_q_len <= FEW_TOKENS:
+        b.recurrence_tokens(rule, q, k, v, gate, state, norm_weight, float(eps), y, batch, state_slots)
+        return y
+    o = torch.empty((T, H, E), dtype=torch.float32, device=q.device)
+    b.recurrence_chunks(rule, q, k, v, state, o, batch, state_slots)
+    b.readout_norm(o, gate, norm_weight, y, float(eps))
+    return y
+
 
 # ------------------------------------------------------------------ layers that are not the pre-norm kind
 def _float32(t: torch.Tensor, name: str, shape: tuple) -> None:
@@ -1679,6 +1907,42 @@ def rotary_split_write(qkv: torch.Tensor, bias: torch.Tensor | None, qk_freqs: t
                                      slot_mapping if with_kv else None, q_out, k_cache if with_kv else None,
                                      v_cache if with_kv else None, num_heads, num_kv_heads, head_dim, value_dim, with_kv,
                                      **({"more_columns": int(more_columns)} if more_columns else {}), **more)
+    return q_out
+
+
+def normed_split_write(qkv: torch.Tensor, bias: torch.Tensor | None, q_norm: torch.Tensor, k_norm: torch.Tensor, eps: float,
+                       freqs: torch.Tensor | None, gain: float, positions: torch.Tensor, slot_mapping: torch.Tensor,
+                       k_cache: torch.Tensor, v_cache: torch.Tensor, num_heads: int, num_kv_heads: int, head_dim: int,
+                       value_dim: int, values_from_keys: bool = False, more_columns: int = 0) -> torch.Tensor:
+    """Splits the packed projection q | k | v (followed by ``more_columns`` columns that another reader takes), adds the bias
+    in float, divides all of q by its root mean square over the whole projection (times ``q_norm``, a weight per entry) and
+    all of k by its own (``k_norm``), turns pair (i, i + r) of every query and key head by position * freqs[i] (float64; r of
+    them), cosine and sine times ``gain``, stores keys and values at the step's slots and returns q as [tokens, heads,
+    head_dim]. ``values_from_keys``: there are no value columns; value head g is key head g with its bias, before norm and
+    rotation."""
+    T = qkv.shape[0]
+    nq, nk = num_heads * head_dim, num_kv_heads * head_dim
+    width = nq + nk + (0 if values_from_keys else num_kv_heads * value_dim)
+    _need(not values_from_keys or value_dim == head_dim, "normed_split_write: values that are the keys as projected have the keys' size")
+    _dense(qkv, "normed_split_write: qkv", (T, width + more_columns))
+    dtype_code(qkv)
+    if bias is not None:
+        _dense(bias, "normed_split_write: bias", (width,), qkv.dtype)
+    _float32(q_norm, "normed_split_write: q norm weight", (nq,))
+    _float32(k_norm, "normed_split_write: k norm weight", (nk,))
+    if freqs is not None:
+        _need(2 * freqs.shape[0] <= head_dim, lambda: f"normed_split_write: {2 * freqs.shape[0]} turned entries of {head_dim}")
+        _dense(freqs, "normed_split_write: frequencies", dtype=torch.float64)
+    _dense(positions, "normed_split_write: positions", (T,), torch.int32)
+    _dense(slot_mapping, "normed_split_write: slot_mapping", (T,), torch.int32)
+    for name, cache, size in (("key", k_cache, head_dim), ("value", v_cache, value_dim)):
+        _need(cache.dim() == 4 and tuple(cache.shape[2:]) == (num_kv_heads, size),
+              lambda: f"normed_split_write: {name} cache {tuple(cache.shape)} does not fit {num_kv_heads} heads of {size}")
+        _dense(cache, f"normed_split_write: {name} cache", dtype=qkv.dtype)
+    q_out = torch.empty((T, num_heads, head_dim), dtype=qkv.dtype, device=qkv.device)
+    if T:
+        backend().normed_split_write(qkv, bias, q_norm, k_norm, float(eps), freqs, float(gain), positions, slot_mapping, q_out,
+                                     k_cache, v_cache, num_heads, num_kv_heads, head_dim, value_dim, bool(values_from_keys))
     return q_out
 
 

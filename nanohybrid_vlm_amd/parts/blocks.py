@@ -299,7 +299,11 @@ class SandwichNormsBlock(Part):
     norm_slots = ("mixer_norm", "mixer_out_norm", "feed_forward_norm", "feed_forward_out_norm")
     norms_ahead = True            # the model tells the block which block follows (``next_norm`` is that block's ``norm``)
 
-    def __init__(self, mixer, feed_forward, mixer_norm, mixer_out_norm, feed_forward_norm, feed_forward_out_norm):
+    def __init__(self, mixer, feed_forward, mixer_norm, mixer_out_norm, feed_forward_norm, feed_forward_out_norm,
+                 keeps_unused_norms=()):
+        """``keeps_unused_norms``: the slots whose norms a block without feed-forward holds all the same (a checkpoint that
+        stores them), unused."""
+        self.keeps_unused_norms = tuple(keeps_unused_norms) if feed_forward is None else ()
         self.mixer, self.feed_forward = mixer, feed_forward
         self.mixer_norm, self.mixer_out_norm = mixer_norm, mixer_out_norm
         self.feed_forward_norm, self.feed_forward_out_norm = feed_forward_norm, feed_forward_out_norm
@@ -316,6 +320,7 @@ class SandwichNormsBlock(Part):
         if self.feed_forward is not None:
             out.update({"feed_forward_norm": self.feed_forward_norm, "feed_forward": self.feed_forward,
                         "feed_forward_out_norm": self.feed_forward_out_norm})
+        out.update({slot: getattr(self, slot) for slot in self.keeps_unused_norms})
         return out
 
     def first_read(self) -> tuple:

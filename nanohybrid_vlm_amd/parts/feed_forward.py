@@ -78,56 +78,78 @@ class PlainMLP(Part):
 
 @FEED_FORWARDS.register("routed_experts")
 class RoutedExperts(Part):
-    """``num_experts`` gated feed-forwards of inner size ``expert_size`` without biases, of which every token uses the
+    """``num_experts`` feed-forwards (gated, unless ``gated`` says False) of inner size ``expert_size`` without biases, of which every token uses the
     ``top`` with the largest router logit z_e = router_e . x (+ b_e with ``router_bias``; summed and kept in float32).
     ``scoring`` "sigmoid": the score s_e = sigmoid(z_e), taken as it is (not renormalised); "softmax_of_chosen": the
     scores are the softmax over the chosen logits alone. ``scores_on`` "input": the score multiplies the expert's input,
     y = sum over chosen e of D_e (act(G_e s_e x) * (U_e s_e x)); "output": it weighs the expert's output,
     y = sum over chosen e of s_e D_e (act(G_e x) * (U_e x)). ``shared``: the description of one more feed-forward that
     every token uses and whose result is added (its tensors lie under ``shared.``).
+    ``gated`` False: an expert is D_e act(U_e x). ``scoring`` "softmax": the scores are the softmax over all experts' logits,
+    taken as they are; only with it: ``correction``, a float32 number per expert that is added to the scores for the choice
+    alone; ``groups`` (count, keep), the choice is made among the experts of the ``keep`` best of ``count`` equal runs of
+    neighbours (by their largest score with its correction); ``identity`` n, the router's last n outputs stand for experts
+    without tensors that hand their input on.
     All experts' matrices lie in two tensors, [experts * 2 expert_size, width] (per expert its gate rows, then its
-    up rows) and [experts * width, expert_size]."""
+    up rows; without a gate [experts * expert_size, width]) and [experts * width, expert_size]."""
 
     def __init__(self, hidden_size: int, num_experts: int, top: int, expert_size: int, activation: str = "silu",
                  scoring: str = "sigmoid", scores_on: str = "input", router_bias: bool = False, shared: dict | None = None,
-                 **offered):
-        if not 0 < top <= num_experts or min(hidden_size, expert_size) <= 0:
+                 gated: bool = True, correction: bool = False, groups: tuple | None = None, identity: int = 0, **offered):
+        if not 0 < top <= num_experts + identity or identity < 0 or min(hidden_size, expert_size) <= 0:
             raise ValueError(f"{top} of {num_experts} experts of size {expert_size}")
-        if activation not in ops.ACTIVATIONS:
-            raise ValueError(f"activation {activation!r} is not known ({sorted(ops.ACTIVATIONS)} are)")
-        if scoring not in ops.ROUTER_SCORES:
-            raise ValueError(f"scoring {scoring!r} is not known ({sorted(ops.ROUTER_SCORES)} are)")
+        known = ops.ACTIVATIONS if gated else ops.PLAIN_ACTIVATIONS
+        if activation not in known:
+            raise ValueError(f"activation {activation!r} is not known ({sorted(known)} are)")
+        if scoring not in (*ops.ROUTER_SCORES, "softmax"):
+            raise ValueError(f"scoring {scoring!r} is not known ({sorted((*ops.ROUTER_SCORES, 'softmax'))} are)")
+        if scoring == "softmax":
+            count, keep = groups if groups is not None else (1, 1)
+            if router_bias or scores_on != "output":
+                raise ValueError("scores over all experts weigh the outputs, and their logits have no bias")
+            if not 0 < keep <= count or (num_experts + identity) % count or top > keep * ((num_experts + identity) // count):
+                raise ValueError(f"{top} of {num_experts} experts and {identity} identities, {keep} of {count} groups")
+            self.groups = (count, keep)
+        elif correction or groups is not None or identity:
+            raise ValueError("a correction, groups and identity experts go with scoring 'softmax'")
         if scores_on not in ("input", "output"):
             raise ValueError(f"scores on {scores_on!r}: 'input' and 'output' are known")
         self.hidden_size, self.num_experts, self.top, self.expert_size = hidden_size, num_experts, top, expert_size
         self.activation, self.scoring, self.scores_on, self.has_router_bias = activation, scoring, scores_on, bool(router_bias)
         self.shared = FEED_FORWARDS.build(shared, offered=offered) if shared is not None else None
-        self.router_bias = None
+        self.gated, self.has_correction, self.identity = bool(gated), bool(correction), int(identity)
+        self.router_bias = self.correction = None
 
     def children(self):
         return {"shared": self.shared} if self.shared is not None else {}
 
     def param_specs(self):
         E, F, W = self.num_experts, self.expert_size, self.hidden_size
-        specs = {"router.weight": ParamSpec((E, W)),
-                 "gate_up.weight": ParamSpec((E * 2 * F, W)),
+        specs = {"router.weight": ParamSpec((E + self.identity, W)),
+                 ("gate_up.weight" if self.gated else "up.weight"): ParamSpec((E * (2 if self.gated else 1) * F, W)),
                  "down.weight": ParamSpec((E * W, F))}
         if self.has_router_bias:
             specs["router.bias"] = ParamSpec((E,), init="zeros", always_float32=True)
+        if self.has_correction:
+            specs["router.correction"] = ParamSpec((E + self.identity,), always_float32=True, init_mean=0.0, init_std=0.02)
         return specs
 
     def bind(self, params):
         E, F, W = self.num_experts, self.expert_size, self.hidden_size
         self.router_weight = params["router.weight"]
-        self.router_bias = params.get("router.bias")
-        self.gate_up_weight = params["gate_up.weight"].view(E, 2 * F, W)
+        self.router_bias, self.correction = params.get("router.bias"), params.get("router.correction")
+        self.gate_up_weight = params["gate_up.weight"].view(E, 2 * F, W) if self.gated else params["up.weight"].view(E, F, W)
         self.down_weight = params["down.weight"].view(E, W, F)
 
     def forward(self, x, step):
-        ids, scores = ops.route_topk(ops.linear(x, self.router_weight, out_dtype=torch.float32), self.top,
-                                     bias=self.router_bias, scoring=self.scoring)
+        logits = ops.linear(x, self.router_weight, out_dtype=torch.float32)
+        if self.scoring == "softmax":
+            ids, scores = ops.route_groups(logits, self.top, self.correction, *self.groups)
+        else:
+            ids, scores = ops.route_topk(logits, self.top, bias=self.router_bias, scoring=self.scoring)
         if self.shared is None and self.scores_on == "input":
             return ops.routed_experts(x, ids, scores, self.gate_up_weight, self.down_weight, self.activation)
         add = self.shared.forward(x, step) if self.shared is not None else None
         return ops.routed_experts(x, ids, scores, self.gate_up_weight, self.down_weight, self.activation,
-                                  scores_on=self.scores_on, add=add)
+                                  scores_on=self.scores_on, add=add, **({} if self.gated else {"gated": False}),
+                                  **({"identity": True} if self.identity else {}))

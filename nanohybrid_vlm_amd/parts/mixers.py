@@ -2,7 +2,8 @@
 nanovllm/layers/attention.py:43-75. ``RotaryAttention`` is softmax attention in a more general make (value heads of
 their own size, biases, a window or a chunk, sinks, a bias by distance, turned or mixed values, keys and values lent by
 another layer), ``GatedDeltaRule`` a
-recurrent mixer with a matrix of state per head, ``NormedPair`` two mixers side by side, ``DifferentialAttention`` the
+recurrent mixer with a matrix of state per head, ``Retention`` and ``WKVMixer`` two more without a delta rule,
+``NormedPair`` two mixers side by side, ``DifferentialAttention`` the
 difference of two softmax maps per head over the same values."""
 from __future__ import annotations
 
@@ -108,14 +109,17 @@ class RotaryAttention(Part):
     ``temperature`` (coef, every): queries at position p are multiplied by 1 + coef ln(floor((p + 1) / every) + 1).
     ``mix_values``: "first": the layer's values are kept for later layers of the same step; "later": what is stored (and
     read) is (1 - lam) v + lam v1, v1 the same token's values of the layer that said "first", lam a parameter (the "first"
-    layer holds one as well, unused)."""
+    layer holds one as well, unused). ``projection_norm_eps``: before the rotation all of q and all of k, every head at once,
+    are divided by their root mean squares over the whole projection (this eps under the root) and multiplied by a weight
+    per entry (``q_norm.weight``, ``k_norm.weight``); the encoding is then one with float64 frequencies and a gain
+    (``yarn_frequencies``), pairs are halves."""
 
     def __init__(self, hidden_size: int, num_heads: int, num_kv_heads: int, head_dim: int, value_dim: int, scale: float,
                  bias: bool, position, chunk: int | None = None, window: int | None = None, rotate_values: bool = False,
                  own_kv: bool = True, softcap: float | None = None, sink: float | None = None, head_gate: bool = False,
                  element_gate: bool = False, rotation: str = "halves", unit_norm_eps: float | None = None,
                  values_are_keys: bool = False, learned_sink: bool = False, distance_bias: bool = False,
-                 temperature: tuple | None = None, mix_values: str | None = None):
+                 temperature: tuple | None = None, mix_values: str | None = None, projection_norm_eps: float | None = None):
         if num_heads % num_kv_heads:
             raise ValueError(f"{num_heads} heads are not a multiple of {num_kv_heads} key/value heads")
         if window and chunk:
@@ -128,8 +132,6 @@ class RotaryAttention(Part):
         self.rotate_values, self.own_kv = rotate_values, own_kv
         if softcap is not None and not softcap > 0:
             raise ValueError(f"a cap on the scores must be positive, got {softcap}")
-        if head_gate and bias:
-            raise ValueError("a gate per head and biases are not taken together")
         if element_gate and (head_gate or bias):
             raise ValueError("a gate per entry is not taken together with a gate per head or with biases")
         if rotation not in ("halves", "interleaved"):
@@ -151,6 +153,16 @@ class RotaryAttention(Part):
             raise ValueError("values that are mixed with another layer's are projections of their own, without bias, and not turned")
         self.learned_sink, self.distance_bias, self.mix_values = bool(learned_sink), bool(distance_bias), mix_values
         self.temperature = None if temperature is None else (float(temperature[0]), float(temperature[1]))
+        if projection_norm_eps is not None:
+            if not projection_norm_eps >= 0:
+                raise ValueError(f"the eps of the projections' norm must not be negative, got {projection_norm_eps}")
+            if unit_norm_eps is not None or rotate_values or not own_kv or temperature or mix_values or rotation != "halves":
+                raise ValueError("projections normed as a whole go with keys and values of the layer's own, pairs of halves, and "
+                                 "neither unit norms nor turned, scaled or mixed rows")
+            if position is not None and not hasattr(position, "gain"):
+                raise ValueError("projections normed as a whole are turned by an encoding with float64 frequencies and a gain")
+        self.projection_norm_eps = projection_norm_eps
+        self.q_norm = self.k_norm = None
         self.qkv_weight = self.qkv_bias = self.o_weight = None
         self.sinks = self.slopes = self.vmix = None
 
@@ -171,6 +183,9 @@ class RotaryAttention(Part):
             specs["qkv.bias"] = ParamSpec((self._packed_width(),), init="zeros")
         if self.learned_sink:
             specs["sink"] = ParamSpec((self.num_heads,), always_float32=True, init_mean=0.0, init_std=1.0)
+        if self.projection_norm_eps is not None:
+            specs["q_norm.weight"] = ParamSpec((self.num_heads * self.head_dim,), init="norm", always_float32=True)
+            specs["k_norm.weight"] = ParamSpec((self.num_kv_heads * self.head_dim,), init="norm", always_float32=True)
         if self.mix_values:
             specs["vmix"] = ParamSpec((), always_float32=True, init_mean=0.4, init_std=0.1)
         return specs
@@ -179,6 +194,7 @@ class RotaryAttention(Part):
         self.qkv_weight, self.o_weight = params["qkv.weight"], params["o.weight"]
         self.qkv_bias = params.get("qkv.bias")
         self.sinks, self.vmix = params.get("sink"), params.get("vmix")
+        self.q_norm, self.k_norm = params.get("q_norm.weight"), params.get("k_norm.weight")
         if self.distance_bias:
             self.slopes = distance_slopes(self.num_heads).to(self.qkv_weight.device)
 
@@ -203,6 +219,13 @@ class RotaryAttention(Part):
             raise ValueError("a layer that mixes values runs before the layer whose values it mixes in")
         return {"mix": (step.scratch["first_values"], self.vmix)}
 
+    def _split_write(self, qkv, bias, freqs, v_freqs, writes, gates, step, tables, cache):
+        return ops.rotary_split_write(qkv, bias, freqs, v_freqs, step.token_positions, tables.slot_mapping, cache.k, cache.v,
+                                      self.num_heads, self.num_kv_heads, self.head_dim, self.value_dim, with_kv=writes,
+                                      more_columns=gates, interleaved=self.rotation == "interleaved",
+                                      unit_eps=self.unit_norm_eps, values_from_keys=self.values_are_keys,
+                                      temperature=self.temperature, **self._values_to_mix(qkv, step))
+
     def forward(self, x, step, cache: CacheView, add_to=None):
         tables = step.groups[cache.group]
         writes = self.own_kv and cache.writes
@@ -218,11 +241,15 @@ class RotaryAttention(Part):
             self.qkv_bias[:self.num_heads * self.head_dim].contiguous()
         freqs = self.position.frequencies() if self.position is not None and self.position.rotary_dim else None
         v_freqs = self.position.frequencies_for(self.value_dim) if self.rotate_values else None
-        q = ops.rotary_split_write(qkv, bias, freqs, v_freqs, step.token_positions, tables.slot_mapping, cache.k, cache.v,
-                                   self.num_heads, self.num_kv_heads, self.head_dim, self.value_dim, with_kv=writes,
-                                   more_columns=gates, interleaved=self.rotation == "interleaved",
-                                   unit_eps=self.unit_norm_eps, values_from_keys=self.values_are_keys,
-                                   temperature=self.temperature, **self._values_to_mix(qkv, step))
+        if self.projection_norm_eps is not None:
+            if not writes:
+                raise ValueError("a layer whose projections are normed as a whole keeps its own keys and values")
+            q = ops.normed_split_write(qkv, self.qkv_bias, self.q_norm, self.k_norm, self.projection_norm_eps, freqs,
+                                       self.position.gain() if freqs is not None else 1.0, step.token_positions,
+                                       tables.slot_mapping, cache.k, cache.v, self.num_heads, self.num_kv_heads, self.head_dim,
+                                       self.value_dim, values_from_keys=self.values_are_keys, more_columns=gates)
+        else:
+            q = self._split_write(qkv, bias, freqs, v_freqs, writes, gates, step, tables, cache)
         # (the gates stay where the projection left them: the attention kernels read them from the packed rows)
         o = ops.paged_attention(q, cache.k, cache.v, step.attention, tables.block_tables, self.scale, self.window, self.chunk,
                                 softcap=self.softcap, sink=self.sinks if self.learned_sink else self.sink,
@@ -390,6 +417,93 @@ class GatedDeltaRule(Part):
                                  cache.state["kept"], cache.state["S"], step.attention, step.state_slots, self.num_heads,
                                  self.num_kv_heads, self.head_dim, self.value_dim, x.dtype,
                                  decay_per_head=self.decay_per_head, gate_activation=self.gate_activation)
+        return ops.linear(y, self.o_weight)
+
+
+@MIXERS.register("retention")
+class Retention(Part):
+    """A recurrent mixer with a fixed decay per head: per head a matrix S[head_dim, value_dim] of float32 state per request,
+        S_t = decay_h S_(t-1) + k_t v_t^T,   o_t = S_t^T q_t,
+    q and k turned by the position (``position``: an encoding with float64 frequencies and no gain; None or a rotary size of
+    0: not turned) and k times head_dim^(-1/2). Every head's read-out is divided by its root mean square (``eps``), times
+    silu(G x), and projected. The packed projection's rows are q | k | v | g."""
+
+    def __init__(self, hidden_size: int, num_heads: int, head_dim: int, value_dim: int, decay, eps: float, position=None):
+        decay = [float(g) for g in decay]
+        if len(decay) != num_heads or min(decay) < 0 or max(decay) > 1:
+            raise ValueError(f"{num_heads} decays between 0 and 1 are needed, got {decay}")
+        if head_dim > ops.RECURRENCE_KEY_DIM:
+            raise ValueError(f"key heads of up to {ops.RECURRENCE_KEY_DIM} entries are taken, got {head_dim}")
+        if position is not None and getattr(position, "gain", lambda: None)() != 1.0:
+            raise ValueError("the rotation of this mixer is one with float64 frequencies and without a gain")
+        self.hidden_size, self.num_heads, self.head_dim, self.value_dim = hidden_size, num_heads, head_dim, value_dim
+        self.decay, self.eps, self.position = decay, eps, position
+        self.log2_decay = None
+
+    def param_specs(self):
+        H, D, E, W = self.num_heads, self.head_dim, self.value_dim, self.hidden_size
+        return {"in.weight": ParamSpec((2 * H * (D + E), W)), "o.weight": ParamSpec((W, H * E))}
+
+    def bind(self, params):
+        super().bind(params)
+        # (no decay at all is 2^-1000, which is 0 in float; a logarithm of minus infinity would make 0 * inf of it)
+        logs = torch.log2(torch.tensor(self.decay, dtype=torch.float64).clamp(min=2.0 ** -1000))
+        self.log2_decay = logs.to(torch.float32).to(self.in_weight.device)
+
+    def cache_need(self):
+        return StateNeed({"S": ((self.num_heads, self.value_dim, self.head_dim), torch.float32)})
+
+    def forward(self, x, step, cache: CacheView):
+        H, D, E = self.num_heads, self.head_dim, self.value_dim
+        proj = ops.linear(x, self.in_weight)
+        q, k, v, g = proj.split([H * D, H * D, H * E, H * E], dim=1)
+        freqs = self.position.frequencies() if self.position is not None and self.position.rotary_dim else None
+        rule = ops.Retention(self.log2_decay, freqs, step.token_positions, D ** -0.5)
+        y = ops.linear_recurrence(rule, q, k, v, g, cache.state["S"], self.eps, step.attention, step.state_slots, x.dtype)
+        return ops.linear(y, self.o_weight)
+
+
+@MIXERS.register("wkv")
+class WKVMixer(Part):
+    """A recurrent mixer with a decay per key channel that the token sets, and a bonus for the token itself: each of r, k, v, g
+    and the decays reads its own mix x + (x' - x) mu of the row and the request's row before (``mu``, five rows in that
+    order; zeros before position 0); per head a matrix S[head_dim, head_dim] of float32 state per request,
+        o_t = (S_(t-1) + diag(u) k_t v_t^T)^T r_t,   S_t = diag(w_t) S_(t-1) + k_t v_t^T,
+    w = exp(-exp(W2 tanh(W1 mix) + w0)), W1 of ``decay_rank`` rows. Every head's read-out is divided by its root mean
+    square (``eps``), times a weight per entry, times silu(G mix), and projected. The packed input matrix is
+    r | k | v | g | W1; the last row is kept beside S."""
+
+    MIXES = ("r", "k", "v", "g", "w")
+
+    def __init__(self, hidden_size: int, num_heads: int, head_dim: int, decay_rank: int, eps: float, position=None):
+        if head_dim > ops.RECURRENCE_KEY_DIM:
+            raise ValueError(f"heads of up to {ops.RECURRENCE_KEY_DIM} entries are taken, got {head_dim}")
+        if min(hidden_size, num_heads, head_dim, decay_rank) <= 0:
+            raise ValueError(f"sizes must be positive: width {hidden_size}, {num_heads} heads of {head_dim}, rank {decay_rank}")
+        self.hidden_size, self.num_heads, self.head_dim, self.decay_rank, self.eps = hidden_size, num_heads, head_dim, decay_rank, eps
+
+    def param_specs(self):
+        W, n, R = self.hidden_size, self.num_heads * self.head_dim, self.decay_rank
+        return {
+            "mu": ParamSpec((len(self.MIXES) * W,), always_float32=True, init_mean=0.5, init_std=0.2),
+            "in.weight": ParamSpec((4 * n + R, W)),
+            "w2.weight": ParamSpec((n, R)),
+            "w0": ParamSpec((n,), always_float32=True, init_mean=-3.0, init_std=1.5),
+            "u": ParamSpec((self.num_heads, self.head_dim), always_float32=True, init_mean=0.5, init_std=0.3),
+            "norm.weight": ParamSpec((n,), init="norm", always_float32=True),
+            "o.weight": ParamSpec((W, n)),
+        }
+
+    def cache_need(self):
+        H, D = self.num_heads, self.head_dim
+        return StateNeed({"S": ((H, D, D), torch.float32), "row": ((self.hidden_size,), torch.float32)})
+
+    def forward(self, x, step, cache: CacheView):
+        mixed = ops.token_shift(x, self.mu.view(len(self.MIXES), self.hidden_size), cache.state["row"], step.attention,
+                                step.state_slots)
+        r, k, v, g, z = ops.banded_linear(mixed, self.in_weight, self.num_heads * self.head_dim)
+        y = ops.linear_recurrence(ops.WKV(z, self.w2_weight, self.w0, self.u), r, k, v, g, cache.state["S"], self.eps,
+                                  step.attention, step.state_slots, x.dtype, norm_weight=self.norm_weight)
         return ops.linear(y, self.o_weight)
 
 

@@ -110,15 +110,21 @@ class LayerNorm(Part):
 class StreamRMSNorm(Part):
     """y = x / sqrt(mean(x^2) + eps) * weight of a float32 stream, given as rows of the model's element type;
     statistics and weight are float32. A block that carries several streams reads this norm's weight and eps and
-    takes the norm in its own kernel (``ops.streams_step``); ``forward`` is the same for one stream."""
+    takes the norm in its own kernel (``ops.streams_step``); ``forward`` is the same for one stream. ``zero_centred``: the
+    stored weight is its distance from one (one is added, in float32, when the weights are bound)."""
 
-    def __init__(self, size: int, eps: float):
-        self.size, self.eps = size, eps
+    def __init__(self, size: int, eps: float, zero_centred: bool = False):
+        self.size, self.eps, self.zero_centred = size, eps, bool(zero_centred)
         self.weight = None
         self.row_dtype = None         # set when the model's weights are bound
 
     def param_specs(self):
+        if self.zero_centred:
+            return {"weight": ParamSpec((self.size,), always_float32=True, init_mean=0.0, init_std=0.1)}
         return {"weight": ParamSpec((self.size,), init="norm", always_float32=True)}
+
+    def bind(self, params):
+        self.weight = params["weight"] + 1.0 if self.zero_centred else params["weight"]
 
     def forward(self, x, out_dtype=None) -> torch.Tensor:
         if x.dtype != torch.float32:

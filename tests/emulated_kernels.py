@@ -180,6 +180,8 @@ class EmulatedBackend:
 
     @staticmethod
     def _act(z, act):
+        if act == 2:
+            return torch.relu(z) ** 2
         if act == 1:
             return 0.5 * z * (1.0 + torch.tanh(0.7978845608028654 * (z + 0.044715 * z ** 3)))
         return z * torch.sigmoid(z)
@@ -251,25 +253,117 @@ class EmulatedBackend:
         chosen = torch.gather(logits, 1, order)
         scores.copy_(torch.sigmoid(chosen) if mode == 0 else torch.softmax(chosen, dim=-1))
 
-    def experts_gate_up(self, h, ids, scores, gate_up, u, act):
+    def route_groups(self, logits, correction, ids, scores, groups, keep):
+        s = torch.softmax(logits, dim=-1)
+        c = s + (correction if correction is not None else 0.0)
+        T, E = c.shape
+        best = c.view(T, groups, E // groups).max(-1).values
+        kept = torch.sort(best, dim=-1, descending=True, stable=True).indices[:, :keep]
+        is_open = torch.zeros(T, groups, dtype=torch.bool).scatter_(1, kept, True).repeat_interleave(E // groups, dim=1)
+        order = torch.sort(c.masked_fill(~is_open, -math.inf), dim=-1, descending=True, stable=True).indices[:, :ids.shape[1]]
+        ids.copy_(order.to(torch.int32))
+        scores.copy_(torch.gather(s, 1, order))
+
+    def experts_gate_up(self, h, ids, scores, gate_up, u, act, gated=True):
         T, top = ids.shape
-        F = gate_up.shape[1] // 2
+        F = gate_up.shape[1] // (2 if gated else 1)
         for t in range(T):
             for j in range(top):
                 e, s = int(ids[t, j]), (scores[t, j] if scores is not None else 1.0)
+                if e >= gate_up.shape[0]:
+                    u[t * top + j] = float("nan")          # (an expert without matrices has no inner row)
+                    continue
                 gu = gate_up[e].float() @ h[t].float()
-                u[t * top + j] = (self._act(s * gu[:F], act) * (s * gu[F:])).to(u.dtype)
+                u[t * top + j] = (self._act(s * gu[:F], act) * ((s * gu[F:]) if gated else 1.0)).to(u.dtype)
 
-    def experts_down(self, u, ids, down, out, weights=None, add=None):
+    def experts_down(self, u, ids, down, out, weights=None, add=None, self_rows=None):
         T, top = ids.shape
         for t in range(T):
             total = torch.zeros(out.shape[1])
             for j in range(top):
-                one = down[int(ids[t, j])].float() @ u[t * top + j].float()
+                e = int(ids[t, j])
+                one = self_rows[t].float() if e >= down.shape[0] else down[e].float() @ u[t * top + j].float()
                 total = total + (one if weights is None else weights[t, j] * one)
             if add is not None:
                 total = total + add[t].float()
             out[t] = total.to(out.dtype)
+
+    # -- linear recurrences: request by request and token by token
+    def token_shift(self, h, mu, kept, out, batch, state_slots):
+        for r in range(batch.num_requests):
+            first, end = int(batch.cu_seqlens_q[r]), int(batch.cu_seqlens_q[r + 1])
+            if end <= first:
+                continue
+            slot = int(state_slots[r])
+            before = torch.zeros_like(kept[slot]) if int(batch.positions[first]) == 0 else kept[slot].clone()
+            for t in range(first, end):
+                x = h[t].float()
+                out[:, t] = (x + (before - x) * mu).to(out.dtype)
+                before = x
+            kept[slot] = before
+
+    def _recurrence(self, rule, q, k, v, state, batch, state_slots):
+        from nanohybrid_vlm_amd.native import ops
+        _, H, E, D = state.shape
+        T = q.shape[0]
+        q, k, v = q.float().reshape(T, H, D), k.float().reshape(T, H, D), v.float().reshape(T, H, E)
+        fixed = isinstance(rule, ops.Retention)
+        if fixed:
+            if rule.freqs is not None:
+                n = 2 * rule.freqs.shape[0]
+                q, k = (torch.cat((self._turn_pairs(x[..., :n], rule.positions, rule.freqs, 1.0, True), x[..., n:]), dim=-1) for x in (q, k))
+            k = k * rule.k_scale
+            decay = torch.exp2(rule.log2_decay)[None, :, None].expand(T, H, D)
+        else:
+            decay = torch.exp(-torch.exp(torch.tanh(rule.z) @ rule.w2.float().T + rule.w0)).view(T, H, D)
+        out = torch.zeros(T, H, E)
+        for r in range(batch.num_requests):
+            first, end = int(batch.cu_seqlens_q[r]), int(batch.cu_seqlens_q[r + 1])
+            if end <= first:
+                continue
+            slot = int(state_slots[r])
+            S = torch.zeros(H, E, D) if int(batch.positions[first]) == 0 else state[slot].clone()
+            for t in range(first, end):
+                kv = v[t][:, :, None] * k[t][:, None, :]
+                new = S * decay[t][:, None, :] + kv
+                out[t] = ((new if fixed else S + kv * rule.u[:, None, :]) * q[t][:, None, :]).sum(-1)
+                S = new
+            state[slot] = S
+        return out
+
+    def readout_norm(self, o, gate, w, y, eps):
+        T = o.shape[0]
+        z = gate.float()
+        r = (o * torch.rsqrt(o.pow(2).mean(-1, keepdim=True) + eps)).reshape(T, -1)
+        y.copy_((r * (w if w is not None else 1.0) * z * torch.sigmoid(z)).to(y.dtype))
+
+    def recurrence_tokens(self, rule, q, k, v, gate, state, norm_w, eps, y, batch, state_slots):
+        self.readout_norm(self._recurrence(rule, q, k, v, state, batch, state_slots), gate, norm_w, y, eps)
+
+    def recurrence_chunks(self, rule, q, k, v, state, out, batch, state_slots):
+        out.copy_(self._recurrence(rule, q, k, v, state, batch, state_slots))
+
+    def normed_split_write(self, qkv, bias, wq, wk, eps, freqs, gain, positions, slot_mapping, q_out, k_cache, v_cache, Hq, Hkv,
+                           D, E, values_from_keys):
+        T, dt = qkv.shape[0], qkv.dtype
+        nq, nk = Hq * D, Hkv * D
+        width = nq + nk + (0 if values_from_keys else Hkv * E)
+        x = qkv[:, :width].float() + (bias.float() if bias is not None else 0.0)
+
+        def prepared(t, w, heads):
+            t = (t / torch.sqrt(t.pow(2).mean(-1, keepdim=True) + eps) * w).reshape(T, heads, D)
+            if freqs is None:
+                return t
+            n = 2 * freqs.shape[0]
+            return torch.cat((self._turn_pairs(t[..., :n], positions, freqs, gain, True), t[..., n:]), dim=-1)
+
+        q_out.copy_(prepared(x[:, :nq], wq, Hq).to(dt))
+        k = prepared(x[:, nq:nq + nk], wk, Hkv)
+        v = (x[:, nq:nq + nk] if values_from_keys else x[:, nq + nk:]).reshape(T, Hkv, E)
+        ok = slot_mapping >= 0
+        slots = slot_mapping[ok].long()
+        k_cache.view(-1, Hkv, D)[slots] = k[ok].to(dt)
+        v_cache.view(-1, Hkv, E)[slots] = v[ok].to(dt)
 
     @staticmethod
     def _turned(t, positions, freqs, sign=1.0):
