@@ -19,10 +19,11 @@ For these two ``value`` is generated tokens a second over the whole run, prompts
 ``--workload projections`` is a diagnosis, not the benchmark: a layer's matrix products alone, cold, beside a kernel
 that only reads the same bytes (see ``bench_projections``).
 
-``--workload design --shape D-1b|D-8b [--layers L]``, D one of pevazen, fazovik, vugelix, pukarax and gabelorn: a model of
+``--workload design --shape D-1b|D-8b [--layers L]``, D one of pevazen, fazovik, vugelix, pukarax, gabelorn and zigelorn: a model of
 that design (see ``architectures/``) beside a Qwen3 model (for Vugelix:
 a Pevazen model of pairs of mixers; for Pukarax: a Fazovik model, whose feed-forwards are dense and routed in turn as
-well; for Gabelorn: a Fazovik model with dense feed-forwards and a Qwen3 model) of the same width, heads, feed-forward size, experts, vocabulary and number of layers: one prompt of ``--prompt-tokens`` in one step, decoding at
+well; for Gabelorn: a Fazovik model with dense feed-forwards and a Qwen3 model; for Zigelorn: a Pukarax model and a Pevazen
+model of pairs of mixers) of the same width, heads, feed-forward size, experts, vocabulary and number of layers: one prompt of ``--prompt-tokens`` in one step, decoding at
 ``--batch`` requests, and the time of every own kernel in one eager step of each kind (see ``bench_design``).
 """
 import argparse
@@ -423,7 +424,7 @@ def bench_design(args):
     from nanohybrid_vlm_amd.engine.runner import StepEntry
     from nanohybrid_vlm_amd.native import ops
 
-    name = args.shape if args.shape.startswith(("pevazen", "fazovik", "vugelix", "pukarax", "gabelorn")) else "pevazen-1b"
+    name = args.shape if args.shape.startswith(("pevazen", "fazovik", "vugelix", "pukarax", "gabelorn", "zigelorn")) else "pevazen-1b"
     design = name.split("-")[0]
     new = json.loads(json.dumps(named_shapes()[name]))
     layers = args.layers or min(8, len(new["layers"]))
@@ -441,6 +442,26 @@ def bench_design(args):
         twin = {"architecture": "Fazovik", "layers": [{"type": "latent_attention", "mixer": mixer, "mlp": {"kind": "dense", "ff": ff}}] * layers,
                 "norm": {"eps": 1e-6}, "vocab": new["vocab"], "width": new["width"]}
         further = [("qwen3", qwen3_shape(layers, new["width"], b["heads"], b["kv_heads"], b["dim"], ff, vocab=new["vocab"]))]
+    elif design == "zigelorn":
+        # Pukarax is as this design is in its layers' norms, in attention whose values are its keys and in routed experts (gated
+        # ones, whose scores are a softmax over the chosen); Pevazen's pairs hold a recurrence with a state of the same size
+        beside = "pukarax"
+        mixers = {layer["type"]: layer["mixer"] for layer in new["layers"]}
+        a, r = mixers.get("attention") or named_shapes()[name]["layers"][2]["mixer"], mixers["wkv"]
+        mixer = {"dim": a["dim"], "heads": a["heads"], "kv_heads": a["kv_heads"], "mask": a["mask"], "scale": a["scale"], "vdim": a["dim"],
+                 "rot": {"base": a["rot"]["base"], "dims": a["rot"]["dims"]}}
+        entries, pairs = [], []
+        for layer in new["layers"]:
+            mlp = layer["mlp"]
+            if mlp["kind"] == "moe":
+                mlp = {"kind": "moe", "expert": mlp["expert"], "router": {key: mlp["router"][key] for key in ("experts", "top")}}
+            entries.append({"type": "attention_2", "mixer": mixer, "mlp": mlp})
+            right = {"conv": 4, "dim": r["dim"], "heads": r["heads"], "kv_heads": r["heads"], "vdim": r["dim"],
+                     "decay_rank": r["decay_rank"], "gate_rank": r["decay_rank"]}
+            pairs.append({"type": "parallel", "mixer": {"left": mixer, "right": right},
+                          "mlp": {"kind": "dense", "ff": new["layers"][0]["mlp"]["ff"]}})
+        twin = {"architecture": "Pukarax", "layers": entries, "norm": {"eps": 1e-6}, "vocab": new["vocab"], "width": new["width"]}
+        further = [("pevazen", dict(twin, architecture="Pevazen", layers=pairs))]
     elif design == "vugelix":
         # the closest model the engine has is Pevazen's pair of mixers (attention beside a gated delta rule): the twin is
         # made of such layers alone, with this design's heads and head sizes on both sides, a chunk as long as the

@@ -752,7 +752,8 @@ int nhv_gemm_fewrows_launch(bool glu, const void* x, const void* w, const void* 
   if (f.band_rows) {
     // (a block's tiles lie in one band)
     if (glu || fused || f.band_rows % 16 != 0) return nhv_fail("few-rows gemm: bands of %d rows (multiples of 16, no gate, no fusion)", f.band_rows);
-    if (f.band_rows % 32 == 0 && (N + 15) / 16 > 512) launch<2, 8, 2, false>(s, x, w, bias, y, M, N, K, out_dtype, false, f);
+    const Plan p = plan(false, M, N, K);
+    if (f.band_rows % 32 == 0 && p.nt == 2) launch<2, 8, 2, false>(s, x, w, bias, y, M, N, K, out_dtype, false, f);
     else launch<1, 8, 8, false>(s, x, w, bias, y, M, N, K, out_dtype, false, f);
     return 0;
   }

@@ -27,7 +27,6 @@ typedef __attribute__((__vector_size__(4 * sizeof(float)))) float floatx4;
 
 #define NHV_LOG2E 1.4426950408889634f
 #define NHV_CHUNK 16
-#define NHV_RANK_PIECE 64
 
 __device__ __forceinline__ float exp2_of(float x) { return __builtin_amdgcn_exp2f(x); }   // (x <= 0; tiny results may become 0)
 __device__ __forceinline__ float silu_of(float z) { return z / (1.0f + expf(-z)); }
@@ -116,103 +115,136 @@ struct RecurrenceIn {
 };
 
 
+// four consecutive entries (``whole``: they start at a multiple of four, else one by one, those from n on being zeros)
+template <typename T>
+__device__ __forceinline__ floatx4 four_of(const T* p, int n, bool whole) {
+  struct alignas(sizeof(T) * 4) Pack { T e[4]; };
+  floatx4 v;
+  if (whole) {
+    const Pack x = *reinterpret_cast<const Pack*>(p);
+#pragma unroll
+    for (int i = 0; i < 4; ++i) v[i] = to_f32(x.e[i]);
+  } else {
+#pragma unroll
+    for (int i = 0; i < 4; ++i) v[i] = i < n ? to_f32(p[i]) : 0.f;
+  }
+  return v;
+}
+
 // ---------------------------------------------------------------- portions of prompts: all chunks at once
 // One block of 256 threads per (chunk, head, request). A chunk's place in the outputs: cu[req] / 16 + req + its number in
-// the request (places never overlap: a request of n tokens has at most floor(n / 16) + 1 chunks).
+// the request (places never overlap: a request of n tokens has at most floor(n / 16) + 1 chunks). ``whole``: rows, heads and
+// ranks are whole groups of four entries.
 template <typename T, typename TW, int KIND>
 __global__ __launch_bounds__(256) void recurrence_prepare_kernel(const RecurrenceIn in, float* __restrict__ r_out,
                                                                  float* __restrict__ k_out, float* __restrict__ a_out,
                                                                  float* __restrict__ decay_out, const int* __restrict__ cu,
-                                                                 int H, int D, int Dp) {
+                                                                 int H, int D, int Dp, int whole, int whole_rank) {
   extern __shared__ __attribute__((aligned(16))) float lds[];
-  const int req = blockIdx.z, h = blockIdx.y;
-  const int first = cu[req], t0 = first + blockIdx.x * NHV_CHUNK, end = cu[req + 1];
+  const int req = blockIdx.z, h = blockIdx.x;
+  const int first = cu[req], t0 = first + blockIdx.y * NHV_CHUNK, end = cu[req + 1];
   if (t0 >= end) return;                     // (the same for the whole block)
   const int n = min(NHV_CHUNK, end - t0);
-  const size_t place = ((size_t)(first / NHV_CHUNK) + req + blockIdx.x) * H + h;
-  const int tid = threadIdx.x, LD = D | 1;   // (rows of an odd number of floats: sixteen rows lie in sixteen banks)
+  const size_t place = ((size_t)(first / NHV_CHUNK) + req + blockIdx.y) * H + h;
+  const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63, col = lane & 15, grp = lane >> 4;
+  const int LD = Dp + 4;                     // (an odd number of groups of four: sixteen rows' groups lie in sixty-four banks)
   float* rs = lds;
   float* ks = rs + NHV_CHUNK * LD;
   float* ls = ks + NHV_CHUNK * LD;           // kind 1: running sums of the decays' logarithms, the token's own included
   const T* q = (const T*)in.q + (size_t)h * D;
   const T* k = (const T*)in.k + (size_t)h * D;
-  if (KIND == 0) {
-    const int half = in.rot / 2, per = D - half;
-    for (int x = tid; x < NHV_CHUNK * per; x += 256) {
-      const int t = x / per, i = x % per;
-      const size_t at = (size_t)(t0 + t) * in.ld;
-      if (i < half) {
-        float q1 = 0.f, q2 = 0.f, k1 = 0.f, k2 = 0.f, sn = 0.f, cs = 0.f;
-        if (t < n) {
-          nhv_turn_angle<float>(in.turn_positions[t0 + t], in.freqs[i], 1.0f, &sn, &cs);
-          q1 = to_f32(q[at + i]); q2 = to_f32(q[at + i + half]);
-          k1 = to_f32(k[at + i]); k2 = to_f32(k[at + i + half]);
-        }
-        rs[t * LD + i] = q1 * cs - q2 * sn;
-        rs[t * LD + i + half] = q2 * cs + q1 * sn;
-        ks[t * LD + i] = (k1 * cs - k2 * sn) * in.k_scale;
-        ks[t * LD + i + half] = (k2 * cs + k1 * sn) * in.k_scale;
-      } else {
-        rs[t * LD + i + half] = t < n ? to_f32(q[at + i + half]) : 0.f;
-        ks[t * LD + i + half] = t < n ? to_f32(k[at + i + half]) * in.k_scale : 0.f;
+  const floatx4 zero = {0.f, 0.f, 0.f, 0.f};
+  const int fours = Dp / 4;
+  if (KIND == 1) {
+    // the decays' linear part tanh(z) w2^T on the matrix cores: a wave takes every fourth tile of 16 channels
+    constexpr int MAX_TILES = 4;
+    floatx4 acc[MAX_TILES];
+#pragma unroll
+    for (int i = 0; i < MAX_TILES; ++i) acc[i] = zero;
+    const float* z = in.z + (size_t)(t0 + min(col, n - 1)) * in.z_ld;
+    for (int r0 = 0; r0 < in.rank; r0 += 16) {
+      const int r = r0 + grp * 4;
+      floatx4 x, w[MAX_TILES];
+#pragma unroll
+      for (int j = 0; j < 4; ++j) x[j] = r + j < in.rank ? z[r + j] : 0.f;
+#pragma unroll
+      for (int i = 0; i < MAX_TILES; ++i) {
+        const int d = (wave + 4 * i) * 16 + col;
+        w[i] = (d < D && r < in.rank) ? four_of((const TW*)in.w2 + ((size_t)h * D + d) * in.rank + r, in.rank - r, whole_rank) : zero;
+      }
+#pragma unroll
+      for (int j = 0; j < 4; ++j) x[j] = tanhf(x[j]);
+#pragma unroll
+      for (int i = 0; i < MAX_TILES; ++i)
+        if ((wave + 4 * i) * 16 < Dp)
+#pragma unroll
+          for (int j = 0; j < 4; ++j) acc[i] = __builtin_amdgcn_mfma_f32_16x16x4f32(x[j], w[i][j], acc[i], 0, 0, 0);
+    }
+    // a lane holds channel d at the tokens 4 grp .. 4 grp + 3: sums along them, then over the groups before
+#pragma unroll
+    for (int i = 0; i < MAX_TILES; ++i) {
+      const int d = (wave + 4 * i) * 16 + col;
+      if (d - col >= Dp) continue;           // (the same for the whole wave)
+      const float w0 = d < D ? in.w0[h * D + d] : 0.f;
+      float run[4], sum = 0.f;
+#pragma unroll
+      for (int j = 0; j < 4; ++j) {
+        const bool real = d < D && grp * 4 + j < n;
+        sum += real ? -NHV_LOG2E * expf(acc[i][j] + w0) : 0.f;
+        run[j] = sum;
+      }
+      const float s0 = __shfl(sum, col, NHV_WAVE), s1 = __shfl(sum, col + 16, NHV_WAVE), s2 = __shfl(sum, col + 32, NHV_WAVE);
+      const float before = grp == 0 ? 0.f : grp == 1 ? s0 : grp == 2 ? s0 + s1 : s0 + s1 + s2;
+#pragma unroll
+      for (int j = 0; j < 4; ++j) ls[(grp * 4 + j) * LD + d] = before + run[j];
+    }
+  }
+  const int half = KIND == 0 ? in.rot / 2 : 0;
+  if (KIND == 0 && half > 0) {
+    const bool fast = whole && half % 4 == 0;
+    for (int x = tid; x < NHV_CHUNK * (fast ? half / 4 : half); x += 256) {
+      const int per = fast ? half / 4 : half;
+      const int t = x / per, i = (x % per) * (fast ? 4 : 1);
+      const size_t at = (size_t)(t0 + t) * in.ld + i;
+      floatx4 q1 = zero, q2 = zero, k1 = zero, k2 = zero;
+      if (t < n) {
+        const int count = fast ? 4 : 1;
+        q1 = four_of(q + at, count, fast); q2 = four_of(q + at + half, count, fast);
+        k1 = four_of(k + at, count, fast); k2 = four_of(k + at + half, count, fast);
+      }
+#pragma unroll
+      for (int j = 0; j < 4; ++j) {
+        if (j > 0 && !fast) break;
+        float sn = 0.f, cs = 1.f;
+        if (t < n) nhv_turn_angle<float>(in.turn_positions[t0 + t], in.freqs[i + j], 1.0f, &sn, &cs);
+        rs[t * LD + i + j] = q1[j] * cs - q2[j] * sn;
+        rs[t * LD + i + j + half] = q2[j] * cs + q1[j] * sn;
+        ks[t * LD + i + j] = (k1[j] * cs - k2[j] * sn) * in.k_scale;
+        ks[t * LD + i + j + half] = (k2[j] * cs + k1[j] * sn) * in.k_scale;
       }
     }
-  } else {
-    for (int x = tid; x < NHV_CHUNK * D; x += 256) {
-      const int t = x / D, d = x % D;
+  }
+  {                                          // what is not turned, and the places beyond D
+    const float k_scale = KIND == 0 ? in.k_scale : 1.0f;
+    const int start = 2 * half, f0 = start / 4;
+    const bool fast = whole && start % 4 == 0;
+    for (int x = tid; x < NHV_CHUNK * (fours - f0); x += 256) {
+      const int t = x / (fours - f0), d = (x % (fours - f0) + f0) * 4;
       const size_t at = (size_t)(t0 + t) * in.ld + d;
-      rs[t * LD + d] = t < n ? to_f32(q[at]) : 0.f;
-      ks[t * LD + d] = t < n ? to_f32(k[at]) : 0.f;
-    }
-    // the decays' linear part: a thread takes channel d of some of the tokens
-    constexpr int TLD = NHV_RANK_PIECE + 4;
-    float* th = lds + ((3 * NHV_CHUNK * LD + 3) & ~3);
-    int groups = 256 / D;
-    if (groups < 1) groups = 1;
-    if (groups > NHV_CHUNK) groups = NHV_CHUNK;
-    const int per = (NHV_CHUNK + groups - 1) / groups;
-    const int d = tid % D, tok0 = (tid / D) * per;
-    const bool works = tid < D * groups && tok0 < NHV_CHUNK;
-    const TW* w2 = (const TW*)in.w2 + ((size_t)h * D + d) * in.rank;
-    float acc[NHV_CHUNK];
+      if (fast) {
+        const bool real = t < n && d < D;
+        *reinterpret_cast<floatx4*>(&rs[t * LD + d]) = real ? four_of(q + at, 4, true) : zero;
+        floatx4 kv = real ? four_of(k + at, 4, true) : zero;
+        kv *= k_scale;
+        *reinterpret_cast<floatx4*>(&ks[t * LD + d]) = kv;
+      } else {
 #pragma unroll
-    for (int i = 0; i < NHV_CHUNK; ++i) acc[i] = 0.f;
-    for (int r0 = 0; r0 < in.rank; r0 += NHV_RANK_PIECE) {
-      const int piece = min(NHV_RANK_PIECE, in.rank - r0);
-      for (int x = tid; x < NHV_CHUNK * NHV_RANK_PIECE; x += 256) {
-        const int t = x / NHV_RANK_PIECE, r = x % NHV_RANK_PIECE;
-        th[t * TLD + r] = (t < n && r < piece) ? tanhf(in.z[(size_t)(t0 + t) * in.z_ld + r0 + r]) : 0.f;
-      }
-      __syncthreads();
-      if (works) {
-        for (int r = 0; r < piece; r += 4) {
-          float w[4];
-#pragma unroll
-          for (int i = 0; i < 4; ++i) w[i] = r + i < piece ? to_f32(w2[r0 + r + i]) : 0.f;
-#pragma unroll
-          for (int i = 0; i < NHV_CHUNK; ++i) {
-            if (i < per && tok0 + i < NHV_CHUNK) {
-              const float4 x = *reinterpret_cast<const float4*>(&th[(tok0 + i) * TLD + r]);
-              acc[i] = fmaf(w[0], x.x, fmaf(w[1], x.y, fmaf(w[2], x.z, fmaf(w[3], x.w, acc[i]))));
-            }
-          }
+        for (int j = 0; j < 4; ++j) {
+          if (d + j < start) continue;
+          const bool real = t < n && d + j < D;
+          rs[t * LD + d + j] = real ? to_f32(q[at + j]) : 0.f;
+          ks[t * LD + d + j] = real ? to_f32(k[at + j]) * k_scale : 0.f;
         }
-      }
-      __syncthreads();
-    }
-    if (works) {
-      const float w0 = in.w0[h * D + d];
-#pragma unroll
-      for (int i = 0; i < NHV_CHUNK; ++i)
-        if (i < per && tok0 + i < NHV_CHUNK) ls[(tok0 + i) * LD + d] = tok0 + i < n ? -NHV_LOG2E * expf(acc[i] + w0) : 0.f;
-    }
-    __syncthreads();
-    if (tid < D) {
-      float sum = 0.f;
-#pragma unroll
-      for (int t = 0; t < NHV_CHUNK; ++t) {
-        sum += ls[t * LD + tid];
-        ls[t * LD + tid] = sum;
       }
     }
   }
@@ -222,29 +254,49 @@ __global__ __launch_bounds__(256) void recurrence_prepare_kernel(const Recurrenc
     const int t = tid >> 4, j = tid & 15;
     float sum = 0.f;
     if (t < n && j <= t) {
+      const float* rt = rs + t * LD;
+      const float* kj = ks + j * LD;
+      floatx4 part = zero;
       if (KIND == 0) {
-        for (int d = 0; d < D; ++d) sum = fmaf(rs[t * LD + d], ks[j * LD + d], sum);
-        sum *= exp2_of(l2 * (float)(t - j));
+        for (int d = 0; d < Dp; d += 4) part += *reinterpret_cast<const floatx4*>(rt + d) * *reinterpret_cast<const floatx4*>(kj + d);
+        sum = (part[0] + part[1] + part[2] + part[3]) * exp2_of(l2 * (float)(t - j));
       } else if (j == t) {
-        for (int d = 0; d < D; ++d) sum = fmaf(rs[t * LD + d] * in.u[h * D + d], ks[t * LD + d], sum);
+        for (int d = 0; d < D; ++d) sum = fmaf(rt[d] * in.u[h * D + d], kj[d], sum);
       } else {
-        for (int d = 0; d < D; ++d)
-          sum = fmaf(rs[t * LD + d] * exp2_of(ls[(t - 1) * LD + d] - ls[j * LD + d]), ks[j * LD + d], sum);
+        const float* lt = ls + (t - 1) * LD;
+        const float* lj = ls + j * LD;
+#pragma unroll 2
+        for (int d = 0; d < Dp; d += 4) {
+          const floatx4 x = *reinterpret_cast<const floatx4*>(lt + d) - *reinterpret_cast<const floatx4*>(lj + d);
+          floatx4 e;
+#pragma unroll
+          for (int i = 0; i < 4; ++i) e[i] = exp2_of(x[i]);
+          part += *reinterpret_cast<const floatx4*>(rt + d) * *reinterpret_cast<const floatx4*>(kj + d) * e;
+        }
+        sum = part[0] + part[1] + part[2] + part[3];
       }
     }
     a_out[place * 256 + tid] = sum;
   }
-  for (int x = tid; x < NHV_CHUNK * Dp; x += 256) {
-    const int t = x / Dp, d = x % Dp;
-    float r = 0.f, kk = 0.f;
-    if (t < n && d < D) {
-      const float from_start = KIND == 0 ? l2 * (float)(t + 1) : (t > 0 ? ls[(t - 1) * LD + d] : 0.f);
-      const float to_end = KIND == 0 ? l2 * (float)(n - 1 - t) : ls[(n - 1) * LD + d] - ls[t * LD + d];
-      r = rs[t * LD + d] * exp2_of(from_start);
-      kk = ks[t * LD + d] * exp2_of(to_end);
+  for (int x = tid; x < NHV_CHUNK * fours; x += 256) {
+    const int t = x / fours, d = (x % fours) * 4;
+    floatx4 r = *reinterpret_cast<const floatx4*>(&rs[t * LD + d]);
+    if (KIND == 0) {
+      r *= exp2_of(l2 * (float)(t + 1));
+    } else if (t > 0) {
+      const floatx4 before = *reinterpret_cast<const floatx4*>(&ls[(t - 1) * LD + d]);
+#pragma unroll
+      for (int j = 0; j < 4; ++j) r[j] *= exp2_of(before[j]);
     }
-    r_out[place * NHV_CHUNK * Dp + x] = r;
-    k_out[place * NHV_CHUNK * Dp + x] = kk;
+    *reinterpret_cast<floatx4*>(r_out + place * NHV_CHUNK * Dp + x * 4) = r;
+  }
+  for (int x = tid; x < Dp * 4; x += 256) {  // keys lie with a channel's sixteen tokens together
+    const int t = (x & 3) * 4, d = x >> 2;
+    floatx4 kk;
+#pragma unroll
+    for (int j = 0; j < 4; ++j)              // (rows beyond n are zeros)
+      kk[j] = ks[(t + j) * LD + d] * exp2_of(KIND == 0 ? l2 * (float)max(n - 1 - t - j, 0) : ls[(n - 1) * LD + d] - ls[(t + j) * LD + d]);
+    *reinterpret_cast<floatx4*>(k_out + place * NHV_CHUNK * Dp + x * 4) = kk;
   }
   for (int d = tid; d < Dp; d += 256)
     decay_out[place * Dp + d] = d < D ? exp2_of(KIND == 0 ? l2 * (float)n : ls[(n - 1) * LD + d]) : 0.f;
@@ -254,16 +306,27 @@ __global__ __launch_bounds__(256) void recurrence_prepare_kernel(const Recurrenc
 // A block owns 16 columns of S (value channels) of one head of one request; its four waves share D in tiles of 16 rows,
 // TPW tiles a wave, which stay in registers as the result of the matrix cores' products: lane l holds S[16 tile + 4 (l / 16) + i,
 // column l % 16]. With the rows of D taken in that same order the tile is also the right-hand operand of R S as it stands.
-// The waves' shares of O meet in LDS (two buffers, one barrier a chunk) and are added in the order of the waves.
+// The waves' shares of O meet in LDS (two buffers, one barrier a chunk) and are added in the order of the waves. What a
+// chunk needs is asked for AHEAD chunks before it is used. EVEN: every wave has TPW tiles. Blocks of one head are a multiple of the number of heads
+// apart, so that with a multiple of eight heads they share an XCD's L2.
 template <typename T, int TPW>
-__global__ __launch_bounds__(256) void recurrence_chunks_kernel(const float* __restrict__ r_in, const float* __restrict__ k_in,
+struct ChunkOperands {
+  floatx4 r[TPW], g[TPW], kk[TPW];
+  T v[4], v_mine;
+  float a;
+};
+
+// (two waves a SIMD at least: with at most 256 registers a wave the products' sums stay in ordinary registers)
+template <typename T, int TPW, bool EVEN>
+__global__ __launch_bounds__(256, 2) void recurrence_chunks_kernel(const float* __restrict__ r_in, const float* __restrict__ k_in,
                                                                 const float* __restrict__ a_in, const float* __restrict__ decay_in,
                                                                 const T* __restrict__ v, long long ld, float* __restrict__ state,
                                                                 float* __restrict__ out, const int* __restrict__ positions,
                                                                 const int* __restrict__ cu, const int* __restrict__ state_slots,
                                                                 int H, int D, int Dp, int E) {
+  constexpr int AHEAD = TPW <= 2 ? 3 : 2;
   __shared__ float red[2][4][NHV_CHUNK][17];
-  const int req = blockIdx.z, h = blockIdx.y, e0 = blockIdx.x * 16;
+  const int req = blockIdx.z, h = blockIdx.x, e0 = blockIdx.y * 16;
   const int first = cu[req], end = cu[req + 1];
   if (end <= first) return;                  // (the same for the whole block)
   const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63, col = lane & 15, grp = lane >> 4;
@@ -281,67 +344,69 @@ __global__ __launch_bounds__(256) void recurrence_chunks_kernel(const float* __r
     }
   const int chunks = (end - first + NHV_CHUNK - 1) / NHV_CHUNK;
   const size_t place0 = (size_t)(first / NHV_CHUNK) + req;
-  floatx4 r[TPW], g[TPW];
-  float kk[TPW][4], vv[4];
-  float a = 0.f;
-  const T* vcol = v + (size_t)h * E + e0 + (column ? col : 0);
-  auto ask = [&](int c) {
+  ChunkOperands<T, TPW> ops[AHEAD];
+  const T* vcol = v + (size_t)h * E + e0 + (column ? col : 0);      // (a lane beyond E works on a column that it does not write)
+  auto ask = [&](ChunkOperands<T, TPW>& x, int c) {
+    c = min(c, chunks - 1);                  // (always asked, so that the loop's waits count the same loads on every way)
     const size_t place = (place0 + c) * H + h;
     const int t0 = first + c * NHV_CHUNK;
 #pragma unroll
     for (int i = 0; i < TPW; ++i) {
-      if (tile0 + i < tiles) {
-        const int d = (tile0 + i) * 16;
-        r[i] = *reinterpret_cast<const floatx4*>(r_in + (place * NHV_CHUNK + col) * Dp + d + grp * 4);
-        g[i] = *reinterpret_cast<const floatx4*>(decay_in + place * Dp + d + grp * 4);
-#pragma unroll
-        for (int j = 0; j < 4; ++j) kk[i][j] = k_in[(place * NHV_CHUNK + grp * 4 + j) * Dp + d + col];
-      } else {
-        r[i] = g[i] = floatx4{0.f, 0.f, 0.f, 0.f};
-#pragma unroll
-        for (int j = 0; j < 4; ++j) kk[i][j] = 0.f;
-      }
+      const int d = (EVEN ? tile0 + i : min(tile0 + i, tiles - 1)) * 16;      // (a wave without a tile leaves it unused)
+      x.r[i] = *reinterpret_cast<const floatx4*>(r_in + (place * NHV_CHUNK + col) * Dp + d + grp * 4);
+      x.g[i] = *reinterpret_cast<const floatx4*>(decay_in + place * Dp + d + grp * 4);
+      x.kk[i] = *reinterpret_cast<const floatx4*>(k_in + (place * Dp + d + col) * NHV_CHUNK + grp * 4);
     }
+    // (rows beyond the request meet zeros in A and K: the request's last row stands in for them)
 #pragma unroll
-    for (int j = 0; j < 4; ++j) {
-      const int t = t0 + grp * 4 + j;
-      vv[j] = (column && t < end) ? to_f32(vcol[(size_t)t * ld]) : 0.f;
-    }
-    a = a_in[place * 256 + col * 16 + grp * 4 + wave];
+    for (int j = 0; j < 4; ++j) x.v[j] = vcol[(size_t)min(t0 + grp * 4 + j, end - 1) * ld];
+    x.v_mine = vcol[(size_t)min(t0 + grp * 4 + wave, end - 1) * ld];
+    x.a = a_in[place * 256 + col * 16 + grp * 4 + wave];
   };
-  ask(0);
-  for (int c = 0; c < chunks; ++c) {
+  auto step = [&](ChunkOperands<T, TPW>& x, int c) {
+    float vv[4];
+#pragma unroll
+    for (int j = 0; j < 4; ++j) vv[j] = to_f32(x.v[j]);
     floatx4 o = {0.f, 0.f, 0.f, 0.f}, o2 = {0.f, 0.f, 0.f, 0.f};
     // this wave's share of A V: the tokens 4 grp + wave
-    o2 = __builtin_amdgcn_mfma_f32_16x16x4f32(a, wave == 0 ? vv[0] : wave == 1 ? vv[1] : wave == 2 ? vv[2] : vv[3], o2, 0, 0, 0);
+    o2 = __builtin_amdgcn_mfma_f32_16x16x4f32(x.a, to_f32(x.v_mine), o2, 0, 0, 0);
 #pragma unroll
     for (int i = 0; i < TPW; ++i) {
-      o = __builtin_amdgcn_mfma_f32_16x16x4f32(r[i][0], S[i][0], o, 0, 0, 0);
-      o2 = __builtin_amdgcn_mfma_f32_16x16x4f32(r[i][1], S[i][1], o2, 0, 0, 0);
-      o = __builtin_amdgcn_mfma_f32_16x16x4f32(r[i][2], S[i][2], o, 0, 0, 0);
-      o2 = __builtin_amdgcn_mfma_f32_16x16x4f32(r[i][3], S[i][3], o2, 0, 0, 0);
+      if (!EVEN && tile0 + i >= tiles) continue;      // (the same for the whole wave)
+      o = __builtin_amdgcn_mfma_f32_16x16x4f32(x.r[i][0], S[i][0], o, 0, 0, 0);
+      o2 = __builtin_amdgcn_mfma_f32_16x16x4f32(x.r[i][1], S[i][1], o2, 0, 0, 0);
+      o = __builtin_amdgcn_mfma_f32_16x16x4f32(x.r[i][2], S[i][2], o, 0, 0, 0);
+      o2 = __builtin_amdgcn_mfma_f32_16x16x4f32(x.r[i][3], S[i][3], o2, 0, 0, 0);
     }
 #pragma unroll
-    for (int i = 0; i < TPW; ++i) {
-#pragma unroll
-      for (int j = 0; j < 4; ++j) S[i][j] *= g[i][j];
-    }
+    for (int i = 0; i < TPW; ++i) S[i] *= x.g[i];
 #pragma unroll
     for (int j = 0; j < 4; ++j)
 #pragma unroll
-      for (int i = 0; i < TPW; ++i) S[i] = __builtin_amdgcn_mfma_f32_16x16x4f32(kk[i][j], vv[j], S[i], 0, 0, 0);
-    if (c + 1 < chunks) ask(c + 1);
+      for (int i = 0; i < TPW; ++i)
+        if (EVEN || tile0 + i < tiles) S[i] = __builtin_amdgcn_mfma_f32_16x16x4f32(x.kk[i][j], vv[j], S[i], 0, 0, 0);
+    ask(x, c + AHEAD);
 #pragma unroll
     for (int j = 0; j < 4; ++j) red[c & 1][wave][grp * 4 + j][col] = o[j] + o2[j];
-    __syncthreads();
+    // a barrier for LDS alone: __syncthreads would also wait for the loads that were asked for ahead. A buffer is written
+    // again two chunks later, past the next barrier, which a wave reaches with its reads of the buffer done.
+    asm volatile("s_waitcnt lgkmcnt(0)\n\ts_barrier" ::: "memory");
     const int t = first + c * NHV_CHUNK + (tid >> 4), e = e0 + (tid & 15);
-    if (t < end && e < E) {
-      float sum = 0.f;
+    float sum = 0.f;
 #pragma unroll
-      for (int w = 0; w < 4; ++w) sum += red[c & 1][w][tid >> 4][tid & 15];
-      out[((size_t)t * H + h) * E + e] = sum;
-    }
+    for (int w = 0; w < 4; ++w) sum += red[c & 1][w][tid >> 4][tid & 15];
+    if (t < end && e < E) out[((size_t)t * H + h) * E + e] = sum;
+  };
+#pragma unroll
+  for (int i = 0; i < AHEAD; ++i) ask(ops[i], i);
+  int c = 0;
+  for (; c + AHEAD <= chunks; c += AHEAD) {
+#pragma unroll
+    for (int i = 0; i < AHEAD; ++i) step(ops[i], c + i);
   }
+#pragma unroll
+  for (int i = 0; i < AHEAD - 1; ++i)
+    if (c + i < chunks) step(ops[i], c + i);
 #pragma unroll
   for (int i = 0; i < TPW; ++i)
 #pragma unroll
@@ -353,13 +418,14 @@ __global__ __launch_bounds__(256) void recurrence_chunks_kernel(const float* __r
 
 // ---------------------------------------------------------------- steps of a few tokens a request: one launch
 // A block per (head, request). Token by token: the token's vectors go to LDS (turned; decays worked out), then every column
-// of S meets them: a column belongs to R adjacent lanes of 16 entries each, columns beyond the block's lanes come in
-// further passes; then the read-outs' norm and gate.
+// of S meets them: a column belongs to R adjacent lanes of 16 entries each (in fours, the lanes' fours side by side: a load
+// takes whole lines), columns beyond the block's lanes come in further passes; then the read-outs' norm and gate.
 template <typename T, typename TW, typename TO, int KIND, int R>
 __global__ __launch_bounds__(1024) void recurrence_tokens_kernel(const RecurrenceIn in, float* __restrict__ state,
                                                                  const float* __restrict__ norm_w, float eps, TO* __restrict__ y,
                                                                  const int* __restrict__ positions, const int* __restrict__ cu,
-                                                                 const int* __restrict__ state_slots, int H, int D, int E) {
+                                                                 const int* __restrict__ state_slots, int H, int D, int E,
+                                                                 int whole_rank) {
   extern __shared__ __attribute__((aligned(16))) float lds[];
   __shared__ float scratch[16];
   const int req = blockIdx.y, h = blockIdx.x;
@@ -379,30 +445,63 @@ __global__ __launch_bounds__(1024) void recurrence_tokens_kernel(const Recurrenc
     const T* q = (const T*)in.q + (size_t)t * in.ld + (size_t)h * D;
     const T* k = (const T*)in.k + (size_t)t * in.ld + (size_t)h * D;
     float bonus = 0.f;                       // this thread's share of what the token's own k v^T counts for
+    // the first columns' state is asked for before anything else
+    const bool fresh = t == first && positions[t] == 0;
+    const int cols = threads / R, part = tid % R;
+    float S[16];
+    auto take = [&](int e0) {
+      const int e = e0 + tid / R;
+      const float* from = head + (size_t)(e < E ? e : 0) * D + part * 4;
+      const bool there = !fresh && e < E && tid / R < cols;
+#pragma unroll
+      for (int i = 0; i < 16; i += 4) {
+        const int d = part * 4 + i * R;
+        if (whole4) {
+          const float4 s4 = (there && d < D) ? *reinterpret_cast<const float4*>(from + i * R) : float4{0.f, 0.f, 0.f, 0.f};
+          S[i] = s4.x; S[i + 1] = s4.y; S[i + 2] = s4.z; S[i + 3] = s4.w;
+        } else {
+#pragma unroll
+          for (int j = 0; j < 4; ++j) S[i + j] = (there && d + j < D) ? from[i * R + j] : 0.f;
+        }
+      }
+    };
+    take(0);
+    // and so are the first columns' value, and the gates and norm weights that the results meet at the end
+    const T* v_row = (const T*)in.v + (size_t)t * in.ld + (size_t)h * E;
+    const T* g_row = (const T*)in.g + (size_t)t * in.ld + (size_t)h * E;
+    const bool column0 = tid / R < cols && tid / R < E;
+    const T v_first = v_row[column0 ? tid / R : 0], g_first = g_row[tid < E ? tid : 0];
+    const float w_first = norm_w ? norm_w[(size_t)h * E + (tid < E ? tid : 0)] : 1.0f;
     if (KIND == 1) {
       for (int r = tid; r < in.rank; r += threads) zs[r] = tanhf(in.z[(size_t)t * in.z_ld + r]);
       __syncthreads();
-      // four lanes a channel
-      for (int x = tid; x < Dl * 4; x += threads) {
-        const int d = x >> 2;
-        float sum = 0.f;
+      // eight lanes a channel, each four of 32 entries at a time
+      for (int x = tid; x < Dl * 8; x += threads) {
+        const int d = x >> 3;
+        float sum = 0.f, rr = 0.f, kk = 0.f, w0 = 0.f, u = 0.f;
         if (d < D) {
+          if ((x & 7) == 0) {
+            rr = to_f32(q[d]);
+            kk = to_f32(k[d]);
+            w0 = in.w0[h * D + d];
+            u = in.u[h * D + d];
+          }
           const TW* w2 = (const TW*)in.w2 + ((size_t)h * D + d) * in.rank;
-#pragma unroll 4
-          for (int r = x & 3; r < in.rank; r += 4) sum = fmaf(to_f32(w2[r]), zs[r], sum);
+#pragma unroll 2
+          for (int r = (x & 7) * 4; r < in.rank; r += 32) {
+            const floatx4 w = four_of(w2 + r, in.rank - r, whole_rank);
+#pragma unroll
+            for (int i = 0; i < 4; ++i) sum = fmaf(w[i], r + i < in.rank ? zs[r + i] : 0.f, sum);
+          }
         }
         sum += __shfl_xor(sum, 1, NHV_WAVE);
         sum += __shfl_xor(sum, 2, NHV_WAVE);
-        if ((x & 3) == 0) {
-          float rr = 0.f, kk = 0.f;
-          if (d < D) {
-            rr = to_f32(q[d]);
-            kk = to_f32(k[d]);
-            bonus = fmaf(rr * in.u[h * D + d], kk, bonus);
-          }
+        sum += __shfl_xor(sum, 4, NHV_WAVE);
+        if ((x & 7) == 0) {
+          bonus = fmaf(rr * u, kk, bonus);
           qs[d] = rr;
           ks[d] = kk;
-          gs[d] = d < D ? exp2_of(-NHV_LOG2E * expf(sum + in.w0[h * D + d])) : 0.f;
+          gs[d] = d < D ? exp2_of(-NHV_LOG2E * expf(sum + w0)) : 0.f;
         }
       }
     } else {
@@ -429,30 +528,17 @@ __global__ __launch_bounds__(1024) void recurrence_tokens_kernel(const Recurrenc
       }
     }
     bonus = block_sum(bonus, scratch);       // (its barriers also make the vectors visible)
-    const bool fresh = t == first && positions[t] == 0;
-    const int cols = threads / R, part = tid % R;
     float ss = 0.f;
     for (int e0 = 0; e0 < E; e0 += cols) {
       const int e = e0 + tid / R;
       const bool column = e < E && tid / R < cols;
-      float* mine = head + (size_t)(column ? e : 0) * D + part * 16;
-      float S[16];
-#pragma unroll
-      for (int i = 0; i < 16; i += 4) {
-        const int d = part * 16 + i;
-        if (whole4) {
-          const float4 s4 = (!fresh && column && d < D) ? *reinterpret_cast<const float4*>(mine + i) : float4{0.f, 0.f, 0.f, 0.f};
-          S[i] = s4.x; S[i + 1] = s4.y; S[i + 2] = s4.z; S[i + 3] = s4.w;
-        } else {
-#pragma unroll
-          for (int j = 0; j < 4; ++j) S[i + j] = (!fresh && column && d + j < D) ? mine[i + j] : 0.f;
-        }
-      }
-      const float vv = column ? to_f32(((const T*)in.v)[(size_t)t * in.ld + (size_t)h * E + e]) : 0.f;
+      float* mine = head + (size_t)(column ? e : 0) * D + part * 4;
+      if (e0 > 0) take(e0);
+      const float vv = !column ? 0.f : e0 == 0 ? to_f32(v_first) : to_f32(v_row[e]);
       float sum = 0.f;
 #pragma unroll
       for (int i = 0; i < 16; i += 4) {
-        const int d = part * 16 + i;
+        const int d = part * 4 + i * R;
         const float4 q4 = *reinterpret_cast<const float4*>(&qs[d]), k4 = *reinterpret_cast<const float4*>(&ks[d]),
                      g4 = *reinterpret_cast<const float4*>(&gs[d]);
         sum = fmaf(q4.x, S[i], fmaf(q4.y, S[i + 1], fmaf(q4.z, S[i + 2], fmaf(q4.w, S[i + 3], sum))));
@@ -467,13 +553,13 @@ __global__ __launch_bounds__(1024) void recurrence_tokens_kernel(const Recurrenc
       if (column) {
 #pragma unroll
         for (int i = 0; i < 16; i += 4) {
-          const int d = part * 16 + i;
+          const int d = part * 4 + i * R;
           if (whole4) {
-            if (d < D) *reinterpret_cast<float4*>(mine + i) = float4{S[i], S[i + 1], S[i + 2], S[i + 3]};
+            if (d < D) *reinterpret_cast<float4*>(mine + i * R) = float4{S[i], S[i + 1], S[i + 2], S[i + 3]};
           } else {
 #pragma unroll
             for (int j = 0; j < 4; ++j)
-              if (d + j < D) mine[i + j] = S[i + j];
+              if (d + j < D) mine[i * R + j] = S[i + j];
           }
         }
         if (part == 0) {
@@ -484,8 +570,9 @@ __global__ __launch_bounds__(1024) void recurrence_tokens_kernel(const Recurrenc
     }
     const float inv = 1.0f / sqrtf(block_sum(ss, scratch) / (float)E + eps);
     for (int e = tid; e < E; e += threads) {
-      const float gate = silu_of(to_f32(((const T*)in.g)[(size_t)t * in.ld + (size_t)h * E + e]));
-      y[((size_t)t * H + h) * E + e] = from_f32<TO>(os[e] * inv * (norm_w ? norm_w[(size_t)h * E + e] : 1.0f) * gate);
+      const float z = to_f32(e == tid ? g_first : g_row[e]);
+      const float w = e == tid ? w_first : norm_w ? norm_w[(size_t)h * E + e] : 1.0f;
+      y[((size_t)t * H + h) * E + e] = from_f32<TO>(os[e] * inv * w * silu_of(z));
     }
     __syncthreads();                         // (the next token's vectors take this one's place)
   }
@@ -529,7 +616,7 @@ static RecurrenceIn recurrence_in(const void* q, const void* k, const void* v, c
               name ": %d turned entries of %d", rot, D);                                                                    \
   NHV_REQUIRE(kind == 0 || (z && w2 && w0 && u && rank > 0 && z_ld >= rank), name ": decays of rank %d", rank)
 
-// Chunks' places: T / 16 + B + 1. r_out, k_out [places, H, 16, Dp], a_out [places, H, 16, 16], decay_out [places, H, Dp], Dp the
+// Chunks' places: T / 16 + B + 1. r_out [places, H, 16, Dp], k_out [places, H, Dp, 16], a_out [places, H, 16, 16], decay_out [places, H, Dp], Dp the
 // head size rounded up to a multiple of 16.
 extern "C" int nhv_recurrence_prepare(int kind, const void* q, const void* k, long long ld, int dtype, const void* log2_decay,
                                       const void* freqs, const void* turn_positions, int rot, float k_scale, const void* z,
@@ -542,13 +629,17 @@ extern "C" int nhv_recurrence_prepare(int kind, const void* q, const void* k, lo
   const RecurrenceIn in = recurrence_in(q, k, nullptr, nullptr, ld, log2_decay, freqs, turn_positions, rot, k_scale, z, z_ld, w2,
                                         rank, w0, u);
   const int Dp = (D + 15) / 16 * 16;
-  const size_t lds = ((((kind == 1 ? 3 : 2) * NHV_CHUNK * (size_t)(D | 1)) + 3) / 4 * 4 +
-                      (kind == 1 ? NHV_CHUNK * (NHV_RANK_PIECE + 4) : 0)) * sizeof(float);
-  const dim3 grid((max_q_len + NHV_CHUNK - 1) / NHV_CHUNK, H, B);
+  const size_t lds = (size_t)(kind == 1 ? 3 : 2) * NHV_CHUNK * (Dp + 4) * sizeof(float);
+  const int chunks = (max_q_len + NHV_CHUNK - 1) / NHV_CHUNK;
+  NHV_REQUIRE(chunks <= 65535, "recurrence_prepare: a portion of %d tokens is beyond this kernel's grid", max_q_len);
+  const dim3 grid(H, chunks, B);
+  const size_t item = dtype == NHV_F32 ? 4 : 2, w_item = w2_dtype == NHV_F32 ? 4 : 2;
+  const int whole = D % 4 == 0 && ld % 4 == 0 && (((uintptr_t)q | (uintptr_t)k) % (4 * item)) == 0;
+  const int whole_rank = rank % 4 == 0 && (uintptr_t)w2 % (4 * w_item) == 0;
   hipStream_t s = (hipStream_t)stream;
 #define LAUNCH(TT, TTW, KIND)                                                                                            \
   hipLaunchKernelGGL((recurrence_prepare_kernel<TT, TTW, KIND>), grid, dim3(256), lds, s, in, (float*)r_out, (float*)k_out, \
-                     (float*)a_out, (float*)decay_out, (const int*)cu, H, D, Dp)
+                     (float*)a_out, (float*)decay_out, (const int*)cu, H, D, Dp, whole, whole_rank)
   if (kind == 0) { if (dtype == NHV_F32) LAUNCH(float, float, 0); else LAUNCH(bf16_t, bf16_t, 0); }
   else if (w2_dtype == NHV_F32) { if (dtype == NHV_F32) LAUNCH(float, float, 1); else LAUNCH(bf16_t, float, 1); }
   else if (w2_dtype == NHV_BF16) { if (dtype == NHV_F32) LAUNCH(float, bf16_t, 1); else LAUNCH(bf16_t, bf16_t, 1); }
@@ -564,21 +655,24 @@ extern "C" int nhv_recurrence_chunks(const void* r_in, const void* k_in, const v
   NHV_REQUIRE(B > 0 && H > 0 && D > 0 && E > 0 && B <= 65535 && H <= 65535 && D <= 256 && ld >= (long long)H * E,
               "recurrence_chunks: bad sizes B=%d H=%d D=%d (up to 256) E=%d, rows of %lld", B, H, D, E, ld);
   const int Dp = (D + 15) / 16 * 16, tpw = (Dp / 16 + 3) / 4;
-  const dim3 grid((E + 15) / 16, H, B);
+  const dim3 grid(H, (E + 15) / 16, B);
   hipStream_t s = (hipStream_t)stream;
-#define LAUNCH(TT, N)                                                                                                     \
-  hipLaunchKernelGGL((recurrence_chunks_kernel<TT, N>), grid, dim3(256), 0, s, (const float*)r_in, (const float*)k_in,    \
+#define LAUNCH(TT, N, EVEN)                                                                                                  \
+  hipLaunchKernelGGL((recurrence_chunks_kernel<TT, N, EVEN>), grid, dim3(256), 0, s, (const float*)r_in, (const float*)k_in,    \
                      (const float*)a_in, (const float*)decay_in, (const TT*)v, ld, (float*)state, (float*)out,            \
                      (const int*)positions, (const int*)cu, (const int*)state_slots, H, D, Dp, E)
-#define BY_TILES(TT)          \
-  if (tpw == 1) LAUNCH(TT, 1); \
-  else if (tpw == 2) LAUNCH(TT, 2); \
-  else if (tpw == 3) LAUNCH(TT, 3); \
-  else LAUNCH(TT, 4)
+  const bool even = Dp / 16 == 4 * tpw;
+#define BY_EVEN(TT, N) { if (even) LAUNCH(TT, N, true); else LAUNCH(TT, N, false); }
+#define BY_TILES(TT)            \
+  if (tpw == 1) BY_EVEN(TT, 1)  \
+  else if (tpw == 2) BY_EVEN(TT, 2) \
+  else if (tpw == 3) BY_EVEN(TT, 3) \
+  else BY_EVEN(TT, 4)
   if (dtype == NHV_F32) { BY_TILES(float); }
   else if (dtype == NHV_BF16) { BY_TILES(bf16_t); }
   else return nhv_fail("recurrence_chunks: unknown dtype %d", dtype);
 #undef BY_TILES
+#undef BY_EVEN
 #undef LAUNCH
   NHV_LAUNCH_CHECK("recurrence_chunks");
   return 0;
@@ -600,11 +694,12 @@ extern "C" int nhv_recurrence_tokens(int kind, const void* q, const void* k, con
   if (threads < 128) threads = 128;
   const size_t lds = (3 * (size_t)R * 16 + E + (kind == 1 ? rank : 0)) * sizeof(float);
   NHV_REQUIRE(lds <= 60 * 1024, "recurrence_tokens: value heads of %d and decays of rank %d are beyond this kernel", E, rank);
+  const int whole_rank = rank % 4 == 0 && (uintptr_t)w2 % (w2_dtype == NHV_F32 ? 16 : 8) == 0;
   const dim3 grid(H, B);
   hipStream_t s = (hipStream_t)stream;
 #define LAUNCH(TT, TTW, TTO, KIND, RR)                                                                                      \
   hipLaunchKernelGGL((recurrence_tokens_kernel<TT, TTW, TTO, KIND, RR>), grid, dim3(threads), lds, s, in, (float*)state,    \
-                     (const float*)norm_w, eps, (TTO*)y, (const int*)positions, (const int*)cu, (const int*)state_slots, H, D, E)
+                     (const float*)norm_w, eps, (TTO*)y, (const int*)positions, (const int*)cu, (const int*)state_slots, H, D, E, whole_rank)
 #define BY_R(TT, TTW, TTO, KIND)                       \
   switch (R) {                                         \
     case 1: LAUNCH(TT, TTW, TTO, KIND, 1); break;      \

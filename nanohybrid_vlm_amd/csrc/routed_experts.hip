@@ -633,9 +633,54 @@ __global__ void experts_combine_kernel(const float* __restrict__ y, bf16_t* __re
   }
 }
 
+// The same four entries at a time (rows of a multiple of four); blockIdx.y walks over tokens.
+__global__ __launch_bounds__(256) void experts_combine_vec_kernel(const float* __restrict__ y, bf16_t* __restrict__ out, int W, int top,
+                                                                  int T, const float* __restrict__ weights,
+                                                                  const bf16_t* __restrict__ add, const int* __restrict__ ids, int E,
+                                                                  const bf16_t* __restrict__ self) {
+  struct alignas(8) Pack { bf16_t e[4]; };
+  const int n = (blockIdx.x * 256 + threadIdx.x) * 4;
+  if (n >= W) return;
+  for (int t = blockIdx.y; t < T; t += gridDim.y) {
+    const size_t at = (size_t)t * W + n;
+    floatx4 sum = {0.f, 0.f, 0.f, 0.f};
+    for (int j = 0; j < top; ++j) {
+      const size_t pair = (size_t)t * top + j;
+      floatx4 v;
+      if (self && ids[pair] >= E) {
+        const Pack p = *reinterpret_cast<const Pack*>(self + at);
+#pragma unroll
+        for (int i = 0; i < 4; ++i) v[i] = (float)p.e[i];
+      } else {
+        v = *reinterpret_cast<const floatx4*>(y + pair * W + n);
+      }
+      const float w = weights ? weights[pair] : 1.0f;
+#pragma unroll
+      for (int i = 0; i < 4; ++i) sum[i] += weights ? w * v[i] : v[i];
+    }
+    Pack o;
+    if (add) {
+      const Pack p = *reinterpret_cast<const Pack*>(add + at);
+#pragma unroll
+      for (int i = 0; i < 4; ++i) sum[i] += (float)p.e[i];
+    }
+#pragma unroll
+    for (int i = 0; i < 4; ++i) o.e[i] = (bf16_t)sum[i];
+    *reinterpret_cast<Pack*>(out + at) = o;
+  }
+}
+
 extern "C" int nhv_experts_combine(const void* y, void* out, int T, int W, int top, const void* weights, const void* add,
                                    const void* ids, int E, const void* self, void* stream) {
   NHV_REQUIRE(T > 0 && W > 0 && top > 0, "experts_combine: bad sizes T=%d W=%d top=%d", T, W, top);
+  NHV_REQUIRE(!self || ids, "experts_combine: identity experts are told by their numbers");
+  if (W % 4 == 0 && (((uintptr_t)y % 16) | (((uintptr_t)out | (uintptr_t)add | (uintptr_t)self) % 8)) == 0) {
+    hipLaunchKernelGGL(experts_combine_vec_kernel, dim3((W / 4 + 255) / 256, T < 65535 ? T : 65535), dim3(256), 0, (hipStream_t)stream,
+                       (const float*)y, (bf16_t*)out, W, top, T, (const float*)weights, (const bf16_t*)add, (const int*)ids, E,
+                       (const bf16_t*)self);
+    NHV_LAUNCH_CHECK("experts_combine");
+    return 0;
+  }
   const size_t total = (size_t)T * W;
   const int blocks = (int)((total + 255) / 256 > 65535 * 4 ? 65535 * 4 : (total + 255) / 256);
   hipLaunchKernelGGL(experts_combine_kernel, dim3(blocks), dim3(256), 0, (hipStream_t)stream, (const float*)y, (bf16_t*)out,

@@ -421,6 +421,84 @@ __global__ __launch_bounds__(256) void normed_split_write_kernel(const T* __rest
     for (int c = threadIdx.x; c < Hkv * E; c += 256) v_cache[(size_t)slot * Hkv * E + c] = from_f32<T>(value(nq + nk + c));
 }
 
+// The same where heads and halves are whole pieces of eight entries: a thread moves eight entries at a time, the row waits in
+// LDS as floats for its sums of squares (a pair's two entries lie in different threads' pieces).
+template <typename T>
+__global__ __launch_bounds__(1024) void normed_split_write_vec_kernel(const T* __restrict__ qkv, int ld, const T* __restrict__ bias,
+                                                                      const float* __restrict__ wq, const float* __restrict__ wk,
+                                                                      float eps, const double* __restrict__ freqs, int rot,
+                                                                      float gain, const int* __restrict__ positions,
+                                                                      const int* __restrict__ slot_mapping, T* __restrict__ q_out,
+                                                                      T* __restrict__ k_cache, T* __restrict__ v_cache, int nq,
+                                                                      int nk, int nv, int D, int v_from_k) {
+  struct alignas(sizeof(T) * 8) Pack { T e[8]; };
+  extern __shared__ __attribute__((aligned(16))) float row_s[];      // nq + nk values, then rot / 2 sines and as many cosines
+  __shared__ float scratch[16];
+  const int t = blockIdx.x, half = rot / 2, n = nq + nk, threads = blockDim.x;
+  float* sines = row_s + n;
+  float* cosines = sines + half;
+  const T* row = qkv + (size_t)t * ld;
+  const int slot = slot_mapping[t];
+  float sq = 0.f, sk = 0.f;
+  for (int c = threadIdx.x * 8; c < n + nv; c += threads * 8) {
+    float v[8];
+    split_load8(row + c, v);
+    if (bias) {
+      float b[8];
+      split_load8(bias + c, b);
+#pragma unroll
+      for (int i = 0; i < 8; ++i) v[i] += b[i];
+    }
+    float ss = 0.f;
+#pragma unroll
+    for (int i = 0; i < 8; ++i) ss = fmaf(v[i], v[i], ss);
+    if (c < nq) sq += ss;
+    else if (c < n) sk += ss;
+    if (c < n) {
+      *reinterpret_cast<float4*>(row_s + c) = float4{v[0], v[1], v[2], v[3]};
+      *reinterpret_cast<float4*>(row_s + c + 4) = float4{v[4], v[5], v[6], v[7]};
+    }
+    if (slot >= 0 && (v_from_k ? (c >= nq && c < n) : c >= n)) {     // (a row that stores nothing: padding of a recorded step)
+      Pack out;
+#pragma unroll
+      for (int i = 0; i < 8; ++i) out.e[i] = from_f32<T>(v[i]);
+      *reinterpret_cast<Pack*>(v_cache + (v_from_k ? (size_t)slot * nk + (c - nq) : (size_t)slot * nv + (c - n))) = out;
+    }
+  }
+  for (int i = threadIdx.x; i < half; i += threads) nhv_turn_angle<float>(positions[t], freqs[i], gain, &sines[i], &cosines[i]);
+  const float rq = 1.0f / sqrtf(block_sum(sq, scratch) / (float)nq + eps);
+  const float rk = 1.0f / sqrtf(block_sum(sk, scratch) / (float)nk + eps);    // (its barriers show the row and the sines as well)
+  for (int c = threadIdx.x * 8; c < (slot < 0 ? nq : n); c += threads * 8) {
+    const bool key = c >= nq;
+    const int in_head = c % D;
+    const float* w = key ? wk + (c - nq) : wq + c;
+    const float r = key ? rk : rq;
+    const int other = in_head < half ? half : -half;                 // where the pairs' other entries lie
+    float v[8], wv[8];
+    split_load8(row_s + c, v);
+    split_load8(w, wv);
+#pragma unroll
+    for (int i = 0; i < 8; ++i) v[i] *= r * wv[i];
+    if (in_head < rot) {
+      float x[8], sn[8], cs[8];
+      split_load8(row_s + c + other, x);
+      split_load8(w + other, wv);
+      const int p = in_head < half ? in_head : in_head - half;
+      split_load8(sines + p, sn);
+      split_load8(cosines + p, cs);
+#pragma unroll
+      for (int i = 0; i < 8; ++i) {
+        const float y = x[i] * r * wv[i];
+        v[i] = in_head < half ? v[i] * cs[i] - y * sn[i] : v[i] * cs[i] + y * sn[i];
+      }
+    }
+    Pack out;
+#pragma unroll
+    for (int i = 0; i < 8; ++i) out.e[i] = from_f32<T>(v[i]);
+    *reinterpret_cast<Pack*>(key ? k_cache + (size_t)slot * nk + (c - nq) : q_out + (size_t)t * nq + c) = out;
+  }
+}
+
 extern "C" int nhv_normed_split_write(const void* qkv, long long ld, const void* bias, const void* wq, const void* wk, float eps,
                                       const void* freqs, int rot, float gain, const void* positions, const void* slot_mapping,
                                       void* q_out, void* k_cache, void* v_cache, int T, int Hq, int Hkv, int D, int E,
@@ -431,6 +509,26 @@ extern "C" int nhv_normed_split_write(const void* qkv, long long ld, const void*
   NHV_REQUIRE(ld >= (long long)(Hq + Hkv) * D + (v_from_k ? 0 : Hkv * E) && ld < (1ll << 31), "normed_split_write: rows of %lld entries", ld);
   NHV_REQUIRE(wq && wk && slot_mapping && k_cache && v_cache && eps >= 0.f, "normed_split_write: norm weights, slots and caches are needed");
   hipStream_t s = (hipStream_t)stream;
+  const size_t item = dtype == NHV_F32 ? 4 : 2;
+  const uintptr_t starts = (uintptr_t)qkv | (uintptr_t)bias | (uintptr_t)q_out | (uintptr_t)k_cache | (uintptr_t)v_cache;
+  const uintptr_t w_starts = (uintptr_t)wq | (uintptr_t)wk;
+  const int nq = Hq * D, nk = Hkv * D, nv = v_from_k ? 0 : Hkv * E;
+  const size_t row_lds = ((size_t)nq + nk + rot) * sizeof(float);
+  if (D % 8 == 0 && rot % 16 == 0 && (v_from_k || E % 8 == 0) && ld % 8 == 0 && starts % (8 * item) == 0 && w_starts % 32 == 0 &&
+      row_lds <= 60 * 1024 &&
+      (dtype == NHV_F32 || dtype == NHV_BF16)) {
+    int threads = ((nq + nk + nv) / 8 + 63) / 64 * 64;
+    if (threads > 1024) threads = 1024;
+#define LAUNCH_VEC(TT)                                                                                                    \
+  hipLaunchKernelGGL(normed_split_write_vec_kernel<TT>, dim3(T), dim3(threads), row_lds, s, (const TT*)qkv, (int)ld,      \
+                     (const TT*)bias, (const float*)wq, (const float*)wk, eps, (const double*)freqs, rot, gain,           \
+                     (const int*)positions, (const int*)slot_mapping, (TT*)q_out, (TT*)k_cache, (TT*)v_cache, nq, nk, nv, D, v_from_k)
+    if (dtype == NHV_F32) LAUNCH_VEC(float);
+    else LAUNCH_VEC(bf16_t);
+#undef LAUNCH_VEC
+    NHV_LAUNCH_CHECK("normed_split_write_vec");
+    return 0;
+  }
 #define LAUNCH(TT)                                                                                                        \
   hipLaunchKernelGGL(normed_split_write_kernel<TT>, dim3(T), dim3(256), (size_t)rot * sizeof(float), s, (const TT*)qkv, (int)ld, \
                      (const TT*)bias, (const float*)wq, (const float*)wk, eps, (const double*)freqs, rot, gain,           \
