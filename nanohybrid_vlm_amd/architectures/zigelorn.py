@@ -206,8 +206,9 @@ def parse_config(raw: dict, shapes: dict | None = None) -> ZigelornConfig:
             raise ConfigError(f"{_where(i, 'mixer')} is missing")
         if j is not None and (not isinstance(j, int) or isinstance(j, bool) or not 0 <= j < i or layers[j].weights_of is not None):
             raise ConfigError(f"{_where(i, 'weights_of')}: {j!r} must name an earlier layer with tensors of its own")
-        mixer, mlp = _MIXERS[kind](i if j is None else j, m, shapes), _mlp(i, entry.get("mlp"))
-        if j is not None and (kind, mixer, mlp) != (layers[j].type, layers[j].mixer, layers[j].mlp):
+        mlp, same = _mlp(i, entry.get("mlp")), j is None or kind == layers[j].type
+        mixer = _MIXERS[kind](i if j is None else j, m, shapes) if same else None
+        if j is not None and (not same or (mixer, mlp) != (layers[j].mixer, layers[j].mlp)):
             raise ConfigError(f"{_where(i, 'weights_of')}: the entry must equal layer {j}'s, whose weights it runs")
         spare = tuple(n for n in ("norm2", "norm2b") if mlp is None and j is None and shapes is not None and f"l{i}.{n}" in shapes)
         layers.append(LayerSizes(kind, mixer, mlp, j, spare))
