@@ -204,8 +204,10 @@ def parse_config(raw: dict, shapes: dict | None = None) -> ZigelornConfig:
             raise ConfigError(f"{_where(i, 'type')}: {kind!r} is not known ({sorted(_MIXERS)} are)")
         if not isinstance(m, dict):
             raise ConfigError(f"{_where(i, 'mixer')} is missing")
-        if j is not None and (not isinstance(j, int) or isinstance(j, bool) or not 0 <= j < i or layers[j].weights_of is not None):
-            raise ConfigError(f"{_where(i, 'weights_of')}: {j!r} must name an earlier layer with tensors of its own")
+        if j is not None and (not isinstance(j, int) or isinstance(j, bool) or not 0 <= j < i):
+            raise ConfigError(f"{_where(i, 'weights_of')}: {j!r} must name an earlier layer")
+        if j is not None and layers[j].weights_of is not None:
+            j = layers[j].weights_of                         # (a layer that itself runs another one's weights: that one's)
         mlp, same = _mlp(i, entry.get("mlp")), j is None or kind == layers[j].type
         mixer = _MIXERS[kind](i if j is None else j, m, shapes) if same else None
         if j is not None and (not same or (mixer, mlp) != (layers[j].mixer, layers[j].mlp)):

@@ -345,23 +345,47 @@ __global__ __launch_bounds__(256, 2) void recurrence_chunks_kernel(const float* 
   const int chunks = (end - first + NHV_CHUNK - 1) / NHV_CHUNK;
   const size_t place0 = (size_t)(first / NHV_CHUNK) + req;
   ChunkOperands<T, TPW> ops[AHEAD];
-  const T* vcol = v + (size_t)h * E + e0 + (column ? col : 0);      // (a lane beyond E works on a column that it does not write)
-  auto ask = [&](ChunkOperands<T, TPW>& x, int c) {
+  // what a lane reads of a chunk lies at offsets that do not change, from bases that are the same for the whole block
+  const int r_at = col * Dp + tile0 * 16 + grp * 4, k_at = (tile0 * 16 + col) * NHV_CHUNK + grp * 4, g_at = tile0 * 16 + grp * 4;
+  const int a_at = col * 16 + grp * 4 + wave;
+  const int spare = (EVEN ? 0 : tiles) - 1;  // (a wave without a tile reads the last one's and leaves it unused)
+  const T* vbase = v + (size_t)first * ld + (size_t)h * E + e0;
+  const int row = (int)ld, vlast = (end - first - 1) * row + (column ? col : 0);       // (a lane beyond E works on a column that it does not write)
+  int v_at[4], v_mine_at = (grp * 4 + wave) * row + (column ? col : 0);
+#pragma unroll
+  for (int j = 0; j < 4; ++j) v_at[j] = (grp * 4 + j) * row + (column ? col : 0);
+  auto ask = [&](ChunkOperands<T, TPW>& x, int c) {      // (in the order of the chunks)
     c = min(c, chunks - 1);                  // (always asked, so that the loop's waits count the same loads on every way)
     const size_t place = (place0 + c) * H + h;
-    const int t0 = first + c * NHV_CHUNK;
+    const float* rb = r_in + place * NHV_CHUNK * Dp;
+    const float* kb = k_in + place * NHV_CHUNK * Dp;
+    const float* gb = decay_in + place * Dp;
 #pragma unroll
     for (int i = 0; i < TPW; ++i) {
-      const int d = (EVEN ? tile0 + i : min(tile0 + i, tiles - 1)) * 16;      // (a wave without a tile leaves it unused)
-      x.r[i] = *reinterpret_cast<const floatx4*>(r_in + (place * NHV_CHUNK + col) * Dp + d + grp * 4);
-      x.g[i] = *reinterpret_cast<const floatx4*>(decay_in + place * Dp + d + grp * 4);
-      x.kk[i] = *reinterpret_cast<const floatx4*>(k_in + (place * Dp + d + col) * NHV_CHUNK + grp * 4);
+      const int back = EVEN ? 0 : max(tile0 + i - spare, 0);
+      x.r[i] = *reinterpret_cast<const floatx4*>(rb + (r_at + (i - back) * 16));
+      x.g[i] = *reinterpret_cast<const floatx4*>(gb + (g_at + (i - back) * 16));
+      x.kk[i] = *reinterpret_cast<const floatx4*>(kb + (k_at + (i - back) * 16 * NHV_CHUNK));
     }
     // (rows beyond the request meet zeros in A and K: the request's last row stands in for them)
 #pragma unroll
-    for (int j = 0; j < 4; ++j) x.v[j] = vcol[(size_t)min(t0 + grp * 4 + j, end - 1) * ld];
-    x.v_mine = vcol[(size_t)min(t0 + grp * 4 + wave, end - 1) * ld];
-    x.a = a_in[place * 256 + col * 16 + grp * 4 + wave];
+    for (int j = 0; j < 4; ++j) {
+      x.v[j] = vbase[min(v_at[j], vlast)];
+      v_at[j] += NHV_CHUNK * row;
+    }
+    x.v_mine = vbase[min(v_mine_at, vlast)];
+    v_mine_at += NHV_CHUNK * row;
+    x.a = a_in[place * 256 + a_at];
+  };
+  const int o_at = (tid >> 4) * H * E + (tid & 15);
+  // the waves' shares of chunk c added up and written
+  auto emit = [&](int c) {
+    const int t = first + c * NHV_CHUNK + (tid >> 4), e = e0 + (tid & 15);
+    float sum = 0.f;
+#pragma unroll
+    for (int w = 0; w < 4; ++w) sum += red[c & 1][w][tid >> 4][tid & 15];
+    float* ob = out + ((size_t)(first + c * NHV_CHUNK) * H + h) * E + e0;
+    if (t < end && e < E) ob[o_at] = sum;
   };
   auto step = [&](ChunkOperands<T, TPW>& x, int c) {
     float vv[4];
@@ -386,16 +410,12 @@ __global__ __launch_bounds__(256, 2) void recurrence_chunks_kernel(const float* 
       for (int i = 0; i < TPW; ++i)
         if (EVEN || tile0 + i < tiles) S[i] = __builtin_amdgcn_mfma_f32_16x16x4f32(x.kk[i][j], vv[j], S[i], 0, 0, 0);
     ask(x, c + AHEAD);
+    if (c > 0) emit(c - 1);                  // (while the products are under way)
 #pragma unroll
     for (int j = 0; j < 4; ++j) red[c & 1][wave][grp * 4 + j][col] = o[j] + o2[j];
-    // a barrier for LDS alone: __syncthreads would also wait for the loads that were asked for ahead. A buffer is written
-    // again two chunks later, past the next barrier, which a wave reaches with its reads of the buffer done.
+    // a barrier for LDS alone: __syncthreads would also wait for the loads that were asked for ahead. A buffer's sums are read
+    // in the step after (below), before that step's barrier, and written again only behind it.
     asm volatile("s_waitcnt lgkmcnt(0)\n\ts_barrier" ::: "memory");
-    const int t = first + c * NHV_CHUNK + (tid >> 4), e = e0 + (tid & 15);
-    float sum = 0.f;
-#pragma unroll
-    for (int w = 0; w < 4; ++w) sum += red[c & 1][w][tid >> 4][tid & 15];
-    if (t < end && e < E) out[((size_t)t * H + h) * E + e] = sum;
   };
 #pragma unroll
   for (int i = 0; i < AHEAD; ++i) ask(ops[i], i);
@@ -407,6 +427,7 @@ __global__ __launch_bounds__(256, 2) void recurrence_chunks_kernel(const float* 
 #pragma unroll
   for (int i = 0; i < AHEAD - 1; ++i)
     if (c + i < chunks) step(ops[i], c + i);
+  emit(chunks - 1);
 #pragma unroll
   for (int i = 0; i < TPW; ++i)
 #pragma unroll
@@ -651,9 +672,11 @@ extern "C" int nhv_recurrence_prepare(int kind, const void* q, const void* k, lo
 
 extern "C" int nhv_recurrence_chunks(const void* r_in, const void* k_in, const void* a_in, const void* decay_in, const void* v,
                                      long long ld, int dtype, void* state, void* out, const void* positions, const void* cu,
-                                     const void* state_slots, int B, int H, int D, int E, void* stream) {
+                                     const void* state_slots, int B, int H, int D, int E, int max_q_len, void* stream) {
   NHV_REQUIRE(B > 0 && H > 0 && D > 0 && E > 0 && B <= 65535 && H <= 65535 && D <= 256 && ld >= (long long)H * E,
               "recurrence_chunks: bad sizes B=%d H=%d D=%d (up to 256) E=%d, rows of %lld", B, H, D, E, ld);
+  // (offsets of up to four chunks beyond the portion are counted in 32 bits)
+  NHV_REQUIRE(max_q_len > 0 && (max_q_len + 80ll) * ld < (1ll << 31), "recurrence_chunks: a portion of %d rows of %lld entries", max_q_len, ld);
   const int Dp = (D + 15) / 16 * 16, tpw = (Dp / 16 + 3) / 4;
   const dim3 grid(H, (E + 15) / 16, B);
   hipStream_t s = (hipStream_t)stream;

@@ -485,7 +485,7 @@ class NativeBackend:
                    _stream())
         self._call("nhv_recurrence_chunks", _ptr(r_s), _ptr(k_s), _ptr(a), _ptr(decay), _ptr(v), ctypes.c_longlong(v.stride(0)),
                    dtype_code(v), _ptr(state), _ptr(out), _ptr(batch.positions), _ptr(batch.cu_seqlens_q), _ptr(state_slots), B,
-                   H, D, E, _stream())
+                   H, D, E, max(1, batch.max_q_len), _stream())
 
     def readout_norm(self, o, gate, w, y, eps):
         T, H, E = o.shape

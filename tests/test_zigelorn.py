@@ -464,7 +464,10 @@ def test_configuration_and_names():
     cfg = arch.parse_config(zc.CONFIG_A, spare)
     assert set(arch.checkpoint_names(cfg)) == set(spare)
     assert {s.param for s in arch.checkpoint_names(cfg).values()} == set(DecoderModel(arch.build_spec(cfg)).all_param_specs())
-    for change, match in ((lambda c: c["layers"][5].update(weights_of=3), "weights_of"),
+    chain = json.loads(json.dumps(zc.CONFIG_A))
+    chain["layers"].append(dict(chain["layers"][3], weights_of=3))                # (layer 3 itself runs layer 1's weights)
+    assert arch.parse_config(chain, shapes).layers[6].weights_of == 1
+    for change, match in ((lambda c: c["layers"][5].update(weights_of=5), "weights_of"),
                           (lambda c: c["layers"][5].update(weights_of=1), "must equal"),
                           (lambda c: c["layers"][1].update(type="other"), "not known"),
                           (lambda c: c["layers"][1]["mixer"]["rot"].update(dims=3), "rot.dims"),
