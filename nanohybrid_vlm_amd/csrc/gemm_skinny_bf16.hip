@@ -21,11 +21,12 @@ __device__ __forceinline__ bf16x8 sk_zero8() {
 
 // For 17 to 64 rows of x the rows of x are the larger share of what a wave loads, so here a wave keeps NT
 // tiles of 16 rows of w (and with GLU their partners in the second matrix) against the same rows of x:
-// every load of x serves NT (2 NT) products. The partial sums of the waves meet in LDS one tile at a time.
-template <int MT, int NT, int WAVES, int UNROLL, bool GLU, typename TOut>
+// every load of x serves NT (2 NT) products. The partial sums of the waves meet in LDS one tile at a time. BANDED: x holds
+// several sets of M rows and a block's outputs are made from the set of their band (nhv_gemm_fusion.h).
+template <int MT, int NT, int WAVES, int UNROLL, bool GLU, bool BANDED, typename TOut>
 __global__ __launch_bounds__(64 * WAVES) void gemm_mid_kernel(const bf16_t* __restrict__ x, const bf16_t* __restrict__ w,
                                                               const bf16_t* __restrict__ bias, TOut* __restrict__ y,
-                                                              int M, int N, int K) {
+                                                              int M, int N, int K, int band_rows, int bands) {
   constexpr int NA = GLU ? 2 : 1;
   constexpr int TILES = NA * NT;
   static_assert(MT <= WAVES, "each of the first MT waves finishes one tile of rows of x");
@@ -33,6 +34,7 @@ __global__ __launch_bounds__(64 * WAVES) void gemm_mid_kernel(const bf16_t* __re
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
   const int col = lane & 15, grp = lane >> 4;
   const int n0 = blockIdx.x * 16 * NT;
+  if (BANDED) x += (size_t)min(n0 / band_rows, bands - 1) * M * K;
   const bf16_t* wrow[TILES];
   bool n_ok[NT];
 #pragma unroll
@@ -120,11 +122,11 @@ static void mid_launch(hipStream_t s, const void* x, const void* w, const void* 
   constexpr int WAVES = 8, UNROLL = 2;
   const unsigned blocks = (unsigned)((N + 16 * NT - 1) / (16 * NT));
   if (out_dtype == NHV_BF16)
-    hipLaunchKernelGGL((gemm_mid_kernel<MT, NT, WAVES, UNROLL, GLU, bf16_t>), dim3(blocks), dim3(64 * WAVES), 0, s,
-                       (const bf16_t*)x, (const bf16_t*)w, (const bf16_t*)bias, (bf16_t*)y, M, N, K);
+    hipLaunchKernelGGL((gemm_mid_kernel<MT, NT, WAVES, UNROLL, GLU, false, bf16_t>), dim3(blocks), dim3(64 * WAVES), 0, s,
+                       (const bf16_t*)x, (const bf16_t*)w, (const bf16_t*)bias, (bf16_t*)y, M, N, K, 0, 1);
   else
-    hipLaunchKernelGGL((gemm_mid_kernel<MT, NT, WAVES, UNROLL, GLU, float>), dim3(blocks), dim3(64 * WAVES), 0, s,
-                       (const bf16_t*)x, (const bf16_t*)w, (const bf16_t*)bias, (float*)y, M, N, K);
+    hipLaunchKernelGGL((gemm_mid_kernel<MT, NT, WAVES, UNROLL, GLU, false, float>), dim3(blocks), dim3(64 * WAVES), 0, s,
+                       (const bf16_t*)x, (const bf16_t*)w, (const bf16_t*)bias, (float*)y, M, N, K, 0, 1);
 }
 
 // more than 16 rows: how many tiles of w a wave keeps, by how many blocks that leaves for the chip
@@ -206,13 +208,26 @@ extern "C" int nhv_gemm_fewrows_act_bf16(const void* x, const void* w, void* y, 
   return 0;
 }
 
-// y[M, N] for up to 16 rows of each of ``bands`` sets x [bands, M, K]: outputs band_rows s ... band_rows (s + 1) - 1 from set s,
-// the last set's outputs going on to N. band_rows: a multiple of 16.
+// y[M, N] for up to 64 rows of each of ``bands`` sets x [bands, M, K]: outputs band_rows s ... band_rows (s + 1) - 1 from set s,
+// the last set's outputs going on to N. band_rows: a multiple of 16 (of 32 for more than 16 rows).
 extern "C" int nhv_gemm_fewrows_banded_bf16(const void* x, const void* w, void* y, int M, int N, int K, int bands, int band_rows,
                                             int out_dtype, void* stream) {
   if (sk_check("few-rows gemm in bands", x, w, M, N, K, out_dtype)) return 1;
-  NHV_REQUIRE(M <= 16 && bands > 0 && band_rows > 0 && band_rows % 16 == 0 && (long long)band_rows * (bands - 1) < N,
-              "few-rows gemm in bands: %d rows (up to 16), %d bands of %d rows (a multiple of 16) of %d", M, bands, band_rows, N);
+  NHV_REQUIRE(bands > 0 && band_rows > 0 && band_rows % (M <= 16 ? 16 : 32) == 0 && (long long)band_rows * (bands - 1) < N,
+              "few-rows gemm in bands: %d rows, %d bands of %d rows (a multiple of 16, or of 32 for more than 16 rows) of %d", M, bands,
+              band_rows, N);
+  if (M > 16) {
+    const dim3 grid((N + 31) / 32), block(64 * 8);
+    hipStream_t s = (hipStream_t)stream;
+#define LAUNCH(MT, TT)                                                                                                  \
+  hipLaunchKernelGGL((gemm_mid_kernel<MT, 2, 8, 2, false, true, TT>), grid, block, 0, s, (const bf16_t*)x, (const bf16_t*)w, \
+                     (const bf16_t*)nullptr, (TT*)y, M, N, K, band_rows, bands)
+    if (out_dtype == NHV_F32) { if (M <= 32) LAUNCH(2, float); else LAUNCH(4, float); }
+    else { if (M <= 32) LAUNCH(2, bf16_t); else LAUNCH(4, bf16_t); }
+#undef LAUNCH
+    NHV_LAUNCH_CHECK("gemm_mid_banded_bf16");
+    return 0;
+  }
   NhvGemmFusion f = {};
   f.band_rows = band_rows;
   f.bands = bands;

@@ -713,7 +713,9 @@ extern "C" int nhv_recurrence_tokens(int kind, const void* q, const void* k, con
   int R = 1;
   while (R * 16 < D) R <<= 1;
   int threads = (E * R + 63) / 64 * 64;
-  if (threads > 1024) threads = 1024;
+  // (with blocks enough for two a compute unit, smaller ones, so that one's loads fall into the other's waits)
+  const int most = (long long)B * H >= 512 ? 512 : 1024;
+  if (threads > most) threads = most;
   if (threads < 128) threads = 128;
   const size_t lds = (3 * (size_t)R * 16 + E + (kind == 1 ? rank : 0)) * sizeof(float);
   NHV_REQUIRE(lds <= 60 * 1024, "recurrence_tokens: value heads of %d and decays of rank %d are beyond this kernel", E, rank);

@@ -443,9 +443,9 @@ class NativeBackend:
 
     def banded_linear(self, x, w, out, band_rows) -> bool:
         """One product whose outputs are made from several sets of rows (x [sets, rows, in]; ``band_rows`` outputs a set, the
-        last set has the rest), if this batch is one for the few-rows kernel; else False."""
+        last set has the rest), if this batch is one for the kernels of up to 64 rows; else False."""
         sets, M, K = x.shape
-        if not (x.dtype == torch.bfloat16 and M <= self.few_rows and K % 8 == 0 and band_rows % 16 == 0
+        if not (x.dtype == torch.bfloat16 and M <= 64 and K % 8 == 0 and band_rows % (16 if M <= self.few_rows else 32) == 0
                 and x.data_ptr() % 16 == 0 and w.data_ptr() % 16 == 0):
             return False
         self._call("nhv_gemm_fewrows_banded_bf16", _ptr(x), _ptr(w), _ptr(out), M, w.shape[0], K, sets, band_rows,
@@ -1674,8 +1674,8 @@ def _recurrence_batch(name: str, T: int, batch: AttentionBatch, state_slots: tor
 def banded_linear(x: torch.Tensor, w: torch.Tensor, band_rows: int) -> list[torch.Tensor]:
     """One product per set of rows: x [n, rows, in], w [out, in] whose outputs i * band_rows ... belong to set i and all outputs
     from (n - 1) * band_rows on to the last set. Returns n tensors [rows, its outputs] (rows may lie further apart than
-    that; the first n - 1 are alike in type and spacing), the last one float32. Few rows in bfloat16: one kernel, and
-    all of them float32."""
+    that; the first n - 1 are alike in type and spacing), the last one float32. Up to 64 rows in bfloat16: one kernel,
+    and all of them float32."""
     _need(x.dim() == 3 and w.dim() == 2 and x.shape[2] == w.shape[1], lambda: f"banded_linear: x {tuple(x.shape)} and w {tuple(w.shape)}")
     n, M, _ = x.shape
     N, last = w.shape[0], (n - 1) * band_rows

@@ -137,7 +137,8 @@ def test_token_shift(where, kernels, W):
 
 
 @pytest.mark.parametrize("where", WHERE)
-@pytest.mark.parametrize("rows,band,last,K", [(1, 16, 5, 40), (8, 32, 64, 128), (16, 48, 1, 64), (5, 24, 7, 40), (3, 16, 8, 36), (40, 32, 8, 64)])
+@pytest.mark.parametrize("rows,band,last,K", [(1, 16, 5, 40), (8, 32, 64, 128), (16, 48, 1, 64), (5, 24, 7, 40), (3, 16, 8, 36), (40, 32, 8, 64), (17, 64, 3, 200),
+                                                    (64, 32, 40, 72), (20, 48, 8, 64), (65, 32, 4, 64)])
 def test_products_in_bands(where, kernels, rows, band, last, K):
     """Outputs made from several sets of rows, in one kernel for few rows and sizes that it takes, else product by product."""
     device, dtype = where
